@@ -611,6 +611,126 @@ LH_API int lh_flash_attention_windowed_split_into(lh_batch* batch, const lh_buff
                                                   uint32_t num_kv_heads, uint32_t window, uint32_t num_splits);
 LH_API uint32_t lh_flash_split_count(uint32_t eff_seq_len);
 
+/* ---- models with plain bf16 weights (no counterpart in the reference: its decoder has quantized weights only) ----
+ * Weights are bf16 [out, in] row-major; activations and caches are bf16 (LH_BF16) or, for a run in full 32-bit
+ * precision, f32 (LH_F32); the residual stream, norm weights, biases, router logits and recurrent states are f32.
+ *
+ * The columns of a product are described by `count` (1..4) segments: ns[i] columns of the stacked weight matrix each,
+ * with an activation (LH_ACT_*), an output buffer and a layout.  heads[i] / padded[i]: column c of the segment lands at
+ * (c / heads[i]) * padded[i] + c % heads[i] of the output row, so that a head's values can be padded to a multiple the
+ * next kernel wants (equal values: no padding).
+ *   LH_ROWS               output row m is row m
+ *   LH_ROWS_AT_POSITION   output row *position + m (key cache)
+ *   LH_BLOCKS_AT_POSITION value cache: blocks of 32 positions, [block][column][32], the 32 in the order the attention
+ *                         kernels read them
+ * Rows past the end of an output buffer are dropped by the kernel. */
+#define LH_ACT_NONE 0
+#define LH_ACT_SILU 1
+#define LH_ACT_GELU_TANH 2
+#define LH_ACT_RELU_SQUARED 3
+#define LH_ACT_SIGMOID 4
+#define LH_ROWS 0
+#define LH_ROWS_AT_POSITION 1
+#define LH_BLOCKS_AT_POSITION 2
+/* output[r] = table[rows[r]] as f32 (row index clamped to the last row) */
+LH_API int lh_embed_rows_bf16_into(lh_batch* batch, const lh_buffer* table, uint32_t table_rows, uint32_t cols,
+                                   const lh_buffer* rows, uint32_t n_rows, lh_buffer* output);
+/* t = input[row] (+ add[row]), stored to `store` when given (may be `input`); output = t / sqrt(mean(t^2) + eps) * weight.
+ * `row_index` (device u32, may be null) picks the input rows. */
+LH_API int lh_norm_rows_f32_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* add, const lh_buffer* weight,
+                                 lh_buffer* store, const lh_buffer* row_index, lh_buffer* output, int output_dtype,
+                                 uint32_t dim, uint32_t rows, float eps);
+/* output = input / sqrt(mean(input^2) + eps) * weight * sigmoid(gate); input f32, gate and output of `dtype` */
+LH_API int lh_gated_norm_rows_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, const lh_buffer* weight,
+                                   lh_buffer* output, int dtype, uint32_t dim, uint32_t rows, float eps);
+/* output[m] = act(input[m, k] . weight^T + bias) by segments; bias f32 [sum ns] or null.  `accumulate` adds to an f32
+ * output instead of storing. */
+LH_API int lh_linear_rows_into(lh_batch* batch, const lh_buffer* input, int input_dtype, const lh_buffer* weight,
+                               const lh_buffer* bias, uint32_t m, uint32_t k, uint32_t count, const uint32_t* ns,
+                               const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
+                               const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype, int accumulate,
+                               const lh_buffer* position);
+/* The same for one row, with the step before it done while the vector is staged:
+ *   plain   x = input (of input_dtype)
+ *   norm    x = rms_norm(input + add) * norm_weight, input f32, `add` may be null; input + add goes to `store` when given
+ *           (which must not be `input`: every workgroup reads it)
+ *   gated   x = rms_norm(input) * norm_weight * sigmoid(gate), input f32, gate of gate_dtype */
+LH_API int lh_linear_vector_into(lh_batch* batch, const lh_buffer* input, int input_dtype, const lh_buffer* weight,
+                                 const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
+                                 const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
+                                 const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype, int accumulate,
+                                 const lh_buffer* position);
+LH_API int lh_linear_norm_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* add, lh_buffer* store,
+                                      const lh_buffer* norm_weight, float eps, const lh_buffer* weight,
+                                      const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
+                                      const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
+                                      const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
+                                      int accumulate, const lh_buffer* position);
+LH_API int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, int gate_dtype,
+                                       const lh_buffer* norm_weight, float eps, const lh_buffer* weight,
+                                       const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
+                                       const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
+                                       const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
+                                       int accumulate, const lh_buffer* position);
+
+/* Causal softmax attention of `rows` queries at positions *position + r over the caches above, `maps` (1 or 2) score maps
+ * per head over the same values.  q [rows, heads, maps, dim_padded], keys [position, kv_heads, maps, dim_padded] and
+ * values [position / 32, kv_heads, vdim_padded, 32], all of `dtype`; output [rows, heads, vdim].  dim is padded to 32,
+ * 64, 128 or a multiple of 128, vdim to a multiple of 32 (lh_attention_padded_dim / _vdim).
+ *   maps 1: output = the softmax average.
+ *   maps 2 (differential attention): o = a1 - lambda * a2, then o / sqrt(mean(o^2) + eps) * out_scale over the head.
+ * `capacity` positions are held by the caches; `max_position` bounds *position (it sizes the launch; a recorded batch
+ * gives the largest it will be replayed with). */
+LH_API uint32_t lh_attention_padded_dim(uint32_t dim);
+LH_API uint32_t lh_attention_padded_vdim(uint32_t vdim);
+LH_API int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* keys, const lh_buffer* values,
+                                  lh_buffer* output, int dtype, const lh_buffer* position, uint32_t max_position,
+                                  uint32_t rows, uint32_t heads, uint32_t kv_heads, uint32_t maps, uint32_t dim,
+                                  uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps);
+
+/* Linear attention with a fixed decay per head: S = decay * S + k v^T, o = S^T q, token by token from the state left by
+ * the call before.  q, k [rows, heads, dim_padded], v [rows, heads, vdim] of `dtype`; state f32 [heads, vdim, dim_padded]
+ * (read and written); output f32 [rows, heads, vdim].  dim_padded is lh_linear_attention_padded_dim(dim).
+ *   recurrent  one launch that walks the rows; any dtype
+ *   chunked    blocks of 64 rows on the matrix cores: every chunk's contribution to the state, a scan over the chunks,
+ *              then all outputs.  bf16, dim <= 256.  `decay_powers` f32 [heads, 65] holds decay^0 .. decay^64;
+ *              `workspace` takes lh_linear_attention_workspace_bytes. */
+LH_API uint32_t lh_linear_attention_padded_dim(uint32_t dim);
+LH_API size_t lh_linear_attention_workspace_bytes(uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
+LH_API int lh_linear_attention_recurrent_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v,
+                                              int dtype, lh_buffer* state, const lh_buffer* decay, lh_buffer* output,
+                                              uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
+LH_API int lh_linear_attention_chunked_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v,
+                                            lh_buffer* state, const lh_buffer* decay_powers, lh_buffer* workspace,
+                                            lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
+
+/* Mixture of experts: scores = sigmoid(router logits), each row takes the `top` largest (ties: the lower index), weighted
+ * by their scores as they are; the weight multiplies the expert's input.  Experts are stacked, up [experts, ff, width]
+ * and down [experts, width, ff], without biases.
+ *   route   logits f32 [rows, experts] -> the rows grouped by expert: plan u32 [lh_moe_plan_words]
+ *   up      hidden[slot] = act(w * (up[e] . input[row])), one slot per (row, choice), in plan order
+ *   down    residual[row] += sum over the row's slots of down[e] . hidden[slot]
+ *   vector  both for one row: the selection is done by every workgroup from the logits; `input` is normed as in
+ *           lh_linear_norm_vector_into */
+LH_API uint32_t lh_moe_plan_words(uint32_t rows, uint32_t experts, uint32_t top);
+LH_API int lh_moe_route_into(lh_batch* batch, const lh_buffer* logits, lh_buffer* plan, uint32_t rows, uint32_t experts,
+                             uint32_t top);
+LH_API int lh_moe_up_into(lh_batch* batch, const lh_buffer* input, int dtype, const lh_buffer* plan, const lh_buffer* up,
+                          lh_buffer* hidden, uint32_t rows, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff,
+                          uint32_t act);
+LH_API int lh_moe_down_into(lh_batch* batch, const lh_buffer* hidden, int dtype, const lh_buffer* plan,
+                            const lh_buffer* down, lh_buffer* slots, lh_buffer* residual, uint32_t rows, uint32_t experts,
+                            uint32_t top, uint32_t width, uint32_t ff);
+LH_API int lh_moe_vector_up_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* norm_weight, float eps,
+                                 const lh_buffer* logits, const lh_buffer* up, lh_buffer* hidden, uint32_t experts,
+                                 uint32_t top, uint32_t width, uint32_t ff, uint32_t act);
+LH_API int lh_moe_vector_down_into(lh_batch* batch, const lh_buffer* hidden, const lh_buffer* logits, const lh_buffer* down,
+                                   lh_buffer* residual, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff);
+
+/* *position += by (u32), and the index of the largest of each row of f32 logits (ties: the lower index) */
+LH_API int lh_advance_position_into(lh_batch* batch, lh_buffer* position, uint32_t by);
+LH_API int lh_argmax_rows_f32_into(lh_batch* batch, const lh_buffer* logits, lh_buffer* index, uint32_t rows, uint32_t n);
+
 #ifdef __cplusplus
 }
 #endif

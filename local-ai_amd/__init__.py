@@ -19,6 +19,7 @@ import numpy as np
 
 _HERE = os.path.dirname(os.path.abspath(__file__))
 LIB_PATH = os.path.join(_HERE, "liblocal_hip.so")
+MODELS_LIB_PATH = os.path.join(_HERE, "liblocal_hip_models.so")   # the bf16-weight kernels alone (native.py)
 
 F16, F32, BF16 = 0, 1, 2
 Q4_0, TQ2_0 = 0, 1
@@ -28,6 +29,10 @@ _DTYPE_SIZE = {F16: 2, F32: 4, BF16: 2}
 SMALLM_MAX_M = 8      # local-metal/src/kernels.rs:6155
 BATCHM_MAX_M = 4      # local-metal/src/kernels.rs:6160
 MULTIVEC_MAX_M = 16   # local-metal/src/kernels.rs:6362
+
+# activations and output layouts of the bf16-weight products (include/local_hip.h)
+ACT_NONE, ACT_SILU, ACT_GELU_TANH, ACT_RELU_SQUARED, ACT_SIGMOID = range(5)
+ROWS, ROWS_AT_POSITION, BLOCKS_AT_POSITION = range(3)
 
 
 class Error(Exception):
@@ -78,20 +83,25 @@ _lib = None
 
 
 def lib() -> C.CDLL:
-    """Load ``liblocal_hip.so``; raises ``LibraryCreation`` when it has not been built."""
+    """Load ``liblocal_hip.so`` (or, where only that has been built, its bf16-weight part); raises ``LibraryCreation``
+    when there is neither."""
     global _lib
     if _lib is None:
-        if not os.path.exists(LIB_PATH):
+        path = LIB_PATH if os.path.exists(LIB_PATH) else MODELS_LIB_PATH
+        if not os.path.exists(path):
             raise LibraryCreation(f"{LIB_PATH} is missing: run __graft_entry__.build() (make -C local-ai_amd/csrc)")
-        _lib = C.CDLL(LIB_PATH)
+        _lib = C.CDLL(path)
         _lib.lh_last_error.restype = C.c_char_p
         _lib.lh_version.restype = C.c_char_p
         _lib.lh_buffer_length.restype = C.c_size_t
         _lib.lh_buffer_device_ptr.restype = C.c_void_p
         _lib.lh_context_stream.restype = C.c_void_p
         for name in ("lh_smallm_max_m", "lh_batchm_max_m", "lh_multivec_max_m", "lh_batch_dispatch_count",
-                     "lh_flash_split_count"):
-            getattr(_lib, name).restype = C.c_uint32
+                     "lh_flash_split_count", "lh_attention_padded_dim", "lh_attention_padded_vdim",
+                     "lh_linear_attention_padded_dim", "lh_moe_plan_words"):
+            if hasattr(_lib, name):
+                getattr(_lib, name).restype = C.c_uint32
+        _lib.lh_linear_attention_workspace_bytes.restype = C.c_size_t
     return _lib
 
 
@@ -303,6 +313,10 @@ class Graph:
 def _handles(bufs):
     arr = (C.c_void_p * len(bufs))(*[b._h for b in bufs])
     return arr
+
+
+def _opt(buf):
+    return buf._h if buf is not None else None
 
 
 class Kernels:
@@ -753,6 +767,99 @@ class Kernels:
                                                               _u32(kv_len), _u32(current_pos), _u32(num_q_heads),
                                                               _u32(num_kv_heads), _u32(window), _u32(num_splits)))
 
+    # -- models with plain bf16 weights: products by column segments (linear_weight.Segments), norms of the f32 residual
+    #    stream, softmax attention over BlockKvCache, linear attention over RecurrentState, mixture of experts --
+    def embed_rows_bf16_into(self, batch, table, table_rows, cols, rows, n_rows, output):
+        _check(self._l.lh_embed_rows_bf16_into(batch._h, table._h, _u32(table_rows), _u32(cols), rows._h, _u32(n_rows), output._h))
+
+    def norm_rows_f32_into(self, batch, input, add, weight, store, row_index, output, output_dtype, dim, rows, eps):
+        _check(self._l.lh_norm_rows_f32_into(batch._h, input._h, _opt(add), weight._h, _opt(store), _opt(row_index), output._h,
+                                             C.c_int(output_dtype), _u32(dim), _u32(rows), C.c_float(eps)))
+
+    def gated_norm_rows_into(self, batch, input, gate, weight, output, dtype, dim, rows, eps):
+        _check(self._l.lh_gated_norm_rows_into(batch._h, input._h, gate._h, weight._h, output._h, C.c_int(dtype), _u32(dim),
+                                               _u32(rows), C.c_float(eps)))
+
+    def linear_rows_into(self, batch, input, input_dtype, weight, bias, m, k, segments, outputs, output_dtype,
+                         accumulate=False, position=None):
+        _check(self._l.lh_linear_rows_into(batch._h, input._h, C.c_int(input_dtype), weight._h, _opt(bias), _u32(m), _u32(k),
+                                           *segments.args, _handles(outputs), C.c_int(output_dtype),
+                                           C.c_int(bool(accumulate)), _opt(position)))
+
+    def linear_vector_into(self, batch, input, input_dtype, weight, bias, k, segments, outputs, output_dtype,
+                           accumulate=False, position=None):
+        _check(self._l.lh_linear_vector_into(batch._h, input._h, C.c_int(input_dtype), weight._h, _opt(bias), _u32(k),
+                                             *segments.args, _handles(outputs), C.c_int(output_dtype),
+                                             C.c_int(bool(accumulate)), _opt(position)))
+
+    def linear_norm_vector_into(self, batch, input, add, store, norm_weight, eps, weight, bias, k, segments, outputs,
+                                output_dtype, accumulate=False, position=None):
+        _check(self._l.lh_linear_norm_vector_into(batch._h, input._h, _opt(add), _opt(store), norm_weight._h, C.c_float(eps),
+                                                  weight._h, _opt(bias), _u32(k), *segments.args, _handles(outputs),
+                                                  C.c_int(output_dtype), C.c_int(bool(accumulate)), _opt(position)))
+
+    def linear_gated_vector_into(self, batch, input, gate, gate_dtype, norm_weight, eps, weight, bias, k, segments, outputs,
+                                 output_dtype, accumulate=False, position=None):
+        _check(self._l.lh_linear_gated_vector_into(batch._h, input._h, gate._h, C.c_int(gate_dtype), norm_weight._h,
+                                                   C.c_float(eps), weight._h, _opt(bias), _u32(k), *segments.args,
+                                                   _handles(outputs), C.c_int(output_dtype), C.c_int(bool(accumulate)),
+                                                   _opt(position)))
+
+    def attention_padded_dim(self, dim):
+        return int(self._l.lh_attention_padded_dim(_u32(dim)))
+
+    def attention_padded_vdim(self, vdim):
+        return int(self._l.lh_attention_padded_vdim(_u32(vdim)))
+
+    def attention_rows_into(self, batch, q, keys, values, output, dtype, position, max_position, rows, heads, kv_heads, maps,
+                            dim, vdim, capacity, scale, lam=0.0, out_scale=1.0, eps=0.0):
+        _check(self._l.lh_attention_rows_into(batch._h, q._h, keys._h, values._h, output._h, C.c_int(dtype), position._h,
+                                              _u32(max_position), _u32(rows), _u32(heads), _u32(kv_heads), _u32(maps),
+                                              _u32(dim), _u32(vdim), _u32(capacity), C.c_float(scale), C.c_float(lam),
+                                              C.c_float(out_scale), C.c_float(eps)))
+
+    def linear_attention_padded_dim(self, dim):
+        return int(self._l.lh_linear_attention_padded_dim(_u32(dim)))
+
+    def linear_attention_workspace_bytes(self, rows, heads, dim, vdim):
+        return int(self._l.lh_linear_attention_workspace_bytes(_u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
+
+    def linear_attention_recurrent_into(self, batch, q, k, v, dtype, state, decay, output, rows, heads, dim, vdim):
+        _check(self._l.lh_linear_attention_recurrent_into(batch._h, q._h, k._h, v._h, C.c_int(dtype), state._h, decay._h,
+                                                          output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
+
+    def linear_attention_chunked_into(self, batch, q, k, v, state, decay_powers, workspace, output, rows, heads, dim, vdim):
+        _check(self._l.lh_linear_attention_chunked_into(batch._h, q._h, k._h, v._h, state._h, decay_powers._h, workspace._h,
+                                                        output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
+
+    def moe_plan_words(self, rows, experts, top):
+        return int(self._l.lh_moe_plan_words(_u32(rows), _u32(experts), _u32(top)))
+
+    def moe_route_into(self, batch, logits, plan, rows, experts, top):
+        _check(self._l.lh_moe_route_into(batch._h, logits._h, plan._h, _u32(rows), _u32(experts), _u32(top)))
+
+    def moe_up_into(self, batch, input, dtype, plan, up, hidden, rows, experts, top, width, ff, act):
+        _check(self._l.lh_moe_up_into(batch._h, input._h, C.c_int(dtype), plan._h, up._h, hidden._h, _u32(rows), _u32(experts),
+                                      _u32(top), _u32(width), _u32(ff), _u32(act)))
+
+    def moe_down_into(self, batch, hidden, dtype, plan, down, slots, residual, rows, experts, top, width, ff):
+        _check(self._l.lh_moe_down_into(batch._h, hidden._h, C.c_int(dtype), plan._h, down._h, _opt(slots), residual._h,
+                                        _u32(rows), _u32(experts), _u32(top), _u32(width), _u32(ff)))
+
+    def moe_vector_up_into(self, batch, input, norm_weight, eps, logits, up, hidden, experts, top, width, ff, act):
+        _check(self._l.lh_moe_vector_up_into(batch._h, input._h, norm_weight._h, C.c_float(eps), logits._h, up._h, hidden._h,
+                                             _u32(experts), _u32(top), _u32(width), _u32(ff), _u32(act)))
+
+    def moe_vector_down_into(self, batch, hidden, logits, down, residual, experts, top, width, ff):
+        _check(self._l.lh_moe_vector_down_into(batch._h, hidden._h, logits._h, down._h, residual._h, _u32(experts), _u32(top),
+                                               _u32(width), _u32(ff)))
+
+    def advance_position_into(self, batch, position, by):
+        _check(self._l.lh_advance_position_into(batch._h, position._h, _u32(by)))
+
+    def argmax_rows_f32_into(self, batch, logits, index, rows, n):
+        _check(self._l.lh_argmax_rows_f32_into(batch._h, logits._h, index._h, _u32(rows), _u32(n)))
+
 
 from . import synth  # noqa: E402  (synthetic inputs of the measured configurations)
 from .quant_weight import QuantWeight  # noqa: E402
@@ -761,3 +868,4 @@ from . import gguf, weights  # noqa: E402  (GGUF reader and weight loader: gguf.
 from . import layer  # noqa: E402  (decoder layer: layer.rs)
 from . import pipeline  # noqa: E402  (decode core of the token loop: pipeline.rs)
 from .layer import LayerParams, LayerWeights, ScratchBuffers, BatchScratch, TransformerLayer  # noqa: E402
+from . import linear_weight, mixers, stack_pipeline, registry, generation  # noqa: E402  (models with bf16 weights, serving loop)

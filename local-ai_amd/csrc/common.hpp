@@ -172,9 +172,10 @@ int lh_upload_descriptors(lh_context* ctx, const void* host, size_t bytes, void*
 int lh_raise_dynamic_lds(lh_context* ctx, const void* kernel, size_t bytes, const char* op);
 
 // Resolves the calling device's copy of the attention kernels' static scratch array (attention_tq.hip); the device must be current.
-int lh_attention_static_scratch_init(int device);
+// (Weak, like the next: a library linked without the quantized-cache attention kernels has neither.)
+__attribute__((weak)) int lh_attention_static_scratch_init(int device);
 // Raises the dynamic-LDS limit of the attention kernels that need more than the default (attention_tq_mfma.hip); ctx's device must be current.
-int lh_attention_kernels_init(lh_context* ctx);
+__attribute__((weak)) int lh_attention_kernels_init(lh_context* ctx);
 
 static inline size_t lh_dtype_size(lh_dtype t) { return t == LH_F32 ? 4 : 2; }
 

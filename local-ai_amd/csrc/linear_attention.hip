@@ -1,0 +1,352 @@
+// Linear attention with a fixed decay per head: S_t = decay S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  The state is f32,
+// kept as [head][value column][DQ key columns] (the key columns that exist, then zeros).
+//
+// Recurrent form: one workgroup per head and 16 value columns; a row of 16 lanes holds one value column's state in
+// registers (DQ / 16 values each) and walks the rows.
+//
+// Chunked form (64 rows a chunk, bf16 inputs on the matrix cores, everything else f32):
+//   1. every chunk's own contribution to the state, U = sum_s decay^(L-1-s) k_s v_s^T (all chunks at once)
+//   2. a scan over the chunks, S <- decay^L S + U, that leaves each chunk's incoming state in place of its U
+//   3. all outputs: o_t = decay^(t+1) S_in^T q_t + sum_(s<=t) decay^(t-s) (q_t . k_s) v_s
+// Where an f32 quantity enters a product (decayed keys, decayed scores, the state) it does so as the sum of three bf16
+// terms, which is all of its 24 bits; the products of bf16 values are exact and summed in f32.
+#include "float_ops.hpp"
+#include <algorithm>
+
+namespace {
+
+constexpr uint32_t kChunk = 64;
+
+template <typename T, int NR>
+__global__ __launch_bounds__(256) void recurrent_kernel(const T* __restrict__ q, const T* __restrict__ k, const T* __restrict__ v, float* __restrict__ state,
+                                                       const float* __restrict__ decay, float* __restrict__ out, uint32_t rows, uint32_t heads, uint32_t dim,
+                                                       uint32_t dq, uint32_t vdim) {
+    const uint32_t vt = (vdim + 15) / 16, h = blockIdx.x / vt, col = (blockIdx.x % vt) * 16 + (threadIdx.x >> 4), part = threadIdx.x & 15;
+    const bool on = col < vdim;
+    const uint32_t c = on ? col : vdim - 1, k0 = part * NR;
+    float* st = state + ((size_t)h * vdim + c) * dq + k0;
+    float s[NR];
+#pragma unroll
+    for (int i = 0; i < NR; i++) s[i] = k0 + i < dq ? st[i] : 0.0f;
+    const float d = decay[h];
+    float kn[NR], qn[NR], vn;
+    auto fetch = [&](uint32_t t) {
+        const size_t row = ((size_t)t * heads + h) * dq + k0;
+#pragma unroll
+        for (int i = 0; i < NR; i++) {
+            const bool in = k0 + i < dim;
+            kn[i] = in ? lh_ld(k, row + i) : 0.0f;
+            qn[i] = in ? lh_ld(q, row + i) : 0.0f;
+        }
+        vn = lh_ld(v, ((size_t)t * heads + h) * vdim + c);
+    };
+    fetch(0);
+    for (uint32_t t = 0; t < rows; t++) {
+        float kc[NR], qc[NR];
+        const float vc = vn;
+#pragma unroll
+        for (int i = 0; i < NR; i++) { kc[i] = kn[i]; qc[i] = qn[i]; }
+        if (t + 1 < rows) fetch(t + 1);
+        float o = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NR; i++) {
+            s[i] = __builtin_fmaf(kc[i], vc, d * s[i]);
+            o = __builtin_fmaf(s[i], qc[i], o);
+        }
+        o = lh_group_sum(o, 16);
+        if (part == 0 && on) out[((size_t)t * heads + h) * vdim + col] = o;
+    }
+    if (on) {
+#pragma unroll
+        for (int i = 0; i < NR; i++) if (k0 + i < dq) st[i] = s[i];
+    }
+}
+
+struct ChunkArgs {
+    const uint16_t *q, *k, *v;
+    float* state;
+    const float* powers;       // [heads][65]
+    float* chunk_state;        // [chunk][heads][vdim][dq]
+    float* out;
+    uint32_t rows, heads, dim, vdim, chunks;
+};
+
+__device__ __forceinline__ lh_bf16x8 bf8(const uint32_t (&w)[4]) {
+    struct { uint32_t v[4]; } t = {{w[0], w[1], w[2], w[3]}};
+    return __builtin_bit_cast(lh_bf16x8, t);
+}
+
+constexpr uint32_t kLdT = kChunk + 8;     // row length of a transposed tile: 16-byte aligned, rows on different banks
+
+// Step 1.  A workgroup takes one chunk of one head and 64 value columns; four waves split the key columns.
+// U^T tiles: row operand = decayed keys (16 key columns x tokens), column operand = values (16 value columns x tokens).
+template <int DQ>
+__global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkArgs a) {
+    __shared__ __align__(16) uint16_t kt[3][32][kLdT], vt[64][kLdT];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t vtiles = (a.vdim + 63) / 64, vb = blockIdx.x % vtiles, h = (blockIdx.x / vtiles) % a.heads, c = blockIdx.x / (vtiles * a.heads);
+    const uint32_t t0 = c * kChunk, L = min(kChunk, a.rows - t0), v0 = vb * 64;
+    const float* pw = a.powers + h * (kChunk + 1);
+    for (uint32_t e = tid; e < 64 * kChunk; e += 256) {
+        const uint32_t s = e >> 6, d = e & 63;
+        vt[d][s] = s < L && v0 + d < a.vdim ? a.v[((size_t)(t0 + s) * a.heads + h) * a.vdim + v0 + d] : 0;
+    }
+    float* U = a.chunk_state + ((size_t)c * a.heads + h) * a.vdim * DQ;
+    for (uint32_t k0 = 0; k0 < DQ; k0 += 32) {
+        __syncthreads();
+        for (uint32_t e = tid; e < 32 * kChunk; e += 256) {
+            const uint32_t s = e >> 5, d = e & 31;
+            float x = 0.0f;
+            if (s < L && k0 + d < a.dim) x = lh_bf2f(a.k[((size_t)(t0 + s) * a.heads + h) * DQ + k0 + d]) * pw[L - 1 - s];
+            const LhSplit3 t = lh_split3(x);
+            kt[0][d][s] = t.hi; kt[1][d][s] = t.mid; kt[2][d][s] = t.lo;
+        }
+        __syncthreads();
+        // the eight 16 x 16 tiles of this 32 x 64 block: wave w takes value tile w of both key tiles
+        lh_f32x4 acc[2] = {(lh_f32x4){0.f, 0.f, 0.f, 0.f}, (lh_f32x4){0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+        for (int ks = 0; ks < 2; ks++) {
+            const uint32_t s = ks * 32 + (lane >> 4) * 8;
+            const lh_bf16x8 vf = *reinterpret_cast<const lh_bf16x8*>(&vt[wave * 16 + (lane & 15)][s]);
+#pragma unroll
+            for (int i = 0; i < 2; i++)
+#pragma unroll
+                for (int p = 0; p < 3; p++)
+                    acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lh_bf16x8*>(&kt[p][i * 16 + (lane & 15)][s]), vf, acc[i], 0, 0, 0);
+        }
+        const uint32_t col = v0 + wave * 16 + (lane & 15);
+        if (col < a.vdim) {
+#pragma unroll
+            for (int i = 0; i < 2; i++)
+                *reinterpret_cast<float4*>(U + (size_t)col * DQ + k0 + i * 16 + (lane >> 4) * 4) = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
+        }
+    }
+}
+
+// Step 2.  A thread owns four neighbouring state values and walks the chunks, eight loads ahead.
+__global__ __launch_bounds__(256) void chunk_scan_kernel(const ChunkArgs a, uint32_t dq) {
+    const size_t per_head4 = (size_t)a.vdim * dq / 4, total4 = per_head4 * a.heads, i = (size_t)blockIdx.x * 256 + threadIdx.x;
+    if (i >= total4) return;
+    const uint32_t h = (uint32_t)(i / per_head4);
+    const float* pw = a.powers + h * (kChunk + 1);
+    const float full = pw[kChunk];
+    float4* st = reinterpret_cast<float4*>(a.state) + i;
+    float4* u = reinterpret_cast<float4*>(a.chunk_state) + i;
+    float4 s = *st;
+    constexpr uint32_t P = 8;
+    for (uint32_t c0 = 0; c0 < a.chunks; c0 += P) {
+        float4 x[P];
+#pragma unroll
+        for (uint32_t j = 0; j < P; j++) x[j] = u[(size_t)min(c0 + j, a.chunks - 1) * total4];
+#pragma unroll
+        for (uint32_t j = 0; j < P; j++) {
+            if (c0 + j >= a.chunks) break;
+            u[(size_t)(c0 + j) * total4] = s;
+            const float d = c0 + j + 1 < a.chunks ? full : pw[a.rows - (a.chunks - 1) * kChunk];
+            s.x = __builtin_fmaf(d, s.x, x[j].x); s.y = __builtin_fmaf(d, s.y, x[j].y);
+            s.z = __builtin_fmaf(d, s.z, x[j].z); s.w = __builtin_fmaf(d, s.w, x[j].w);
+        }
+    }
+    *st = s;
+}
+
+// Step 3.  A workgroup takes one chunk of one head and 64 value columns; wave w the rows 16 w .. 16 w + 15.
+// Scores transposed (row operand keys, column operand queries), so that the decayed scores are in operand order for
+// O^T = V^T P^T, whose k index 8g + j is row 4g + j of the first 16-row tile (j < 4) or 4g + j - 4 of the second.
+template <int DQ>
+__global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkArgs a) {
+    __shared__ __align__(16) uint16_t vt[64][kLdT];            // [value column][32-row half][slot]
+    __shared__ float pws[kChunk + 1];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4;
+    const uint32_t vtiles = (a.vdim + 63) / 64, vb = blockIdx.x % vtiles, h = (blockIdx.x / vtiles) % a.heads, c = blockIdx.x / (vtiles * a.heads);
+    const uint32_t t0 = c * kChunk, L = min(kChunk, a.rows - t0), v0 = vb * 64;
+    for (uint32_t e = tid; e < 64 * kChunk; e += 256) {
+        const uint32_t s = e >> 6, d = e & 63;
+        vt[d][(s & 32) + lh_block_slot(s & 31)] = s < L && v0 + d < a.vdim ? a.v[((size_t)(t0 + s) * a.heads + h) * a.vdim + v0 + d] : 0;
+    }
+    if (tid <= kChunk) pws[tid] = a.powers[h * (kChunk + 1) + tid];
+    __syncthreads();
+    if (wave * 16 >= L) return;
+    const uint32_t t = wave * 16 + (lane & 15), tr = min(t, L - 1);
+    lh_bf16x8 qf[DQ / 32];
+#pragma unroll
+    for (int i = 0; i < DQ / 32; i++) {
+        const uint32_t k = i * 32 + g * 8;
+        uint32_t w[4] = {0u, 0u, 0u, 0u};
+        if (k < a.dim) {
+            const uint4 x = *reinterpret_cast<const uint4*>(a.q + ((size_t)(t0 + tr) * a.heads + h) * DQ + k);
+            w[0] = x.x; w[1] = x.y; w[2] = x.z; w[3] = x.w;
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                if (k + 2 * j >= a.dim) w[j] = 0u;
+                else if (k + 2 * j + 1 >= a.dim) w[j] &= 0xFFFFu;
+            }
+        }
+        qf[i] = bf8(w);
+    }
+    lh_f32x4 o[4];
+    // the state's part, scaled by decay^(t + 1) afterwards
+    const float* S = a.chunk_state + ((size_t)c * a.heads + h) * a.vdim * DQ;
+#pragma unroll
+    for (int d = 0; d < 4; d++) {
+        o[d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+        if (v0 + d * 16 >= a.vdim) continue;
+        const float* srow = S + (size_t)min(v0 + d * 16 + (lane & 15), a.vdim - 1) * DQ + g * 8;
+#pragma unroll
+        for (int i = 0; i < DQ / 32; i++) {
+            const float4 x = *reinterpret_cast<const float4*>(srow + i * 32), y = *reinterpret_cast<const float4*>(srow + i * 32 + 4);
+            const float f[8] = {x.x, x.y, x.z, x.w, y.x, y.y, y.z, y.w};
+            uint32_t p[3][4];
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                const LhSplit3 e = lh_split3(f[2 * j]), m = lh_split3(f[2 * j + 1]);
+                p[0][j] = (uint32_t)e.hi | ((uint32_t)m.hi << 16);
+                p[1][j] = (uint32_t)e.mid | ((uint32_t)m.mid << 16);
+                p[2][j] = (uint32_t)e.lo | ((uint32_t)m.lo << 16);
+            }
+#pragma unroll
+            for (int z = 2; z >= 0; z--) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(bf8(p[z]), qf[i], o[d], 0, 0, 0);
+        }
+    }
+    const float carry = pws[tr + 1];
+#pragma unroll
+    for (int d = 0; d < 4; d++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) o[d][r] *= carry;
+    // the chunk's own rows, 32 at a time
+    for (uint32_t s0 = 0; s0 <= wave * 16 + 15 && s0 < L; s0 += 32) {
+        lh_f32x4 sc[2];
+#pragma unroll
+        for (int u = 0; u < 2; u++) {
+            sc[u] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+            const uint32_t s = min(s0 + u * 16 + (lane & 15), L - 1);
+            const uint16_t* kr = a.k + ((size_t)(t0 + s) * a.heads + h) * DQ + g * 8;
+#pragma unroll
+            for (int i = 0; i < DQ / 32; i++) sc[u] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lh_bf16x8*>(kr + i * 32), qf[i], sc[u], 0, 0, 0);
+        }
+        uint32_t p[3][4];
+#pragma unroll
+        for (int j = 0; j < 4; j++) {
+            LhSplit3 e[2];
+#pragma unroll
+            for (int b = 0; b < 2; b++) {
+                const int n = 2 * j + b;
+                const uint32_t s = s0 + (n >> 2) * 16 + g * 4 + (n & 3);
+                e[b] = lh_split3(s <= t && s < L ? sc[n >> 2][n & 3] * pws[min(t - s, kChunk)] : 0.0f);
+            }
+            p[0][j] = (uint32_t)e[0].hi | ((uint32_t)e[1].hi << 16);
+            p[1][j] = (uint32_t)e[0].mid | ((uint32_t)e[1].mid << 16);
+            p[2][j] = (uint32_t)e[0].lo | ((uint32_t)e[1].lo << 16);
+        }
+#pragma unroll
+        for (int d = 0; d < 4; d++) {
+            const lh_bf16x8 vf = *reinterpret_cast<const lh_bf16x8*>(&vt[d * 16 + (lane & 15)][s0 + g * 8]);
+#pragma unroll
+            for (int z = 2; z >= 0; z--) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, bf8(p[z]), o[d], 0, 0, 0);
+        }
+    }
+    if (t >= L) return;
+    float* out = a.out + ((size_t)(t0 + t) * a.heads + h) * a.vdim + v0;
+#pragma unroll
+    for (int d = 0; d < 4; d++) {
+        const uint32_t col = d * 16 + g * 4;
+        if ((a.vdim & 3) == 0) { if (v0 + col < a.vdim) *reinterpret_cast<float4*>(out + col) = make_float4(o[d][0], o[d][1], o[d][2], o[d][3]); }
+        else {
+#pragma unroll
+            for (int r = 0; r < 4; r++) if (v0 + col + r < a.vdim) out[col + r] = o[d][r];
+        }
+    }
+}
+
+template <int DQ>
+int launch_chunked(lh_context* ctx, const ChunkArgs& a, const char* op) {
+    const uint32_t grid = a.chunks * a.heads * ((a.vdim + 63) / 64);
+    hipLaunchKernelGGL((chunk_state_kernel<DQ>), dim3(grid), dim3(256), 0, ctx->stream, a);
+    int r = lh_check_launch(op);
+    if (r != LH_OK) return r;
+    const size_t total4 = (size_t)a.heads * a.vdim * DQ / 4;
+    hipLaunchKernelGGL(chunk_scan_kernel, dim3((uint32_t)((total4 + 255) / 256)), dim3(256), 0, ctx->stream, a, (uint32_t)DQ);
+    r = lh_check_launch(op);
+    if (r != LH_OK) return r;
+    hipLaunchKernelGGL((chunk_output_kernel<DQ>), dim3(grid), dim3(256), 0, ctx->stream, a);
+    return lh_check_launch(op);
+}
+
+}  // namespace
+
+extern "C" {
+
+uint32_t lh_linear_attention_padded_dim(uint32_t dim) { return dim <= 32 ? 32u : dim <= 64 ? 64u : (dim + 127) / 128 * 128; }
+
+size_t lh_linear_attention_workspace_bytes(uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim) {
+    return (size_t)((rows + kChunk - 1) / kChunk) * heads * vdim * lh_linear_attention_padded_dim(dim) * 4;
+}
+
+int lh_linear_attention_recurrent_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v, int dtype, lh_buffer* state,
+                                       const lh_buffer* decay, lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim) {
+    const char* op = "linear_attention_recurrent";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    LH_REQUIRE(dtype == LH_F32 || dtype == LH_BF16, "%s: dtype %d", op, dtype);
+    LH_REQUIRE(heads > 0 && dim > 0 && dim <= 1024 && vdim > 0, "%s: heads %u, dim %u, vdim %u", op, heads, dim, vdim);
+    if (rows == 0) return LH_OK;
+    const uint32_t dq = lh_linear_attention_padded_dim(dim);
+    const size_t es = dtype == LH_F32 ? 4 : 2;
+    LH_NEED(q, (size_t)rows * heads * dq * es, op, "q");
+    LH_NEED(k, (size_t)rows * heads * dq * es, op, "k");
+    LH_NEED(v, (size_t)rows * heads * vdim * es, op, "v");
+    LH_NEED(state, (size_t)heads * vdim * dq * 4, op, "state");
+    LH_NEED(decay, (size_t)heads * 4, op, "decay");
+    LH_NEED(output, (size_t)rows * heads * vdim * 4, op, "output");
+    const uint64_t grid = (uint64_t)heads * ((vdim + 15) / 16);
+    LH_REQUIRE(grid < 0x7FFFFFFFull, "%s: heads %u, vdim %u", op, heads, vdim);
+#define LH_REC(T, NR_)                                                                                                                               \
+    hipLaunchKernelGGL((recurrent_kernel<T, NR_>), dim3((uint32_t)grid), dim3(256), 0, batch->ctx->stream, (const T*)q->ptr, (const T*)k->ptr,        \
+                       (const T*)v->ptr, (float*)state->ptr, (const float*)decay->ptr, (float*)output->ptr, rows, heads, dim, dq, vdim)
+#define LH_REC_T(T)                       \
+    do {                                  \
+        if (dq <= 32) LH_REC(T, 2);       \
+        else if (dq <= 64) LH_REC(T, 4);  \
+        else if (dq <= 128) LH_REC(T, 8); \
+        else if (dq <= 256) LH_REC(T, 16); \
+        else if (dq <= 512) LH_REC(T, 32); \
+        else LH_REC(T, 64);               \
+    } while (0)
+    if (dtype == LH_F32) LH_REC_T(float);
+    else LH_REC_T(uint16_t);
+#undef LH_REC_T
+#undef LH_REC
+    const int r = lh_check_launch(op);
+    if (r == LH_OK) batch->dispatch_count++;
+    return r;
+}
+
+int lh_linear_attention_chunked_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v, lh_buffer* state,
+                                     const lh_buffer* decay_powers, lh_buffer* workspace, lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim,
+                                     uint32_t vdim) {
+    const char* op = "linear_attention_chunked";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    LH_REQUIRE(heads > 0 && dim > 0 && dim <= 256 && vdim > 0, "%s: heads %u, dim %u, vdim %u", op, heads, dim, vdim);
+    if (rows == 0) return LH_OK;
+    const uint32_t dq = lh_linear_attention_padded_dim(dim);
+    LH_NEED(q, (size_t)rows * heads * dq * 2, op, "q");
+    LH_NEED(k, (size_t)rows * heads * dq * 2, op, "k");
+    LH_NEED(v, (size_t)rows * heads * vdim * 2, op, "v");
+    LH_NEED(state, (size_t)heads * vdim * dq * 4, op, "state");
+    LH_NEED(decay_powers, (size_t)heads * (kChunk + 1) * 4, op, "decay_powers");
+    LH_NEED(workspace, lh_linear_attention_workspace_bytes(rows, heads, dim, vdim), op, "workspace");
+    LH_NEED(output, (size_t)rows * heads * vdim * 4, op, "output");
+    LH_REQUIRE((((uintptr_t)q->ptr | (uintptr_t)k->ptr | (uintptr_t)state->ptr | (uintptr_t)workspace->ptr | (uintptr_t)output->ptr) & 15) == 0,
+               "%s: buffers must be 16-byte aligned", op);
+    ChunkArgs a{(const uint16_t*)q->ptr, (const uint16_t*)k->ptr, (const uint16_t*)v->ptr, (float*)state->ptr, (const float*)decay_powers->ptr,
+                (float*)workspace->ptr, (float*)output->ptr, rows, heads, dim, vdim, (rows + kChunk - 1) / kChunk};
+    LH_REQUIRE((uint64_t)a.chunks * heads * ((vdim + 63) / 64) < 0x7FFFFFFFull, "%s: %u rows", op, rows);
+    int r;
+    if (dq == 32) r = launch_chunked<32>(batch->ctx, a, op);
+    else if (dq == 64) r = launch_chunked<64>(batch->ctx, a, op);
+    else if (dq == 128) r = launch_chunked<128>(batch->ctx, a, op);
+    else r = launch_chunked<256>(batch->ctx, a, op);
+    if (r == LH_OK) batch->dispatch_count += 3;
+    return r;
+}
+
+}  // extern "C"

@@ -140,7 +140,7 @@ int lh_context_create(int device_index, lh_context** out) {
     LH_HIP_TRY(hipGetDeviceProperties(&prop, device_index), LH_ERR_NO_DEVICE, "hipGetDeviceProperties");
     if (strncmp(prop.gcnArchName, "gfx950", 6) != 0)
         return lh_fail(LH_ERR_LIBRARY_CREATION, "kernels are built for gfx950 only, device is %s", prop.gcnArchName);
-    {
+    if (lh_attention_static_scratch_init) {
         const int rs = lh_attention_static_scratch_init(device_index);
         if (rs != LH_OK) return rs;
     }
@@ -195,7 +195,7 @@ int lh_context_create(int device_index, lh_context** out) {
     }
     // The attention kernels with hand-over areas in dynamic LDS get their limit raised here, so that no launch -- in
     // particular none inside a recorded batch or from the entry that may not allocate -- has to do it.
-    {
+    if (lh_attention_kernels_init) {
         const int ra = lh_attention_kernels_init(ctx);
         if (ra != LH_OK) { lh_context_destroy(ctx); return ra; }
     }

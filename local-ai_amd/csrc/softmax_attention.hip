@@ -1,0 +1,581 @@
+// Causal softmax attention over bf16 (or f32) caches, with one or two score maps per head.  With two maps (differential
+// attention) both share the head's values and are combined in the same kernel: o = a1 - lambda a2, an RMS norm over the
+// head, a constant factor.
+//
+// Caches: keys [position][kv head][map][DQ], values in blocks of 32 positions [block][kv head][DV][32] whose 32 entries
+// are in lh_block_slot order.  The queries of one kv head's group are packed: packed row r = query row r / R, head r % R of
+// the group (R heads per kv head), so a tile of 16 packed rows uses the matrix cores fully also for one query row.
+//
+// Matrix-core form (bf16): a step of 32 keys computes S^T = K Q^T (two 16 x 16 tiles; lane = packed row (lane & 15), keys
+// 4g .. 4g + 3 of each tile, g = lane >> 4), so a row's maximum and sum are eight registers and two lane exchanges, and
+// the weights are already where O^T = V^T P^T wants them: its k index 8g + j is key 4g + j of tile 0 (j < 4) or key
+// 4g + j - 4 of tile 1, which is the order of the value blocks.  Scores, weights and sums are f32; a weight enters the
+// product as the sum of two bf16 terms.
+//   attention_tile_kernel   many rows: four waves share key and value blocks through LDS
+//   attention_split_kernel  few rows: every wave walks its own share of the blocks straight from global memory; the
+//                           workgroup's four partial results are merged in LDS, the workgroups' by attention_merge_kernel
+// Plain form (any dtype, any dim): attention_plain_kernel, one workgroup per query row and head.
+#include "float_ops.hpp"
+#include <algorithm>
+#include <cmath>
+
+namespace {
+
+struct AttentionArgs {
+    const void* q;
+    const void* keys;
+    const void* values;
+    void* out;
+    const uint32_t* position;
+    uint32_t rows, heads, kv_heads, maps, dim, dq, vdim, dv, capacity;
+    float scale, lambda, out_scale, eps;
+    float* partial;            // split form: [tile][kv head][split][map][16] (max, sum), then the unnormalised sums [..][16][dv]
+    uint32_t splits;
+};
+
+constexpr float kLog2e = 1.4426950408889634f;
+
+typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
+
+// The B operand of S^T: query values of packed row `row` (zero past the rows and past dim).
+template <int DQ, int MAPS>
+__device__ __forceinline__ void load_queries(lh_bf16x8 (&qf)[MAPS][DQ / 32], const AttentionArgs& a, uint32_t g, uint32_t row, uint32_t lane) {
+    const uint32_t R = a.heads / a.kv_heads, t = row / R, h = g * R + (row - t * R);
+    const bool on = t < a.rows;
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++)
+#pragma unroll
+        for (int c = 0; c < DQ / 32; c++) {
+            const uint32_t k = c * 32 + (lane >> 4) * 8;
+            u32x4 v = {0u, 0u, 0u, 0u};
+            if (on && k < a.dim) {
+                v = *reinterpret_cast<const u32x4*>(static_cast<const uint16_t*>(a.q) + (((size_t)t * a.heads + h) * MAPS + mp) * DQ + k);
+#pragma unroll
+                for (int j = 0; j < 4; j++) {
+                    if (k + 2 * j >= a.dim) v[j] = 0u;
+                    else if (k + 2 * j + 1 >= a.dim) v[j] &= 0xFFFFu;
+                }
+            }
+            qf[mp][c] = __builtin_bit_cast(lh_bf16x8, v);
+        }
+}
+
+// One row tile's running softmax state for one map; every lane holds the values of packed row (lane & 15).
+struct RowState { float m, l; };
+
+// Scores of a 32-key step -> weights in P V operand order, as two bf16 terms; returns the factor for what was summed before.
+// `first` is the step's first key, `limit` the row's last visible key, `bound` whether any lane may have to mask.
+__device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2], RowState& st, float scale2, uint32_t first, uint32_t limit, bool bound, uint32_t lane,
+                                              lh_bf16x8& hi, lh_bf16x8& lo) {
+    float v[8], mx = -INFINITY;
+    const uint32_t g = lane >> 4;
+#pragma unroll
+    for (int i = 0; i < 8; i++) {
+        v[i] = s[i >> 2][i & 3] * scale2;
+        if (bound && first + (i >> 2) * 16 + g * 4 + (i & 3) > limit) v[i] = -INFINITY;
+        mx = fmaxf(mx, v[i]);
+    }
+    mx = fmaxf(mx, lh_swap16_f(mx));
+    mx = fmaxf(mx, lh_swap32_f(mx));
+    const float nm = fmaxf(st.m, mx), base = nm == -INFINITY ? 0.0f : nm;
+    const float alpha = __builtin_amdgcn_exp2f(st.m - base);
+    float sum = 0.0f;
+    uint32_t h[4], l[4];
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const float p0 = __builtin_amdgcn_exp2f(v[2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[2 * i + 1] - base);
+        sum += p0 + p1;
+        h[i] = lh_pack_bf(p0, p1);
+        l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, h[i] << 16), p1 - __builtin_bit_cast(float, h[i] & 0xFFFF0000u));
+    }
+    hi = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
+    lo = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
+    st.l = st.l * alpha + sum;      // this lane's keys only; the four lanes of a row are added at the end
+    st.m = nm;
+    return alpha;
+}
+
+// A finished row: o[i][r] holds value 16 i + 4g + r of packed row (lane & 15), for every map unnormalised with sum l.
+template <int DV, int MAPS>
+__device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)[MAPS][DV / 16], const float (&l)[MAPS], uint32_t g, uint32_t row, uint32_t lane) {
+    const uint32_t R = a.heads / a.kv_heads, t = row / R, h = g * R + (row - t * R);
+    float inv[MAPS];
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) inv[mp] = 1.0f / l[mp];
+    float ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < DV / 16; i++)
+#pragma unroll
+        for (int r = 0; r < 4; r++) {
+            float v = o[0][i][r] * inv[0];
+            if constexpr (MAPS == 2) v -= a.lambda * (o[MAPS - 1][i][r] * inv[MAPS - 1]);
+            o[0][i][r] = v;
+            if ((uint32_t)(i * 16 + (lane >> 4) * 4 + r) < a.vdim) ss += v * v;
+        }
+    float f = 1.0f;
+    if constexpr (MAPS == 2) {
+        ss += lh_swap16_f(ss);
+        ss += lh_swap32_f(ss);
+        f = rsqrtf(ss / (float)a.vdim + a.eps) * a.out_scale;
+    }
+    if (t >= a.rows) return;
+    uint16_t* out = static_cast<uint16_t*>(a.out) + ((size_t)t * a.heads + h) * a.vdim;
+#pragma unroll
+    for (int i = 0; i < DV / 16; i++) {
+        const uint32_t c = i * 16 + (lane >> 4) * 4;
+        if ((a.vdim & 3) == 0) {
+            if (c < a.vdim) *reinterpret_cast<uint2*>(out + c) = make_uint2(lh_pack_bf(o[0][i][0] * f, o[0][i][1] * f), lh_pack_bf(o[0][i][2] * f, o[0][i][3] * f));
+        } else {
+#pragma unroll
+            for (int r = 0; r < 4; r++) if (c + r < a.vdim) out[c + r] = lh_f2bf(o[0][i][r] * f);
+        }
+    }
+}
+
+typedef __attribute__((address_space(1))) const void gvoid;
+typedef __attribute__((address_space(3))) void lvoid;
+
+// RT row tiles of 16 packed rows per wave, four waves; steps of 32 keys through two LDS buffers.  A key row of the buffer is
+// MAPS * DQ / 8 chunks of 16 bytes, chunk c at place c ^ (key & 7) (see linear_mfma_kernel for why and how).
+template <int DQ, int DV, int MAPS, int RT>
+__global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs a) {
+    constexpr int KC = MAPS * DQ / 8, KCH = 32 * KC, VCH = DV * 4;      // chunks per key row; per key block; per value block
+    __shared__ uint4 sm[2][KCH + VCH];
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t R = a.heads / a.kv_heads, packed = a.rows * R, tiles = (packed + 64 * RT - 1) / (64 * RT);
+    const uint32_t g = blockIdx.x % a.kv_heads, tile = tiles - 1 - blockIdx.x / a.kv_heads;    // the long tiles first
+    const uint32_t start = *a.position;
+    const uint32_t row0 = tile * 64 * RT, row_last = min(row0 + 64 * RT, packed) - 1;
+    const uint32_t last_key = min(start + row_last / R, a.capacity - 1), nb = last_key / 32 + 1;
+    const uint32_t wrow = row0 + wave * 16 * RT;
+
+    lh_bf16x8 qf[RT][MAPS][DQ / 32];
+    uint32_t limit[RT];
+#pragma unroll
+    for (int i = 0; i < RT; i++) {
+        const uint32_t row = wrow + i * 16 + (lane & 15);
+        load_queries<DQ, MAPS>(qf[i], a, g, row, lane);
+        limit[i] = min(start + row / R, last_key);
+    }
+    const uint32_t wave_first_limit = start + wrow / R, wave_last = min(start + (wrow + 16 * RT - 1) / R, last_key);
+    lh_f32x4 o[RT][MAPS][DV / 16];
+    RowState st[RT][MAPS];
+#pragma unroll
+    for (int i = 0; i < RT; i++)
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) {
+            st[i][mp] = RowState{-INFINITY, 0.0f};
+#pragma unroll
+            for (int d = 0; d < DV / 16; d++) o[i][mp][d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+        }
+
+    const uint16_t* K = static_cast<const uint16_t*>(a.keys) + (size_t)g * MAPS * DQ;
+    const uint16_t* V = static_cast<const uint16_t*>(a.values) + (size_t)g * DV * 32;
+    const size_t krow = (size_t)a.kv_heads * MAPS * DQ, vblock = (size_t)a.kv_heads * DV * 32;
+    auto load_block = [&](int buf, uint32_t b) {
+#pragma unroll
+        for (int i = 0; i < (KCH + 255) / 256; i++) {
+            if (KCH % 256 != 0 && i * 256 + wave * 64 >= KCH) break;                           // whole waves (KCH is a multiple of 64)
+            const uint32_t c = i * 256 + tid, key = c / KC, place = c % KC, ch = place ^ (key & (KC >= 8 ? 7 : KC - 1));
+            const uint32_t p = min(b * 32 + key, last_key);                                     // keys past the last are masked
+            __builtin_amdgcn_global_load_lds((gvoid*)(K + p * krow + ch * 8), (lvoid*)&sm[buf][i * 256 + wave * 64], 16, 0, 0);
+        }
+#pragma unroll
+        for (int i = 0; i < (VCH + 255) / 256; i++) {
+            if (VCH % 256 != 0 && i * 256 + wave * 64 >= VCH) break;
+            __builtin_amdgcn_global_load_lds((gvoid*)(V + b * vblock + (i * 256 + tid) * 8), (lvoid*)&sm[buf][KCH + i * 256 + wave * 64], 16, 0, 0);
+        }
+    };
+    const float scale2 = a.scale * kLog2e;
+    load_block(0, 0);
+    for (uint32_t b = 0; b < nb; b++) {
+        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        __syncthreads();
+        if (b + 1 < nb) load_block((b + 1) & 1, b + 1);
+        if (b * 32 > wave_last) continue;                                                       // nothing here is visible to this wave
+        const uint4* ks = sm[b & 1];
+        const uint4* vs = ks + KCH;
+        const bool bound = b * 32 + 31 > wave_first_limit;
+        lh_bf16x8 hi[RT][MAPS], lo[RT][MAPS];
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) {
+            lh_f32x4 s[RT][2];
+#pragma unroll
+            for (int t = 0; t < 2; t++) {
+#pragma unroll
+                for (int i = 0; i < RT; i++) s[i][t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+                const uint32_t key = t * 16 + (lane & 15);
+#pragma unroll
+                for (int c = 0; c < DQ / 32; c++) {
+                    const uint32_t ch = mp * (DQ / 8) + c * 4 + (lane >> 4);
+                    const lh_bf16x8 kf = __builtin_bit_cast(lh_bf16x8, ks[key * KC + (ch ^ (key & (KC >= 8 ? 7 : KC - 1)))]);
+#pragma unroll
+                    for (int i = 0; i < RT; i++) s[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][mp][c], s[i][t], 0, 0, 0);
+                }
+            }
+#pragma unroll
+            for (int i = 0; i < RT; i++) {
+                const float alpha = softmax_step(s[i], st[i][mp], scale2, b * 32, limit[i], bound, lane, hi[i][mp], lo[i][mp]);
+                if (__ballot(alpha != 1.0f)) {
+#pragma unroll
+                    for (int d = 0; d < DV / 16; d++)
+#pragma unroll
+                        for (int r = 0; r < 4; r++) o[i][mp][d][r] *= alpha;
+                }
+            }
+        }
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++) {
+            const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, vs[(d * 16 + (lane & 15)) * 4 + (lane >> 4)]);
+#pragma unroll
+            for (int i = 0; i < RT; i++)
+#pragma unroll
+                for (int mp = 0; mp < MAPS; mp++) {
+                    o[i][mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[i][mp], o[i][mp][d], 0, 0, 0);
+                    o[i][mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[i][mp], o[i][mp][d], 0, 0, 0);
+                }
+        }
+    }
+#pragma unroll
+    for (int i = 0; i < RT; i++) {
+        float l[MAPS];
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) {
+            l[mp] = st[i][mp].l;
+            l[mp] += lh_swap16_f(l[mp]);
+            l[mp] += lh_swap32_f(l[mp]);
+        }
+        finish_row<DV, MAPS>(a, o[i], l, g, wrow + i * 16 + (lane & 15), lane);
+    }
+}
+
+// grid: row tiles x kv heads x splits.  The blocks of the visible range are dealt out in contiguous runs to the 4 * splits
+// waves of a (tile, kv head); a wave loads a block's operands one block ahead.
+template <int DQ, int DV, int MAPS>
+__global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArgs a) {
+    extern __shared__ float merge[];                          // [4 waves][MAPS][16 rows][DV + 2]: max, sum, values
+    const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
+    const uint32_t split = blockIdx.x % a.splits, g = (blockIdx.x / a.splits) % a.kv_heads, tile = blockIdx.x / (a.splits * a.kv_heads);
+    const uint32_t R = a.heads / a.kv_heads, packed = a.rows * R, start = *a.position;
+    const uint32_t row0 = tile * 16, row_last = min(row0 + 16, packed) - 1, row = row0 + (lane & 15);
+    const uint32_t last_key = min(start + row_last / R, a.capacity - 1), nb = last_key / 32 + 1;
+    const uint32_t limit = min(start + row / R, last_key), first_limit = start + row0 / R;
+    const uint32_t per = (nb + 4 * a.splits - 1) / (4 * a.splits), w = split * 4 + wave;
+    const uint32_t b0 = min(w * per, nb), b1 = min(b0 + per, nb);
+
+    lh_bf16x8 qf[MAPS][DQ / 32];
+    load_queries<DQ, MAPS>(qf, a, g, row, lane);
+    lh_f32x4 o[MAPS][DV / 16];
+    RowState st[MAPS];
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) {
+        st[mp] = RowState{-INFINITY, 0.0f};
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++) o[mp][d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+    }
+    const uint16_t* K = static_cast<const uint16_t*>(a.keys) + (size_t)g * MAPS * DQ + (lane >> 4) * 8;
+    const uint16_t* V = static_cast<const uint16_t*>(a.values) + (size_t)g * DV * 32;
+    const size_t krow = (size_t)a.kv_heads * MAPS * DQ, vblock = (size_t)a.kv_heads * DV * 32;
+    struct Block { u32x4 k[2][MAPS][DQ / 32], v[DV / 16]; };
+    auto issue = [&](Block& f, uint32_t b) {
+#pragma unroll
+        for (int t = 0; t < 2; t++) {
+            const uint32_t p = min(b * 32 + t * 16 + (lane & 15), last_key);
+#pragma unroll
+            for (int mp = 0; mp < MAPS; mp++)
+#pragma unroll
+                for (int c = 0; c < DQ / 32; c++) f.k[t][mp][c] = *reinterpret_cast<const u32x4*>(K + p * krow + mp * DQ + c * 32);
+        }
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++) f.v[d] = *reinterpret_cast<const u32x4*>(V + b * vblock + ((d * 16 + (lane & 15)) * 4 + (lane >> 4)) * 8);
+    };
+    const float scale2 = a.scale * kLog2e;
+    auto consume = [&](const Block& f, uint32_t b) {
+        const bool bound = b * 32 + 31 > first_limit;
+        lh_bf16x8 hi[MAPS], lo[MAPS];
+#pragma unroll
+        for (int mp = 0; mp < MAPS; mp++) {
+            lh_f32x4 s[2];
+#pragma unroll
+            for (int t = 0; t < 2; t++) {
+                s[t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+#pragma unroll
+                for (int c = 0; c < DQ / 32; c++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.k[t][mp][c]), qf[mp][c], s[t], 0, 0, 0);
+            }
+            const float alpha = softmax_step(s, st[mp], scale2, b * 32, limit, bound, lane, hi[mp], lo[mp]);
+            if (__ballot(alpha != 1.0f)) {
+#pragma unroll
+                for (int d = 0; d < DV / 16; d++)
+#pragma unroll
+                    for (int r = 0; r < 4; r++) o[mp][d][r] *= alpha;
+            }
+        }
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++)
+#pragma unroll
+            for (int mp = 0; mp < MAPS; mp++) {
+                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), hi[mp], o[mp][d], 0, 0, 0);
+                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), lo[mp], o[mp][d], 0, 0, 0);
+            }
+    };
+    if (b0 < b1) {
+        Block x, y;
+        issue(x, b0);
+        for (uint32_t b = b0; b < b1; b += 2) {
+            issue(y, min(b + 1, b1 - 1));
+            consume(x, b);
+            if (b + 1 < b1) {
+                issue(x, min(b + 2, b1 - 1));
+                consume(y, b + 1);
+            }
+        }
+    }
+    constexpr uint32_t kRow = DV + 2;
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) {
+        float l = st[mp].l;
+        l += lh_swap16_f(l);
+        l += lh_swap32_f(l);
+        float* d0 = merge + ((wave * MAPS + mp) * 16 + (lane & 15)) * kRow;
+        if (lane < 16) { d0[0] = st[mp].m; d0[1] = l; }
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) d0[2 + d * 16 + (lane >> 4) * 4 + r] = o[mp][d][r];
+    }
+    __syncthreads();
+    // partial record of (tile, kv head, split): [map][16] rows of DV + 2
+    float* rec = a.partial + (size_t)((tile * a.kv_heads + g) * a.splits + split) * MAPS * 16 * kRow;
+    const uint32_t used = row_last - row0 + 1;
+    for (uint32_t i = tid; i < (uint32_t)MAPS * used * DV; i += 256) {
+        const uint32_t mp = i / (used * DV), rr = (i / DV) % used, d = i % DV;
+        float m = -INFINITY, acc = 0.0f, l = 0.0f;
+#pragma unroll
+        for (int wv = 0; wv < 4; wv++) m = fmaxf(m, merge[((wv * MAPS + mp) * 16 + rr) * kRow]);
+        const float base = m == -INFINITY ? 0.0f : m;
+#pragma unroll
+        for (int wv = 0; wv < 4; wv++) {
+            const float* s = merge + ((wv * MAPS + mp) * 16 + rr) * kRow;
+            const float f = __builtin_amdgcn_exp2f(s[0] - base);
+            l += f * s[1];
+            acc += f * s[2 + d];
+        }
+        float* r = rec + (mp * 16 + rr) * kRow;
+        r[2 + d] = acc;
+        if (d == 0) { r[0] = m; r[1] = l; }
+    }
+}
+
+// One workgroup per (query row, head): merges the splits of every map, combines the maps, norms and stores.
+template <int MAPS>
+__global__ __launch_bounds__(256) void attention_merge_kernel(const AttentionArgs a) {
+    __shared__ float factor[MAPS][512], total[MAPS], scratch[4];
+    const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
+    const uint32_t kRow = a.dv + 2, rr = row & 15;
+    const size_t stride = (size_t)MAPS * 16 * kRow;
+    const float* rec = a.partial + (size_t)(((row >> 4) * a.kv_heads + g) * a.splits) * stride + rr * kRow;
+    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
+    if (wave < MAPS) {                                        // splits <= 512
+        const float* r = rec + wave * 16 * kRow;
+        float m = -INFINITY, l = 0.0f;
+        for (uint32_t s = lane; s < a.splits; s += 64) m = fmaxf(m, r[s * stride]);
+        m = lh_group_max(m, 64);
+        for (uint32_t s = lane; s < a.splits; s += 64) {
+            const float f = __builtin_amdgcn_exp2f(r[s * stride] - m);
+            factor[wave][s] = f;
+            l += f * r[s * stride + 1];
+        }
+        l = lh_group_sum(l, 64);
+        if (lane == 0) total[wave] = 1.0f / l;
+    }
+    __syncthreads();
+    float v[4], ss = 0.0f;                                    // vdim <= 1024
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const uint32_t d = threadIdx.x + i * 256;
+        v[i] = 0.0f;
+        if (d >= a.vdim) break;
+        float acc[MAPS] = {};
+        for (uint32_t s = 0; s < a.splits; s++)
+#pragma unroll
+            for (int mp = 0; mp < MAPS; mp++)
+                if (factor[mp][s] != 0.0f) acc[mp] += factor[mp][s] * rec[s * stride + mp * 16 * kRow + 2 + d];
+        v[i] = acc[0] * total[0];
+        if constexpr (MAPS == 2) v[i] -= a.lambda * (acc[MAPS - 1] * total[MAPS - 1]);
+        ss += v[i] * v[i];
+    }
+    float f = 1.0f;
+    if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(ss, scratch) / (float)a.vdim + a.eps) * a.out_scale;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        const uint32_t d = threadIdx.x + i * 256;
+        if (d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v[i] * f);
+    }
+}
+
+// One workgroup per (query row, head), 256 keys at a time; f32 arithmetic throughout.
+template <typename T>
+__global__ __launch_bounds__(256) void attention_plain_kernel(const AttentionArgs a) {
+    extern __shared__ float dyn[];                            // the query's maps * dim values
+    __shared__ float p[2][256], scratch[4];
+    const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, g = h / (a.heads / a.kv_heads), tid = threadIdx.x;
+    const uint32_t start = *a.position, last = min(start + t, a.capacity - 1);
+    const T* q = static_cast<const T*>(a.q) + ((size_t)t * a.heads + h) * a.maps * a.dq;
+    for (uint32_t i = tid; i < a.maps * a.dim; i += 256) dyn[i] = lh_ld(q, (size_t)(i / a.dim) * a.dq + i % a.dim);
+    __syncthreads();
+    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.0f, 0.0f}, acc[2][4] = {};
+    for (uint32_t k0 = 0; k0 <= last; k0 += 256) {
+        const uint32_t n = min(256u, last + 1 - k0);
+        for (uint32_t mp = 0; mp < a.maps; mp++) {
+            float s = -INFINITY;
+            if (tid < n) {
+                const T* k = static_cast<const T*>(a.keys) + (((size_t)(k0 + tid) * a.kv_heads + g) * a.maps + mp) * a.dq;
+                float dot = 0.0f;
+                for (uint32_t i = 0; i < a.dim; i++) dot = __builtin_fmaf(dyn[mp * a.dim + i], lh_ld(k, i), dot);
+                s = dot * a.scale;
+            }
+            float mx = lh_group_max(s, 64);
+            if ((tid & 63) == 0) scratch[tid >> 6] = mx;
+            __syncthreads();
+            mx = fmaxf(fmaxf(scratch[0], scratch[1]), fmaxf(scratch[2], scratch[3]));
+            __syncthreads();
+            const float nm = fmaxf(m[mp], mx), alpha = expf(m[mp] - nm), w = tid < n ? expf(s - nm) : 0.0f;
+            p[mp][tid] = w;
+            const float sum = lh_block_sum(w, scratch);
+            l[mp] = l[mp] * alpha + sum;
+            m[mp] = nm;
+#pragma unroll
+            for (int i = 0; i < 4; i++) acc[mp][i] *= alpha;
+        }
+        __syncthreads();
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const uint32_t d = tid + i * 256;
+            if (d >= a.vdim) break;
+            for (uint32_t j0 = 0; j0 < n; j0 += 32) {          // k0 is a multiple of 32
+                const T* v = static_cast<const T*>(a.values) + ((size_t)((k0 + j0) >> 5) * a.kv_heads * a.dv + (size_t)g * a.dv + d) * 32;
+                for (uint32_t j = 0; j < min(32u, n - j0); j++) {
+                    const float x = lh_ld(v, lh_block_slot(j));
+                    acc[0][i] = __builtin_fmaf(p[0][j0 + j], x, acc[0][i]);
+                    if (a.maps == 2) acc[1][i] = __builtin_fmaf(p[1][j0 + j], x, acc[1][i]);
+                }
+            }
+        }
+        __syncthreads();
+    }
+    float v[4], ss = 0.0f;
+#pragma unroll
+    for (int i = 0; i < 4; i++) {
+        v[i] = acc[0][i] / l[0];
+        if (a.maps == 2) v[i] -= a.lambda * (acc[1][i] / l[1]);
+        if (tid + i * 256 < a.vdim) ss += v[i] * v[i];
+    }
+    float f = 1.0f;
+    if (a.maps == 2) f = rsqrtf(lh_block_sum(ss, scratch) / (float)a.vdim + a.eps) * a.out_scale;
+#pragma unroll
+    for (int i = 0; i < 4; i++)
+        if (tid + i * 256 < a.vdim) lh_st(static_cast<T*>(a.out), ((size_t)t * a.heads + h) * a.vdim + tid + i * 256, v[i] * f);
+}
+
+constexpr uint32_t kMaxSplits = 512;
+
+template <int DQ, int DV, int MAPS>
+int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const char* op, uint32_t& launches) {
+    const uint32_t R = a.heads / a.kv_heads;
+    const uint64_t packed = (uint64_t)a.rows * R;
+    constexpr int RT = DV <= 128 && DQ <= 64 ? 2 : 1;
+    const uint64_t tiles = (packed + 64 * RT - 1) / (64 * RT);
+    const uint32_t max_blocks = (uint32_t)std::min<uint64_t>((uint64_t)max_position + a.rows, a.capacity) / 32 + 1;
+    const bool split = packed <= 64 || (tiles * a.kv_heads < (uint64_t)ctx->cu_count / 4 && packed <= 256);
+    if (!split) {
+        LH_REQUIRE(tiles * a.kv_heads < 0x7FFFFFFFull, "%s: %u rows", op, a.rows);
+        hipLaunchKernelGGL((attention_tile_kernel<DQ, DV, MAPS, RT>), dim3((uint32_t)(tiles * a.kv_heads)), dim3(256), 0, ctx->stream, a);
+        launches = 1;
+        return lh_check_launch(op);
+    }
+    const uint32_t st = (uint32_t)((packed + 15) / 16);
+    const size_t rec = (size_t)st * a.kv_heads * MAPS * 16 * (DV + 2) * 4;
+    // two blocks per wave at least, two workgroups per CU at most
+    uint32_t splits = std::max(1u, std::min({max_blocks / 8, (2u * ctx->cu_count + st * a.kv_heads - 1) / (st * a.kv_heads), kMaxSplits}));
+    splits = (uint32_t)std::min<size_t>(splits, std::max<size_t>(1, ctx->workspace_bytes / rec));
+    LH_REQUIRE(rec * splits <= ctx->workspace_bytes, "%s: %u heads of %u values exceed the workspace", op, a.heads, a.vdim);
+    a.partial = (float*)ctx->workspace;
+    a.splits = splits;
+    constexpr size_t lds = (size_t)4 * MAPS * 16 * (DV + 2) * 4;
+    if (lds > 64 * 1024) {
+        const int r = lh_raise_dynamic_lds(ctx, (const void*)attention_split_kernel<DQ, DV, MAPS>, lds, op);
+        if (r != LH_OK) return r;
+    }
+    hipLaunchKernelGGL((attention_split_kernel<DQ, DV, MAPS>), dim3(st * a.kv_heads * splits), dim3(256), lds, ctx->stream, a);
+    int r = lh_check_launch(op);
+    if (r != LH_OK) return r;
+    hipLaunchKernelGGL((attention_merge_kernel<MAPS>), dim3(a.rows * a.heads), dim3(256), 0, ctx->stream, a);
+    launches = 2;
+    return lh_check_launch(op);
+}
+
+template <int DQ, int DV>
+int launch_maps(lh_context* ctx, AttentionArgs& a, uint32_t mp, const char* op, uint32_t& n) {
+    return a.maps == 2 ? launch_mfma<DQ, DV, 2>(ctx, a, mp, op, n) : launch_mfma<DQ, DV, 1>(ctx, a, mp, op, n);
+}
+template <int DQ>
+int launch_dv(lh_context* ctx, AttentionArgs& a, uint32_t mp, const char* op, uint32_t& n) {
+    switch (a.dv) {
+        case 32: return launch_maps<DQ, 32>(ctx, a, mp, op, n);
+        case 64: return launch_maps<DQ, 64>(ctx, a, mp, op, n);
+        case 128: return launch_maps<DQ, 128>(ctx, a, mp, op, n);
+        default: return launch_maps<DQ, 256>(ctx, a, mp, op, n);
+    }
+}
+
+}  // namespace
+
+extern "C" {
+
+uint32_t lh_attention_padded_dim(uint32_t dim) { return dim <= 32 ? 32u : dim <= 64 ? 64u : (dim + 127) / 128 * 128; }
+uint32_t lh_attention_padded_vdim(uint32_t vdim) { return vdim <= 32 ? 32u : vdim <= 64 ? 64u : vdim <= 128 ? 128u : (vdim + 255) / 256 * 256; }
+
+int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* keys, const lh_buffer* values, lh_buffer* output, int dtype,
+                           const lh_buffer* position, uint32_t max_position, uint32_t rows, uint32_t heads, uint32_t kv_heads, uint32_t maps, uint32_t dim,
+                           uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps) {
+    const char* op = "attention_rows";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    LH_REQUIRE(dtype == LH_F32 || dtype == LH_BF16, "%s: dtype %d", op, dtype);
+    LH_REQUIRE(maps == 1 || maps == 2, "%s: %u maps", op, maps);
+    LH_REQUIRE(kv_heads > 0 && heads > 0 && heads % kv_heads == 0, "%s: heads %u is not a multiple of kv_heads %u", op, heads, kv_heads);
+    LH_REQUIRE(dim > 0 && dim <= 4096 && vdim > 0 && vdim <= 1024, "%s: dim %u, vdim %u", op, dim, vdim);
+    if (rows == 0) return LH_OK;
+    LH_REQUIRE(capacity > 0 && capacity % 32 == 0 && (uint64_t)max_position + rows <= capacity, "%s: positions up to %llu in caches of %u", op,
+               (unsigned long long)max_position + rows, capacity);
+    AttentionArgs a{};
+    a.dq = lh_attention_padded_dim(dim);
+    a.dv = lh_attention_padded_vdim(vdim);
+    const size_t es = dtype == LH_F32 ? 4 : 2;
+    LH_NEED(q, (size_t)rows * heads * maps * a.dq * es, op, "q");
+    LH_NEED(keys, (size_t)capacity * kv_heads * maps * a.dq * es, op, "keys");
+    LH_NEED(values, (size_t)capacity * kv_heads * a.dv * es, op, "values");
+    LH_NEED(output, (size_t)rows * heads * vdim * es, op, "output");
+    LH_NEED(position, 4, op, "position");
+    a.q = q->ptr; a.keys = keys->ptr; a.values = values->ptr; a.out = output->ptr; a.position = (const uint32_t*)position->ptr;
+    a.rows = rows; a.heads = heads; a.kv_heads = kv_heads; a.maps = maps; a.dim = dim; a.vdim = vdim; a.capacity = capacity;
+    a.scale = scale; a.lambda = lambda; a.out_scale = out_scale; a.eps = eps;
+    const bool aligned = (((uintptr_t)a.q | (uintptr_t)a.keys | (uintptr_t)a.values | (uintptr_t)a.out) & 15) == 0;
+    uint32_t launches = 0;
+    int r;
+    if (dtype == LH_BF16 && aligned && a.dq <= 128 && a.dv <= 256) {
+        if (a.dq == 32) r = launch_dv<32>(batch->ctx, a, max_position, op, launches);
+        else if (a.dq == 64) r = launch_dv<64>(batch->ctx, a, max_position, op, launches);
+        else r = launch_dv<128>(batch->ctx, a, max_position, op, launches);
+    } else {
+        LH_REQUIRE((uint64_t)rows * heads < 0x7FFFFFFFull, "%s: %u rows", op, rows);
+        const size_t lds = (size_t)maps * dim * 4;
+        if (dtype == LH_F32) hipLaunchKernelGGL((attention_plain_kernel<float>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
+        else hipLaunchKernelGGL((attention_plain_kernel<uint16_t>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
+        launches = 1;
+        r = lh_check_launch(op);
+    }
+    batch->dispatch_count += launches;
+    return r;
+}
+
+}  // extern "C"
