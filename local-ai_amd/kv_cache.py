@@ -6,7 +6,7 @@ import ctypes as C
 
 import numpy as np
 
-from . import Buffer, InvalidArgument, Kernels, lib
+from . import F32, Buffer, InvalidArgument, Kernels, lib
 
 TQ_SEED = 0x7459C0DE       # quant_cache.rs:30
 DEFAULT_KV_BITS = 2        # quant_cache.rs:37
@@ -303,3 +303,75 @@ class QuantizedUnifiedKvPool:
         for b, stride in ((self.keys_q, self._cb), (self.values_q, self._cb), (self.key_norms, 2),
                           (self.value_norms, 2)):
             b.view(lane * rows * stride, rows * stride).fill_zero()
+
+
+class BlockKvCache:
+    """Keys and values of one softmax-attention layer run for one sequence, unquantized (bf16, or f32 for runs in full
+    precision), in the layouts of ``lh_attention_rows_into``: keys [position][kv head][map][padded dim], values in blocks of
+    32 positions [block][kv head][padded value dim][32]."""
+
+    def __init__(self, ctx, kernels: Kernels, kv_heads: int, maps: int, dim: int, vdim: int, capacity: int, dtype: int):
+        self.capacity = (capacity + 31) // 32 * 32
+        size = 4 if dtype == F32 else 2
+        self.keys = Buffer.empty(ctx, self.capacity * kv_heads * maps * kernels.attention_padded_dim(dim) * size)
+        self.values = Buffer.empty(ctx, self.capacity * kv_heads * kernels.attention_padded_vdim(vdim) * size)
+
+    def reset(self) -> None:
+        """Cleared, not only forgotten: the entries of a block past the last position enter products with weight zero."""
+        self.keys.fill_zero()
+        self.values.fill_zero()
+
+
+class RecurrentState:
+    """The f32 state of one linear-attention layer run for one sequence: [head][value column][padded key dim]."""
+
+    def __init__(self, ctx, kernels: Kernels, heads: int, dim: int, vdim: int):
+        self.state = Buffer.empty(ctx, heads * vdim * kernels.linear_attention_padded_dim(dim) * 4)
+
+    def reset(self) -> None:
+        self.state.fill_zero()
+
+
+class SequenceSlot:
+    """Everything one live sequence holds: a cache or state per layer run, and its position on the host and on the device."""
+
+    def __init__(self, ctx, memories):
+        self.memories = memories
+        self.position_buf = Buffer.empty(ctx, 4)
+        self.position = 0
+        # the slot's recorded decode step, the scratch it was recorded with, and whether a step has run unrecorded
+        self.graph, self.graph_version, self.graph_ready = None, -1, False
+
+    def reset(self) -> None:
+        for m in self.memories:
+            m.reset()
+        self.position_buf.fill_zero()
+        self.position = 0
+
+
+class SlotPool:
+    """Slots for live sequences, made when first needed and used again after they are given back."""
+
+    def __init__(self, make, limit: int):
+        self._make, self.limit = make, limit
+        self._free, self._live = [], set()
+
+    def acquire(self):
+        if self._free:
+            slot = self._free.pop()
+        elif len(self._live) < self.limit:
+            slot = self._make()
+        else:
+            raise InvalidArgument(f"all {self.limit} sequence slots are in use")
+        self._live.add(slot)
+        return slot
+
+    def release(self, slot) -> None:
+        if slot not in self._live:
+            raise InvalidArgument("the slot is not in use")
+        self._live.remove(slot)
+        slot.reset()
+        self._free.append(slot)
+
+    def available(self) -> int:
+        return self.limit - len(self._live)

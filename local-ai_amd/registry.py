@@ -1,0 +1,69 @@
+"""Model registry: the ``architecture`` of a model folder's config.json -> how its configuration is read and which pipeline
+serves it."""
+from __future__ import annotations
+
+import json
+import os
+from typing import Callable, Dict
+
+from . import BF16, Context, InvalidArgument, Io, Kernels
+from .mixers import AttentionSpec, DenseSpec, LayerSpec, LinearAttentionSpec, MoeSpec
+from .safetensors import SafetensorsFile
+from .stack_pipeline import Loop, StackConfig, StackPipeline
+
+ARCHITECTURES: Dict[str, Callable] = {}      # name -> config dict -> StackConfig
+
+
+def register(name: str):
+    def add(reader):
+        ARCHITECTURES[name] = reader
+        return reader
+    return add
+
+
+def read_config(config: dict) -> StackConfig:
+    name = config.get("architecture")
+    if name not in ARCHITECTURES:
+        raise InvalidArgument(f"unknown architecture {name!r} (known: {', '.join(sorted(ARCHITECTURES))})")
+    try:
+        return ARCHITECTURES[name](config)
+    except (KeyError, TypeError) as e:
+        raise InvalidArgument(f"{name}: configuration lacks or misplaces {e}") from e
+
+
+def load_model(path: str, max_tokens: int, dtype: int = BF16, ctx=None, **options) -> StackPipeline:
+    """The pipeline for the model in folder `path` (config.json, model.safetensors)."""
+    try:
+        with open(os.path.join(path, "config.json")) as f:
+            config = json.load(f)
+    except (OSError, ValueError) as e:
+        raise Io(f"{path}: {e}") from e
+    stack = read_config(config)
+    tensors = SafetensorsFile(os.path.join(path, "model.safetensors"))
+    ctx = ctx or Context(0)
+    return StackPipeline(ctx, Kernels(ctx), stack, tensors, max_tokens, dtype, **options)
+
+
+@register("Komirax")
+def komirax(config: dict) -> StackConfig:
+    """Differential-attention and lightning-attention layers in any order, dense or routed feed-forwards, an optional loop."""
+    def mixer(kind, m):
+        if kind == "attention":
+            return AttentionSpec(m["heads"], m["kv_heads"], m["dim"], m["vdim"], m["scale"], maps=2, diff=m["diff"], bias=True)
+        if kind == "lightning":
+            return LinearAttentionSpec(m["heads"], m["dim"], m["vdim"], list(m["decay"]))
+        raise InvalidArgument(f"unknown layer type {kind!r}")
+
+    def feed_forward(f):
+        if f is None:
+            return None
+        if f["kind"] == "dense":
+            return DenseSpec(f["ff"])
+        if f["kind"] == "moe":
+            return MoeSpec(f["router"]["experts"], f["router"]["top"], f["expert"]["ff"])
+        raise InvalidArgument(f"unknown feed-forward {f['kind']!r}")
+
+    layers = [LayerSpec(mixer(l["type"], l["mixer"]), feed_forward(l.get("mlp"))) for l in config["layers"]]
+    loop = config.get("loop")
+    return StackConfig(config["vocab"], config["width"], config["norm"]["eps"], layers,
+                       Loop(loop["start"], loop["stop"], loop["times"]) if loop else None)
