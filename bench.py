@@ -837,6 +837,217 @@ def cpu_baseline_attention(pkg, st, target_s=8.0):
                       f"f32 softmax . V; OpenMP over positions); single thread: {1.0 / single:.2f} tokens/s, {alg / single * 1e-9:.4f} GB/s"}
 
 
+# ---- models with bf16 weights (legs "stack_kernels" and "stack_models", not in the default set) -------------------------------------------------------
+
+class RandomTensors:
+    """Random weights of any shape by name (a repeated block of normal values, 1/sqrt(columns) in size)."""
+
+    def __init__(self, seed=0):
+        self._block = np.random.default_rng(seed).standard_normal(1 << 20).astype(np.float32)
+
+    def f32(self, name, shape):
+        scale = 1.0 / np.sqrt(shape[1]) if len(shape) == 2 else 0.3
+        x = np.resize(np.roll(self._block, hash_of(name)), shape) * np.float32(scale)
+        return x + 1.0 if "norm" in name else x
+
+    def bf16(self, name, shape):
+        from local_ai_amd.safetensors import round_to_bf16
+        return round_to_bf16(self.f32(name, shape))
+
+
+def hash_of(name):
+    return sum((i + 1) * 7919 * ord(c) for i, c in enumerate(name)) % (1 << 20)
+
+
+def random_bits(ctx, pkg, nbytes, seed=0):
+    """Device buffer of bf16 bits (normal values x 2^-6, also sane as f16 bits up to scale)."""
+    from local_ai_amd.safetensors import round_to_bf16
+    block = round_to_bf16(np.random.default_rng(seed).standard_normal(1 << 20).astype(np.float32) / 64)
+    return pkg.Buffer.from_slice(ctx, np.resize(block, nbytes // 2))
+
+
+def bench_stack_kernels(pkg, ctx, K, steps, warmup):
+    """The kernels of a bf16-weight stack, each beside the like kernel of the quantized decoder at the same size: fraction of
+    the HBM peak (one row, decoding) or of the dense f16/bf16 matrix peak (many rows)."""
+    import ctypes as C
+    L, lw, res = pkg.lib(), pkg.linear_weight, {}
+    batch = pkg.CommandBatch(ctx)
+    F16, F32, BF16 = pkg.F16, pkg.F32, pkg.BF16
+
+    def timed(name, fns, byte=None, flop=None):
+        """`fns`: the same call on distinct data, in turn (so that nothing comes from a cache)."""
+        it = [0]
+
+        def step():
+            fns[it[0] % len(fns)]()
+            it[0] += 1
+        _, ev = time_steps(pkg, ctx, step, max(steps, len(fns), 20), warmup)
+        r = {"us": ev * 1e3}
+        if byte:
+            r.update(gbs=byte / (ev * 1e-3) * 1e-9, frac_of_hbm_peak=byte / (ev * 1e-3) * 1e-9 / HBM_PEAK_GBS)
+        if flop:
+            r.update(tflops=flop / (ev * 1e-3) * 1e-12, frac_of_mfma_peak=flop / (ev * 1e-3) * 1e-12 / MFMA_F16_PEAK_TFLOPS)
+        res[name] = r
+        log(f"[bench] stack {name}: " + ", ".join(f"{k} {v:.4g}" for k, v in r.items()))
+
+    # one row
+    for n, k in ((2048, 2048), (8192, 2048), (2048, 8192), (131072, 2048)):
+        byte = n * k * 2
+        reps = max(1, min(64, (1 << 29) // byte))
+        big = random_bits(ctx, pkg, byte * reps)
+        ws = [big.view(i * byte, byte) for i in range(reps)]
+        seg = lw.Segments([lw.Segment(n)])
+        x, nw = pkg.Buffer.from_slice(ctx, np.ones(k, np.float32)), pkg.Buffer.from_slice(ctx, np.ones(k, np.float32))
+        xh, y = pkg.Buffer.from_slice(ctx, np.ones(k, np.float16)), pkg.Buffer.empty(ctx, n * 4)
+        timed(f"row {n}x{k} bf16, norm in front", [lambda w=w: K.linear_norm_vector_into(batch, x, None, None, nw, 1e-6, w, None, k, seg, [y], F32) for w in ws], byte)
+        timed(f"row {n}x{k} bf16, residual add", [lambda w=w: K.linear_vector_into(batch, x, F32, w, None, k, seg, [y], F32, True) for w in ws], byte)
+        timed(f"row {n}x{k} f16 (existing)", [lambda w=w: K.matvec_f32out_offset_into(batch, w, 0, xh, y, n, k) for w in ws], byte)
+        big.free()
+    # many rows
+    for m, k, n in ((256, 2048, 2048), (256, 2048, 8192), (512, 2048, 8192), (2048, 2048, 2048), (2048, 2048, 8192), (2048, 8192, 2048)):
+        x, w, y = random_bits(ctx, pkg, m * k * 2, 1), random_bits(ctx, pkg, n * k * 2, 2), pkg.Buffer.empty(ctx, m * n * 4)
+        seg, flop = lw.Segments([lw.Segment(n)]), 2.0 * m * n * k
+        timed(f"rows {m}x{k}x{n} bf16", [lambda: K.linear_rows_into(batch, x, BF16, w, None, m, k, seg, [y], BF16)], None, flop)
+        timed(f"rows {m}x{k}x{n} bf16, residual add", [lambda: K.linear_rows_into(batch, x, BF16, w, None, m, k, seg, [y], F32, True)], None, flop)
+        timed(f"rows {m}x{k}x{n} f16 (existing)", [lambda: K.matmul_nt_into(batch, x, w, y, m, k, n)], None, flop)
+        q = pkg.QuantWeight.from_bytes(ctx, pkg.synth.weights("tq2_0", n, k, pkg.synth.rng(4, 2)), pkg.TQ2_0, n, k)
+        timed(f"rows {m}x{k}x{n} tq2_0 (existing)", [lambda: q.matmul_nt_into(batch, K, x, y, m)], None, flop)
+    # softmax attention: 16 heads over 4, two maps of 64, values of 128 -- the cache bytes of one map of 128
+    H, G, D, V, T = 16, 4, 64, 128, 32768
+    cap = T + 2304
+    caches = [(random_bits(ctx, pkg, cap * G * 2 * D * 2, i), random_bits(ctx, pkg, cap * G * V * 2, i + 9)) for i in range(8)]
+    q, o = random_bits(ctx, pkg, 2048 * H * 2 * D * 2, 3), pkg.Buffer.empty(ctx, 2048 * H * V * 2)
+    for t, rows in ((T - 1, 1), (4095, 1)):
+        pos, byte = pkg.Buffer.from_slice(ctx, np.array([t], np.uint32)), (t + 1) * G * (2 * D + V) * 2
+        timed(f"attention decode, {t + 1} positions, two maps",
+              [lambda c=c: K.attention_rows_into(batch, q, c[0], c[1], o, BF16, pos, t, 1, H, G, 2, D, V, cap, 0.125, 0.3, 0.7, 1e-6) for c in caches], byte)
+        timed(f"attention decode, {t + 1} positions, f16 (existing)",
+              [lambda c=c: K.flash_decoding_into(batch, q, c[0], c[1], o, 128, t + 1, t, H, G) for c in caches], byte)
+    for t, rows in ((0, 2048), (T, 256), (2048, 2048)):
+        pos = pkg.Buffer.from_slice(ctx, np.array([t], np.uint32))
+        pairs = rows * t + rows * (rows + 1) / 2
+        timed(f"attention prefill, {rows} rows at {t}, two maps",
+              [lambda: K.attention_rows_into(batch, q, caches[0][0], caches[0][1], o, BF16, pos, t, rows, H, G, 2, D, V, cap, 0.125, 0.3, 0.7, 1e-6)],
+              None, pairs * H * 2 * 2 * (D + V))
+    del caches
+    pre = bench_attention_prefill(pkg, ctx, K, steps, warmup)
+    log("[bench] stack tq2 prefill attention 256 x 32768 (existing):", pre)
+    res["tq2 prefill attention 256x32768 (existing)"] = pre
+    # linear attention: 16 heads, 128 x 128
+    H, D = 16, 128
+    q, k, v = (random_bits(ctx, pkg, 4096 * H * D * 2, i) for i in range(3))
+    decay = np.linspace(0.9, 0.999, H)
+    db, pw = pkg.Buffer.from_slice(ctx, decay.astype(np.float32)), pkg.Buffer.from_slice(ctx, (decay[:, None] ** np.arange(65)).astype(np.float32))
+    o = pkg.Buffer.empty(ctx, 4096 * H * D * 4)
+    states = [pkg.Buffer.empty(ctx, H * D * D * 4) for _ in range(64)]
+    timed("linear attention, one row", [lambda s=s: K.linear_attention_recurrent_into(batch, q, k, v, BF16, s, db, o, 1, H, D, D) for s in states], 2 * H * D * D * 4)
+    work = pkg.Buffer.empty(ctx, K.linear_attention_workspace_bytes(4096, H, D, D))
+    for rows in (256, 2048, 4096):
+        # bytes: q, k, v once each by the kernels that need them, the chunk states written and read twice, the outputs
+        byte = rows * H * D * 2 * 5 + 4 * K.linear_attention_workspace_bytes(rows, H, D, D) + rows * H * D * 4
+        timed(f"linear attention, {rows} rows", [lambda: K.linear_attention_chunked_into(batch, q, k, v, states[0], pw, work, o, rows, H, D, D)], byte)
+    # experts: 16 of 2048 -> 1024, two of them
+    E, top, W, F = 16, 2, 2048, 1024
+    up, down = [random_bits(ctx, pkg, E * W * F * 2, i) for i in range(2)], [random_bits(ctx, pkg, E * W * F * 2, i + 5) for i in range(2)]
+    logits = [pkg.Buffer.from_slice(ctx, np.random.default_rng(i).standard_normal((2048, E)).astype(np.float32)) for i in range(13)]
+    x, h, y = random_bits(ctx, pkg, 2048 * W * 2), pkg.Buffer.empty(ctx, 2048 * top * F * 4), pkg.Buffer.empty(ctx, 2048 * W * 4)
+    xf, nw = pkg.Buffer.from_slice(ctx, np.ones(W, np.float32)), pkg.Buffer.from_slice(ctx, np.ones(W, np.float32))
+    slots, plan = pkg.Buffer.empty(ctx, 2048 * top * W * 4), pkg.Buffer.empty(ctx, 4 * K.moe_plan_words(2048, E, top))
+    timed("experts, one row: up", [lambda i=i: K.moe_vector_up_into(batch, xf, nw, 1e-6, logits[i], up[i % 2], h, E, top, W, F, pkg.ACT_RELU_SQUARED) for i in range(13)], top * W * F * 2)
+    timed("experts, one row: down", [lambda i=i: K.moe_vector_down_into(batch, h, logits[i], down[i % 2], y, E, top, W, F) for i in range(13)], top * W * F * 2)
+    for rows in (256, 2048):
+        timed(f"experts, {rows} rows: route", [lambda: K.moe_route_into(batch, logits[0], plan, rows, E, top)])
+        timed(f"experts, {rows} rows: up", [lambda: K.moe_up_into(batch, x, BF16, plan, up[0], h, rows, E, top, W, F, pkg.ACT_RELU_SQUARED)], None, 2.0 * rows * top * W * F)
+        timed(f"experts, {rows} rows: down", [lambda: K.moe_down_into(batch, h, BF16, plan, down[0], slots, y, rows, E, top, W, F)], None, 2.0 * rows * top * W * F)
+    return res
+
+
+def bench_stack_models(pkg, ctx, K, steps, warmup):
+    """Tokens per second of whole stacks with random weights, beside the quantized decoder at equal width, depth and context:
+    decoding (a recorded step each) and prompts in passes of 2048 rows."""
+    A = pkg.mixers
+    res = {}
+    for width, heads, kv, ff, experts in ((1024, 8, 2, 4096, 8), (2048, 16, 4, 8192, 16)):
+        attn = A.AttentionSpec(heads, kv, 64, 128, 0.125, maps=2, diff=0.3, bias=True)
+        lin = A.LinearAttentionSpec(width // 128, 128, 128, list(np.linspace(0.9, 0.999, width // 128)))
+        moe, dense = A.MoeSpec(experts, 2, ff // 8), A.DenseSpec(ff)
+        cfg = pkg.stack_pipeline.StackConfig(32000, width, 1e-6, [A.LayerSpec(m, f) for m, f in ((attn, dense), (lin, dense), (attn, moe), (lin, moe))])
+        T = 4096
+        m = pkg.stack_pipeline.StackPipeline(ctx, K, cfg, RandomTensors(1), T + 512)
+        tokens = [int(t) for t in np.random.default_rng(2).integers(0, 32000, T)]
+        out = {}
+        for rows in (256, 2048):
+            m.max_rows = rows
+
+            def prompt():
+                s = m.new_sequence()
+                m.step(s, tokens, [T - 1])
+                m.end_sequence(s)
+            prompt()
+            t0 = time.perf_counter()
+            for _ in range(3):
+                prompt()
+            out[f"prompt_tokens_per_s_passes_of_{rows}"] = 3 * T / (time.perf_counter() - t0)
+        s = m.new_sequence()
+        m.step(s, tokens)
+        for _ in range(5):
+            m.greedy(s, 1)
+        n = 200
+        t0 = time.perf_counter()
+        for _ in range(n):
+            m.greedy(s, 1)
+        out["decode_us_per_token_with_host"] = (time.perf_counter() - t0) / n * 1e6
+        settle(ctx, s.graph.launch, 100)
+        e0, e1 = pkg.Event(ctx), pkg.Event(ctx)
+        s.position_buf.copy_from_bytes(np.array([T], np.uint32))
+        e0.record()
+        for _ in range(100):
+            s.graph.launch()
+        e1.record()
+        ctx.synchronize()
+        us = e0.elapsed_ms(e1) * 10
+        # bytes a decoded token has to read: every weight but the unchosen experts, the attention caches, the states twice
+        byte = sum(b.bytes() for l in m.layers for b in (l.mixer.out, getattr(l.mixer, "qkv", None) or l.mixer.qkvg)) + m.head.bytes()
+        byte += sum(l.ff.up.bytes() + l.ff.down.bytes() if isinstance(l.ff, A.DenseFeedForward) else 2 * 2 * 2 * width * (ff // 8) for l in m.layers)
+        byte += 2 * T * kv * (2 * 64 + 128) * 2 + 2 * 2 * lin.heads * 128 * 128 * 4
+        out.update(decode_us_per_token=us, decode_tokens_per_s=1e6 / us, decode_dispatches=s.graph.dispatch_count(),
+                   decode_gbs=byte / us * 1e-3, decode_frac_of_hbm_peak=byte / us * 1e-3 / HBM_PEAK_GBS)
+        m.end_sequence(s)
+        del m
+        gcfg = pkg.pipeline.Gemma4QATConfig(vocab_size=32000, hidden_size=width, num_hidden_layers=4, num_attention_heads=width // 256, num_key_value_heads=1,
+                                            head_dim=256, global_head_dim=256, layer_types=["full_attention"] * 4)
+        pipe = pkg.pipeline.DecodePipeline.from_host(ctx, K, gcfg, pkg.synth.decode_model_tensors(gcfg, pkg.synth.rng(3), ff), T + 512)
+        pipe.prefill_prompt(tokens)
+        t0 = time.perf_counter()
+        for _ in range(3):
+            pipe.reset()
+            pipe.prefill_prompt(tokens)
+        out["quantized_prompt_tokens_per_s_passes_of_256"] = 3 * T / (time.perf_counter() - t0)
+        pipe.position = T
+        for _ in range(5):
+            pipe.decode_step(1)
+        t0 = time.perf_counter()
+        for _ in range(n):
+            pipe.decode_step(1)
+        out["quantized_decode_us_per_token_with_host"] = (time.perf_counter() - t0) / n * 1e6
+        batch = pkg.CommandBatch(ctx)
+        batch.begin_capture()
+        pipe.write_logits(pipe.forward_token(1, T, batch=batch), batch=batch)
+        graph = batch.end_capture()
+        settle(ctx, graph.launch, 100)
+        e0.record()
+        for _ in range(100):
+            graph.launch()
+        e1.record()
+        ctx.synchronize()
+        out["quantized_decode_us_per_token"] = e0.elapsed_ms(e1) * 10
+        out["quantized_decode_dispatches"] = graph.dispatch_count()
+        del pipe, graph
+        res[f"width_{width}"] = out
+        log(f"[bench] stack model width {width}:", out)
+    return res
+
+
 def main():
     global SETTLE_MS
     ap = argparse.ArgumentParser()
@@ -854,7 +1065,8 @@ def main():
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--legs", default="matvec,attention,sweep,layer,prefill,glue,decode,lanes,chunk,model,model_lanes",
                     help="comma-separated extra measurements to run besides the headline (for profiling one kernel at a time); "
-                         "model_few_lanes (2 .. 16 sequences at 8k context) is not in the default set")
+                         "model_few_lanes (2 .. 16 sequences at 8k context), stack_kernels and stack_models (models with bf16 "
+                         "weights beside the quantized decoder) are not in the default set")
     args = ap.parse_args()
     SETTLE_MS = args.settle_ms
     if args.gpus != 1:
@@ -959,6 +1171,11 @@ def main():
                                                          lanes=64 if "model_lanes" in legs else 0, defer_tail=not args.no_defer_tail,
                                                          rotate_in_o=not args.no_rotate_in_o)
         log("[bench] model decode:", extra["model_decode_e2b_geometry"])
+
+    if "stack_kernels" in legs:
+        extra["stack_kernels"] = bench_stack_kernels(pkg, ctx, K, args.steps, args.warmup)
+    if "stack_models" in legs:
+        extra["stack_models"] = bench_stack_models(pkg, ctx, K, args.steps, args.warmup)
 
     achieved = head["alg_bytes_per_launch"] / head["ms_per_launch_events"] * 1e-6
     # The other north-star kernels of this run, in the blocks a reader of the line keeps: their rooflines beside the

@@ -55,6 +55,36 @@ __device__ __forceinline__ void tile_of_block(uint32_t mt_n, uint32_t nt_n, uint
     nt = r / m_in;
 }
 
+// Bias, activation and destination of columns n .. n + 3 (those below N) of one row of a product.
+__device__ __forceinline__ void store4(const LhLinear& a, uint32_t slot, uint32_t n, const float4 acc, uint32_t pos0) {
+    const OutRow o = out_row(a, slot);
+    float v[4] = {acc.x, acc.y, acc.z, acc.w};
+#pragma unroll
+    for (int r = 0; r < 4; r++) v[r] = v[r] * o.weight + (a.bias && n + r < a.N ? a.bias[n + r] : 0.0f);
+    if (!a.seg.vec4) {
+#pragma unroll 1
+        for (uint32_t r = 0; r < 4 && n + r < a.N; r++) lh_segment_store(a.seg, o.row, n + r, r == 0 ? v[0] : r == 1 ? v[1] : r == 2 ? v[2] : v[3], pos0);
+        return;
+    }
+    const uint32_t s = lh_segment_of(a.seg, n);              // the four columns are one aligned piece of one segment
+    const uint32_t p = a.seg.layout[s] == LH_ROWS ? o.row : pos0 + o.row;
+    if (p >= a.seg.rows[s]) return;
+    const size_t idx = (size_t)p * a.seg.ld[s] + (n - a.seg.n0[s]);
+    const uint32_t act = a.seg.act[s];
+    if (act != LH_ACT_NONE) {
+#pragma unroll
+        for (int r = 0; r < 4; r++) v[r] = lh_activate(v[r], act);
+    }
+    if (a.seg.f32_out) {
+        float4* d = reinterpret_cast<float4*>(static_cast<float*>(a.seg.out[s]) + idx);
+        float4 t = make_float4(v[0], v[1], v[2], v[3]);
+        if (a.seg.accumulate) { const float4 x = *d; t.x += x.x; t.y += x.y; t.z += x.z; t.w += x.w; }
+        *d = t;
+    } else {
+        *reinterpret_cast<uint2*>(static_cast<uint16_t*>(a.seg.out[s]) + idx) = make_uint2(lh_pack_bf(v[0], v[1]), lh_pack_bf(v[2], v[3]));
+    }
+}
+
 // ---- matrix cores ------------------------------------------------------------------------------------------------------
 // 256 threads, 2 x 2 waves of BM/2 x BN/2 outputs.  A k step is 64 wide: a tile row is eight 16-byte chunks, chunk c of row r
 // kept at place c ^ (r & 7) of its row so that the fragment reads of sixteen rows fall on different banks (the loads
@@ -87,11 +117,18 @@ __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
 
     auto load_step = [&](int buf, uint32_t kt) {
         uint4* base = &sm[buf][wave * 64];
-        const bool past = kt * 64 + src * 8 >= K;            // only in the last step of a ragged K
+        if (kt * 64 + 64 <= K) {
 #pragma unroll
-        for (int i = 0; i < CA; i++) load_lds16(past ? (const void*)&g_zero16 : (const void*)(pa[i] + kt * 64), base + i * 256);
+            for (int i = 0; i < CA; i++) load_lds16(pa[i] + kt * 64, base + i * 256);
 #pragma unroll
-        for (int i = 0; i < CB; i++) load_lds16(past ? (const void*)&g_zero16 : (const void*)(pb[i] + kt * 64), base + (CA + i) * 256);
+            for (int i = 0; i < CB; i++) load_lds16(pb[i] + kt * 64, base + (CA + i) * 256);
+        } else {                                             // the last step of a ragged K: chunks past it read zeros
+            const bool past = kt * 64 + src * 8 >= K;
+#pragma unroll
+            for (int i = 0; i < CA; i++) load_lds16(past ? (const void*)&g_zero16 : (const void*)(pa[i] + kt * 64), base + i * 256);
+#pragma unroll
+            for (int i = 0; i < CB; i++) load_lds16(past ? (const void*)&g_zero16 : (const void*)(pb[i] + kt * 64), base + (CA + i) * 256);
+        }
     };
 
     lh_f32x4 acc[TI][TJ];
@@ -128,40 +165,24 @@ __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
         }
     }
 
-    const uint32_t pos0 = a.seg.position ? *a.seg.position : 0u;
+    // The tile goes through LDS, so that a wave stores whole stretches of a row (and the store code exists once): four columns
+    // of row m are the 16-byte piece n / 4, kept at place (n / 4) ^ (m & 7).
+    __syncthreads();
+    float4* tile = reinterpret_cast<float4*>(&sm[0][0]);
 #pragma unroll
-    for (int i = 0; i < TI; i++) {
-        const uint32_t slot = rt.begin + wm * (BM / 2) + i * 16 + (lane & 15);
-        if (slot >= rt.end) continue;
-        const OutRow o = out_row(a, slot);
+    for (int i = 0; i < TI; i++)
 #pragma unroll
         for (int j = 0; j < TJ; j++) {
-            const uint32_t n = n0 + wn * (BN / 2) + j * 16 + (lane >> 4) * 4;
-            if (n >= a.N) continue;
-            float v[4];
-#pragma unroll
-            for (int r = 0; r < 4; r++) v[r] = acc[i][j][r] * o.weight + (a.bias && n + r < a.N ? a.bias[n + r] : 0.0f);
-            if (a.seg.vec4) {                                // the four columns are one aligned piece of one segment
-                const uint32_t s = lh_segment_of(a.seg, n);
-                const uint32_t p = a.seg.layout[s] == LH_ROWS ? o.row : pos0 + o.row;
-                if (p >= a.seg.rows[s]) continue;
-                const size_t idx = (size_t)p * a.seg.ld[s] + (n - a.seg.n0[s]);
-#pragma unroll
-                for (int r = 0; r < 4; r++) v[r] = lh_activate(v[r], a.seg.act[s]);
-                if (a.seg.f32_out) {
-                    float4* d = reinterpret_cast<float4*>(static_cast<float*>(a.seg.out[s]) + idx);
-                    float4 t = make_float4(v[0], v[1], v[2], v[3]);
-                    if (a.seg.accumulate) { const float4 x = *d; t.x += x.x; t.y += x.y; t.z += x.z; t.w += x.w; }
-                    *d = t;
-                } else {
-                    *reinterpret_cast<uint2*>(static_cast<uint16_t*>(a.seg.out[s]) + idx) = make_uint2(lh_pack_bf(v[0], v[1]), lh_pack_bf(v[2], v[3]));
-                }
-            } else {
-#pragma unroll
-                for (int r = 0; r < 4; r++)
-                    if (n + r < a.N) lh_segment_store(a.seg, o.row, n + r, v[r], pos0);
-            }
+            const uint32_t m = wm * (BM / 2) + i * 16 + (lane & 15), c = (wn * (BN / 2) + j * 16) / 4 + (lane >> 4);
+            tile[m * (BN / 4) + (c ^ (m & 7))] = make_float4(acc[i][j][0], acc[i][j][1], acc[i][j][2], acc[i][j][3]);
         }
+    __syncthreads();
+    const uint32_t pos0 = a.seg.position ? *a.seg.position : 0u;
+#pragma unroll 1
+    for (uint32_t e = tid; e < BM * BN / 4; e += 256) {
+        const uint32_t m = e / (BN / 4), c = e % (BN / 4), n = n0 + c * 4, slot = rt.begin + m;
+        if (slot >= rt.end || n >= a.N) continue;
+        store4(a, slot, n, tile[m * (BN / 4) + (c ^ (m & 7))], pos0);
     }
 }
 
@@ -213,25 +234,6 @@ __global__ __launch_bounds__(256) void linear_plain_kernel(const LhLinear a) {
 }
 
 // ---- one row -----------------------------------------------------------------------------------------------------------
-enum { kPlain = 0, kNorm = 1, kGated = 2 };
-struct VectorStage {
-    const void* x;             // plain: x_f32 ? f32 : bf16; norm, gated: f32
-    uint32_t x_f32;
-    const float* add;          // norm: may be null
-    float* store;              // norm: receives x + add (workgroup 0), may be null
-    const float* norm_weight;
-    const void* gate;          // gated
-    uint32_t gate_f32;
-    float eps;
-};
-
-// Weights are read once per launch: streaming loads.
-__device__ __forceinline__ uint4 ld16_stream(const uint16_t* p) {
-    typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
-    const u32x4_t v = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(p));
-    return make_uint4(v.x, v.y, v.z, v.w);
-}
-
 // Place of element k in the staged vector: the two halves of an 8-element chunk lie in planes of 64 x 16 bytes, so that the
 // 16-byte reads of a wave (lane = chunk) are in order.
 __device__ __forceinline__ uint32_t x_place(uint32_t k) {
@@ -285,6 +287,26 @@ __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, u
     __syncthreads();
 }
 
+// The finished sums of a wave's rows, one per lane, stored 64 at a time: bias, activation and destination then cost one pass
+// for all of them, and no load of that pass has to wait for weights that were requested in between.
+struct RowSums {
+    const LhSegments& seg;
+    const float* bias;
+    const uint32_t lane, step;
+    uint32_t row0, n = 0;
+    float mine = 0.0f;
+    __device__ __forceinline__ void add(float total) {
+        mine = n == lane ? total : mine;
+        if (++n == 64) flush();
+    }
+    __device__ __forceinline__ void flush() {
+        const uint32_t row = row0 + lane * step;
+        if (lane < n) lh_segment_store(seg, 0, row, mine + (bias ? bias[row] : 0.0f), seg.position ? *seg.position : 0u);
+        row0 += n * step;
+        n = 0;
+    }
+};
+
 // A wave takes rows round robin over the grid, 8 weights (16 bytes) per lane and load, NL loads per pass of a row; the loads
 // of the next pass are issued before the arithmetic of the current one.  Past the row's end the address is clamped and the
 // staged vector is zero.  VEC false (K not a multiple of 8): single weights.
@@ -295,11 +317,7 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
     __shared__ float scratch[4];
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     stage_vector<STAGE>(st, xs, scratch, K);
-    const uint32_t pos0 = seg.position ? *seg.position : 0u;
-    auto finish = [&](uint32_t row, float acc) {
-        const float total = lh_group_sum(acc, 64);
-        if (lane == 0) lh_segment_store(seg, 0, row, total + (bias ? bias[row] : 0.0f), pos0);
-    };
+    RowSums sums{seg, bias, lane, gridDim.x * 4, blockIdx.x * 4 + wave};
     if constexpr (VEC) {
         constexpr uint32_t kPass = 512u * NL;
         const uint32_t ppr = (K + kPass - 1) / kPass, row_step = gridDim.x * 4, last = (K >> 3) - 1;
@@ -307,7 +325,7 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
         auto issue = [&](uint4 (&v)[NL], uint32_t r, uint32_t ps) {
             const uint16_t* wr = W + (size_t)r * K;
 #pragma unroll
-            for (int c = 0; c < NL; c++) v[c] = ld16_stream(wr + 8 * min(ps * (kPass >> 3) + 64u * c + lane, last));
+            for (int c = 0; c < NL; c++) v[c] = lh_ld16_stream(wr + 8 * min(ps * (kPass >> 3) + 64u * c + lane, last));
         };
         float acc = 0.0f;
         auto consume = [&](const uint4 (&v)[NL], uint32_t r, uint32_t ps) {
@@ -324,7 +342,7 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
                     acc = __builtin_fmaf(__builtin_bit_cast(float, wv[j] & 0xFFFF0000u), xv[2 * j + 1], acc);
                 }
             }
-            if (ps + 1 == ppr) { finish(r, acc); acc = 0.0f; }
+            if (ps + 1 == ppr) { sums.add(lh_group_sum(acc, 64)); acc = 0.0f; }
         };
         auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {   // false: that was the wave's last pass
             uint32_t nrow = row, npass = pass + 1;
@@ -344,9 +362,41 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
         for (uint32_t row = blockIdx.x * 4 + wave; row < N; row += gridDim.x * 4) {
             float acc = 0.0f;
             for (uint32_t k = lane; k < K; k += 64) acc = __builtin_fmaf(lh_bf2f(W[(size_t)row * K + k]), xs[x_place(k)], acc);
-            finish(row, acc);
+            sums.add(lh_group_sum(acc, 64));
         }
     }
+    sums.flush();
+}
+
+// The same with the vector in registers (K up to 512 * NL): the first row's weights are requested before the vector.
+template <int STAGE, int NL>
+__global__ __launch_bounds__(256) void matvec_bf16_reg_kernel(const VectorStage st, const uint16_t* __restrict__ W, const float* __restrict__ bias, const LhSegments seg,
+                                                             uint32_t N, uint32_t K) {
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row_step = gridDim.x * 4, last = (K >> 3) - 1;
+    auto issue = [&](uint4 (&v)[NL], uint32_t r) {
+        const uint16_t* wr = W + (size_t)r * K;
+#pragma unroll
+        for (int c = 0; c < NL; c++) v[c] = lh_ld16_stream(wr + 8 * min(64u * c + lane, last));
+    };
+    uint32_t row = blockIdx.x * 4 + wave;
+    if (row >= N) return;
+    uint4 p[NL], q[NL];
+    issue(p, row);
+    RowSums sums{seg, bias, lane, row_step, row};
+    float xr[NL][8];
+    lh_vector_registers<STAGE, NL>(st, K, lane, blockIdx.x == 0 && wave == 0 && st.store != nullptr, xr);
+    auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {   // false: that was the wave's last row
+        const bool more = row + row_step < N;
+        if (more) issue(nxt, row + row_step);
+        float acc = 0.0f;
+#pragma unroll
+        for (int c = 0; c < NL; c++) acc = lh_dot8(cur[c], xr[c], acc);
+        sums.add(lh_group_sum(acc, 64));
+        row += row_step;
+        return more;
+    };
+    while (step(p, q) && step(q, p)) {}
+    sums.flush();
 }
 
 constexpr uint32_t kMaxVectorK = 36864;   // 144 KB of staged f32 activations
@@ -356,6 +406,16 @@ int launch_vector(lh_context* ctx, const VectorStage& st, const uint16_t* W, con
     LH_REQUIRE(K > 0 && K <= kMaxVectorK, "%s: k %u outside 1..=%u", op, K, kMaxVectorK);
     const size_t lds = (size_t)(K + 511) / 512 * 512 * 4;
     const bool vec = K % 8 == 0 && ((uintptr_t)W & 15) == 0;
+    if (vec && K <= 4096 && lh_stage_aligned(st)) {
+        const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * (K <= 2048 ? 4 : 2));
+#define LH_MVR(NLOADS) hipLaunchKernelGGL((matvec_bf16_reg_kernel<STAGE, NLOADS>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K)
+        if (K <= 512) LH_MVR(1);
+        else if (K <= 1024) LH_MVR(2);
+        else if (K <= 2048) LH_MVR(4);
+        else LH_MVR(8);
+#undef LH_MVR
+        return lh_check_launch(op);
+    }
     const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * 4);
 #define LH_MV(NLOADS, V)                                                                                                               \
     do {                                                                                                                               \
@@ -427,7 +487,8 @@ int lh_launch_linear(lh_context* ctx, const LhLinear& a, const char* op) {
     if (a.ex.tiles) {
         if (a.ex.tile_rows == 128) { if (tiles(128, 128) >= want) LH_GEMM(128, 128); else LH_GEMM(128, 64); }
         else LH_GEMM(64, 64);
-    } else if (tiles(128, 128) >= want) LH_GEMM(128, 128);
+    } else if (tiles(128, 128) >= 2 * want) LH_GEMM(128, 128);
+    else if (tiles(128, 64) >= want) LH_GEMM(128, 64);
     else if (tiles(64, 64) >= want || a.M > 32) LH_GEMM(64, 64);
     else LH_GEMM(32, 32);
 #undef LH_GEMM

@@ -24,3 +24,95 @@ struct LhLinear {
 };
 int lh_launch_linear(lh_context* ctx, const LhLinear& a, const char* op);
 uint32_t lh_expert_tile_rows(uint32_t slots, uint32_t experts);
+
+// ---- one row: the activation vector in registers -------------------------------------------------------------------------
+// Up to 4096 columns a wave keeps the vector itself: lane l holds the NL chunks of eight elements 8 (64 c + l), which is what
+// it multiplies in every row.  The norm before the product is then a sum over the wave, with no barrier and no LDS.
+enum { kPlain = 0, kNorm = 1, kGated = 2 };
+struct VectorStage {
+    const void* x;             // plain: x_f32 ? f32 : bf16; norm, gated: f32
+    uint32_t x_f32;
+    const float* add;          // norm: may be null
+    float* store;              // norm: receives x + add (workgroup 0), may be null
+    const float* norm_weight;
+    const void* gate;          // gated
+    uint32_t gate_f32;
+    float eps;
+};
+
+__device__ __forceinline__ void lh_ld8(const float* p, float (&v)[8]) {
+    const float4 a = *reinterpret_cast<const float4*>(p), b = *reinterpret_cast<const float4*>(p + 4);
+    v[0] = a.x; v[1] = a.y; v[2] = a.z; v[3] = a.w; v[4] = b.x; v[5] = b.y; v[6] = b.z; v[7] = b.w;
+}
+__device__ __forceinline__ void lh_ld8(const uint16_t* p, float (&v)[8]) {
+    const uint4 a = *reinterpret_cast<const uint4*>(p);
+    const uint32_t w[4] = {a.x, a.y, a.z, a.w};
+#pragma unroll
+    for (int j = 0; j < 4; j++) { v[2 * j] = __builtin_bit_cast(float, w[j] << 16); v[2 * j + 1] = __builtin_bit_cast(float, w[j] & 0xFFFF0000u); }
+}
+
+// K a multiple of 8, all pointers 16-byte aligned; chunks past K are zero.  `store` whether this wave stores x + add.
+template <int STAGE, int NL>
+__device__ __forceinline__ void lh_vector_registers(const VectorStage& st, uint32_t K, uint32_t lane, bool store, float (&xr)[NL][8]) {
+    float w[STAGE == kPlain ? 1 : NL][8], s = 0.0f;
+#pragma unroll
+    for (int c = 0; c < NL; c++) {
+        const uint32_t k = (64 * c + lane) * 8;
+#pragma unroll
+        for (int j = 0; j < 8; j++) xr[c][j] = 0.0f;
+        if (k >= K) continue;
+        if (STAGE == kPlain && !st.x_f32) lh_ld8(static_cast<const uint16_t*>(st.x) + k, xr[c]);
+        else lh_ld8(static_cast<const float*>(st.x) + k, xr[c]);
+        if constexpr (STAGE == kNorm) if (st.add) {
+            float b[8];
+            lh_ld8(st.add + k, b);
+#pragma unroll
+            for (int j = 0; j < 8; j++) xr[c][j] += b[j];
+        }
+        if constexpr (STAGE != kPlain) {
+            lh_ld8(st.norm_weight + k, w[c]);
+            if constexpr (STAGE == kGated) {
+                float g[8];
+                if (st.gate_f32) lh_ld8(static_cast<const float*>(st.gate) + k, g);
+                else lh_ld8(static_cast<const uint16_t*>(st.gate) + k, g);
+#pragma unroll
+                for (int j = 0; j < 8; j++) w[c][j] *= lh_sigmoid(g[j]);
+            }
+#pragma unroll
+            for (int j = 0; j < 8; j++) s += xr[c][j] * xr[c][j];
+        }
+    }
+    if constexpr (STAGE != kPlain) {
+        const float r = rsqrtf(lh_group_sum(s, 64) / (float)K + st.eps);
+#pragma unroll
+        for (int c = 0; c < NL; c++) {
+            const uint32_t k = (64 * c + lane) * 8;
+            if (k >= K) continue;
+            if (STAGE == kNorm && store) {
+                *reinterpret_cast<float4*>(st.store + k) = make_float4(xr[c][0], xr[c][1], xr[c][2], xr[c][3]);
+                *reinterpret_cast<float4*>(st.store + k + 4) = make_float4(xr[c][4], xr[c][5], xr[c][6], xr[c][7]);
+            }
+#pragma unroll
+            for (int j = 0; j < 8; j++) xr[c][j] = xr[c][j] * r * w[c][j];
+        }
+    }
+}
+static inline bool lh_stage_aligned(const VectorStage& st) {
+    return (((uintptr_t)st.x | (uintptr_t)st.add | (uintptr_t)st.store | (uintptr_t)st.norm_weight | (uintptr_t)st.gate) & 15) == 0;
+}
+
+// Weights are read once per launch: streaming loads.
+__device__ __forceinline__ uint4 lh_ld16_stream(const uint16_t* p) {
+    typedef uint32_t u32x4_t __attribute__((ext_vector_type(4)));
+    const u32x4_t v = __builtin_nontemporal_load(reinterpret_cast<const u32x4_t*>(p));
+    return make_uint4(v.x, v.y, v.z, v.w);
+}
+__device__ __forceinline__ float lh_dot8(const uint4& v, const float* x, float acc) {
+    const uint32_t w[4] = {v.x, v.y, v.z, v.w};
+#pragma unroll
+    for (int j = 0; j < 4; j++) {
+        acc = __builtin_fmaf(__builtin_bit_cast(float, w[j] << 16), x[2 * j], acc);
+        acc = __builtin_fmaf(__builtin_bit_cast(float, w[j] & 0xFFFF0000u), x[2 * j + 1], acc);
+    }
+    return acc;
+}

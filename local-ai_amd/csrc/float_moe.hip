@@ -18,25 +18,31 @@ namespace {
 
 constexpr uint32_t kMaxExperts = 1024, kMaxTop = 64;
 
-// The `top` largest of `experts` logits, best first, by one wave; every lane returns with the same ids and weights in LDS.
-// (Sigmoid is monotone, so the logits decide; ties go to the lower index.)
-__device__ void select_experts(const float* logits, uint32_t experts, uint32_t top, uint32_t lane, uint32_t* ids, float* weights) {
-    float v[kMaxExperts / 64];
+// The `top` largest of `experts` logits, best first, by one wave; ids and weights go to LDS or global memory.  (Sigmoid is
+// monotone, so the logits decide; ties go to the lower index.)
+template <uint32_t PER>
+__device__ __forceinline__ void select_experts_of(const float* logits, uint32_t experts, uint32_t top, uint32_t lane, uint32_t* ids, float* weights) {
+    float v[PER];
 #pragma unroll
-    for (uint32_t i = 0; i < kMaxExperts / 64; i++) v[i] = i * 64 + lane < experts ? logits[i * 64 + lane] : -INFINITY;
+    for (uint32_t i = 0; i < PER; i++) v[i] = i * 64 + lane < experts ? logits[i * 64 + lane] : -INFINITY;
     for (uint32_t c = 0; c < top; c++) {
         float best = -INFINITY;
         uint32_t at = 0xFFFFFFFFu;
 #pragma unroll
-        for (uint32_t i = 0; i < kMaxExperts / 64; i++) if (v[i] > best) { best = v[i]; at = i * 64 + lane; }
+        for (uint32_t i = 0; i < PER; i++) if (v[i] > best) { best = v[i]; at = i * 64 + lane; }
         const float m = lh_group_max(best, 64);
         // the lowest index among the lanes that hold the maximum: a minimum as the maximum of the complements
         uint32_t win = ~lh_group_max_u(best == m && at != 0xFFFFFFFFu ? ~at : 0u, 64);
         if (win >= experts) win = min(c, experts - 1);        // no finite logit left
 #pragma unroll
-        for (uint32_t i = 0; i < kMaxExperts / 64; i++) if (i * 64 + lane == win) v[i] = -INFINITY;
-        if (lane == 0) { ids[c] = win; weights[c] = lh_sigmoid(logits[win]); }
+        for (uint32_t i = 0; i < PER; i++) if (i * 64 + lane == win) v[i] = -INFINITY;
+        if (lane == 0) { ids[c] = win; weights[c] = lh_sigmoid(m); }
     }
+}
+__device__ void select_experts(const float* logits, uint32_t experts, uint32_t top, uint32_t lane, uint32_t* ids, float* weights) {
+    if (experts <= 64) select_experts_of<1>(logits, experts, top, lane, ids, weights);
+    else if (experts <= 256) select_experts_of<4>(logits, experts, top, lane, ids, weights);
+    else select_experts_of<kMaxExperts / 64>(logits, experts, top, lane, ids, weights);
 }
 
 __global__ __launch_bounds__(256) void route_kernel(const float* __restrict__ logits, uint32_t* __restrict__ plan, uint32_t rows, uint32_t experts, uint32_t top) {
@@ -144,6 +150,37 @@ __global__ __launch_bounds__(256) void vector_up_kernel(const float* __restrict_
     }
 }
 
+// The same with the normed vector in registers (width a multiple of 8, up to 512 * NL): a workgroup keeps to one expert's rows
+// (blockIdx.y: the choice), and the first row's weights are requested as soon as the selection is known.
+template <int NL>
+__global__ __launch_bounds__(256) void vector_up_reg_kernel(const VectorStage st, const float* __restrict__ logits, const uint16_t* __restrict__ up,
+                                                           float* __restrict__ hidden, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff, uint32_t act) {
+    __shared__ uint32_t ids[4][kMaxTop];
+    __shared__ float weights[4][kMaxTop];
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, c = blockIdx.y, last = (width >> 3) - 1;
+    select_experts(logits, experts, c + 1, lane, ids[wave], weights[wave]);    // every wave for itself: no barrier
+    const uint32_t e = ids[wave][c];
+    const float weight = weights[wave][c];
+    const uint16_t* base = up + (size_t)e * ff * width;
+    uint32_t row = blockIdx.x * 4 + wave;
+    uint4 w[NL];
+    auto issue = [&](uint32_t r) {
+#pragma unroll
+        for (int i = 0; i < NL; i++) w[i] = lh_ld16_stream(base + (size_t)min(r, ff - 1) * width + 8 * min(64u * i + lane, last));
+    };
+    issue(row);
+    float xr[NL][8];
+    lh_vector_registers<kNorm, NL>(st, width, lane, false, xr);
+    for (; row < ff; row += gridDim.x * 4) {
+        float acc = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NL; i++) acc = lh_dot8(w[i], xr[i], acc);
+        if (row + gridDim.x * 4 < ff) issue(row + gridDim.x * 4);
+        acc = lh_group_sum(acc, 64);
+        if (lane == 0) hidden[c * ff + row] = lh_activate(weight * acc, act);
+    }
+}
+
 // residual[r] += sum_c down[e_c][r] . hidden[c]
 __global__ __launch_bounds__(256) void vector_down_kernel(const float* __restrict__ hidden, const float* __restrict__ logits, const uint16_t* __restrict__ down,
                                                          float* __restrict__ residual, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff, uint32_t vec) {
@@ -158,6 +195,43 @@ __global__ __launch_bounds__(256) void vector_down_kernel(const float* __restric
         float v = 0.0f;
         for (uint32_t c = 0; c < top; c++) v += wave_dot(down + ((size_t)ids[c] * width + n) * ff, xs + c * ffp, ff, lane, vec);
         if (lane == 0) residual[n] += v;
+    }
+}
+
+// The same with the hidden values of all choices in registers as one vector of top * ff (ff a multiple of 8): a lane's chunk
+// belongs to one choice, so it has its own place in the weights.
+template <int NL>
+__global__ __launch_bounds__(256) void vector_down_reg_kernel(const float* __restrict__ hidden, const float* __restrict__ logits, const uint16_t* __restrict__ down,
+                                                             float* __restrict__ residual, uint32_t experts, uint32_t top, uint32_t width, uint32_t ff) {
+    __shared__ uint32_t ids[4][kMaxTop];
+    __shared__ float weights[4][kMaxTop];
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, chunks = top * (ff >> 3), row_step = gridDim.x * 4;
+    const VectorStage st{hidden, 1, nullptr, nullptr, nullptr, nullptr, 0, 0.0f};
+    float xr[NL][8];
+    lh_vector_registers<kPlain, NL>(st, top * ff, lane, false, xr);
+    select_experts(logits, experts, top, lane, ids[wave], weights[wave]);
+    const uint16_t* base[NL];
+#pragma unroll
+    for (int i = 0; i < NL; i++) {
+        const uint32_t q = min(64u * i + lane, chunks - 1), c = q / (ff >> 3);
+        base[i] = down + (size_t)ids[wave][c] * width * ff + 8 * (q - c * (ff >> 3));
+    }
+    uint32_t n = blockIdx.x * 4 + wave;
+    if (n >= width) return;
+    uint4 w[NL];
+    auto issue = [&](uint32_t r) {
+#pragma unroll
+        for (int i = 0; i < NL; i++) w[i] = lh_ld16_stream(base[i] + (size_t)r * ff);
+    };
+    issue(n);
+    for (; n < width; n += row_step) {
+        const float before = lane == 0 ? residual[n] : 0.0f;
+        float acc = 0.0f;
+#pragma unroll
+        for (int i = 0; i < NL; i++) acc = lh_dot8(w[i], xr[i], acc);
+        if (n + row_step < width) issue(n + row_step);
+        acc = lh_group_sum(acc, 64);
+        if (lane == 0) residual[n] = before + acc;
     }
 }
 
@@ -288,6 +362,20 @@ int lh_moe_vector_up_into(lh_batch* batch, const lh_buffer* input, const lh_buff
     LH_NEED(logits, (size_t)experts * 4, op, "logits");
     LH_NEED(up, (size_t)experts * ff * width * 2, op, "up");
     LH_NEED(hidden, (size_t)top * ff * 4, op, "hidden");
+    const VectorStage st{input->ptr, 1, nullptr, nullptr, (const float*)norm_weight->ptr, nullptr, 0, eps};
+    if (width % 8 == 0 && width <= 4096 && ((uintptr_t)up->ptr & 15) == 0 && lh_stage_aligned(st)) {
+        const dim3 grid(std::min<uint32_t>((ff + 3) / 4, std::max<uint32_t>(1, (uint32_t)batch->ctx->cu_count * 4 / top)), top);
+#define LH_UP(NL) hipLaunchKernelGGL((vector_up_reg_kernel<NL>), grid, dim3(256), 0, batch->ctx->stream, st, (const float*)logits->ptr, (const uint16_t*)up->ptr, \
+                                     (float*)hidden->ptr, experts, top, width, ff, act)
+        if (width <= 512) LH_UP(1);
+        else if (width <= 1024) LH_UP(2);
+        else if (width <= 2048) LH_UP(4);
+        else LH_UP(8);
+#undef LH_UP
+        LH_TRY(lh_check_launch(op));
+        batch->dispatch_count++;
+        return LH_OK;
+    }
     const size_t lds = (size_t)width * 4;
     LH_TRY(vector_lds(batch->ctx, (const void*)vector_up_kernel, lds, op));
     const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)top * ff + 3) / 4, (uint64_t)batch->ctx->cu_count * 4);
@@ -309,6 +397,19 @@ int lh_moe_vector_down_into(lh_batch* batch, const lh_buffer* hidden, const lh_b
     LH_NEED(logits, (size_t)experts * 4, op, "logits");
     LH_NEED(down, (size_t)experts * ff * width * 2, op, "down");
     LH_NEED(residual, (size_t)width * 4, op, "residual");
+    if (ff % 8 == 0 && (uint64_t)top * ff <= 4096 && (((uintptr_t)down->ptr | (uintptr_t)hidden->ptr) & 15) == 0) {
+        const uint32_t blocks = (uint32_t)std::min<uint64_t>(((uint64_t)width + 3) / 4, (uint64_t)batch->ctx->cu_count * 4);
+#define LH_DOWN(NL) hipLaunchKernelGGL((vector_down_reg_kernel<NL>), dim3(blocks), dim3(256), 0, batch->ctx->stream, (const float*)hidden->ptr, (const float*)logits->ptr, \
+                                       (const uint16_t*)down->ptr, (float*)residual->ptr, experts, top, width, ff)
+        if (top * ff <= 512) LH_DOWN(1);
+        else if (top * ff <= 1024) LH_DOWN(2);
+        else if (top * ff <= 2048) LH_DOWN(4);
+        else LH_DOWN(8);
+#undef LH_DOWN
+        LH_TRY(lh_check_launch(op));
+        batch->dispatch_count++;
+        return LH_OK;
+    }
     const size_t lds = (size_t)top * ((ff + 3) / 4 * 4) * 4;
     LH_TRY(vector_lds(batch->ctx, (const void*)vector_down_kernel, lds, op));
     const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)width + 3) / 4, (uint64_t)batch->ctx->cu_count * 4);

@@ -98,3 +98,31 @@ __device__ __forceinline__ float lh_block_sum(float v, float* scratch) {
     __syncthreads();
     return t;
 }
+
+// Barrier over LDS accesses only: global loads that are on their way stay on their way.
+__device__ __forceinline__ void lh_lds_barrier() { asm volatile("s_waitcnt lgkmcnt(0)\n\ts_barrier" ::: "memory"); }
+
+// Maximum and sum over the four lanes that differ in their 16s and 32s (the column of a 16 x 16 matrix-product tile).
+// v_permlane16_swap / v_permlane32_swap on two copies leave the even and the odd rows (the lower and the upper half) of a
+// value in all rows (both halves).  (The compiler's builtin hands back its first result twice; the wait states before the
+// swap are what the compiler itself puts there.)
+__device__ __forceinline__ void lh_pair16(float v, float& a, float& b) {
+    a = v; b = v;
+    asm("s_nop 1\n\tv_permlane16_swap_b32 %0, %1" : "+v"(a), "+v"(b));
+}
+__device__ __forceinline__ void lh_pair32(float v, float& a, float& b) {
+    a = v; b = v;
+    asm("s_nop 1\n\tv_permlane32_swap_b32 %0, %1" : "+v"(a), "+v"(b));
+}
+__device__ __forceinline__ float lh_column_max(float v) {
+    float a, b;
+    lh_pair16(v, a, b);
+    lh_pair32(fmaxf(a, b), a, b);
+    return fmaxf(a, b);
+}
+__device__ __forceinline__ float lh_column_sum(float v) {
+    float a, b;
+    lh_pair16(v, a, b);
+    lh_pair32(a + b, a, b);
+    return a + b;
+}

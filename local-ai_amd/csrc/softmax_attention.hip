@@ -29,7 +29,7 @@ struct AttentionArgs {
     const uint32_t* position;
     uint32_t rows, heads, kv_heads, maps, dim, dq, vdim, dv, capacity;
     float scale, lambda, out_scale, eps;
-    float* partial;            // split form: [tile][kv head][split][map][16] (max, sum), then the unnormalised sums [..][16][dv]
+    float* partial;            // records [16-row tile][kv head][split][map][16] of dv unnormalised sums, maximum, sum of weights
     uint32_t splits;
 };
 
@@ -60,36 +60,38 @@ __device__ __forceinline__ void load_queries(lh_bf16x8 (&qf)[MAPS][DQ / 32], con
         }
 }
 
-// One row tile's running softmax state for one map; every lane holds the values of packed row (lane & 15).
+// A row tile's running softmax state for one map; every lane holds the values of packed row (lane & 15).
 struct RowState { float m, l; };
 
-// Scores of a 32-key step -> weights in P V operand order, as two bf16 terms; returns the factor for what was summed before.
-// `first` is the step's first key, `limit` the row's last visible key, `bound` whether any lane may have to mask.
-__device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2], RowState& st, float scale2, uint32_t first, uint32_t limit, bool bound, uint32_t lane,
-                                              lh_bf16x8& hi, lh_bf16x8& lo) {
-    float v[8], mx = -INFINITY;
+// Scores of NB steps of 32 keys -> weights in P V operand order, as two bf16 terms; returns the factor for what was summed
+// before.  `first` is the first key, `limit` the row's last visible key, `bound` whether any lane may have to mask.
+template <int NB>
+__device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2 * NB], RowState& st, float scale2, uint32_t first, uint32_t limit, bool bound, uint32_t lane,
+                                              lh_bf16x8 (&hi)[NB], lh_bf16x8 (&lo)[NB]) {
+    float v[8 * NB], mx = -INFINITY;
     const uint32_t g = lane >> 4;
 #pragma unroll
-    for (int i = 0; i < 8; i++) {
+    for (int i = 0; i < 8 * NB; i++) {
         v[i] = s[i >> 2][i & 3] * scale2;
         if (bound && first + (i >> 2) * 16 + g * 4 + (i & 3) > limit) v[i] = -INFINITY;
         mx = fmaxf(mx, v[i]);
     }
-    mx = fmaxf(mx, lh_swap16_f(mx));
-    mx = fmaxf(mx, lh_swap32_f(mx));
-    const float nm = fmaxf(st.m, mx), base = nm == -INFINITY ? 0.0f : nm;
+    const float nm = fmaxf(st.m, lh_column_max(mx)), base = nm == -INFINITY ? 0.0f : nm;
     const float alpha = __builtin_amdgcn_exp2f(st.m - base);
     float sum = 0.0f;
-    uint32_t h[4], l[4];
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const float p0 = __builtin_amdgcn_exp2f(v[2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[2 * i + 1] - base);
-        sum += p0 + p1;
-        h[i] = lh_pack_bf(p0, p1);
-        l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, h[i] << 16), p1 - __builtin_bit_cast(float, h[i] & 0xFFFF0000u));
+    for (int b = 0; b < NB; b++) {
+        uint32_t h[4], l[4];
+#pragma unroll
+        for (int i = 0; i < 4; i++) {
+            const float p0 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i + 1] - base);
+            sum += p0 + p1;
+            h[i] = lh_pack_bf(p0, p1);
+            l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, h[i] << 16), p1 - __builtin_bit_cast(float, h[i] & 0xFFFF0000u));
+        }
+        hi[b] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
+        lo[b] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
     }
-    hi = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
-    lo = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
     st.l = st.l * alpha + sum;      // this lane's keys only; the four lanes of a row are added at the end
     st.m = nm;
     return alpha;
@@ -114,8 +116,7 @@ __device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)
         }
     float f = 1.0f;
     if constexpr (MAPS == 2) {
-        ss += lh_swap16_f(ss);
-        ss += lh_swap32_f(ss);
+        ss = lh_column_sum(ss);
         f = rsqrtf(ss / (float)a.vdim + a.eps) * a.out_scale;
     }
     if (t >= a.rows) return;
@@ -135,117 +136,111 @@ __device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)
 typedef __attribute__((address_space(1))) const void gvoid;
 typedef __attribute__((address_space(3))) void lvoid;
 
-// RT row tiles of 16 packed rows per wave, four waves; steps of 32 keys through two LDS buffers.  A key row of the buffer is
-// MAPS * DQ / 8 chunks of 16 bytes, chunk c at place c ^ (key & 7) (see linear_mfma_kernel for why and how).
-template <int DQ, int DV, int MAPS, int RT>
+// 64 packed rows, 16 per wave; steps of 32 * NB keys through two LDS buffers.  A key row of the buffer is MAPS * DQ / 8 chunks
+// of 16 bytes, chunk c at place c ^ (key & 7) (see linear_mfma_kernel for why and how).  With more than one split a
+// workgroup takes its share of the key steps and leaves partial records.
+template <int DQ, int DV, int MAPS, int NB>
 __global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs a) {
-    constexpr int KC = MAPS * DQ / 8, KCH = 32 * KC, VCH = DV * 4;      // chunks per key row; per key block; per value block
+    constexpr int KC = MAPS * DQ / 8, KCH = 32 * NB * KC, VB = DV * 4, VCH = NB * VB;    // chunks per key row; per step: keys, values
+    constexpr uint32_t kSwizzle = KC >= 8 ? 7 : KC - 1;
     __shared__ uint4 sm[2][KCH + VCH];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const uint32_t R = a.heads / a.kv_heads, packed = a.rows * R, tiles = (packed + 64 * RT - 1) / (64 * RT);
-    const uint32_t g = blockIdx.x % a.kv_heads, tile = tiles - 1 - blockIdx.x / a.kv_heads;    // the long tiles first
+    const uint32_t R = a.heads / a.kv_heads, packed = a.rows * R, tiles = (packed + 63) / 64;
+    const uint32_t split = blockIdx.x % a.splits, gt = blockIdx.x / a.splits;
+    const uint32_t g = gt % a.kv_heads, tile = tiles - 1 - gt / a.kv_heads;              // the long tiles first
     const uint32_t start = *a.position;
-    const uint32_t row0 = tile * 64 * RT, row_last = min(row0 + 64 * RT, packed) - 1;
-    const uint32_t last_key = min(start + row_last / R, a.capacity - 1), nb = last_key / 32 + 1;
-    const uint32_t wrow = row0 + wave * 16 * RT;
+    const uint32_t row0 = tile * 64, row_last = min(row0 + 64, packed) - 1;
+    const uint32_t last_key = min(start + row_last / R, a.capacity - 1), last_block = last_key / 32, nstep = last_block / NB + 1;
+    const uint32_t per = (nstep + a.splits - 1) / a.splits, s0 = min(split * per, nstep), s1 = min(s0 + per, nstep);
+    const uint32_t wrow = row0 + wave * 16, row = wrow + (lane & 15);
 
-    lh_bf16x8 qf[RT][MAPS][DQ / 32];
-    uint32_t limit[RT];
+    lh_bf16x8 qf[MAPS][DQ / 32];
+    load_queries<DQ, MAPS>(qf, a, g, row, lane);
+    const uint32_t limit = min(start + row / R, last_key), first_limit = start + wrow / R, wave_last = min(start + (wrow + 15) / R, last_key);
+    lh_f32x4 o[MAPS][DV / 16];
+    RowState st[MAPS];
 #pragma unroll
-    for (int i = 0; i < RT; i++) {
-        const uint32_t row = wrow + i * 16 + (lane & 15);
-        load_queries<DQ, MAPS>(qf[i], a, g, row, lane);
-        limit[i] = min(start + row / R, last_key);
+    for (int mp = 0; mp < MAPS; mp++) {
+        st[mp] = RowState{-INFINITY, 0.0f};
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++) o[mp][d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
     }
-    const uint32_t wave_first_limit = start + wrow / R, wave_last = min(start + (wrow + 16 * RT - 1) / R, last_key);
-    lh_f32x4 o[RT][MAPS][DV / 16];
-    RowState st[RT][MAPS];
-#pragma unroll
-    for (int i = 0; i < RT; i++)
-#pragma unroll
-        for (int mp = 0; mp < MAPS; mp++) {
-            st[i][mp] = RowState{-INFINITY, 0.0f};
-#pragma unroll
-            for (int d = 0; d < DV / 16; d++) o[i][mp][d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
-        }
 
     const uint16_t* K = static_cast<const uint16_t*>(a.keys) + (size_t)g * MAPS * DQ;
     const uint16_t* V = static_cast<const uint16_t*>(a.values) + (size_t)g * DV * 32;
     const size_t krow = (size_t)a.kv_heads * MAPS * DQ, vblock = (size_t)a.kv_heads * DV * 32;
-    auto load_block = [&](int buf, uint32_t b) {
+    auto load_step = [&](int buf, uint32_t s) {
 #pragma unroll
         for (int i = 0; i < (KCH + 255) / 256; i++) {
-            if (KCH % 256 != 0 && i * 256 + wave * 64 >= KCH) break;                           // whole waves (KCH is a multiple of 64)
-            const uint32_t c = i * 256 + tid, key = c / KC, place = c % KC, ch = place ^ (key & (KC >= 8 ? 7 : KC - 1));
-            const uint32_t p = min(b * 32 + key, last_key);                                     // keys past the last are masked
+            if (KCH % 256 != 0 && i * 256 + wave * 64 >= KCH) break;                     // whole waves (KCH is a multiple of 64)
+            const uint32_t c = i * 256 + tid, key = c / KC, ch = (c % KC) ^ (key & kSwizzle);
+            const uint32_t p = min(s * (32 * NB) + key, last_key);                        // keys past the last are masked
             __builtin_amdgcn_global_load_lds((gvoid*)(K + p * krow + ch * 8), (lvoid*)&sm[buf][i * 256 + wave * 64], 16, 0, 0);
         }
 #pragma unroll
         for (int i = 0; i < (VCH + 255) / 256; i++) {
             if (VCH % 256 != 0 && i * 256 + wave * 64 >= VCH) break;
-            __builtin_amdgcn_global_load_lds((gvoid*)(V + b * vblock + (i * 256 + tid) * 8), (lvoid*)&sm[buf][KCH + i * 256 + wave * 64], 16, 0, 0);
+            const uint32_t c = i * 256 + tid;
+            __builtin_amdgcn_global_load_lds((gvoid*)(V + min(s * NB + c / VB, last_block) * vblock + (c % VB) * 8), (lvoid*)&sm[buf][KCH + i * 256 + wave * 64], 16, 0, 0);
         }
     };
     const float scale2 = a.scale * kLog2e;
-    load_block(0, 0);
-    for (uint32_t b = 0; b < nb; b++) {
+    if (s0 < s1) load_step(s0 & 1, s0);
+    for (uint32_t s = s0; s < s1; s++) {
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
         __syncthreads();
-        if (b + 1 < nb) load_block((b + 1) & 1, b + 1);
-        if (b * 32 > wave_last) continue;                                                       // nothing here is visible to this wave
-        const uint4* ks = sm[b & 1];
+        if (s + 1 < s1) load_step((s + 1) & 1, s + 1);
+        const uint32_t first = s * (32 * NB);
+        if (first > wave_last) continue;                                                  // nothing here is visible to this wave
+        const uint4* ks = sm[s & 1];
         const uint4* vs = ks + KCH;
-        const bool bound = b * 32 + 31 > wave_first_limit;
-        lh_bf16x8 hi[RT][MAPS], lo[RT][MAPS];
+        const bool bound = first + 32 * NB - 1 > first_limit;
+        lh_bf16x8 hi[MAPS][NB], lo[MAPS][NB];
 #pragma unroll
         for (int mp = 0; mp < MAPS; mp++) {
-            lh_f32x4 s[RT][2];
+            lh_f32x4 sc[2 * NB];
 #pragma unroll
-            for (int t = 0; t < 2; t++) {
-#pragma unroll
-                for (int i = 0; i < RT; i++) s[i][t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+            for (int t = 0; t < 2 * NB; t++) {
+                sc[t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
                 const uint32_t key = t * 16 + (lane & 15);
 #pragma unroll
                 for (int c = 0; c < DQ / 32; c++) {
                     const uint32_t ch = mp * (DQ / 8) + c * 4 + (lane >> 4);
-                    const lh_bf16x8 kf = __builtin_bit_cast(lh_bf16x8, ks[key * KC + (ch ^ (key & (KC >= 8 ? 7 : KC - 1)))]);
-#pragma unroll
-                    for (int i = 0; i < RT; i++) s[i][t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(kf, qf[i][mp][c], s[i][t], 0, 0, 0);
+                    sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, ks[key * KC + (ch ^ (key & kSwizzle))]), qf[mp][c], sc[t], 0, 0, 0);
                 }
             }
+            const float alpha = softmax_step<NB>(sc, st[mp], scale2, first, limit, bound, lane, hi[mp], lo[mp]);
+            if (__ballot(alpha != 1.0f)) {
 #pragma unroll
-            for (int i = 0; i < RT; i++) {
-                const float alpha = softmax_step(s[i], st[i][mp], scale2, b * 32, limit[i], bound, lane, hi[i][mp], lo[i][mp]);
-                if (__ballot(alpha != 1.0f)) {
+                for (int d = 0; d < DV / 16; d++)
 #pragma unroll
-                    for (int d = 0; d < DV / 16; d++)
-#pragma unroll
-                        for (int r = 0; r < 4; r++) o[i][mp][d][r] *= alpha;
-                }
+                    for (int r = 0; r < 4; r++) o[mp][d][r] *= alpha;
             }
         }
 #pragma unroll
-        for (int d = 0; d < DV / 16; d++) {
-            const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, vs[(d * 16 + (lane & 15)) * 4 + (lane >> 4)]);
+        for (int b = 0; b < NB; b++)
 #pragma unroll
-            for (int i = 0; i < RT; i++)
+            for (int d = 0; d < DV / 16; d++) {
+                const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, vs[b * VB + (d * 16 + (lane & 15)) * 4 + (lane >> 4)]);
 #pragma unroll
                 for (int mp = 0; mp < MAPS; mp++) {
-                    o[i][mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[i][mp], o[i][mp][d], 0, 0, 0);
-                    o[i][mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[i][mp], o[i][mp][d], 0, 0, 0);
+                    o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[mp][b], o[mp][d], 0, 0, 0);
+                    o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[mp][b], o[mp][d], 0, 0, 0);
                 }
-        }
+            }
     }
+    float l[MAPS];
 #pragma unroll
-    for (int i = 0; i < RT; i++) {
-        float l[MAPS];
+    for (int mp = 0; mp < MAPS; mp++) l[mp] = lh_column_sum(st[mp].l);
+    if (a.splits == 1) { finish_row<DV, MAPS>(a, o, l, g, row, lane); return; }
+    if (row >= packed) return;
+    constexpr uint32_t kRow = DV + 4;
 #pragma unroll
-        for (int mp = 0; mp < MAPS; mp++) {
-            l[mp] = st[i][mp].l;
-            l[mp] += lh_swap16_f(l[mp]);
-            l[mp] += lh_swap32_f(l[mp]);
-        }
-        finish_row<DV, MAPS>(a, o[i], l, g, wrow + i * 16 + (lane & 15), lane);
+    for (int mp = 0; mp < MAPS; mp++) {
+        float* r = a.partial + ((((size_t)(wrow >> 4) * a.kv_heads + g) * a.splits + split) * MAPS + mp) * 16 * kRow + (lane & 15) * kRow;
+#pragma unroll
+        for (int d = 0; d < DV / 16; d++) *reinterpret_cast<float4*>(r + d * 16 + (lane >> 4) * 4) = make_float4(o[mp][d][0], o[mp][d][1], o[mp][d][2], o[mp][d][3]);
+        if (lane < 16) { r[DV] = st[mp].m; r[DV + 1] = l[mp]; }
     }
 }
 
@@ -253,7 +248,7 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs
 // waves of a (tile, kv head); a wave loads a block's operands one block ahead.
 template <int DQ, int DV, int MAPS>
 __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArgs a) {
-    extern __shared__ float merge[];                          // [4 waves][MAPS][16 rows][DV + 2]: max, sum, values
+    extern __shared__ __align__(16) float merge[];                          // [4 waves][MAPS][16 rows][DV + 4]: values, maximum, sum
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
     const uint32_t split = blockIdx.x % a.splits, g = (blockIdx.x / a.splits) % a.kv_heads, tile = blockIdx.x / (a.splits * a.kv_heads);
     const uint32_t R = a.heads / a.kv_heads, packed = a.rows * R, start = *a.position;
@@ -292,7 +287,7 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
     const float scale2 = a.scale * kLog2e;
     auto consume = [&](const Block& f, uint32_t b) {
         const bool bound = b * 32 + 31 > first_limit;
-        lh_bf16x8 hi[MAPS], lo[MAPS];
+        lh_bf16x8 hi[MAPS][1], lo[MAPS][1];
 #pragma unroll
         for (int mp = 0; mp < MAPS; mp++) {
             lh_f32x4 s[2];
@@ -302,7 +297,7 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
 #pragma unroll
                 for (int c = 0; c < DQ / 32; c++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.k[t][mp][c]), qf[mp][c], s[t], 0, 0, 0);
             }
-            const float alpha = softmax_step(s, st[mp], scale2, b * 32, limit, bound, lane, hi[mp], lo[mp]);
+            const float alpha = softmax_step<1>(s, st[mp], scale2, b * 32, limit, bound, lane, hi[mp], lo[mp]);
             if (__ballot(alpha != 1.0f)) {
 #pragma unroll
                 for (int d = 0; d < DV / 16; d++)
@@ -314,8 +309,8 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
         for (int d = 0; d < DV / 16; d++)
 #pragma unroll
             for (int mp = 0; mp < MAPS; mp++) {
-                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), hi[mp], o[mp][d], 0, 0, 0);
-                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), lo[mp], o[mp][d], 0, 0, 0);
+                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), hi[mp][0], o[mp][d], 0, 0, 0);
+                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), lo[mp][0], o[mp][d], 0, 0, 0);
             }
     };
     if (b0 < b1) {
@@ -330,87 +325,100 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
             }
         }
     }
-    constexpr uint32_t kRow = DV + 2;
+    constexpr uint32_t kRow = DV + 4;
 #pragma unroll
     for (int mp = 0; mp < MAPS; mp++) {
-        float l = st[mp].l;
-        l += lh_swap16_f(l);
-        l += lh_swap32_f(l);
+        const float l = lh_column_sum(st[mp].l);
         float* d0 = merge + ((wave * MAPS + mp) * 16 + (lane & 15)) * kRow;
-        if (lane < 16) { d0[0] = st[mp].m; d0[1] = l; }
+        if (lane < 16) { d0[DV] = st[mp].m; d0[DV + 1] = l; }
 #pragma unroll
-        for (int d = 0; d < DV / 16; d++)
-#pragma unroll
-            for (int r = 0; r < 4; r++) d0[2 + d * 16 + (lane >> 4) * 4 + r] = o[mp][d][r];
+        for (int d = 0; d < DV / 16; d++) *reinterpret_cast<float4*>(d0 + d * 16 + (lane >> 4) * 4) = make_float4(o[mp][d][0], o[mp][d][1], o[mp][d][2], o[mp][d][3]);
     }
     __syncthreads();
-    // partial record of (tile, kv head, split): [map][16] rows of DV + 2
     float* rec = a.partial + (size_t)((tile * a.kv_heads + g) * a.splits + split) * MAPS * 16 * kRow;
     const uint32_t used = row_last - row0 + 1;
     for (uint32_t i = tid; i < (uint32_t)MAPS * used * DV; i += 256) {
         const uint32_t mp = i / (used * DV), rr = (i / DV) % used, d = i % DV;
         float m = -INFINITY, acc = 0.0f, l = 0.0f;
 #pragma unroll
-        for (int wv = 0; wv < 4; wv++) m = fmaxf(m, merge[((wv * MAPS + mp) * 16 + rr) * kRow]);
+        for (int wv = 0; wv < 4; wv++) m = fmaxf(m, merge[((wv * MAPS + mp) * 16 + rr) * kRow + DV]);
         const float base = m == -INFINITY ? 0.0f : m;
 #pragma unroll
         for (int wv = 0; wv < 4; wv++) {
             const float* s = merge + ((wv * MAPS + mp) * 16 + rr) * kRow;
-            const float f = __builtin_amdgcn_exp2f(s[0] - base);
-            l += f * s[1];
-            acc += f * s[2 + d];
+            const float f = __builtin_amdgcn_exp2f(s[DV] - base);
+            l += f * s[DV + 1];
+            acc += f * s[d];
         }
         float* r = rec + (mp * 16 + rr) * kRow;
-        r[2 + d] = acc;
-        if (d == 0) { r[0] = m; r[1] = l; }
+        r[d] = acc;
+        if (d == 0) { r[DV] = m; r[DV + 1] = l; }
     }
 }
 
-// One workgroup per (query row, head): merges the splits of every map, combines the maps, norms and stores.
+// One workgroup per (query row, head): merges the splits of every map, combines the maps, norms and stores.  Groups of dv / 4
+// threads take the splits in turn, four values a thread, several loads on their way; the groups are added through LDS.
+constexpr uint32_t kMergeThreads = 512;
 template <int MAPS>
-__global__ __launch_bounds__(256) void attention_merge_kernel(const AttentionArgs a) {
-    __shared__ float factor[MAPS][512], total[MAPS], scratch[4];
+__global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const AttentionArgs a) {
+    __shared__ float factor[MAPS][512], total[MAPS], scratch[kMergeThreads / 64];
+    __shared__ float4 sums[MAPS][kMergeThreads];
     const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
-    const uint32_t kRow = a.dv + 2, rr = row & 15;
+    const uint32_t kRow = a.dv + 4, rr = row & 15;
     const size_t stride = (size_t)MAPS * 16 * kRow;
     const float* rec = a.partial + (size_t)(((row >> 4) * a.kv_heads + g) * a.splits) * stride + rr * kRow;
     const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
     if (wave < MAPS) {                                        // splits <= 512
-        const float* r = rec + wave * 16 * kRow;
-        float m = -INFINITY, l = 0.0f;
-        for (uint32_t s = lane; s < a.splits; s += 64) m = fmaxf(m, r[s * stride]);
+        const float* r = rec + wave * 16 * kRow + a.dv;
+        float m = -INFINITY, l = 0.0f, mine[8], ml[8];
+#pragma unroll
+        for (uint32_t i = 0; i < 8; i++) {
+            const uint32_t s = i * 64 + lane;
+            mine[i] = -INFINITY; ml[i] = 0.0f;
+            if (i * 64 >= a.splits) break;
+            if (s < a.splits) { const float2 x = *reinterpret_cast<const float2*>(r + s * stride); mine[i] = x.x; ml[i] = x.y; }
+            m = fmaxf(m, mine[i]);
+        }
         m = lh_group_max(m, 64);
-        for (uint32_t s = lane; s < a.splits; s += 64) {
-            const float f = __builtin_amdgcn_exp2f(r[s * stride] - m);
-            factor[wave][s] = f;
-            l += f * r[s * stride + 1];
+#pragma unroll
+        for (uint32_t i = 0; i < 8; i++) {
+            if (i * 64 >= a.splits) break;
+            const float f = __builtin_amdgcn_exp2f(mine[i] - m);
+            if (i * 64 + lane < a.splits) factor[wave][i * 64 + lane] = f;
+            l += f * ml[i];
         }
         l = lh_group_sum(l, 64);
         if (lane == 0) total[wave] = 1.0f / l;
     }
     __syncthreads();
-    float v[4], ss = 0.0f;                                    // vdim <= 1024
+    const uint32_t quads = a.dv / 4, groups = kMergeThreads / quads, grp = threadIdx.x / quads, q = threadIdx.x % quads;   // quads <= 64
+    float4 acc[MAPS];
 #pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const uint32_t d = threadIdx.x + i * 256;
-        v[i] = 0.0f;
-        if (d >= a.vdim) break;
-        float acc[MAPS] = {};
-        for (uint32_t s = 0; s < a.splits; s++)
+    for (int mp = 0; mp < MAPS; mp++) acc[mp] = make_float4(0.f, 0.f, 0.f, 0.f);
+#pragma unroll 4
+    for (uint32_t s = grp; s < a.splits; s += groups)
 #pragma unroll
-            for (int mp = 0; mp < MAPS; mp++)
-                if (factor[mp][s] != 0.0f) acc[mp] += factor[mp][s] * rec[s * stride + mp * 16 * kRow + 2 + d];
-        v[i] = acc[0] * total[0];
-        if constexpr (MAPS == 2) v[i] -= a.lambda * (acc[MAPS - 1] * total[MAPS - 1]);
-        ss += v[i] * v[i];
+        for (int mp = 0; mp < MAPS; mp++) {
+            const float4 x = *reinterpret_cast<const float4*>(rec + s * stride + mp * 16 * kRow + q * 4);
+            const float f = factor[mp][s];
+            acc[mp].x += f * x.x; acc[mp].y += f * x.y; acc[mp].z += f * x.z; acc[mp].w += f * x.w;
+        }
+#pragma unroll
+    for (int mp = 0; mp < MAPS; mp++) sums[mp][threadIdx.x] = acc[mp];
+    __syncthreads();
+    float v = 0.0f;
+    const uint32_t d = threadIdx.x;                           // dv <= 256
+    if (d < a.vdim) {
+        float s[MAPS] = {};
+        for (uint32_t i = 0; i < groups; i++)
+#pragma unroll
+            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sums[mp][i * quads])[d];
+        v = s[0] * total[0];
+        if constexpr (MAPS == 2) v -= a.lambda * (s[MAPS - 1] * total[MAPS - 1]);
     }
     float f = 1.0f;
-    if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(ss, scratch) / (float)a.vdim + a.eps) * a.out_scale;
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        const uint32_t d = threadIdx.x + i * 256;
-        if (d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v[i] * f);
-    }
+    if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(v * v, scratch) / (float)a.vdim + a.eps) * a.out_scale;
+    if (d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
 }
 
 // One workgroup per (query row, head), 256 keys at a time; f32 arithmetic throughout.
@@ -482,36 +490,39 @@ constexpr uint32_t kMaxSplits = 512;
 template <int DQ, int DV, int MAPS>
 int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const char* op, uint32_t& launches) {
     const uint32_t R = a.heads / a.kv_heads;
-    const uint64_t packed = (uint64_t)a.rows * R;
-    constexpr int RT = DV <= 128 && DQ <= 64 ? 2 : 1;
-    const uint64_t tiles = (packed + 64 * RT - 1) / (64 * RT);
+    const uint64_t packed = (uint64_t)a.rows * R, tiles16 = (packed + 15) / 16, cus = ctx->cu_count;
     const uint32_t max_blocks = (uint32_t)std::min<uint64_t>((uint64_t)max_position + a.rows, a.capacity) / 32 + 1;
-    const bool split = packed <= 64 || (tiles * a.kv_heads < (uint64_t)ctx->cu_count / 4 && packed <= 256);
-    if (!split) {
-        LH_REQUIRE(tiles * a.kv_heads < 0x7FFFFFFFull, "%s: %u rows", op, a.rows);
-        hipLaunchKernelGGL((attention_tile_kernel<DQ, DV, MAPS, RT>), dim3((uint32_t)(tiles * a.kv_heads)), dim3(256), 0, ctx->stream, a);
-        launches = 1;
+    const size_t rec = (size_t)tiles16 * a.kv_heads * MAPS * 16 * (DV + 4) * 4;
+    const uint32_t room = (uint32_t)std::min<size_t>(ctx->workspace_bytes / rec, kMaxSplits);
+    auto merge = [&]() {
+        hipLaunchKernelGGL((attention_merge_kernel<MAPS>), dim3(a.rows * a.heads), dim3(kMergeThreads), 0, ctx->stream, a);
+        launches++;
         return lh_check_launch(op);
-    }
-    const uint32_t st = (uint32_t)((packed + 15) / 16);
-    const size_t rec = (size_t)st * a.kv_heads * MAPS * 16 * (DV + 2) * 4;
-    // two blocks per wave at least, two workgroups per CU at most
-    uint32_t splits = std::max(1u, std::min({max_blocks / 8, (2u * ctx->cu_count + st * a.kv_heads - 1) / (st * a.kv_heads), kMaxSplits}));
-    splits = (uint32_t)std::min<size_t>(splits, std::max<size_t>(1, ctx->workspace_bytes / rec));
-    LH_REQUIRE(rec * splits <= ctx->workspace_bytes, "%s: %u heads of %u values exceed the workspace", op, a.heads, a.vdim);
+    };
     a.partial = (float*)ctx->workspace;
-    a.splits = splits;
-    constexpr size_t lds = (size_t)4 * MAPS * 16 * (DV + 2) * 4;
+    launches = 1;
+    if (packed > 64) {
+        constexpr int NB = MAPS * DQ + DV <= 256 ? 2 : 1;
+        const uint64_t groups = (packed + 63) / 64 * a.kv_heads;
+        // a share of eight key steps at least, and no more workgroups than two per CU
+        a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({2 * cus / groups, max_blocks / (8 * NB), room}));
+        LH_REQUIRE(groups * a.splits < 0x7FFFFFFFull, "%s: %u rows", op, a.rows);
+        hipLaunchKernelGGL((attention_tile_kernel<DQ, DV, MAPS, NB>), dim3((uint32_t)(groups * a.splits)), dim3(256), 0, ctx->stream, a);
+        const int r = lh_check_launch(op);
+        return r != LH_OK || a.splits == 1 ? r : merge();
+    }
+    // two blocks per wave at least, no more workgroups than one per CU
+    const uint64_t groups = tiles16 * a.kv_heads;
+    LH_REQUIRE(room >= 1, "%s: %u heads of %u values exceed the workspace", op, a.heads, a.vdim);
+    a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({max_blocks / 8, (cus + groups - 1) / groups, room}));
+    constexpr size_t lds = (size_t)4 * MAPS * 16 * (DV + 4) * 4;
     if (lds > 64 * 1024) {
         const int r = lh_raise_dynamic_lds(ctx, (const void*)attention_split_kernel<DQ, DV, MAPS>, lds, op);
         if (r != LH_OK) return r;
     }
-    hipLaunchKernelGGL((attention_split_kernel<DQ, DV, MAPS>), dim3(st * a.kv_heads * splits), dim3(256), lds, ctx->stream, a);
-    int r = lh_check_launch(op);
-    if (r != LH_OK) return r;
-    hipLaunchKernelGGL((attention_merge_kernel<MAPS>), dim3(a.rows * a.heads), dim3(256), 0, ctx->stream, a);
-    launches = 2;
-    return lh_check_launch(op);
+    hipLaunchKernelGGL((attention_split_kernel<DQ, DV, MAPS>), dim3((uint32_t)(groups * a.splits)), dim3(256), lds, ctx->stream, a);
+    const int r = lh_check_launch(op);
+    return r != LH_OK ? r : merge();
 }
 
 template <int DQ, int DV>
