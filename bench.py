@@ -962,7 +962,7 @@ def bench_stack_kernels(pkg, ctx, K, steps, warmup):
     return res
 
 
-def bench_stack_models(pkg, ctx, K, steps, warmup):
+def bench_stack_models(pkg, ctx, K, steps, warmup, graphs=True):
     """Tokens per second of whole stacks with random weights, beside the quantized decoder at equal width, depth and context:
     decoding (a recorded step each) and prompts in passes of 2048 rows."""
     A = pkg.mixers
@@ -973,7 +973,7 @@ def bench_stack_models(pkg, ctx, K, steps, warmup):
         moe, dense = A.MoeSpec(experts, 2, ff // 8), A.DenseSpec(ff)
         cfg = pkg.stack_pipeline.StackConfig(32000, width, 1e-6, [A.LayerSpec(m, f) for m, f in ((attn, dense), (lin, dense), (attn, moe), (lin, moe))])
         T = 4096
-        m = pkg.stack_pipeline.StackPipeline(ctx, K, cfg, RandomTensors(1), T + 512)
+        m = pkg.stack_pipeline.StackPipeline(ctx, K, cfg, RandomTensors(1), T + 512, graphs=graphs)
         tokens = [int(t) for t in np.random.default_rng(2).integers(0, 32000, T)]
         out = {}
         for rows in (256, 2048):
@@ -997,21 +997,22 @@ def bench_stack_models(pkg, ctx, K, steps, warmup):
         for _ in range(n):
             m.greedy(s, 1)
         out["decode_us_per_token_with_host"] = (time.perf_counter() - t0) / n * 1e6
-        settle(ctx, s.graph.launch, 100)
-        e0, e1 = pkg.Event(ctx), pkg.Event(ctx)
-        s.position_buf.copy_from_bytes(np.array([T], np.uint32))
-        e0.record()
-        for _ in range(100):
-            s.graph.launch()
-        e1.record()
-        ctx.synchronize()
-        us = e0.elapsed_ms(e1) * 10
         # bytes a decoded token has to read: every weight but the unchosen experts, the attention caches, the states twice
         byte = sum(b.bytes() for l in m.layers for b in (l.mixer.out, getattr(l.mixer, "qkv", None) or l.mixer.qkvg)) + m.head.bytes()
         byte += sum(l.ff.up.bytes() + l.ff.down.bytes() if isinstance(l.ff, A.DenseFeedForward) else 2 * 2 * 2 * width * (ff // 8) for l in m.layers)
         byte += 2 * T * kv * (2 * 64 + 128) * 2 + 2 * 2 * lin.heads * 128 * 128 * 4
-        out.update(decode_us_per_token=us, decode_tokens_per_s=1e6 / us, decode_dispatches=s.graph.dispatch_count(),
-                   decode_gbs=byte / us * 1e-3, decode_frac_of_hbm_peak=byte / us * 1e-3 / HBM_PEAK_GBS)
+        if graphs:
+            settle(ctx, s.graph.launch, 100)
+            e0, e1 = pkg.Event(ctx), pkg.Event(ctx)
+            s.position_buf.copy_from_bytes(np.array([T], np.uint32))
+            e0.record()
+            for _ in range(100):
+                s.graph.launch()
+            e1.record()
+            ctx.synchronize()
+            us = e0.elapsed_ms(e1) * 10
+            out.update(decode_us_per_token=us, decode_tokens_per_s=1e6 / us, decode_dispatches=s.graph.dispatch_count(),
+                       decode_gbs=byte / us * 1e-3, decode_frac_of_hbm_peak=byte / us * 1e-3 / HBM_PEAK_GBS)
         m.end_sequence(s)
         del m
         gcfg = pkg.pipeline.Gemma4QATConfig(vocab_size=32000, hidden_size=width, num_hidden_layers=4, num_attention_heads=width // 256, num_key_value_heads=1,
@@ -1030,19 +1031,21 @@ def bench_stack_models(pkg, ctx, K, steps, warmup):
         for _ in range(n):
             pipe.decode_step(1)
         out["quantized_decode_us_per_token_with_host"] = (time.perf_counter() - t0) / n * 1e6
-        batch = pkg.CommandBatch(ctx)
-        batch.begin_capture()
-        pipe.write_logits(pipe.forward_token(1, T, batch=batch), batch=batch)
-        graph = batch.end_capture()
-        settle(ctx, graph.launch, 100)
-        e0.record()
-        for _ in range(100):
-            graph.launch()
-        e1.record()
-        ctx.synchronize()
-        out["quantized_decode_us_per_token"] = e0.elapsed_ms(e1) * 10
-        out["quantized_decode_dispatches"] = graph.dispatch_count()
-        del pipe, graph
+        if graphs:
+            batch = pkg.CommandBatch(ctx)
+            batch.begin_capture()
+            pipe.write_logits(pipe.forward_token(1, T, batch=batch), batch=batch)
+            graph = batch.end_capture()
+            settle(ctx, graph.launch, 100)
+            e0.record()
+            for _ in range(100):
+                graph.launch()
+            e1.record()
+            ctx.synchronize()
+            out["quantized_decode_us_per_token"] = e0.elapsed_ms(e1) * 10
+            out["quantized_decode_dispatches"] = graph.dispatch_count()
+            del graph
+        del pipe
         res[f"width_{width}"] = out
         log(f"[bench] stack model width {width}:", out)
     return res
@@ -1175,7 +1178,7 @@ def main():
     if "stack_kernels" in legs:
         extra["stack_kernels"] = bench_stack_kernels(pkg, ctx, K, args.steps, args.warmup)
     if "stack_models" in legs:
-        extra["stack_models"] = bench_stack_models(pkg, ctx, K, args.steps, args.warmup)
+        extra["stack_models"] = bench_stack_models(pkg, ctx, K, args.steps, args.warmup, graphs=not args.no_graph)
 
     achieved = head["alg_bytes_per_launch"] / head["ms_per_launch_events"] * 1e-6
     # The other north-star kernels of this run, in the blocks a reader of the line keeps: their rooflines beside the

@@ -77,7 +77,13 @@ __global__ __launch_bounds__(1024) void argmax_rows_kernel(const float* __restri
     const float* row = x + (size_t)blockIdx.x * n;
     float best = -INFINITY;
     uint32_t at = 0xFFFFFFFFu;
-    for (uint32_t i = threadIdx.x; i < n; i += 1024) { const float v = row[i]; if (v > best || at == 0xFFFFFFFFu) { best = v; at = i; } }
+    for (uint32_t i0 = threadIdx.x; i0 < n; i0 += 16 * 1024) {   // sixteen loads on their way at a time
+        float v[16];
+#pragma unroll
+        for (uint32_t j = 0; j < 16; j++) v[j] = row[min(i0 + j * 1024, n - 1)];
+#pragma unroll
+        for (uint32_t j = 0; j < 16; j++) if (i0 + j * 1024 < n && (v[j] > best || at == 0xFFFFFFFFu)) { best = v[j]; at = i0 + j * 1024; }
+    }
     sv[threadIdx.x] = best; si[threadIdx.x] = at;
     __syncthreads();
     for (uint32_t h = 512; h > 0; h >>= 1) {

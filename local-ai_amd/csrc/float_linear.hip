@@ -88,12 +88,16 @@ __device__ __forceinline__ void store4(const LhLinear& a, uint32_t slot, uint32_
 // ---- matrix cores ------------------------------------------------------------------------------------------------------
 // 256 threads, 2 x 2 waves of BM/2 x BN/2 outputs.  A k step is 64 wide: a tile row is eight 16-byte chunks, chunk c of row r
 // kept at place c ^ (r & 7) of its row so that the fragment reads of sixteen rows fall on different banks (the loads
-// write LDS in order, so the permutation is applied to their global addresses).  Two buffers, one barrier per step.
+// write LDS in order, so the permutation is applied to their global addresses).  NS buffers, one barrier per step: step kt is
+// multiplied while the loads of the NS - 1 steps after it are on their way.
 // The weights are the MFMA's row operand: lane = output row (lane & 15), four consecutive output columns per tile.
-template <int BM, int BN>
+template <int N> __device__ __forceinline__ void wait_loads() { asm volatile("s_waitcnt vmcnt(%0)" :: "n"(N) : "memory"); }
+
+template <int BM, int BN, int NS>
 __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
     constexpr int TI = BM / 32, TJ = BN / 32, CA = BM / 32, CB = BN / 32;
-    __shared__ uint4 sm[2][(BM + BN) * 8];
+    static_assert(NS * (BM + BN) * 128 >= BM * BN * 4, "the output tile must fit the staging buffers");
+    __shared__ uint4 sm[NS][(BM + BN) * 8];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, wm = wave >> 1, wn = wave & 1;
     const uint32_t mt_n = a.ex.tiles ? a.ex.n_tiles : (a.M + BM - 1) / BM, nt_n = (a.N + BN - 1) / BN;
     uint32_t mt, nt;
@@ -137,12 +141,16 @@ __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
 #pragma unroll
         for (int j = 0; j < TJ; j++) acc[i][j] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
 
-    load_step(0, 0);
+#pragma unroll
+    for (int i = 0; i < NS - 1; i++) if (i < (int)nk) load_step(i, i);
+    uint32_t buf = 0;
     for (uint32_t kt = 0; kt < nk; kt++) {
-        asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        __syncthreads();
-        if (kt + 1 < nk) load_step((kt + 1) & 1, kt + 1);
-        const uint4* as = sm[kt & 1];
+        if (kt + NS - 1 <= nk) wait_loads<(NS - 2) * (CA + CB)>();   // step kt has arrived; the later steps may still be coming
+        else wait_loads<0>();
+        lh_lds_barrier();
+        if (kt + NS - 1 < nk) load_step(buf == 0 ? NS - 1 : buf - 1, kt + NS - 1);
+        const uint4* as = sm[buf];
+        buf = buf + 1 == NS ? 0 : buf + 1;
         const uint4* bs = as + BM * 8;
 #pragma unroll
         for (int ks = 0; ks < 2; ks++) {
@@ -399,6 +407,51 @@ __global__ __launch_bounds__(256) void matvec_bf16_reg_kernel(const VectorStage 
     sums.flush();
 }
 
+// Rows longer than a wave's registers: the four waves of a workgroup take a quarter of the columns each, and the quarters of up to 64 rows meet in LDS.  Plain vectors only: a norm would need all quarters.
+template <int NL>
+__global__ __launch_bounds__(256) void matvec_bf16_quarter_kernel(const VectorStage st, const uint16_t* __restrict__ W, const float* __restrict__ bias, const LhSegments seg,
+                                                                 uint32_t N, uint32_t K, uint32_t quarter) {
+    __shared__ float sums[4][64];
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, k0 = wave * quarter, len = k0 < K ? min(quarter, K - k0) : 0u;   // quarter: a multiple of 8
+    const uint32_t last = len ? (len >> 3) - 1 : 0u, kb = len ? k0 : 0u;
+    auto issue = [&](uint4 (&v)[NL], uint32_t r) {
+        const uint16_t* wr = W + (size_t)r * K + kb;
+#pragma unroll
+        for (int c = 0; c < NL; c++) v[c] = lh_ld16_stream(wr + 8 * min(64u * c + lane, last));
+    };
+    uint32_t row = blockIdx.x, base = blockIdx.x, n = 0;
+    uint4 p[NL], q[NL];
+    issue(p, row);
+    VectorStage part = st;
+    part.x = st.x_f32 ? (const void*)(static_cast<const float*>(st.x) + kb) : (const void*)(static_cast<const uint16_t*>(st.x) + kb);
+    float xr[NL][8], mine = 0.0f;
+    lh_vector_registers<kPlain, NL>(part, len, lane, false, xr);
+    auto flush = [&]() {
+        sums[wave][lane] = mine;
+        __syncthreads();
+        const uint32_t r = base + lane * gridDim.x;
+        if (wave == 0 && lane < n)
+            lh_segment_store(seg, 0, r, ((sums[0][lane] + sums[1][lane]) + (sums[2][lane] + sums[3][lane])) + (bias ? bias[r] : 0.0f), seg.position ? *seg.position : 0u);
+        __syncthreads();
+        base += n * gridDim.x;
+        n = 0;
+    };
+    auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {
+        const bool more = row + gridDim.x < N;
+        if (more) issue(nxt, row + gridDim.x);
+        float acc = 0.0f;
+#pragma unroll
+        for (int c = 0; c < NL; c++) acc = lh_dot8(cur[c], xr[c], acc);
+        acc = lh_group_sum(acc, 64);
+        mine = n == lane ? acc : mine;
+        if (++n == 64) flush();
+        row += gridDim.x;
+        return more;
+    };
+    while (step(p, q) && step(q, p)) {}
+    if (n) flush();
+}
+
 constexpr uint32_t kMaxVectorK = 36864;   // 144 KB of staged f32 activations
 
 template <int STAGE>
@@ -414,6 +467,13 @@ int launch_vector(lh_context* ctx, const VectorStage& st, const uint16_t* W, con
         else if (K <= 2048) LH_MVR(4);
         else LH_MVR(8);
 #undef LH_MVR
+        return lh_check_launch(op);
+    }
+    if (STAGE == kPlain && vec && K <= 16384 && lh_stage_aligned(st)) {
+        const uint32_t quarter = ((K + 3) / 4 + 7) / 8 * 8, grid = (uint32_t)std::min<uint64_t>(N, (uint64_t)ctx->cu_count * 4);
+        if (quarter <= 1024) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<2>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else if (quarter <= 2048) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<4>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else hipLaunchKernelGGL((matvec_bf16_quarter_kernel<8>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
         return lh_check_launch(op);
     }
     const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * 4);
@@ -477,20 +537,20 @@ int lh_launch_linear(lh_context* ctx, const LhLinear& a, const char* op) {
         return lh_check_launch(op);
     }
     auto tiles = [&](uint32_t bm, uint32_t bn) { return (uint64_t)(a.ex.tiles ? a.ex.n_tiles : (a.M + bm - 1) / bm) * ((a.N + bn - 1) / bn); };
-#define LH_GEMM(BM_, BN_)                                                                                               \
+#define LH_GEMM(BM_, BN_, NS_)                                                                                             \
     do {                                                                                                                \
         const uint64_t grid = tiles(BM_, BN_);                                                                          \
         LH_REQUIRE(grid < 0x7FFFFFFFull, "%s: %u x %u outputs", op, a.M, a.N);                                          \
-        if (grid) hipLaunchKernelGGL((linear_mfma_kernel<BM_, BN_>), dim3((uint32_t)grid), dim3(256), 0, ctx->stream, a); \
+        if (grid) hipLaunchKernelGGL((linear_mfma_kernel<BM_, BN_, NS_>), dim3((uint32_t)grid), dim3(256), 0, ctx->stream, a); \
     } while (0)
     const uint64_t want = (uint64_t)ctx->cu_count;
     if (a.ex.tiles) {
-        if (a.ex.tile_rows == 128) { if (tiles(128, 128) >= want) LH_GEMM(128, 128); else LH_GEMM(128, 64); }
-        else LH_GEMM(64, 64);
-    } else if (tiles(128, 128) >= 2 * want) LH_GEMM(128, 128);
-    else if (tiles(128, 64) >= want) LH_GEMM(128, 64);
-    else if (tiles(64, 64) >= want || a.M > 32) LH_GEMM(64, 64);
-    else LH_GEMM(32, 32);
+        if (a.ex.tile_rows == 128) { if (tiles(128, 128) >= want) LH_GEMM(128, 128, 2); else LH_GEMM(128, 64, 3); }
+        else LH_GEMM(64, 64, 4);
+    } else if (tiles(128, 128) >= 2 * want) LH_GEMM(128, 128, 2);
+    else if (tiles(128, 64) >= want) LH_GEMM(128, 64, 3);
+    else if (tiles(64, 64) >= want || a.M > 32) LH_GEMM(64, 64, 4);
+    else LH_GEMM(32, 32, 4);
 #undef LH_GEMM
     return lh_check_launch(op);
 }

@@ -78,49 +78,80 @@ __device__ __forceinline__ lh_bf16x8 bf8(const uint32_t (&w)[4]) {
 
 constexpr uint32_t kLdT = kChunk + 8;     // row length of a transposed tile: 16-byte aligned, rows on different banks
 
-// Step 1.  A workgroup takes one chunk of one head and 64 value columns; four waves split the key columns.
-// U^T tiles: row operand = decayed keys (16 key columns x tokens), column operand = values (16 value columns x tokens).
+// 64 rows of 64 value columns, transposed into LDS: thread t brings in rows t / 8 and t / 8 + 32, eight columns each.
+struct ValueTile { uint4 x[2]; };
+__device__ __forceinline__ void load_values(ValueTile& f, const ChunkArgs& a, uint32_t t0, uint32_t L, uint32_t h, uint32_t v0, uint32_t tid) {
+    const uint32_t d = v0 + (tid & 7) * 8;
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const uint32_t s = (tid >> 3) + 32 * i;
+        f.x[i] = make_uint4(0u, 0u, 0u, 0u);
+        if (s >= L || d >= a.vdim) continue;
+        const uint16_t* p = a.v + ((size_t)(t0 + s) * a.heads + h) * a.vdim + d;
+        if ((a.vdim & 7) == 0) f.x[i] = *reinterpret_cast<const uint4*>(p);
+        else {
+            uint32_t w[4] = {0u, 0u, 0u, 0u};
+#pragma unroll
+            for (uint32_t j = 0; j < 8; j++) if (d + j < a.vdim) w[j >> 1] |= (uint32_t)p[j] << (16 * (j & 1));
+            f.x[i] = make_uint4(w[0], w[1], w[2], w[3]);
+        }
+    }
+}
+template <bool SLOTS>
+__device__ __forceinline__ void park_values(const ValueTile& f, uint16_t (&vt)[64][kLdT], uint32_t tid) {
+#pragma unroll
+    for (int i = 0; i < 2; i++) {
+        const uint32_t s = (tid >> 3) + 32 * i, place = SLOTS ? (s & 32) + lh_block_slot(s & 31) : s;
+        const uint32_t w[4] = {f.x[i].x, f.x[i].y, f.x[i].z, f.x[i].w};
+#pragma unroll
+        for (uint32_t j = 0; j < 8; j++) vt[(tid & 7) * 8 + j][place] = (uint16_t)(w[j >> 1] >> (16 * (j & 1)));
+    }
+}
+
+// Step 1.  A workgroup takes one chunk of one head, 32 key columns and 64 value columns; wave w the value columns 16 w ..
+// 16 w + 15.  Row operand = decayed keys (16 key columns x rows), column operand = values (16 value columns x rows).
 template <int DQ>
 __global__ __launch_bounds__(256) void chunk_state_kernel(const ChunkArgs a) {
     __shared__ __align__(16) uint16_t kt[3][32][kLdT], vt[64][kLdT];
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6;
-    const uint32_t vtiles = (a.vdim + 63) / 64, vb = blockIdx.x % vtiles, h = (blockIdx.x / vtiles) % a.heads, c = blockIdx.x / (vtiles * a.heads);
+    const uint32_t vtiles = (a.vdim + 63) / 64, k0 = blockIdx.x % (DQ / 32) * 32, r = blockIdx.x / (DQ / 32);
+    const uint32_t vb = r % vtiles, h = (r / vtiles) % a.heads, c = r / (vtiles * a.heads);
     const uint32_t t0 = c * kChunk, L = min(kChunk, a.rows - t0), v0 = vb * 64;
-    const float* pw = a.powers + h * (kChunk + 1);
-    for (uint32_t e = tid; e < 64 * kChunk; e += 256) {
-        const uint32_t s = e >> 6, d = e & 63;
-        vt[d][s] = s < L && v0 + d < a.vdim ? a.v[((size_t)(t0 + s) * a.heads + h) * a.vdim + v0 + d] : 0;
-    }
-    float* U = a.chunk_state + ((size_t)c * a.heads + h) * a.vdim * DQ;
-    for (uint32_t k0 = 0; k0 < DQ; k0 += 32) {
-        __syncthreads();
-        for (uint32_t e = tid; e < 32 * kChunk; e += 256) {
-            const uint32_t s = e >> 5, d = e & 31;
-            float x = 0.0f;
-            if (s < L && k0 + d < a.dim) x = lh_bf2f(a.k[((size_t)(t0 + s) * a.heads + h) * DQ + k0 + d]) * pw[L - 1 - s];
-            const LhSplit3 t = lh_split3(x);
-            kt[0][d][s] = t.hi; kt[1][d][s] = t.mid; kt[2][d][s] = t.lo;
+    ValueTile f;
+    load_values(f, a, t0, L, h, v0, tid);
+    {   // eight key columns of one row per thread
+        const uint32_t s = tid >> 2, d = (tid & 3) * 8;
+        uint4 x = make_uint4(0u, 0u, 0u, 0u);
+        float p = 0.0f;
+        if (s < L) {
+            x = *reinterpret_cast<const uint4*>(a.k + ((size_t)(t0 + s) * a.heads + h) * DQ + k0 + d);
+            p = a.powers[h * (kChunk + 1) + L - 1 - s];
         }
-        __syncthreads();
-        // the eight 16 x 16 tiles of this 32 x 64 block: wave w takes value tile w of both key tiles
-        lh_f32x4 acc[2] = {(lh_f32x4){0.f, 0.f, 0.f, 0.f}, (lh_f32x4){0.f, 0.f, 0.f, 0.f}};
+        const uint32_t w[4] = {x.x, x.y, x.z, x.w};
 #pragma unroll
-        for (int ks = 0; ks < 2; ks++) {
-            const uint32_t s = ks * 32 + (lane >> 4) * 8;
-            const lh_bf16x8 vf = *reinterpret_cast<const lh_bf16x8*>(&vt[wave * 16 + (lane & 15)][s]);
-#pragma unroll
-            for (int i = 0; i < 2; i++)
-#pragma unroll
-                for (int p = 0; p < 3; p++)
-                    acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lh_bf16x8*>(&kt[p][i * 16 + (lane & 15)][s]), vf, acc[i], 0, 0, 0);
-        }
-        const uint32_t col = v0 + wave * 16 + (lane & 15);
-        if (col < a.vdim) {
-#pragma unroll
-            for (int i = 0; i < 2; i++)
-                *reinterpret_cast<float4*>(U + (size_t)col * DQ + k0 + i * 16 + (lane >> 4) * 4) = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
+        for (uint32_t j = 0; j < 8; j++) {
+            const LhSplit3 e = lh_split3(s < L && k0 + d + j < a.dim ? lh_bf2f((uint16_t)(w[j >> 1] >> (16 * (j & 1)))) * p : 0.0f);
+            kt[0][d + j][s] = e.hi; kt[1][d + j][s] = e.mid; kt[2][d + j][s] = e.lo;
         }
     }
+    park_values<false>(f, vt, tid);
+    __syncthreads();
+    lh_f32x4 acc[2] = {(lh_f32x4){0.f, 0.f, 0.f, 0.f}, (lh_f32x4){0.f, 0.f, 0.f, 0.f}};
+#pragma unroll
+    for (int ks = 0; ks < 2; ks++) {
+        const uint32_t s = ks * 32 + (lane >> 4) * 8;
+        const lh_bf16x8 vf = *reinterpret_cast<const lh_bf16x8*>(&vt[wave * 16 + (lane & 15)][s]);
+#pragma unroll
+        for (int i = 0; i < 2; i++)
+#pragma unroll
+            for (int p = 0; p < 3; p++)
+                acc[i] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(*reinterpret_cast<const lh_bf16x8*>(&kt[p][i * 16 + (lane & 15)][s]), vf, acc[i], 0, 0, 0);
+    }
+    const uint32_t col = v0 + wave * 16 + (lane & 15);
+    if (col >= a.vdim) return;
+    float* U = a.chunk_state + ((size_t)c * a.heads + h) * a.vdim * DQ + (size_t)col * DQ + k0 + (lane >> 4) * 4;
+#pragma unroll
+    for (int i = 0; i < 2; i++) *reinterpret_cast<float4*>(U + i * 16) = make_float4(acc[i][0], acc[i][1], acc[i][2], acc[i][3]);
 }
 
 // Step 2.  A thread owns four neighbouring state values and walks the chunks, eight loads ahead.
@@ -160,13 +191,9 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkArgs a) {
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4;
     const uint32_t vtiles = (a.vdim + 63) / 64, vb = blockIdx.x % vtiles, h = (blockIdx.x / vtiles) % a.heads, c = blockIdx.x / (vtiles * a.heads);
     const uint32_t t0 = c * kChunk, L = min(kChunk, a.rows - t0), v0 = vb * 64;
-    for (uint32_t e = tid; e < 64 * kChunk; e += 256) {
-        const uint32_t s = e >> 6, d = e & 63;
-        vt[d][(s & 32) + lh_block_slot(s & 31)] = s < L && v0 + d < a.vdim ? a.v[((size_t)(t0 + s) * a.heads + h) * a.vdim + v0 + d] : 0;
-    }
+    ValueTile f;
+    load_values(f, a, t0, L, h, v0, tid);
     if (tid <= kChunk) pws[tid] = a.powers[h * (kChunk + 1) + tid];
-    __syncthreads();
-    if (wave * 16 >= L) return;
     const uint32_t t = wave * 16 + (lane & 15), tr = min(t, L - 1);
     lh_bf16x8 qf[DQ / 32];
 #pragma unroll
@@ -184,6 +211,9 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkArgs a) {
         }
         qf[i] = bf8(w);
     }
+    park_values<true>(f, vt, tid);
+    __syncthreads();
+    if (wave * 16 >= L) return;
     lh_f32x4 o[4];
     // the state's part, scaled by decay^(t + 1) afterwards
     const float* S = a.chunk_state + ((size_t)c * a.heads + h) * a.vdim * DQ;
@@ -261,7 +291,7 @@ __global__ __launch_bounds__(256) void chunk_output_kernel(const ChunkArgs a) {
 template <int DQ>
 int launch_chunked(lh_context* ctx, const ChunkArgs& a, const char* op) {
     const uint32_t grid = a.chunks * a.heads * ((a.vdim + 63) / 64);
-    hipLaunchKernelGGL((chunk_state_kernel<DQ>), dim3(grid), dim3(256), 0, ctx->stream, a);
+    hipLaunchKernelGGL((chunk_state_kernel<DQ>), dim3(grid * (DQ / 32)), dim3(256), 0, ctx->stream, a);
     int r = lh_check_launch(op);
     if (r != LH_OK) return r;
     const size_t total4 = (size_t)a.heads * a.vdim * DQ / 4;
@@ -335,11 +365,11 @@ int lh_linear_attention_chunked_into(lh_batch* batch, const lh_buffer* q, const 
     LH_NEED(decay_powers, (size_t)heads * (kChunk + 1) * 4, op, "decay_powers");
     LH_NEED(workspace, lh_linear_attention_workspace_bytes(rows, heads, dim, vdim), op, "workspace");
     LH_NEED(output, (size_t)rows * heads * vdim * 4, op, "output");
-    LH_REQUIRE((((uintptr_t)q->ptr | (uintptr_t)k->ptr | (uintptr_t)state->ptr | (uintptr_t)workspace->ptr | (uintptr_t)output->ptr) & 15) == 0,
+    LH_REQUIRE((((uintptr_t)q->ptr | (uintptr_t)k->ptr | (uintptr_t)v->ptr | (uintptr_t)state->ptr | (uintptr_t)workspace->ptr | (uintptr_t)output->ptr) & 15) == 0,
                "%s: buffers must be 16-byte aligned", op);
     ChunkArgs a{(const uint16_t*)q->ptr, (const uint16_t*)k->ptr, (const uint16_t*)v->ptr, (float*)state->ptr, (const float*)decay_powers->ptr,
                 (float*)workspace->ptr, (float*)output->ptr, rows, heads, dim, vdim, (rows + kChunk - 1) / kChunk};
-    LH_REQUIRE((uint64_t)a.chunks * heads * ((vdim + 63) / 64) < 0x7FFFFFFFull, "%s: %u rows", op, rows);
+    LH_REQUIRE((uint64_t)a.chunks * heads * ((vdim + 63) / 64) * 8 < 0x7FFFFFFFull, "%s: %u rows", op, rows);
     int r;
     if (dq == 32) r = launch_chunked<32>(batch->ctx, a, op);
     else if (dq == 64) r = launch_chunked<64>(batch->ctx, a, op);

@@ -511,10 +511,10 @@ int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const 
         const int r = lh_check_launch(op);
         return r != LH_OK || a.splits == 1 ? r : merge();
     }
-    // two blocks per wave at least, no more workgroups than one per CU
+    // one block per wave at least, no more workgroups than one per CU
     const uint64_t groups = tiles16 * a.kv_heads;
     LH_REQUIRE(room >= 1, "%s: %u heads of %u values exceed the workspace", op, a.heads, a.vdim);
-    a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({max_blocks / 8, (cus + groups - 1) / groups, room}));
+    a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({max_blocks / 4, (cus + groups - 1) / groups, room}));
     constexpr size_t lds = (size_t)4 * MAPS * 16 * (DV + 4) * 4;
     if (lds > 64 * 1024) {
         const int r = lh_raise_dynamic_lds(ctx, (const void*)attention_split_kernel<DQ, DV, MAPS>, lds, op);
