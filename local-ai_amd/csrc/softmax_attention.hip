@@ -10,7 +10,7 @@
 // 4g .. 4g + 3 of each tile, g = lane >> 4), so a row's maximum and sum are eight registers and two lane exchanges, and
 // the weights are already where O^T = V^T P^T wants them: its k index 8g + j is key 4g + j of tile 0 (j < 4) or key
 // 4g + j - 4 of tile 1, which is the order of the value blocks.  Scores, weights and sums are f32; a weight enters the
-// product as the sum of two bf16 terms.
+// product as the sum of three bf16 terms, which is all of its 24 bits.
 //   attention_tile_kernel   many rows: four waves share key and value blocks through LDS
 //   attention_split_kernel  few rows: every wave walks its own share of the blocks straight from global memory; the
 //                           workgroup's four partial results are merged in LDS, the workgroups' by attention_merge_kernel
@@ -63,11 +63,11 @@ __device__ __forceinline__ void load_queries(lh_bf16x8 (&qf)[MAPS][DQ / 32], con
 // A row tile's running softmax state for one map; every lane holds the values of packed row (lane & 15).
 struct RowState { float m, l; };
 
-// Scores of NB steps of 32 keys -> weights in P V operand order, as two bf16 terms; returns the factor for what was summed
+// Scores of NB steps of 32 keys -> weights in P V operand order, as three bf16 terms; returns the factor for what was summed
 // before.  `first` is the first key, `limit` the row's last visible key, `bound` whether any lane may have to mask.
 template <int NB>
 __device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2 * NB], RowState& st, float scale2, uint32_t first, uint32_t limit, bool bound, uint32_t lane,
-                                              lh_bf16x8 (&hi)[NB], lh_bf16x8 (&lo)[NB]) {
+                                              lh_bf16x8 (&w)[NB][3]) {
     float v[8 * NB], mx = -INFINITY;
     const uint32_t g = lane >> 4;
 #pragma unroll
@@ -81,16 +81,19 @@ __device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2 * NB], RowState& s
     float sum = 0.0f;
 #pragma unroll
     for (int b = 0; b < NB; b++) {
-        uint32_t h[4], l[4];
+        uint32_t h[4], m[4], l[4];
 #pragma unroll
         for (int i = 0; i < 4; i++) {
-            const float p0 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i + 1] - base);
+            float p0 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i + 1] - base);
             sum += p0 + p1;
             h[i] = lh_pack_bf(p0, p1);
-            l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, h[i] << 16), p1 - __builtin_bit_cast(float, h[i] & 0xFFFF0000u));
+            p0 -= __builtin_bit_cast(float, h[i] << 16); p1 -= __builtin_bit_cast(float, h[i] & 0xFFFF0000u);
+            m[i] = lh_pack_bf(p0, p1);
+            l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, m[i] << 16), p1 - __builtin_bit_cast(float, m[i] & 0xFFFF0000u));
         }
-        hi[b] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
-        lo[b] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
+        w[b][0] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
+        w[b][1] = __builtin_bit_cast(lh_bf16x8, (u32x4){m[0], m[1], m[2], m[3]});
+        w[b][2] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
     }
     st.l = st.l * alpha + sum;      // this lane's keys only; the four lanes of a row are added at the end
     st.m = nm;
@@ -140,7 +143,7 @@ typedef __attribute__((address_space(3))) void lvoid;
 // of 16 bytes, chunk c at place c ^ (key & 7) (see linear_mfma_kernel for why and how).  With more than one split a
 // workgroup takes its share of the key steps and leaves partial records.
 template <int DQ, int DV, int MAPS, int NB>
-__global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs a) {
+__global__ __launch_bounds__(256, MAPS * DV <= 256 ? 2 : 1) void attention_tile_kernel(const AttentionArgs a) {
     constexpr int KC = MAPS * DQ / 8, KCH = 32 * NB * KC, VB = DV * 4, VCH = NB * VB;    // chunks per key row; per step: keys, values
     constexpr uint32_t kSwizzle = KC >= 8 ? 7 : KC - 1;
     __shared__ uint4 sm[2][KCH + VCH];
@@ -195,9 +198,9 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs
         const uint4* ks = sm[s & 1];
         const uint4* vs = ks + KCH;
         const bool bound = first + 32 * NB - 1 > first_limit;
-        lh_bf16x8 hi[MAPS][NB], lo[MAPS][NB];
 #pragma unroll
-        for (int mp = 0; mp < MAPS; mp++) {
+        for (int mp = 0; mp < MAPS; mp++) {                                               // (a map at a time: the registers of two halve the waves)
+            lh_bf16x8 w[NB][3];
             lh_f32x4 sc[2 * NB];
 #pragma unroll
             for (int t = 0; t < 2 * NB; t++) {
@@ -209,25 +212,22 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs
                     sc[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, ks[key * KC + (ch ^ (key & kSwizzle))]), qf[mp][c], sc[t], 0, 0, 0);
                 }
             }
-            const float alpha = softmax_step<NB>(sc, st[mp], scale2, first, limit, bound, lane, hi[mp], lo[mp]);
+            const float alpha = softmax_step<NB>(sc, st[mp], scale2, first, limit, bound, lane, w);
             if (__ballot(alpha != 1.0f)) {
 #pragma unroll
                 for (int d = 0; d < DV / 16; d++)
 #pragma unroll
                     for (int r = 0; r < 4; r++) o[mp][d][r] *= alpha;
             }
-        }
 #pragma unroll
-        for (int b = 0; b < NB; b++)
+            for (int b = 0; b < NB; b++)
 #pragma unroll
-            for (int d = 0; d < DV / 16; d++) {
-                const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, vs[b * VB + (d * 16 + (lane & 15)) * 4 + (lane >> 4)]);
+                for (int d = 0; d < DV / 16; d++) {
+                    const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, vs[b * VB + (d * 16 + (lane & 15)) * 4 + (lane >> 4)]);
 #pragma unroll
-                for (int mp = 0; mp < MAPS; mp++) {
-                    o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, hi[mp][b], o[mp][d], 0, 0, 0);
-                    o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, lo[mp][b], o[mp][d], 0, 0, 0);
+                    for (int z = 2; z >= 0; z--) o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, w[b][z], o[mp][d], 0, 0, 0);
                 }
-            }
+        }
     }
     float l[MAPS];
 #pragma unroll
@@ -245,7 +245,7 @@ __global__ __launch_bounds__(256) void attention_tile_kernel(const AttentionArgs
 }
 
 // grid: row tiles x kv heads x splits.  The blocks of the visible range are dealt out in contiguous runs to the 4 * splits
-// waves of a (tile, kv head); a wave loads a block's operands one block ahead.
+// waves of a (tile, kv head); where two blocks' operands fit the registers a wave loads one block ahead.
 template <int DQ, int DV, int MAPS>
 __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArgs a) {
     extern __shared__ __align__(16) float merge[];                          // [4 waves][MAPS][16 rows][DV + 4]: values, maximum, sum
@@ -287,7 +287,7 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
     const float scale2 = a.scale * kLog2e;
     auto consume = [&](const Block& f, uint32_t b) {
         const bool bound = b * 32 + 31 > first_limit;
-        lh_bf16x8 hi[MAPS][1], lo[MAPS][1];
+        lh_bf16x8 w[MAPS][1][3];
 #pragma unroll
         for (int mp = 0; mp < MAPS; mp++) {
             lh_f32x4 s[2];
@@ -297,7 +297,7 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
 #pragma unroll
                 for (int c = 0; c < DQ / 32; c++) s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.k[t][mp][c]), qf[mp][c], s[t], 0, 0, 0);
             }
-            const float alpha = softmax_step<1>(s, st[mp], scale2, b * 32, limit, bound, lane, hi[mp], lo[mp]);
+            const float alpha = softmax_step<1>(s, st[mp], scale2, b * 32, limit, bound, lane, w[mp]);
             if (__ballot(alpha != 1.0f)) {
 #pragma unroll
                 for (int d = 0; d < DV / 16; d++)
@@ -309,11 +309,18 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
         for (int d = 0; d < DV / 16; d++)
 #pragma unroll
             for (int mp = 0; mp < MAPS; mp++) {
-                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), hi[mp][0], o[mp][d], 0, 0, 0);
-                o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), lo[mp][0], o[mp][d], 0, 0, 0);
+#pragma unroll
+                for (int z = 2; z >= 0; z--)
+                    o[mp][d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(__builtin_bit_cast(lh_bf16x8, f.v[d]), w[mp][0][z], o[mp][d], 0, 0, 0);
             }
     };
-    if (b0 < b1) {
+    if constexpr (sizeof(Block) > 256) {                      // two blocks would not fit the registers
+        for (uint32_t b = b0; b < b1; b++) {
+            Block x;
+            issue(x, b);
+            consume(x, b);
+        }
+    } else if (b0 < b1) {
         Block x, y;
         issue(x, b0);
         for (uint32_t b = b0; b < b1; b += 2) {

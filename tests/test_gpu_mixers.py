@@ -55,7 +55,8 @@ def values_from_cache(flat, cols):
 # ---- products ----------------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", ["bf16", "f32"])
 @pytest.mark.parametrize("m,k,n", [(1, 64, 48), (2, 256, 200), (31, 72, 33), (33, 40, 70), (64, 520, 130), (65, 64, 64), (129, 200, 257),
-                                   (300, 136, 2052), (7, 60, 45), (140, 7, 9), (2100, 128, 2048)])
+                                   (300, 136, 2052), (7, 60, 45), (140, 7, 9), (2100, 128, 2048),
+                                   (1, 4104, 300), (1, 5000, 17), (1, 8192, 70), (1, 16384, 9), (1, 20008, 5), (1, 16, 270000), (600, 2048, 1100)])
 def test_linear_rows(ai, gpu, dtype, m, k, n):
     ctx, K = gpu
     dt = ai.BF16 if dtype == "bf16" else ai.F32
@@ -231,7 +232,7 @@ def test_attention_shapes(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, star
     attention_case(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, start, rows, 256)
 
 
-@pytest.mark.parametrize("dim,vdim", [(32, 32), (32, 128), (32, 256), (64, 32), (64, 64), (64, 256), (128, 32), (128, 64), (128, 128), (136, 64), (48, 300)])
+@pytest.mark.parametrize("dim,vdim", [(32, 32), (32, 128), (32, 256), (64, 32), (64, 64), (64, 256), (128, 32), (128, 64), (128, 128), (128, 256), (136, 64), (48, 300)])
 @pytest.mark.parametrize("rows", [1, 150])
 @pytest.mark.parametrize("maps", [1, 2])
 def test_attention_every_head_size(ai, gpu, maps, dim, vdim, rows):
@@ -308,7 +309,8 @@ def test_linear_attention_forms(ai, gpu, heads, dim, vdim, cuts):
 # ---- mixture of experts ------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", ["bf16", "f32"])
 @pytest.mark.parametrize("rows,experts,top,width,ff", [(2, 5, 2, 64, 48), (7, 3, 3, 40, 33), (65, 12, 1, 64, 96), (300, 4, 2, 64, 72), (600, 2, 1, 32, 40),
-                                                       (33, 70, 8, 32, 16), (130, 130, 3, 24, 24), (5, 1, 1, 60, 20), (90, 6, 2, 136, 257)])
+                                                       (33, 70, 8, 32, 16), (130, 130, 3, 24, 24), (5, 1, 1, 60, 20), (90, 6, 2, 136, 257),
+                                                       (3, 300, 4, 24, 16), (2, 4, 3, 4104, 40), (2, 6, 3, 64, 1500)])
 def test_mixture_of_experts(ai, gpu, dtype, rows, experts, top, width, ff):
     ctx, K = gpu
     dt = ai.BF16 if dtype == "bf16" else ai.F32
