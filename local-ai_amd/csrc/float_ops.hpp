@@ -104,15 +104,16 @@ __device__ __forceinline__ void lh_lds_barrier() { asm volatile("s_waitcnt lgkmc
 
 // Maximum and sum over the four lanes that differ in their 16s and 32s (the column of a 16 x 16 matrix-product tile).
 // v_permlane16_swap / v_permlane32_swap on two copies leave the even and the odd rows (the lower and the upper half) of a
-// value in all rows (both halves).  (The compiler's builtin hands back its first result twice; the wait states before the
-// swap are what the compiler itself puts there.)
+// value in all rows (both halves).
 __device__ __forceinline__ void lh_pair16(float v, float& a, float& b) {
-    a = v; b = v;
-    asm("s_nop 1\n\tv_permlane16_swap_b32 %0, %1" : "+v"(a), "+v"(b));
+    const auto r = __builtin_amdgcn_permlane16_swap(__builtin_bit_cast(uint32_t, v), __builtin_bit_cast(uint32_t, v), false, false);
+    const uint32_t x = r[0], y = r[1];      // (__builtin_bit_cast of a vector's element reads element 0, whichever is named)
+    a = __builtin_bit_cast(float, x); b = __builtin_bit_cast(float, y);
 }
 __device__ __forceinline__ void lh_pair32(float v, float& a, float& b) {
-    a = v; b = v;
-    asm("s_nop 1\n\tv_permlane32_swap_b32 %0, %1" : "+v"(a), "+v"(b));
+    const auto r = __builtin_amdgcn_permlane32_swap(__builtin_bit_cast(uint32_t, v), __builtin_bit_cast(uint32_t, v), false, false);
+    const uint32_t x = r[0], y = r[1];      // (__builtin_bit_cast of a vector's element reads element 0, whichever is named)
+    a = __builtin_bit_cast(float, x); b = __builtin_bit_cast(float, y);
 }
 __device__ __forceinline__ float lh_column_max(float v) {
     float a, b;
