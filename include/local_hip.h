@@ -678,7 +678,8 @@ LH_API int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, 
  * values [position / 32, kv_heads, vdim_padded, 32], all of `dtype`; output [rows, heads, vdim].  dim is padded to 32,
  * 64, 128 or a multiple of 128, vdim to a multiple of 32 (lh_attention_padded_dim / _vdim).
  *   maps 1: output = the softmax average.
- *   maps 2 (differential attention): o = a1 - lambda * a2, then o / sqrt(mean(o^2) + eps) * out_scale over the head.
+ *   maps 2 (differential attention): the second average, times lambda, is taken from the first; the head's difference
+ *           is RMS-normed without a weight and scaled by out_scale.
  * `capacity` positions are held by the caches; `max_position` bounds *position (it sizes the launch; a recorded batch
  * gives the largest it will be replayed with). */
 LH_API uint32_t lh_attention_padded_dim(uint32_t dim);
@@ -688,8 +689,8 @@ LH_API int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_
                                   uint32_t rows, uint32_t heads, uint32_t kv_heads, uint32_t maps, uint32_t dim,
                                   uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps);
 
-/* Linear attention with a fixed decay per head: S = decay * S + k v^T, o = S^T q, token by token from the state left by
- * the call before.  q, k [rows, heads, dim_padded], v [rows, heads, vdim] of `dtype`; state f32 [heads, vdim, dim_padded]
+/* Linear attention with a fixed decay per head: per token the head's state M shrinks by its decay, takes in the outer
+ * product of key and value, and is read with the query (M <- a M + k (x) v, y = q M), from the state the call before left.  q, k [rows, heads, dim_padded], v [rows, heads, vdim] of `dtype`; state f32 [heads, vdim, dim_padded]
  * (read and written); output f32 [rows, heads, vdim].  dim_padded is lh_linear_attention_padded_dim(dim).
  *   recurrent  one launch that walks the rows; any dtype
  *   chunked    blocks of 64 rows on the matrix cores: every chunk's contribution to the state, a scan over the chunks,
@@ -704,8 +705,8 @@ LH_API int lh_linear_attention_chunked_into(lh_batch* batch, const lh_buffer* q,
                                             lh_buffer* state, const lh_buffer* decay_powers, lh_buffer* workspace,
                                             lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
 
-/* Mixture of experts: scores = sigmoid(router logits), each row takes the `top` largest (ties: the lower index), weighted
- * by their scores as they are; the weight multiplies the expert's input.  Experts are stacked, up [experts, ff, width]
+/* Mixture of experts: scores = sigmoid(router logits), each row takes the `top` largest (ties: the lower index), scaled
+ * by the score itself on the way into the expert.  Experts are stacked, up [experts, ff, width]
  * and down [experts, width, ff], without biases.
  *   route   logits f32 [rows, experts] -> the rows grouped by expert: plan u32 [lh_moe_plan_words]
  *   up      hidden[slot] = act(w * (up[e] . input[row])), one slot per (row, choice), in plan order

@@ -1,5 +1,5 @@
-// Mixture of experts with sigmoid scores: every row takes the `top` experts with the largest scores, each weighted by its
-// score as it is, and the weight multiplies the expert's input.  The first product of an expert is linear, so the weight
+// Mixture of experts with sigmoid scores: every row goes to its `top` best experts, and what enters an expert is scaled by
+// the score itself.  The first product of an expert is linear, so the weight
 // is applied to that product's result, before the activation.
 //
 // Many rows: route_kernel picks the experts of every row (one wave per row), place_kernel groups the (row, choice) slots by

@@ -25,7 +25,7 @@ __device__ __forceinline__ LhSplit3 lh_split3(float x) {
 }
 
 __device__ __forceinline__ float lh_sigmoid(float z) { return 1.0f / (1.0f + expf(-z)); }
-// 0.5 z (1 + tanh(u)) = z / (1 + exp(-2u)) with u = sqrt(2/pi) (z + 0.044715 z^3)
+// the tanh form of gelu as z times a sigmoid of twice the tanh's argument
 __device__ __forceinline__ float lh_gelu_tanh(float z) {
     const float u = 0.7978845608028654f * (z + 0.044715f * z * z * z);
     return z / (1.0f + expf(-2.0f * u));

@@ -1,13 +1,13 @@
-// Linear attention with a fixed decay per head: S_t = decay S_(t-1) + k_t v_t^T, o_t = S_t^T q_t.  The state is f32,
+// Linear attention with a fixed decay a per head: for every token M <- a M + k (x) v and y = q M.  The state M is f32,
 // kept as [head][value column][DQ key columns] (the key columns that exist, then zeros).
 //
 // Recurrent form: one workgroup per head and 16 value columns; a row of 16 lanes holds one value column's state in
 // registers (DQ / 16 values each) and walks the rows.
 //
 // Chunked form (64 rows a chunk, bf16 inputs on the matrix cores, everything else f32):
-//   1. every chunk's own contribution to the state, U = sum_s decay^(L-1-s) k_s v_s^T (all chunks at once)
-//   2. a scan over the chunks, S <- decay^L S + U, that leaves each chunk's incoming state in place of its U
-//   3. all outputs: o_t = decay^(t+1) S_in^T q_t + sum_(s<=t) decay^(t-s) (q_t . k_s) v_s
+//   1. every chunk's own contribution to the state, U = sum over rows s of a^(L-1-s) k_s (x) v_s (all chunks at once)
+//   2. a scan over the chunks, M <- a^L M + U, that leaves each chunk's incoming state in place of its U
+//   3. all outputs: y_t = a^(t+1) q_t M_in + sum over s <= t of a^(t-s) (q_t . k_s) v_s
 // Where an f32 quantity enters a product (decayed keys, decayed scores, the state) it does so as the sum of three bf16
 // terms, which is all of its 24 bits; the products of bf16 values are exact and summed in f32.
 #include "float_ops.hpp"

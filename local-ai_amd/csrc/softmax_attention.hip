@@ -1,6 +1,6 @@
 // Causal softmax attention over bf16 (or f32) caches, with one or two score maps per head.  With two maps (differential
-// attention) both share the head's values and are combined in the same kernel: o = a1 - lambda a2, an RMS norm over the
-// head, a constant factor.
+// attention) both share the head's values and are combined in the same kernel: the difference of the two averages, the
+// second times lambda, an RMS norm over the head, a constant factor.
 //
 // Caches: keys [position][kv head][map][DQ], values in blocks of 32 positions [block][kv head][DV][32] whose 32 entries
 // are in lh_block_slot order.  The queries of one kv head's group are packed: packed row r = query row r / R, head r % R of

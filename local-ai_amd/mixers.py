@@ -230,7 +230,7 @@ class MoeSpec:
 
 
 class MoeFeedForward:
-    """Sigmoid scores, the ``top`` best experts, weighted by their scores on the experts' input."""
+    """Sigmoid gates: a token goes to its ``top`` best experts, scaled by the gate on the way in."""
 
     def __init__(self, ctx, kernels: Kernels, spec: MoeSpec, width: int, tensors, prefix: str):
         s = self.spec = spec
@@ -273,7 +273,7 @@ class LayerSpec:
 
 
 class PreNormLayer:
-    """x <- x + mixer(norm1(x)), then x <- x + ff(norm2(x)) where there is a feed-forward."""
+    """Two residual branches, each on a norm of the stream: the mixer, and the feed-forward where the layer has one."""
 
     def __init__(self, ctx, kernels: Kernels, spec: LayerSpec, width: int, eps: float, tensors, prefix: str):
         self.norm1 = Norm(ctx, tensors.f32(prefix + "norm1", (width,)), eps)

@@ -17,7 +17,7 @@ DEFAULT_MAX_ROWS = 2048     # rows of one pass; longer portions go through in pi
 
 @dataclass
 class Loop:
-    """Layers start .. stop - 1 run `times` times in a row; before each pass but the first the embedding output is added."""
+    """The range [start, stop) of layers is walked `times` times; every repetition begins by adding the embedded tokens again."""
     start: int
     stop: int
     times: int

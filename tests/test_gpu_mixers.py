@@ -217,7 +217,7 @@ def attention_case(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, start, rows
         j = h // (heads // kv_heads)
         a = [O.causal_softmax_attention(q[:, h, m], k[:, j, m], v[:, j], scale, start) for m in range(maps)]
         want[:, h] = a[0] if maps == 1 else O.unit_rms(a[0] - lam * a[1], eps) * out_scale
-    # over a thousand random keys a1 - lambda a2 is small and its norm enlarges the rounding of both sums about thirtyfold
+    # over a thousand random keys the difference of the two averages is small and its norm enlarges the rounding of both sums about thirtyfold
     close(got, want, BF16_TOL if dt == ai.BF16 else F32_TOL if maps == 1 else 1e-4, "attention")
     if spike is not None and maps == 1:
         close(got[spike[0]].reshape(kv_heads, -1, vdim), v[spike[1]][:, None].repeat(heads // kv_heads, 1), 0.03, "the far key's value")
@@ -226,7 +226,7 @@ def attention_case(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, start, rows
 
 @pytest.mark.parametrize("dtype", ["bf16", "f32"])
 @pytest.mark.parametrize("maps", [1, 2])
-@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(4, 4, 32, 64), (6, 2, 24, 40), (8, 1, 64, 128), (3, 3, 8, 16), (4, 2, 128, 256), (5, 1, 20, 33), (34, 2, 16, 24)])
+@pytest.mark.parametrize("heads,kv_heads,dim,vdim", [(3, 3, 32, 64), (6, 2, 24, 40), (8, 1, 64, 128), (3, 3, 8, 16), (4, 2, 128, 256), (5, 1, 20, 33), (34, 2, 16, 24)])
 @pytest.mark.parametrize("start,rows", [(0, 1), (31, 1), (32, 2), (95, 34), (0, 97), (63, 190)])
 def test_attention_shapes(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, start, rows):
     attention_case(ai, gpu, dtype, maps, heads, kv_heads, dim, vdim, start, rows, 256)
@@ -270,7 +270,7 @@ def test_attention_rejects(ai, gpu):
 
 
 # ---- linear attention --------------------------------------------------------------------------------------------------
-@pytest.mark.parametrize("heads,dim,vdim", [(4, 32, 32), (3, 20, 33), (2, 64, 128), (1, 128, 80), (2, 200, 48), (2, 8, 100)])
+@pytest.mark.parametrize("heads,dim,vdim", [(4, 32, 48), (3, 20, 33), (2, 64, 128), (1, 128, 80), (2, 200, 48), (2, 8, 100)])
 @pytest.mark.parametrize("cuts", [[1, 1, 1], [16, 2], [64], [17, 65, 130], [63, 1, 64], [300]])
 def test_linear_attention_forms(ai, gpu, heads, dim, vdim, cuts):
     """Recurrent in both types and chunked, in portions: the outputs, and the state after every portion."""
@@ -308,7 +308,7 @@ def test_linear_attention_forms(ai, gpu, heads, dim, vdim, cuts):
 
 # ---- mixture of experts ------------------------------------------------------------------------------------------------
 @pytest.mark.parametrize("dtype", ["bf16", "f32"])
-@pytest.mark.parametrize("rows,experts,top,width,ff", [(2, 5, 2, 64, 48), (7, 3, 3, 40, 33), (65, 12, 1, 64, 96), (300, 4, 2, 64, 72), (600, 2, 1, 32, 40),
+@pytest.mark.parametrize("rows,experts,top,width,ff", [(2, 5, 2, 64, 48), (7, 3, 3, 40, 33), (65, 11, 1, 64, 88), (300, 4, 2, 64, 72), (600, 2, 1, 32, 40),
                                                        (33, 70, 8, 32, 16), (130, 130, 3, 24, 24), (5, 1, 1, 60, 20), (90, 6, 2, 136, 257),
                                                        (3, 300, 4, 24, 16), (2, 4, 3, 4104, 40), (2, 6, 3, 64, 1500)])
 def test_mixture_of_experts(ai, gpu, dtype, rows, experts, top, width, ff):
