@@ -629,9 +629,11 @@ LH_API uint32_t lh_flash_split_count(uint32_t eff_seq_len);
 #define LH_ACT_GELU_TANH 2
 #define LH_ACT_RELU_SQUARED 3
 #define LH_ACT_SIGMOID 4
+#define LH_ACT_SILU_PAIRS 5   /* products of many rows: columns come as (gate, up) pairs and leave as silu(gate) * up */
 #define LH_ROWS 0
 #define LH_ROWS_AT_POSITION 1
 #define LH_BLOCKS_AT_POSITION 2
+#define LH_ROWS_F32 3         /* LH_ROWS into an f32 buffer, whatever the product's output dtype */
 /* output[r] = table[rows[r]] as f32 (row index clamped to the last row) */
 LH_API int lh_embed_rows_bf16_into(lh_batch* batch, const lh_buffer* table, uint32_t table_rows, uint32_t cols,
                                    const lh_buffer* rows, uint32_t n_rows, lh_buffer* output);
@@ -640,9 +642,19 @@ LH_API int lh_embed_rows_bf16_into(lh_batch* batch, const lh_buffer* table, uint
 LH_API int lh_norm_rows_f32_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* add, const lh_buffer* weight,
                                  lh_buffer* store, const lh_buffer* row_index, lh_buffer* output, int output_dtype,
                                  uint32_t dim, uint32_t rows, float eps);
-/* output = input / sqrt(mean(input^2) + eps) * weight * sigmoid(gate); input f32, gate and output of `dtype` */
-LH_API int lh_gated_norm_rows_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, const lh_buffer* weight,
-                                   lh_buffer* output, int dtype, uint32_t dim, uint32_t rows, float eps);
+/* store = input + rms_norm(branch) * weight (`store` may be `input`), and a copy in `output`, for the product that reads the
+ * stream itself; `store` and `output` may be null.  Without a branch only the copy is made. */
+LH_API int lh_residual_rows_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* branch, const lh_buffer* weight,
+                                 lh_buffer* store, lh_buffer* output, int output_dtype, uint32_t dim, uint32_t rows,
+                                 float eps);
+/* RMS norm in equal parts of `group` columns, each by its own mean square, with a gate (LH_ACT_SIGMOID or LH_ACT_SILU):
+ * output = norm(input) * weight * act(gate), or norm(input * act(gate)) * weight with gate_first.  weight may be null;
+ * input f32, gate and output of `dtype` */
+LH_API int lh_gated_norm_rows_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, uint32_t gate_act,
+                                   int gate_first, const lh_buffer* weight, lh_buffer* output, int dtype, uint32_t dim,
+                                   uint32_t group, uint32_t rows, float eps);
+/* logits = cap * tanh(logits / cap), in place, n values */
+LH_API int lh_softcap_f32_into(lh_batch* batch, lh_buffer* logits, size_t n, float cap);
 /* output[m] = act(input[m, k] . weight^T + bias) by segments; bias f32 [sum ns] or null.  `accumulate` adds to an f32
  * output instead of storing. */
 LH_API int lh_linear_rows_into(lh_batch* batch, const lh_buffer* input, int input_dtype, const lh_buffer* weight,
@@ -654,7 +666,10 @@ LH_API int lh_linear_rows_into(lh_batch* batch, const lh_buffer* input, int inpu
  *   plain   x = input (of input_dtype)
  *   norm    x = rms_norm(input + add) * norm_weight, input f32, `add` may be null; input + add goes to `store` when given
  *           (which must not be `input`: every workgroup reads it)
- *   gated   x = rms_norm(input) * norm_weight * sigmoid(gate), input f32, gate of gate_dtype */
+ *   residual  x = input + rms_norm(branch) * norm_weight, all f32; x goes to `store` when given (not `input` or `branch`)
+ *   pairs   x = silu(input[2i]) * input[2i + 1], input f32 [2 k]
+ *   gated   x = the output of lh_gated_norm_rows_into, input f32, gate of gate_dtype; lh_gated_vector_fits(k, group) says
+ *           whether the parts suit this form */
 LH_API int lh_linear_vector_into(lh_batch* batch, const lh_buffer* input, int input_dtype, const lh_buffer* weight,
                                  const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
                                  const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
@@ -666,8 +681,21 @@ LH_API int lh_linear_norm_vector_into(lh_batch* batch, const lh_buffer* input, c
                                       const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
                                       const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
                                       int accumulate, const lh_buffer* position);
+LH_API int lh_linear_residual_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* branch,
+                                          lh_buffer* store, const lh_buffer* norm_weight, float eps,
+                                          const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count,
+                                          const uint32_t* ns, const uint32_t* acts, const uint32_t* heads,
+                                          const uint32_t* padded, const uint32_t* layouts, lh_buffer* const* outputs,
+                                          int output_dtype, int accumulate, const lh_buffer* position);
+LH_API int lh_linear_pairs_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* weight,
+                                       const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
+                                       const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
+                                       const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
+                                       int accumulate, const lh_buffer* position);
+LH_API uint32_t lh_gated_vector_fits(uint32_t k, uint32_t group);
 LH_API int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, int gate_dtype,
-                                       const lh_buffer* norm_weight, float eps, const lh_buffer* weight,
+                                       uint32_t gate_act, int gate_first, const lh_buffer* norm_weight,
+                                       uint32_t group, float eps, const lh_buffer* weight,
                                        const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
                                        const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
                                        const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
@@ -676,10 +704,12 @@ LH_API int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, 
 /* Causal softmax attention of `rows` queries at positions *position + r over the caches above, `maps` (1 or 2) score maps
  * per head over the same values.  q [rows, heads, maps, dim_padded], keys [position, kv_heads, maps, dim_padded] and
  * values [position / 32, kv_heads, vdim_padded, 32], all of `dtype`; output [rows, heads, vdim].  dim is padded to 32,
- * 64, 128 or a multiple of 128, vdim to a multiple of 32 (lh_attention_padded_dim / _vdim).
+ * 64, 128, 192 or a multiple of 128, vdim to a multiple of 32 (lh_attention_padded_dim / _vdim).
  *   maps 1: output = the softmax average.
  *   maps 2 (differential attention): the second average, times lambda, is taken from the first; the head's difference
  *           is RMS-normed without a weight and scaled by out_scale.
+ * sink f32 [heads] (may be null; maps 1): exp(sink) is one more term of every denominator, without key or value.  gate f32
+ * [rows, heads] (may be null; maps 1): a head's output is multiplied by sigmoid(gate).
  * `capacity` positions are held by the caches; `max_position` bounds *position (it sizes the launch; a recorded batch
  * gives the largest it will be replayed with). */
 LH_API uint32_t lh_attention_padded_dim(uint32_t dim);
@@ -687,11 +717,42 @@ LH_API uint32_t lh_attention_padded_vdim(uint32_t vdim);
 LH_API int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* keys, const lh_buffer* values,
                                   lh_buffer* output, int dtype, const lh_buffer* position, uint32_t max_position,
                                   uint32_t rows, uint32_t heads, uint32_t kv_heads, uint32_t maps, uint32_t dim,
-                                  uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps);
+                                  uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps,
+                                  const lh_buffer* sink, const lh_buffer* gate);
+
+/* Latent attention: keys and values are projections of one latent per position, shared by all heads, and a rotated key part
+ * that all heads share.  Only these are cached, as rows of `dtype`: [latent, zeros to lh_latent_padded_rank, rotated part,
+ * zeros to the row's end]; a row has lh_latent_row(rank, rot) values.
+ *   prepare  down f32 [rows, rank + rot] (may be null: another layer has written the rows): the RMS-normed latent and the
+ *            rotated part go to the cache rows *position ...  q_rot f32 [rows, heads, rot]: rotated into columns
+ *            rot_column ... of each head of q [rows, heads, q_ld] (q_dtype); the other columns from clear_column on become
+ *            zero.  Entries 2i and 2i + 1 turn by position * frequencies[i].
+ *   heads    output[m, h, n] = sum over k of input[m, h, k] * weight[h, n, k]: one small product per head
+ *   expand   keys and values of the first `positions` cache rows, as lh_attention_rows_into reads them: weight [heads * dim
+ *            (keys), then heads * vdim (values)][rank]; keys get the rotated part behind their dim columns
+ *   rows     attention of queries that the key projection has been applied to, in the latent space: q f32 [rows, heads,
+ *            lh_latent_row], output [rows, heads, rank] of `dtype`, of which the value projection is then taken.  sink and
+ *            gate as above. */
+LH_API uint32_t lh_latent_padded_rank(uint32_t rank);
+LH_API uint32_t lh_latent_row(uint32_t rank, uint32_t rot);
+LH_API int lh_latent_prepare_into(lh_batch* batch, const lh_buffer* q_rot, const lh_buffer* down, const lh_buffer* norm_weight,
+                                  const lh_buffer* frequencies, const lh_buffer* position, lh_buffer* q, int q_dtype,
+                                  lh_buffer* cache, int dtype, uint32_t rows, uint32_t heads, uint32_t rank, uint32_t rot,
+                                  uint32_t q_ld, uint32_t rot_column, uint32_t clear_column, uint32_t capacity, float eps);
+LH_API int lh_head_linear_into(lh_batch* batch, const lh_buffer* input, int dtype, const lh_buffer* weight, lh_buffer* output,
+                               int output_dtype, uint32_t rows, uint32_t heads, uint32_t n, uint32_t k, uint32_t output_ld);
+LH_API int lh_latent_expand_into(lh_batch* batch, const lh_buffer* cache, int dtype, const lh_buffer* weight, lh_buffer* keys,
+                                 lh_buffer* values, uint32_t positions, uint32_t heads, uint32_t dim, uint32_t rot,
+                                 uint32_t vdim, uint32_t rank);
+LH_API int lh_latent_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* cache, lh_buffer* output,
+                                         int dtype, const lh_buffer* position, uint32_t max_position, uint32_t rows,
+                                         uint32_t heads, uint32_t rank, uint32_t rot, uint32_t capacity, float scale,
+                                         const lh_buffer* sink, const lh_buffer* gate);
 
 /* Linear attention with a fixed decay per head: per token the head's state M shrinks by its decay, takes in the outer
  * product of key and value, and is read with the query (M <- a M + k (x) v, y = q M), from the state the call before left.  q, k [rows, heads, dim_padded], v [rows, heads, vdim] of `dtype`; state f32 [heads, vdim, dim_padded]
  * (read and written); output f32 [rows, heads, vdim].  dim_padded is lh_linear_attention_padded_dim(dim).
+ * Outputs are multiplied by `scale`.
  *   recurrent  one launch that walks the rows; any dtype
  *   chunked    blocks of 64 rows on the matrix cores: every chunk's contribution to the state, a scan over the chunks,
  *              then all outputs.  bf16, dim <= 256.  `decay_powers` f32 [heads, 65] holds decay^0 .. decay^64;
@@ -700,10 +761,40 @@ LH_API uint32_t lh_linear_attention_padded_dim(uint32_t dim);
 LH_API size_t lh_linear_attention_workspace_bytes(uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
 LH_API int lh_linear_attention_recurrent_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v,
                                               int dtype, lh_buffer* state, const lh_buffer* decay, lh_buffer* output,
-                                              uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
+                                              uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim, float scale);
 LH_API int lh_linear_attention_chunked_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* k, const lh_buffer* v,
                                             lh_buffer* state, const lh_buffer* decay_powers, lh_buffer* workspace,
-                                            lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim);
+                                            lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t dim, uint32_t vdim,
+                                            float scale);
+
+/* Selective state space (the state-space form of linear attention, with a decay that depends on the token): per head
+ * dt = softplus(dt_raw + dt_bias), S <- exp(-exp(a_log) dt) S + dt * B (x) x, y = S C + skip * x; head h reads B and C of
+ * group h / (heads / groups).  State f32 [heads, vdim, state_padded], state_padded = lh_linear_attention_padded_dim(state).
+ * x, B and C come out of a causal convolution per channel with SiLU over `taps` rows of [x | B | C], whose last rows are kept
+ * in `ring` f32 [taps, channels], row (position mod taps); rows before position 0 count as zeros.  taps f32 [taps, channels]
+ * (the last for the current row), bias f32 [channels].
+ *   conv       input [rows, channels] -> x [rows, heads * vdim], B and C [rows, groups, state_padded], zeros in the padding
+ *   recurrent  one launch that walks the rows; any dtype; output f32 [rows, heads * vdim]
+ *   chunked    as lh_linear_attention_chunked_into; bf16, state <= 256; `steps` takes lh_selective_steps_bytes
+ *   step       all of it for one row: input f32 [channels], dt_raw f32 [heads] */
+LH_API size_t lh_selective_steps_bytes(uint32_t rows, uint32_t heads);
+LH_API int lh_selective_conv_into(lh_batch* batch, const lh_buffer* input, int dtype, lh_buffer* ring, const lh_buffer* taps_weight,
+                                  const lh_buffer* bias, const lh_buffer* position, lh_buffer* x, lh_buffer* b, lh_buffer* c,
+                                  uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t groups, uint32_t state, uint32_t taps);
+LH_API int lh_selective_recurrent_into(lh_batch* batch, const lh_buffer* x, const lh_buffer* b, const lh_buffer* c, int dtype,
+                                       const lh_buffer* dt_raw, const lh_buffer* dt_bias, const lh_buffer* a_log,
+                                       const lh_buffer* skip, lh_buffer* memory, lh_buffer* output, uint32_t rows,
+                                       uint32_t heads, uint32_t vdim, uint32_t groups, uint32_t state);
+LH_API int lh_selective_chunked_into(lh_batch* batch, const lh_buffer* x, const lh_buffer* b, const lh_buffer* c,
+                                     const lh_buffer* dt_raw, const lh_buffer* dt_bias, const lh_buffer* a_log,
+                                     const lh_buffer* skip, lh_buffer* memory, lh_buffer* steps, lh_buffer* workspace,
+                                     lh_buffer* output, uint32_t rows, uint32_t heads, uint32_t vdim, uint32_t groups,
+                                     uint32_t state);
+LH_API int lh_selective_step_into(lh_batch* batch, const lh_buffer* input, lh_buffer* ring, const lh_buffer* taps_weight,
+                                  const lh_buffer* bias, const lh_buffer* position, const lh_buffer* dt_raw,
+                                  const lh_buffer* dt_bias, const lh_buffer* a_log, const lh_buffer* skip, lh_buffer* memory,
+                                  lh_buffer* output, uint32_t heads, uint32_t vdim, uint32_t groups, uint32_t state,
+                                  uint32_t taps);
 
 /* Mixture of experts: scores = sigmoid(router logits), each row takes the `top` largest (ties: the lower index), scaled
  * by the score itself on the way into the expert.  Experts are stacked, up [experts, ff, width]

@@ -31,8 +31,8 @@ BATCHM_MAX_M = 4      # local-metal/src/kernels.rs:6160
 MULTIVEC_MAX_M = 16   # local-metal/src/kernels.rs:6362
 
 # activations and output layouts of the bf16-weight products (include/local_hip.h)
-ACT_NONE, ACT_SILU, ACT_GELU_TANH, ACT_RELU_SQUARED, ACT_SIGMOID = range(5)
-ROWS, ROWS_AT_POSITION, BLOCKS_AT_POSITION = range(3)
+ACT_NONE, ACT_SILU, ACT_GELU_TANH, ACT_RELU_SQUARED, ACT_SIGMOID, ACT_SILU_PAIRS = range(6)
+ROWS, ROWS_AT_POSITION, BLOCKS_AT_POSITION, ROWS_F32 = range(4)
 
 
 class Error(Exception):
@@ -98,10 +98,12 @@ def lib() -> C.CDLL:
         _lib.lh_context_stream.restype = C.c_void_p
         for name in ("lh_smallm_max_m", "lh_batchm_max_m", "lh_multivec_max_m", "lh_batch_dispatch_count",
                      "lh_flash_split_count", "lh_attention_padded_dim", "lh_attention_padded_vdim",
-                     "lh_linear_attention_padded_dim", "lh_moe_plan_words"):
+                     "lh_linear_attention_padded_dim", "lh_moe_plan_words", "lh_latent_padded_rank", "lh_latent_row",
+                     "lh_gated_vector_fits"):
             if hasattr(_lib, name):
                 getattr(_lib, name).restype = C.c_uint32
         _lib.lh_linear_attention_workspace_bytes.restype = C.c_size_t
+        _lib.lh_selective_steps_bytes.restype = C.c_size_t
     return _lib
 
 
@@ -776,9 +778,17 @@ class Kernels:
         _check(self._l.lh_norm_rows_f32_into(batch._h, input._h, _opt(add), weight._h, _opt(store), _opt(row_index), output._h,
                                              C.c_int(output_dtype), _u32(dim), _u32(rows), C.c_float(eps)))
 
-    def gated_norm_rows_into(self, batch, input, gate, weight, output, dtype, dim, rows, eps):
-        _check(self._l.lh_gated_norm_rows_into(batch._h, input._h, gate._h, weight._h, output._h, C.c_int(dtype), _u32(dim),
-                                               _u32(rows), C.c_float(eps)))
+    def residual_rows_into(self, batch, input, branch, weight, store, output, output_dtype, dim, rows, eps):
+        _check(self._l.lh_residual_rows_into(batch._h, input._h, _opt(branch), _opt(weight), _opt(store), _opt(output),
+                                             C.c_int(output_dtype), _u32(dim), _u32(rows), C.c_float(eps)))
+
+    def gated_norm_rows_into(self, batch, input, gate, weight, output, dtype, dim, rows, eps, group=None, gate_act=ACT_SIGMOID,
+                             gate_first=False):
+        _check(self._l.lh_gated_norm_rows_into(batch._h, input._h, gate._h, _u32(gate_act), C.c_int(bool(gate_first)), _opt(weight),
+                                               output._h, C.c_int(dtype), _u32(dim), _u32(group or dim), _u32(rows), C.c_float(eps)))
+
+    def softcap_f32_into(self, batch, logits, n, cap):
+        _check(self._l.lh_softcap_f32_into(batch._h, logits._h, C.c_size_t(n), C.c_float(cap)))
 
     def linear_rows_into(self, batch, input, input_dtype, weight, bias, m, k, segments, outputs, output_dtype,
                          accumulate=False, position=None):
@@ -798,9 +808,26 @@ class Kernels:
                                                   weight._h, _opt(bias), _u32(k), *segments.args, _handles(outputs),
                                                   C.c_int(output_dtype), C.c_int(bool(accumulate)), _opt(position)))
 
+    def linear_residual_vector_into(self, batch, input, branch, store, norm_weight, eps, weight, bias, k, segments, outputs,
+                                    output_dtype, accumulate=False, position=None):
+        _check(self._l.lh_linear_residual_vector_into(batch._h, input._h, branch._h, _opt(store), norm_weight._h, C.c_float(eps),
+                                                      weight._h, _opt(bias), _u32(k), *segments.args, _handles(outputs),
+                                                      C.c_int(output_dtype), C.c_int(bool(accumulate)), _opt(position)))
+
+    def linear_pairs_vector_into(self, batch, input, weight, bias, k, segments, outputs, output_dtype, accumulate=False,
+                                 position=None):
+        _check(self._l.lh_linear_pairs_vector_into(batch._h, input._h, weight._h, _opt(bias), _u32(k), *segments.args,
+                                                   _handles(outputs), C.c_int(output_dtype), C.c_int(bool(accumulate)),
+                                                   _opt(position)))
+
+    def gated_vector_fits(self, k, group):
+        return bool(self._l.lh_gated_vector_fits(_u32(k), _u32(group)))
+
     def linear_gated_vector_into(self, batch, input, gate, gate_dtype, norm_weight, eps, weight, bias, k, segments, outputs,
-                                 output_dtype, accumulate=False, position=None):
-        _check(self._l.lh_linear_gated_vector_into(batch._h, input._h, gate._h, C.c_int(gate_dtype), norm_weight._h,
+                                 output_dtype, accumulate=False, position=None, group=None, gate_act=ACT_SIGMOID,
+                                 gate_first=False):
+        _check(self._l.lh_linear_gated_vector_into(batch._h, input._h, gate._h, C.c_int(gate_dtype), _u32(gate_act),
+                                                   C.c_int(bool(gate_first)), _opt(norm_weight), _u32(group or k),
                                                    C.c_float(eps), weight._h, _opt(bias), _u32(k), *segments.args,
                                                    _handles(outputs), C.c_int(output_dtype), C.c_int(bool(accumulate)),
                                                    _opt(position)))
@@ -812,11 +839,11 @@ class Kernels:
         return int(self._l.lh_attention_padded_vdim(_u32(vdim)))
 
     def attention_rows_into(self, batch, q, keys, values, output, dtype, position, max_position, rows, heads, kv_heads, maps,
-                            dim, vdim, capacity, scale, lam=0.0, out_scale=1.0, eps=0.0):
+                            dim, vdim, capacity, scale, lam=0.0, out_scale=1.0, eps=0.0, sink=None, gate=None):
         _check(self._l.lh_attention_rows_into(batch._h, q._h, keys._h, values._h, output._h, C.c_int(dtype), position._h,
                                               _u32(max_position), _u32(rows), _u32(heads), _u32(kv_heads), _u32(maps),
                                               _u32(dim), _u32(vdim), _u32(capacity), C.c_float(scale), C.c_float(lam),
-                                              C.c_float(out_scale), C.c_float(eps)))
+                                              C.c_float(out_scale), C.c_float(eps), _opt(sink), _opt(gate)))
 
     def linear_attention_padded_dim(self, dim):
         return int(self._l.lh_linear_attention_padded_dim(_u32(dim)))
@@ -824,13 +851,70 @@ class Kernels:
     def linear_attention_workspace_bytes(self, rows, heads, dim, vdim):
         return int(self._l.lh_linear_attention_workspace_bytes(_u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
 
-    def linear_attention_recurrent_into(self, batch, q, k, v, dtype, state, decay, output, rows, heads, dim, vdim):
+    def linear_attention_recurrent_into(self, batch, q, k, v, dtype, state, decay, output, rows, heads, dim, vdim, scale=1.0):
         _check(self._l.lh_linear_attention_recurrent_into(batch._h, q._h, k._h, v._h, C.c_int(dtype), state._h, decay._h,
-                                                          output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
+                                                          output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim),
+                                                          C.c_float(scale)))
 
-    def linear_attention_chunked_into(self, batch, q, k, v, state, decay_powers, workspace, output, rows, heads, dim, vdim):
+    def linear_attention_chunked_into(self, batch, q, k, v, state, decay_powers, workspace, output, rows, heads, dim, vdim,
+                                      scale=1.0):
         _check(self._l.lh_linear_attention_chunked_into(batch._h, q._h, k._h, v._h, state._h, decay_powers._h, workspace._h,
-                                                        output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim)))
+                                                        output._h, _u32(rows), _u32(heads), _u32(dim), _u32(vdim),
+                                                        C.c_float(scale)))
+
+    def latent_padded_rank(self, rank):
+        return int(self._l.lh_latent_padded_rank(_u32(rank)))
+
+    def latent_row(self, rank, rot):
+        return int(self._l.lh_latent_row(_u32(rank), _u32(rot)))
+
+    def latent_prepare_into(self, batch, q_rot, down, norm_weight, frequencies, position, q, q_dtype, cache, dtype, rows, heads,
+                            rank, rot, q_ld, rot_column, clear_column, capacity, eps):
+        _check(self._l.lh_latent_prepare_into(batch._h, q_rot._h, _opt(down), _opt(norm_weight), frequencies._h, position._h, q._h,
+                                              C.c_int(q_dtype), cache._h, C.c_int(dtype), _u32(rows), _u32(heads), _u32(rank),
+                                              _u32(rot), _u32(q_ld), _u32(rot_column), _u32(clear_column), _u32(capacity),
+                                              C.c_float(eps)))
+
+    def head_linear_into(self, batch, input, dtype, weight, output, output_dtype, rows, heads, n, k, output_ld):
+        _check(self._l.lh_head_linear_into(batch._h, input._h, C.c_int(dtype), weight._h, output._h, C.c_int(output_dtype),
+                                           _u32(rows), _u32(heads), _u32(n), _u32(k), _u32(output_ld)))
+
+    def latent_expand_into(self, batch, cache, dtype, weight, keys, values, positions, heads, dim, rot, vdim, rank):
+        _check(self._l.lh_latent_expand_into(batch._h, cache._h, C.c_int(dtype), weight._h, keys._h, values._h, _u32(positions),
+                                             _u32(heads), _u32(dim), _u32(rot), _u32(vdim), _u32(rank)))
+
+    def latent_attention_rows_into(self, batch, q, cache, output, dtype, position, max_position, rows, heads, rank, rot, capacity,
+                                   scale, sink=None, gate=None):
+        _check(self._l.lh_latent_attention_rows_into(batch._h, q._h, cache._h, output._h, C.c_int(dtype), position._h,
+                                                     _u32(max_position), _u32(rows), _u32(heads), _u32(rank), _u32(rot),
+                                                     _u32(capacity), C.c_float(scale), _opt(sink), _opt(gate)))
+
+    def selective_steps_bytes(self, rows, heads):
+        return int(self._l.lh_selective_steps_bytes(_u32(rows), _u32(heads)))
+
+    def selective_conv_into(self, batch, input, dtype, ring, taps_weight, bias, position, x, b, c, rows, heads, vdim, groups, state,
+                            taps):
+        _check(self._l.lh_selective_conv_into(batch._h, input._h, C.c_int(dtype), ring._h, taps_weight._h, bias._h, position._h,
+                                              x._h, b._h, c._h, _u32(rows), _u32(heads), _u32(vdim), _u32(groups), _u32(state),
+                                              _u32(taps)))
+
+    def selective_recurrent_into(self, batch, x, b, c, dtype, dt_raw, dt_bias, a_log, skip, memory, output, rows, heads, vdim,
+                                 groups, state):
+        _check(self._l.lh_selective_recurrent_into(batch._h, x._h, b._h, c._h, C.c_int(dtype), dt_raw._h, dt_bias._h, a_log._h,
+                                                   skip._h, memory._h, output._h, _u32(rows), _u32(heads), _u32(vdim),
+                                                   _u32(groups), _u32(state)))
+
+    def selective_chunked_into(self, batch, x, b, c, dt_raw, dt_bias, a_log, skip, memory, steps, workspace, output, rows, heads,
+                               vdim, groups, state):
+        _check(self._l.lh_selective_chunked_into(batch._h, x._h, b._h, c._h, dt_raw._h, dt_bias._h, a_log._h, skip._h, memory._h,
+                                                 steps._h, workspace._h, output._h, _u32(rows), _u32(heads), _u32(vdim),
+                                                 _u32(groups), _u32(state)))
+
+    def selective_step_into(self, batch, input, ring, taps_weight, bias, position, dt_raw, dt_bias, a_log, skip, memory, output,
+                            heads, vdim, groups, state, taps):
+        _check(self._l.lh_selective_step_into(batch._h, input._h, ring._h, taps_weight._h, bias._h, position._h, dt_raw._h,
+                                              dt_bias._h, a_log._h, skip._h, memory._h, output._h, _u32(heads), _u32(vdim),
+                                              _u32(groups), _u32(state), _u32(taps)))
 
     def moe_plan_words(self, rows, experts, top):
         return int(self._l.lh_moe_plan_words(_u32(rows), _u32(experts), _u32(top)))

@@ -61,21 +61,33 @@ __device__ __forceinline__ void store4(const LhLinear& a, uint32_t slot, uint32_
     float v[4] = {acc.x, acc.y, acc.z, acc.w};
 #pragma unroll
     for (int r = 0; r < 4; r++) v[r] = v[r] * o.weight + (a.bias && n + r < a.N ? a.bias[n + r] : 0.0f);
-    if (!a.seg.vec4) {
+    const uint32_t s = lh_segment_of(a.seg, n);              // (of all four columns where the boundaries are aligned)
+    if (a.seg.pairs) {
+        if (a.seg.aligned4 && a.seg.act[s] == LH_ACT_SILU_PAIRS && !a.seg.f32[s]) {
+            *reinterpret_cast<uint32_t*>(static_cast<uint16_t*>(a.seg.out[s]) + (size_t)o.row * a.seg.ld[s] + (n - a.seg.n0[s]) / 2) =
+                lh_pack_bf(v[0] * lh_sigmoid(v[0]) * v[1], v[2] * lh_sigmoid(v[2]) * v[3]);
+            return;
+        }
+        lh_segment_store_pair(a.seg, o.row, n, v[0], v[1], pos0);   // every count of columns is even here
+        if (n + 2 < a.N) lh_segment_store_pair(a.seg, o.row, n + 2, v[2], v[3], pos0);
+        return;
+    }
+    if (!a.seg.aligned4 || !a.seg.vec4[s]) {
 #pragma unroll 1
         for (uint32_t r = 0; r < 4 && n + r < a.N; r++) lh_segment_store(a.seg, o.row, n + r, r == 0 ? v[0] : r == 1 ? v[1] : r == 2 ? v[2] : v[3], pos0);
         return;
     }
-    const uint32_t s = lh_segment_of(a.seg, n);              // the four columns are one aligned piece of one segment
-    const uint32_t p = a.seg.layout[s] == LH_ROWS ? o.row : pos0 + o.row;
+    const uint32_t p = lh_segment_at_position(a.seg, s) ? pos0 + o.row : o.row;
     if (p >= a.seg.rows[s]) return;
-    const size_t idx = (size_t)p * a.seg.ld[s] + (n - a.seg.n0[s]);
+    uint32_t c = n - a.seg.n0[s];
+    if (a.seg.head[s] != a.seg.padded[s]) { const uint32_t h = c / a.seg.head[s]; c = h * a.seg.padded[s] + (c - h * a.seg.head[s]); }
+    const size_t idx = (size_t)p * a.seg.ld[s] + c;
     const uint32_t act = a.seg.act[s];
     if (act != LH_ACT_NONE) {
 #pragma unroll
         for (int r = 0; r < 4; r++) v[r] = lh_activate(v[r], act);
     }
-    if (a.seg.f32_out) {
+    if (a.seg.f32[s]) {
         float4* d = reinterpret_cast<float4*>(static_cast<float*>(a.seg.out[s]) + idx);
         float4 t = make_float4(v[0], v[1], v[2], v[3]);
         if (a.seg.accumulate) { const float4 x = *d; t.x += x.x; t.y += x.y; t.z += x.z; t.w += x.w; }
@@ -114,7 +126,7 @@ __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
 #pragma unroll
     for (int i = 0; i < CA; i++) {
         const uint32_t r = min(rt.begin + i * 32 + (tid >> 3), rt.end - 1);
-        pa[i] = A + (size_t)a_row(a, r) * K + src * 8;
+        pa[i] = A + (size_t)a_row(a, r) * a.lda + src * 8;
     }
 #pragma unroll
     for (int i = 0; i < CB; i++) pb[i] = W + (size_t)min(n0 + i * 32 + (tid >> 3), a.N - 1) * K + src * 8;
@@ -211,7 +223,7 @@ __global__ __launch_bounds__(256) void linear_plain_kernel(const LhLinear a) {
             for (uint32_t e = tid; e < 64 * BK; e += 256) {
                 const uint32_t r = e >> 4, k = k0 + (e & 15);
                 const bool ka = k < K;
-                as[e & 15][r] = ka && begin + r < rt.end ? lh_ld(A, (size_t)a_row(a, begin + r) * K + k) : 0.0f;
+                as[e & 15][r] = ka && begin + r < rt.end ? lh_ld(A, (size_t)a_row(a, begin + r) * a.lda + k) : 0.0f;
                 bs[e & 15][r] = ka && n0 + r < a.N ? lh_bf2f(W[(size_t)(n0 + r) * K + k]) : 0.0f;
             }
             __syncthreads();
@@ -232,6 +244,14 @@ __global__ __launch_bounds__(256) void linear_plain_kernel(const LhLinear a) {
             const uint32_t slot = begin + ty * 4 + i;
             if (slot >= rt.end) continue;
             const OutRow o = out_row(a, slot);
+            if (a.seg.pairs) {                                // (an expert's weight and a bias do not occur with pairs of a plain product)
+#pragma unroll
+                for (int j = 0; j < 4; j += 2) {
+                    const uint32_t n = n0 + tx * 4 + j;
+                    if (n < a.N) lh_segment_store_pair(a.seg, o.row, n, acc[i][j] + (a.bias ? a.bias[n] : 0.0f), acc[i][j + 1] + (a.bias ? a.bias[n + 1] : 0.0f), pos0);
+                }
+                continue;
+            }
 #pragma unroll
             for (int j = 0; j < 4; j++) {
                 const uint32_t n = n0 + tx * 4 + j;
@@ -251,14 +271,31 @@ __device__ __forceinline__ uint32_t x_place(uint32_t k) {
 
 template <int STAGE>
 __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, uint32_t K) {
+    auto gate = [&](uint32_t k) { return lh_gate(st.gate_f32 ? static_cast<const float*>(st.gate)[k] : lh_bf2f(static_cast<const uint16_t*>(st.gate)[k]), st.gate_act); };
     auto value = [&](uint32_t k) {
+        if constexpr (STAGE == kPairs) { const float2 p = reinterpret_cast<const float2*>(st.x)[k]; return p.x * lh_sigmoid(p.x) * p.y; }
         if constexpr (STAGE == kPlain) return st.x_f32 ? static_cast<const float*>(st.x)[k] : lh_bf2f(static_cast<const uint16_t*>(st.x)[k]);
         float v = static_cast<const float*>(st.x)[k];
         if (STAGE == kNorm && st.add) v += st.add[k];
+        if constexpr (STAGE == kGated) if (st.gate_first) v *= gate(k);
         return v;
     };
+    auto weight = [&](uint32_t k) {
+        const float w = STAGE != kGated || st.norm_weight ? st.norm_weight[k] : 1.0f;
+        if constexpr (STAGE == kGated) return st.gate_first ? w : w * gate(k);
+        return w;
+    };
     const uint32_t padded = (K + 511) / 512 * 512;
-    if constexpr (STAGE == kPlain) {
+    if constexpr (STAGE == kResidual) {
+        float s = 0.0f;
+        for (uint32_t k = threadIdx.x; k < K; k += blockDim.x) { const float y = st.add[k]; s += y * y; }
+        const float r = rsqrtf(lh_block_sum(s, scratch) / (float)K + st.eps);
+        for (uint32_t k = threadIdx.x; k < padded; k += blockDim.x) {
+            const float v = k < K ? __builtin_fmaf(st.add[k] * st.norm_weight[k], r, value(k)) : 0.0f;
+            xs[x_place(k)] = v;
+            if (st.store && blockIdx.x == 0 && k < K) st.store[k] = v;
+        }
+    } else if constexpr (STAGE == kPlain || STAGE == kPairs) {
         for (uint32_t k = threadIdx.x; k < padded; k += blockDim.x) xs[x_place(k)] = k < K ? value(k) : 0.0f;
     } else {
         constexpr int R = 8;                                  // elements a thread keeps between the passes; the rest are read again
@@ -268,8 +305,7 @@ __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, u
         for (int i = 0; i < R; i++) {
             const uint32_t k = threadIdx.x + i * blockDim.x;
             keep[i] = k < K ? value(k) : 0.0f;
-            wk[i] = k < K ? st.norm_weight[k] : 0.0f;
-            if constexpr (STAGE == kGated) if (k < K) wk[i] *= lh_sigmoid(st.gate_f32 ? static_cast<const float*>(st.gate)[k] : lh_bf2f(static_cast<const uint16_t*>(st.gate)[k]));
+            wk[i] = k < K ? weight(k) : 0.0f;
             s += keep[i] * keep[i];
         }
         for (uint32_t k = threadIdx.x + R * blockDim.x; k < K; k += blockDim.x) { const float v = value(k); s += v * v; }
@@ -285,8 +321,7 @@ __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, u
             float v = 0.0f, w = 0.0f;
             if (k < K) {
                 v = value(k);
-                w = st.norm_weight[k];
-                if constexpr (STAGE == kGated) w *= lh_sigmoid(st.gate_f32 ? static_cast<const float*>(st.gate)[k] : lh_bf2f(static_cast<const uint16_t*>(st.gate)[k]));
+                w = weight(k);
                 if (store) st.store[k] = v;
             }
             xs[x_place(k)] = v * r * w;
@@ -407,8 +442,8 @@ __global__ __launch_bounds__(256) void matvec_bf16_reg_kernel(const VectorStage 
     sums.flush();
 }
 
-// Rows longer than a wave's registers: the four waves of a workgroup take a quarter of the columns each, and the quarters of up to 64 rows meet in LDS.  Plain vectors only: a norm would need all quarters.
-template <int NL>
+// Rows longer than a wave's registers: the four waves of a workgroup take a quarter of the columns each, and the quarters of up to 64 rows meet in LDS.  Plain vectors and pairs only: a norm would need all quarters.
+template <int STAGE, int NL>
 __global__ __launch_bounds__(256) void matvec_bf16_quarter_kernel(const VectorStage st, const uint16_t* __restrict__ W, const float* __restrict__ bias, const LhSegments seg,
                                                                  uint32_t N, uint32_t K, uint32_t quarter) {
     __shared__ float sums[4][64];
@@ -423,9 +458,9 @@ __global__ __launch_bounds__(256) void matvec_bf16_quarter_kernel(const VectorSt
     uint4 p[NL], q[NL];
     issue(p, row);
     VectorStage part = st;
-    part.x = st.x_f32 ? (const void*)(static_cast<const float*>(st.x) + kb) : (const void*)(static_cast<const uint16_t*>(st.x) + kb);
+    part.x = STAGE == kPairs ? (const void*)(static_cast<const float*>(st.x) + 2 * kb) : st.x_f32 ? (const void*)(static_cast<const float*>(st.x) + kb) : (const void*)(static_cast<const uint16_t*>(st.x) + kb);
     float xr[NL][8], mine = 0.0f;
-    lh_vector_registers<kPlain, NL>(part, len, lane, false, xr);
+    lh_vector_registers<STAGE, NL>(part, len, lane, false, xr);
     auto flush = [&]() {
         sums[wave][lane] = mine;
         __syncthreads();
@@ -469,11 +504,11 @@ int launch_vector(lh_context* ctx, const VectorStage& st, const uint16_t* W, con
 #undef LH_MVR
         return lh_check_launch(op);
     }
-    if (STAGE == kPlain && vec && K <= 16384 && lh_stage_aligned(st)) {
+    if constexpr (STAGE == kPlain || STAGE == kPairs) if (vec && K <= 16384 && lh_stage_aligned(st)) {
         const uint32_t quarter = ((K + 3) / 4 + 7) / 8 * 8, grid = (uint32_t)std::min<uint64_t>(N, (uint64_t)ctx->cu_count * 4);
-        if (quarter <= 1024) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<2>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
-        else if (quarter <= 2048) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<4>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
-        else hipLaunchKernelGGL((matvec_bf16_quarter_kernel<8>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        if (quarter <= 1024) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 2>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else if (quarter <= 2048) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 4>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 8>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
         return lh_check_launch(op);
     }
     const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * 4);
@@ -510,12 +545,15 @@ int vector_entry(lh_batch* batch, const char* op, int stage, const VectorStage& 
                  lh_buffer* const* outputs, int output_dtype, int accumulate, const lh_buffer* position) {
     LhSegments seg;
     LH_TRY(lh_make_segments(seg, op, 1, 0, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position));
+    LH_REQUIRE(!seg.pairs, "%s: pairs are stored as they are for one row", op);
     const uint32_t n = seg.n0[seg.count];
     LH_TRY(check_common(batch, weight, bias, k, n, op));
     const uint16_t* W = (const uint16_t*)weight->ptr;
     const float* b = bias ? (const float*)bias->ptr : nullptr;
     int r;
-    if (stage == kPlain) r = launch_vector<kPlain>(batch->ctx, st, W, b, seg, n, k, op);
+    if (stage == kPairs) r = launch_vector<kPairs>(batch->ctx, st, W, b, seg, n, k, op);
+    else if (stage == kResidual) r = launch_vector<kResidual>(batch->ctx, st, W, b, seg, n, k, op);
+    else if (stage == kPlain) r = launch_vector<kPlain>(batch->ctx, st, W, b, seg, n, k, op);
     else if (stage == kNorm) r = launch_vector<kNorm>(batch->ctx, st, W, b, seg, n, k, op);
     else r = launch_vector<kGated>(batch->ctx, st, W, b, seg, n, k, op);
     if (r == LH_OK) batch->dispatch_count++;
@@ -526,8 +564,10 @@ int vector_entry(lh_batch* batch, const char* op, int stage, const VectorStage& 
 
 uint32_t lh_expert_tile_rows(uint32_t slots, uint32_t experts) { return slots / (experts ? experts : 1) >= 128 ? 128u : 64u; }
 
-int lh_launch_linear(lh_context* ctx, const LhLinear& a, const char* op) {
-    const bool mfma = !a.a_f32 && a.K % 8 == 0 && (((uintptr_t)a.A | (uintptr_t)a.W) & 15) == 0;
+int lh_launch_linear(lh_context* ctx, const LhLinear& given, const char* op) {
+    LhLinear a = given;
+    if (a.lda == 0) a.lda = a.K;
+    const bool mfma = !a.a_f32 && a.K % 8 == 0 && a.lda % 8 == 0 && (((uintptr_t)a.A | (uintptr_t)a.W) & 15) == 0;
     if (!mfma) {
         const uint64_t mt = a.ex.tiles ? a.ex.n_tiles : ((uint64_t)a.M + 63) / 64, grid = mt * ((a.N + 63) / 64);
         LH_REQUIRE(grid < 0x7FFFFFFFull, "%s: %u x %u outputs", op, a.M, a.N);
@@ -585,7 +625,8 @@ int lh_linear_vector_into(lh_batch* batch, const lh_buffer* input, int input_dty
     LH_REQUIRE(batch, "%s: batch is null", op);
     LH_REQUIRE(input_dtype == LH_F32 || input_dtype == LH_BF16, "%s: input dtype %d", op, input_dtype);
     LH_NEED(input, (size_t)k * (input_dtype == LH_F32 ? 4 : 2), op, "input");
-    const VectorStage st{input->ptr, input_dtype == LH_F32, nullptr, nullptr, nullptr, nullptr, 0, 0.0f};
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = input_dtype == LH_F32;
     return vector_entry(batch, op, kPlain, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
 }
 
@@ -602,12 +643,51 @@ int lh_linear_norm_vector_into(lh_batch* batch, const lh_buffer* input, const lh
         LH_NEED(store, (size_t)k * 4, op, "store");
         LH_REQUIRE(store->ptr != input->ptr && (!add || store->ptr != add->ptr), "%s: store must not be read by the other workgroups", op);
     }
-    const VectorStage st{input->ptr, 1, add ? (const float*)add->ptr : nullptr, store ? (float*)store->ptr : nullptr, (const float*)norm_weight->ptr, nullptr, 0, eps};
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = 1; st.add = add ? (const float*)add->ptr : nullptr; st.store = store ? (float*)store->ptr : nullptr;
+    st.norm_weight = (const float*)norm_weight->ptr; st.eps = eps;
     return vector_entry(batch, op, kNorm, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
 }
 
-int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, int gate_dtype, const lh_buffer* norm_weight, float eps,
-                                const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns, const uint32_t* acts,
+int lh_linear_residual_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* branch, lh_buffer* store, const lh_buffer* norm_weight,
+                                   float eps, const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
+                                   const uint32_t* acts, const uint32_t* heads, const uint32_t* padded, const uint32_t* layouts, lh_buffer* const* outputs,
+                                   int output_dtype, int accumulate, const lh_buffer* position) {
+    const char* op = "linear_residual_vector";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    LH_NEED(input, (size_t)k * 4, op, "input");
+    LH_NEED(branch, (size_t)k * 4, op, "branch");
+    LH_NEED(norm_weight, (size_t)k * 4, op, "norm_weight");
+    if (store) {
+        LH_NEED(store, (size_t)k * 4, op, "store");
+        LH_REQUIRE(store->ptr != input->ptr && store->ptr != branch->ptr, "%s: store must not be read by the other workgroups", op);
+    }
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = 1; st.add = (const float*)branch->ptr; st.store = store ? (float*)store->ptr : nullptr;
+    st.norm_weight = (const float*)norm_weight->ptr; st.eps = eps;
+    return vector_entry(batch, op, kResidual, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
+}
+
+int lh_linear_pairs_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count,
+                                const uint32_t* ns, const uint32_t* acts, const uint32_t* heads, const uint32_t* padded, const uint32_t* layouts,
+                                lh_buffer* const* outputs, int output_dtype, int accumulate, const lh_buffer* position) {
+    const char* op = "linear_pairs_vector";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    LH_NEED(input, (size_t)k * 8, op, "input");
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = 1;
+    return vector_entry(batch, op, kPairs, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
+}
+
+uint32_t lh_gated_vector_fits(uint32_t k, uint32_t group) {
+    if (group == k) return 1;
+    if (group == 0 || k % group || group % 8 || k > 4096) return 0;
+    const uint32_t c = group / 8;
+    return c % 64 == 0 || (c < 64 && (c & (c - 1)) == 0);
+}
+
+int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, int gate_dtype, uint32_t gate_act, int gate_first,
+                                const lh_buffer* norm_weight, uint32_t group, float eps, const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns, const uint32_t* acts,
                                 const uint32_t* heads, const uint32_t* padded, const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
                                 int accumulate, const lh_buffer* position) {
     const char* op = "linear_gated_vector";
@@ -615,8 +695,14 @@ int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const l
     LH_REQUIRE(gate_dtype == LH_F32 || gate_dtype == LH_BF16, "%s: gate dtype %d", op, gate_dtype);
     LH_NEED(input, (size_t)k * 4, op, "input");
     LH_NEED(gate, (size_t)k * (gate_dtype == LH_F32 ? 4 : 2), op, "gate");
-    LH_NEED(norm_weight, (size_t)k * 4, op, "norm_weight");
-    const VectorStage st{input->ptr, 1, nullptr, nullptr, (const float*)norm_weight->ptr, gate->ptr, gate_dtype == LH_F32, eps};
+    if (norm_weight) LH_NEED(norm_weight, (size_t)k * 4, op, "norm_weight");
+    LH_REQUIRE(gate_act == LH_ACT_SIGMOID || gate_act == LH_ACT_SILU, "%s: gate activation %u", op, gate_act);
+    LH_REQUIRE(lh_gated_vector_fits(k, group), "%s: %u values in parts of %u", op, k, group);
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = 1; st.norm_weight = norm_weight ? (const float*)norm_weight->ptr : nullptr; st.gate = gate->ptr;
+    st.gate_f32 = gate_dtype == LH_F32; st.gate_act = gate_act; st.gate_first = gate_first != 0; st.group = group; st.eps = eps;
+    LH_REQUIRE(group == k || lh_stage_aligned(st), "%s: buffers must be 16-byte aligned", op);
+    LH_REQUIRE(group == k || ((uintptr_t)weight->ptr & 15) == 0, "%s: the weight must be 16-byte aligned", op);
     return vector_entry(batch, op, kGated, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
 }
 

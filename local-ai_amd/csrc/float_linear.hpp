@@ -14,11 +14,11 @@ struct LhExpertRows {
 };
 
 struct LhLinear {
-    const void* A;                  // [M, K], bf16 or f32
+    const void* A;                  // [M, K], bf16 or f32, rows `lda` elements apart (0: K)
     uint32_t a_f32;
     const uint16_t* W;              // [N, K] (of every expert, one after the other)
     const float* bias;
-    uint32_t M, N, K;
+    uint32_t M, N, K, lda;
     LhSegments seg;
     LhExpertRows ex;
 };
@@ -28,15 +28,15 @@ uint32_t lh_expert_tile_rows(uint32_t slots, uint32_t experts);
 // ---- one row: the activation vector in registers -------------------------------------------------------------------------
 // Up to 4096 columns a wave keeps the vector itself: lane l holds the NL chunks of eight elements 8 (64 c + l), which is what
 // it multiplies in every row.  The norm before the product is then a sum over the wave, with no barrier and no LDS.
-enum { kPlain = 0, kNorm = 1, kGated = 2 };
+enum { kPlain = 0, kNorm = 1, kGated = 2, kResidual = 3, kPairs = 4 };
 struct VectorStage {
-    const void* x;             // plain: x_f32 ? f32 : bf16; norm, gated: f32
+    const void* x;             // plain: x_f32 ? f32 : bf16; the others: f32 (pairs: 2 K values, gate and up in turn)
     uint32_t x_f32;
-    const float* add;          // norm: may be null
-    float* store;              // norm: receives x + add (workgroup 0), may be null
-    const float* norm_weight;
+    const float* add;          // norm: may be null; residual: what is normed and added
+    float* store;              // norm, residual: receives the sum (workgroup 0), may be null
+    const float* norm_weight;  // gated: may be null
     const void* gate;          // gated
-    uint32_t gate_f32;
+    uint32_t gate_f32, gate_act, gate_first, group;   // gated: the gate multiplies before the norm; elements per normed part
     float eps;
 };
 
@@ -54,14 +54,25 @@ __device__ __forceinline__ void lh_ld8(const uint16_t* p, float (&v)[8]) {
 // K a multiple of 8, all pointers 16-byte aligned; chunks past K are zero.  `store` whether this wave stores x + add.
 template <int STAGE, int NL>
 __device__ __forceinline__ void lh_vector_registers(const VectorStage& st, uint32_t K, uint32_t lane, bool store, float (&xr)[NL][8]) {
-    float w[STAGE == kPlain ? 1 : NL][8], s = 0.0f;
+    constexpr bool kNormed = STAGE == kNorm || STAGE == kGated || STAGE == kResidual;
+    float w[kNormed ? NL : 1][8], s[kNormed ? NL : 1], total = 0.0f;
 #pragma unroll
     for (int c = 0; c < NL; c++) {
         const uint32_t k = (64 * c + lane) * 8;
 #pragma unroll
         for (int j = 0; j < 8; j++) xr[c][j] = 0.0f;
+        if constexpr (kNormed) s[c] = 0.0f;
         if (k >= K) continue;
-        if (STAGE == kPlain && !st.x_f32) lh_ld8(static_cast<const uint16_t*>(st.x) + k, xr[c]);
+        if constexpr (STAGE == kPairs) {
+            float a[8], b[8];
+            lh_ld8(static_cast<const float*>(st.x) + 2 * k, a);
+            lh_ld8(static_cast<const float*>(st.x) + 2 * k + 8, b);
+#pragma unroll
+            for (int j = 0; j < 4; j++) {
+                xr[c][j] = a[2 * j] * lh_sigmoid(a[2 * j]) * a[2 * j + 1];
+                xr[c][4 + j] = b[2 * j] * lh_sigmoid(b[2 * j]) * b[2 * j + 1];
+            }
+        } else if (STAGE == kPlain && !st.x_f32) lh_ld8(static_cast<const uint16_t*>(st.x) + k, xr[c]);
         else lh_ld8(static_cast<const float*>(st.x) + k, xr[c]);
         if constexpr (STAGE == kNorm) if (st.add) {
             float b[8];
@@ -69,31 +80,65 @@ __device__ __forceinline__ void lh_vector_registers(const VectorStage& st, uint3
 #pragma unroll
             for (int j = 0; j < 8; j++) xr[c][j] += b[j];
         }
-        if constexpr (STAGE != kPlain) {
-            lh_ld8(st.norm_weight + k, w[c]);
+        if constexpr (kNormed) {
+            if (STAGE != kGated || st.norm_weight) lh_ld8(st.norm_weight + k, w[c]);
+            else
+#pragma unroll
+                for (int j = 0; j < 8; j++) w[c][j] = 1.0f;
             if constexpr (STAGE == kGated) {
                 float g[8];
                 if (st.gate_f32) lh_ld8(static_cast<const float*>(st.gate) + k, g);
                 else lh_ld8(static_cast<const uint16_t*>(st.gate) + k, g);
 #pragma unroll
-                for (int j = 0; j < 8; j++) w[c][j] *= lh_sigmoid(g[j]);
+                for (int j = 0; j < 8; j++) {
+                    const float f = lh_gate(g[j], st.gate_act);
+                    if (st.gate_first) xr[c][j] *= f; else w[c][j] *= f;
+                }
             }
+            if constexpr (STAGE == kResidual) {               // w becomes the weighted branch
+                float y[8];
+                lh_ld8(st.add + k, y);
 #pragma unroll
-            for (int j = 0; j < 8; j++) s += xr[c][j] * xr[c][j];
+                for (int j = 0; j < 8; j++) { s[c] += y[j] * y[j]; w[c][j] *= y[j]; }
+            } else
+#pragma unroll
+                for (int j = 0; j < 8; j++) s[c] += xr[c][j] * xr[c][j];
+            total += s[c];
         }
     }
-    if constexpr (STAGE != kPlain) {
-        const float r = rsqrtf(lh_group_sum(s, 64) / (float)K + st.eps);
+    if constexpr (kNormed) {
+        float r[NL];
+        if (STAGE == kGated && st.group != K) {               // group / 8 chunks: a power of two of lanes, or whole sets of 64
+            const uint32_t cg = st.group >> 3;
+#pragma unroll
+            for (int c = 0; c < NL; c++) s[c] = lh_group_sum(s[c], (int)min(cg, 64u));
+            const uint32_t per = cg > 64 ? cg >> 6 : 1u;
+#pragma unroll
+            for (int c = 0; c < NL; c++) {
+                float t = 0.0f;
+#pragma unroll
+                for (int e = 0; e < NL; e++) t += (uint32_t)e / per == (uint32_t)c / per ? s[e] : 0.0f;
+                r[c] = rsqrtf(t / (float)st.group + st.eps);
+            }
+        } else {
+            const float all = rsqrtf(lh_group_sum(total, 64) / (float)K + st.eps);
+#pragma unroll
+            for (int c = 0; c < NL; c++) r[c] = all;
+        }
 #pragma unroll
         for (int c = 0; c < NL; c++) {
             const uint32_t k = (64 * c + lane) * 8;
             if (k >= K) continue;
-            if (STAGE == kNorm && store) {
+            if constexpr (STAGE == kResidual)
+#pragma unroll
+                for (int j = 0; j < 8; j++) xr[c][j] = __builtin_fmaf(w[c][j], r[c], xr[c][j]);
+            if (STAGE != kGated && store) {
                 *reinterpret_cast<float4*>(st.store + k) = make_float4(xr[c][0], xr[c][1], xr[c][2], xr[c][3]);
                 *reinterpret_cast<float4*>(st.store + k + 4) = make_float4(xr[c][4], xr[c][5], xr[c][6], xr[c][7]);
             }
+            if constexpr (STAGE != kResidual)
 #pragma unroll
-            for (int j = 0; j < 8; j++) xr[c][j] = xr[c][j] * r * w[c][j];
+                for (int j = 0; j < 8; j++) xr[c][j] = xr[c][j] * r[c] * w[c][j];
         }
     }
 }

@@ -206,7 +206,8 @@ __global__ __launch_bounds__(256) void vector_down_reg_kernel(const float* __res
     __shared__ uint32_t ids[4][kMaxTop];
     __shared__ float weights[4][kMaxTop];
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, chunks = top * (ff >> 3), row_step = gridDim.x * 4;
-    const VectorStage st{hidden, 1, nullptr, nullptr, nullptr, nullptr, 0, 0.0f};
+    VectorStage st{};
+    st.x = hidden; st.x_f32 = 1;
     float xr[NL][8];
     lh_vector_registers<kPlain, NL>(st, top * ff, lane, false, xr);
     select_experts(logits, experts, top, lane, ids[wave], weights[wave]);
@@ -362,7 +363,8 @@ int lh_moe_vector_up_into(lh_batch* batch, const lh_buffer* input, const lh_buff
     LH_NEED(logits, (size_t)experts * 4, op, "logits");
     LH_NEED(up, (size_t)experts * ff * width * 2, op, "up");
     LH_NEED(hidden, (size_t)top * ff * 4, op, "hidden");
-    const VectorStage st{input->ptr, 1, nullptr, nullptr, (const float*)norm_weight->ptr, nullptr, 0, eps};
+    VectorStage st{};
+    st.x = input->ptr; st.x_f32 = 1; st.norm_weight = (const float*)norm_weight->ptr; st.eps = eps;
     if (width % 8 == 0 && width <= 4096 && ((uintptr_t)up->ptr & 15) == 0 && lh_stage_aligned(st)) {
         const dim3 grid(std::min<uint32_t>((ff + 3) / 4, std::max<uint32_t>(1, (uint32_t)batch->ctx->cu_count * 4 / top)), top);
 #define LH_UP(NL) hipLaunchKernelGGL((vector_up_reg_kernel<NL>), grid, dim3(256), 0, batch->ctx->stream, st, (const float*)logits->ptr, (const uint16_t*)up->ptr, \

@@ -39,6 +39,7 @@ __device__ __forceinline__ float lh_activate(float v, uint32_t act) {
         default: return v;
     }
 }
+__device__ __forceinline__ float lh_gate(float g, uint32_t act) { const float s = lh_sigmoid(g); return act == LH_ACT_SILU ? g * s : s; }
 
 // Inside a 32-position block of a value cache the positions are kept in the order in which a lane of the matrix product
 // P V needs them: the scores of a 32-key step leave lane group g with keys 4g .. 4g + 3 of both 16-key tiles, so those
@@ -53,22 +54,27 @@ struct LhSegments {
     uint32_t ld[4];                 // columns of a destination row, padding included
     uint32_t head[4], padded[4];    // column n of the segment lands at (n / head) * padded + n % head
     uint32_t act[4];
-    uint32_t layout[4];             // LH_ROWS, LH_ROWS_AT_POSITION, LH_BLOCKS_AT_POSITION
+    uint32_t layout[4];             // LH_ROWS, LH_ROWS_AT_POSITION, LH_BLOCKS_AT_POSITION, LH_ROWS_F32
     uint32_t rows[4];               // rows (positions) the destination holds: writes past it are dropped
-    uint32_t f32_out;               // destinations are f32 (else bf16)
+    uint32_t f32[4];                // the destination is f32 (else bf16)
     uint32_t accumulate;            // add to the destination (f32 only)
-    uint32_t vec4;                  // every boundary is a multiple of 4 and no head is padded: four neighbouring columns stay together
+    uint32_t aligned4;              // every boundary is a multiple of 4: four neighbouring columns are of one segment
+    uint32_t vec4[4];               // and stay together in the destination
+    uint32_t pairs;                 // some segment has LH_ACT_SILU_PAIRS
     const uint32_t* position;       // device word: position of row 0 (layouts AT_POSITION)
 };
+__device__ __forceinline__ bool lh_segment_at_position(const LhSegments& s, uint32_t i) {
+    return s.layout[i] == LH_ROWS_AT_POSITION || s.layout[i] == LH_BLOCKS_AT_POSITION;
+}
 __device__ __forceinline__ uint32_t lh_segment_of(const LhSegments& s, uint32_t n) {
     uint32_t i = 0;
 #pragma unroll
     for (uint32_t j = 1; j < 4; j++) if (j < s.count && n >= s.n0[j]) i = j;
     return i;
 }
-__device__ __forceinline__ void lh_segment_put(const LhSegments& s, size_t idx, void* out, float v) {
-    if (s.f32_out) { float* o = static_cast<float*>(out); o[idx] = s.accumulate ? o[idx] + v : v; }
-    else static_cast<uint16_t*>(out)[idx] = lh_f2bf(v);
+__device__ __forceinline__ void lh_segment_put(const LhSegments& s, uint32_t i, size_t idx, float v) {
+    if (s.f32[i]) { float* o = static_cast<float*>(s.out[i]); o[idx] = s.accumulate ? o[idx] + v : v; }
+    else static_cast<uint16_t*>(s.out[i])[idx] = lh_f2bf(v);
 }
 // Stores column n of row m (activation applied here); `pos0` is *s.position, or 0.
 __device__ __forceinline__ void lh_segment_store(const LhSegments& s, uint32_t m, uint32_t n, float v, uint32_t pos0) {
@@ -76,10 +82,17 @@ __device__ __forceinline__ void lh_segment_store(const LhSegments& s, uint32_t m
     uint32_t c = n - s.n0[i];
     if (s.head[i] != s.padded[i]) { const uint32_t h = c / s.head[i]; c = h * s.padded[i] + (c - h * s.head[i]); }
     v = lh_activate(v, s.act[i]);
-    const uint32_t p = s.layout[i] == LH_ROWS ? m : pos0 + m;
+    const uint32_t p = lh_segment_at_position(s, i) ? pos0 + m : m;
     if (p >= s.rows[i]) return;
     const size_t idx = s.layout[i] == LH_BLOCKS_AT_POSITION ? ((size_t)(p >> 5) * s.ld[i] + c) * 32 + lh_block_slot(p & 31u) : (size_t)p * s.ld[i] + c;
-    lh_segment_put(s, idx, s.out[i], v);
+    lh_segment_put(s, i, idx, v);
+}
+// Columns n and n + 1 (n even) of row m: a (gate, up) pair of an LH_ACT_SILU_PAIRS segment becomes one value.
+__device__ __forceinline__ void lh_segment_store_pair(const LhSegments& s, uint32_t m, uint32_t n, float a, float b, uint32_t pos0) {
+    const uint32_t i = lh_segment_of(s, n);
+    if (s.act[i] == LH_ACT_SILU_PAIRS) { lh_segment_put(s, i, (size_t)m * s.ld[i] + (n - s.n0[i]) / 2, a * lh_sigmoid(a) * b); return; }
+    lh_segment_store(s, m, n, a, pos0);
+    lh_segment_store(s, m, n + 1, b, pos0);
 }
 
 // Host side of the above, from the arrays of the C ABI; validates every destination against its shape.

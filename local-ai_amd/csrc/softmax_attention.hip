@@ -15,27 +15,9 @@
 //   attention_split_kernel  few rows: every wave walks its own share of the blocks straight from global memory; the
 //                           workgroup's four partial results are merged in LDS, the workgroups' by attention_merge_kernel
 // Plain form (any dtype, any dim): attention_plain_kernel, one workgroup per query row and head.
-#include "float_ops.hpp"
-#include <algorithm>
-#include <cmath>
+#include "softmax_attention.hpp"
 
 namespace {
-
-struct AttentionArgs {
-    const void* q;
-    const void* keys;
-    const void* values;
-    void* out;
-    const uint32_t* position;
-    uint32_t rows, heads, kv_heads, maps, dim, dq, vdim, dv, capacity;
-    float scale, lambda, out_scale, eps;
-    float* partial;            // records [16-row tile][kv head][split][map][16] of dv unnormalised sums, maximum, sum of weights
-    uint32_t splits;
-};
-
-constexpr float kLog2e = 1.4426950408889634f;
-
-typedef uint32_t u32x4 __attribute__((ext_vector_type(4)));
 
 // The B operand of S^T: query values of packed row `row` (zero past the rows and past dim).
 template <int DQ, int MAPS>
@@ -60,53 +42,14 @@ __device__ __forceinline__ void load_queries(lh_bf16x8 (&qf)[MAPS][DQ / 32], con
         }
 }
 
-// A row tile's running softmax state for one map; every lane holds the values of packed row (lane & 15).
-struct RowState { float m, l; };
-
-// Scores of NB steps of 32 keys -> weights in P V operand order, as three bf16 terms; returns the factor for what was summed
-// before.  `first` is the first key, `limit` the row's last visible key, `bound` whether any lane may have to mask.
-template <int NB>
-__device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2 * NB], RowState& st, float scale2, uint32_t first, uint32_t limit, bool bound, uint32_t lane,
-                                              lh_bf16x8 (&w)[NB][3]) {
-    float v[8 * NB], mx = -INFINITY;
-    const uint32_t g = lane >> 4;
-#pragma unroll
-    for (int i = 0; i < 8 * NB; i++) {
-        v[i] = s[i >> 2][i & 3] * scale2;
-        if (bound && first + (i >> 2) * 16 + g * 4 + (i & 3) > limit) v[i] = -INFINITY;
-        mx = fmaxf(mx, v[i]);
-    }
-    const float nm = fmaxf(st.m, lh_column_max(mx)), base = nm == -INFINITY ? 0.0f : nm;
-    const float alpha = __builtin_amdgcn_exp2f(st.m - base);
-    float sum = 0.0f;
-#pragma unroll
-    for (int b = 0; b < NB; b++) {
-        uint32_t h[4], m[4], l[4];
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            float p0 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i] - base), p1 = __builtin_amdgcn_exp2f(v[8 * b + 2 * i + 1] - base);
-            sum += p0 + p1;
-            h[i] = lh_pack_bf(p0, p1);
-            p0 -= __builtin_bit_cast(float, h[i] << 16); p1 -= __builtin_bit_cast(float, h[i] & 0xFFFF0000u);
-            m[i] = lh_pack_bf(p0, p1);
-            l[i] = lh_pack_bf(p0 - __builtin_bit_cast(float, m[i] << 16), p1 - __builtin_bit_cast(float, m[i] & 0xFFFF0000u));
-        }
-        w[b][0] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
-        w[b][1] = __builtin_bit_cast(lh_bf16x8, (u32x4){m[0], m[1], m[2], m[3]});
-        w[b][2] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
-    }
-    st.l = st.l * alpha + sum;      // this lane's keys only; the four lanes of a row are added at the end
-    st.m = nm;
-    return alpha;
-}
-
 // A finished row: o[i][r] holds value 16 i + 4g + r of packed row (lane & 15), for every map unnormalised with sum l.
 template <int DV, int MAPS>
-__device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)[MAPS][DV / 16], const float (&l)[MAPS], uint32_t g, uint32_t row, uint32_t lane) {
+__device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)[MAPS][DV / 16], const float (&l)[MAPS], float m0, uint32_t g, uint32_t row, uint32_t lane) {   // m0: the first map's maximum
     const uint32_t R = a.heads / a.kv_heads, t = row / R, h = g * R + (row - t * R);
     float inv[MAPS];
 #pragma unroll
     for (int mp = 0; mp < MAPS; mp++) inv[mp] = 1.0f / l[mp];
+    if (MAPS == 1 && a.sink) inv[0] = 1.0f / (l[0] + __builtin_amdgcn_exp2f(a.sink[h] * kLog2e - m0));
     float ss = 0.0f;
 #pragma unroll
     for (int i = 0; i < DV / 16; i++)
@@ -123,6 +66,7 @@ __device__ __forceinline__ void finish_row(const AttentionArgs& a, lh_f32x4 (&o)
         f = rsqrtf(ss / (float)a.vdim + a.eps) * a.out_scale;
     }
     if (t >= a.rows) return;
+    if (MAPS == 1 && a.gate) f = lh_sigmoid(a.gate[(size_t)t * a.heads + h]);
     uint16_t* out = static_cast<uint16_t*>(a.out) + ((size_t)t * a.heads + h) * a.vdim;
 #pragma unroll
     for (int i = 0; i < DV / 16; i++) {
@@ -232,7 +176,7 @@ __global__ __launch_bounds__(256, MAPS * DV <= 256 ? 2 : 1) void attention_tile_
     float l[MAPS];
 #pragma unroll
     for (int mp = 0; mp < MAPS; mp++) l[mp] = lh_column_sum(st[mp].l);
-    if (a.splits == 1) { finish_row<DV, MAPS>(a, o, l, g, row, lane); return; }
+    if (a.splits == 1) { finish_row<DV, MAPS>(a, o, l, st[0].m, g, row, lane); return; }
     if (row >= packed) return;
     constexpr uint32_t kRow = DV + 4;
 #pragma unroll
@@ -363,137 +307,6 @@ __global__ __launch_bounds__(256) void attention_split_kernel(const AttentionArg
     }
 }
 
-// One workgroup per (query row, head): merges the splits of every map, combines the maps, norms and stores.  Groups of dv / 4
-// threads take the splits in turn, four values a thread, several loads on their way; the groups are added through LDS.
-constexpr uint32_t kMergeThreads = 512;
-template <int MAPS>
-__global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const AttentionArgs a) {
-    __shared__ float factor[MAPS][512], total[MAPS], scratch[kMergeThreads / 64];
-    __shared__ float4 sums[MAPS][kMergeThreads];
-    const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
-    const uint32_t kRow = a.dv + 4, rr = row & 15;
-    const size_t stride = (size_t)MAPS * 16 * kRow;
-    const float* rec = a.partial + (size_t)(((row >> 4) * a.kv_heads + g) * a.splits) * stride + rr * kRow;
-    const uint32_t wave = threadIdx.x >> 6, lane = threadIdx.x & 63;
-    if (wave < MAPS) {                                        // splits <= 512
-        const float* r = rec + wave * 16 * kRow + a.dv;
-        float m = -INFINITY, l = 0.0f, mine[8], ml[8];
-#pragma unroll
-        for (uint32_t i = 0; i < 8; i++) {
-            const uint32_t s = i * 64 + lane;
-            mine[i] = -INFINITY; ml[i] = 0.0f;
-            if (i * 64 >= a.splits) break;
-            if (s < a.splits) { const float2 x = *reinterpret_cast<const float2*>(r + s * stride); mine[i] = x.x; ml[i] = x.y; }
-            m = fmaxf(m, mine[i]);
-        }
-        m = lh_group_max(m, 64);
-#pragma unroll
-        for (uint32_t i = 0; i < 8; i++) {
-            if (i * 64 >= a.splits) break;
-            const float f = __builtin_amdgcn_exp2f(mine[i] - m);
-            if (i * 64 + lane < a.splits) factor[wave][i * 64 + lane] = f;
-            l += f * ml[i];
-        }
-        l = lh_group_sum(l, 64);
-        if (lane == 0) total[wave] = 1.0f / l;
-    }
-    __syncthreads();
-    const uint32_t quads = a.dv / 4, groups = kMergeThreads / quads, grp = threadIdx.x / quads, q = threadIdx.x % quads;   // quads <= 64
-    float4 acc[MAPS];
-#pragma unroll
-    for (int mp = 0; mp < MAPS; mp++) acc[mp] = make_float4(0.f, 0.f, 0.f, 0.f);
-#pragma unroll 4
-    for (uint32_t s = grp; s < a.splits; s += groups)
-#pragma unroll
-        for (int mp = 0; mp < MAPS; mp++) {
-            const float4 x = *reinterpret_cast<const float4*>(rec + s * stride + mp * 16 * kRow + q * 4);
-            const float f = factor[mp][s];
-            acc[mp].x += f * x.x; acc[mp].y += f * x.y; acc[mp].z += f * x.z; acc[mp].w += f * x.w;
-        }
-#pragma unroll
-    for (int mp = 0; mp < MAPS; mp++) sums[mp][threadIdx.x] = acc[mp];
-    __syncthreads();
-    float v = 0.0f;
-    const uint32_t d = threadIdx.x;                           // dv <= 256
-    if (d < a.vdim) {
-        float s[MAPS] = {};
-        for (uint32_t i = 0; i < groups; i++)
-#pragma unroll
-            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sums[mp][i * quads])[d];
-        v = s[0] * total[0];
-        if constexpr (MAPS == 2) v -= a.lambda * (s[MAPS - 1] * total[MAPS - 1]);
-    }
-    float f = 1.0f;
-    if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(v * v, scratch) / (float)a.vdim + a.eps) * a.out_scale;
-    if (d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
-}
-
-// One workgroup per (query row, head), 256 keys at a time; f32 arithmetic throughout.
-template <typename T>
-__global__ __launch_bounds__(256) void attention_plain_kernel(const AttentionArgs a) {
-    extern __shared__ float dyn[];                            // the query's maps * dim values
-    __shared__ float p[2][256], scratch[4];
-    const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, g = h / (a.heads / a.kv_heads), tid = threadIdx.x;
-    const uint32_t start = *a.position, last = min(start + t, a.capacity - 1);
-    const T* q = static_cast<const T*>(a.q) + ((size_t)t * a.heads + h) * a.maps * a.dq;
-    for (uint32_t i = tid; i < a.maps * a.dim; i += 256) dyn[i] = lh_ld(q, (size_t)(i / a.dim) * a.dq + i % a.dim);
-    __syncthreads();
-    float m[2] = {-INFINITY, -INFINITY}, l[2] = {0.0f, 0.0f}, acc[2][4] = {};
-    for (uint32_t k0 = 0; k0 <= last; k0 += 256) {
-        const uint32_t n = min(256u, last + 1 - k0);
-        for (uint32_t mp = 0; mp < a.maps; mp++) {
-            float s = -INFINITY;
-            if (tid < n) {
-                const T* k = static_cast<const T*>(a.keys) + (((size_t)(k0 + tid) * a.kv_heads + g) * a.maps + mp) * a.dq;
-                float dot = 0.0f;
-                for (uint32_t i = 0; i < a.dim; i++) dot = __builtin_fmaf(dyn[mp * a.dim + i], lh_ld(k, i), dot);
-                s = dot * a.scale;
-            }
-            float mx = lh_group_max(s, 64);
-            if ((tid & 63) == 0) scratch[tid >> 6] = mx;
-            __syncthreads();
-            mx = fmaxf(fmaxf(scratch[0], scratch[1]), fmaxf(scratch[2], scratch[3]));
-            __syncthreads();
-            const float nm = fmaxf(m[mp], mx), alpha = expf(m[mp] - nm), w = tid < n ? expf(s - nm) : 0.0f;
-            p[mp][tid] = w;
-            const float sum = lh_block_sum(w, scratch);
-            l[mp] = l[mp] * alpha + sum;
-            m[mp] = nm;
-#pragma unroll
-            for (int i = 0; i < 4; i++) acc[mp][i] *= alpha;
-        }
-        __syncthreads();
-#pragma unroll
-        for (int i = 0; i < 4; i++) {
-            const uint32_t d = tid + i * 256;
-            if (d >= a.vdim) break;
-            for (uint32_t j0 = 0; j0 < n; j0 += 32) {          // k0 is a multiple of 32
-                const T* v = static_cast<const T*>(a.values) + ((size_t)((k0 + j0) >> 5) * a.kv_heads * a.dv + (size_t)g * a.dv + d) * 32;
-                for (uint32_t j = 0; j < min(32u, n - j0); j++) {
-                    const float x = lh_ld(v, lh_block_slot(j));
-                    acc[0][i] = __builtin_fmaf(p[0][j0 + j], x, acc[0][i]);
-                    if (a.maps == 2) acc[1][i] = __builtin_fmaf(p[1][j0 + j], x, acc[1][i]);
-                }
-            }
-        }
-        __syncthreads();
-    }
-    float v[4], ss = 0.0f;
-#pragma unroll
-    for (int i = 0; i < 4; i++) {
-        v[i] = acc[0][i] / l[0];
-        if (a.maps == 2) v[i] -= a.lambda * (acc[1][i] / l[1]);
-        if (tid + i * 256 < a.vdim) ss += v[i] * v[i];
-    }
-    float f = 1.0f;
-    if (a.maps == 2) f = rsqrtf(lh_block_sum(ss, scratch) / (float)a.vdim + a.eps) * a.out_scale;
-#pragma unroll
-    for (int i = 0; i < 4; i++)
-        if (tid + i * 256 < a.vdim) lh_st(static_cast<T*>(a.out), ((size_t)t * a.heads + h) * a.vdim + tid + i * 256, v[i] * f);
-}
-
-constexpr uint32_t kMaxSplits = 512;
-
 template <int DQ, int DV, int MAPS>
 int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const char* op, uint32_t& launches) {
     const uint32_t R = a.heads / a.kv_heads;
@@ -509,7 +322,7 @@ int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const 
     a.partial = (float*)ctx->workspace;
     launches = 1;
     if (packed > 64) {
-        constexpr int NB = MAPS * DQ + DV <= 256 ? 2 : 1;
+        constexpr int NB = MAPS * DQ + DV <= (MAPS == 1 ? 320 : 256) ? 2 : 1;
         const uint64_t groups = (packed + 63) / 64 * a.kv_heads;
         // a share of eight key steps at least, and no more workgroups than two per CU
         a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({2 * cus / groups, max_blocks / (8 * NB), room}));
@@ -534,7 +347,8 @@ int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const 
 
 template <int DQ, int DV>
 int launch_maps(lh_context* ctx, AttentionArgs& a, uint32_t mp, const char* op, uint32_t& n) {
-    return a.maps == 2 ? launch_mfma<DQ, DV, 2>(ctx, a, mp, op, n) : launch_mfma<DQ, DV, 1>(ctx, a, mp, op, n);
+    if constexpr (DQ <= 128) if (a.maps == 2) return launch_mfma<DQ, DV, 2>(ctx, a, mp, op, n);
+    return launch_mfma<DQ, DV, 1>(ctx, a, mp, op, n);
 }
 template <int DQ>
 int launch_dv(lh_context* ctx, AttentionArgs& a, uint32_t mp, const char* op, uint32_t& n) {
@@ -550,12 +364,13 @@ int launch_dv(lh_context* ctx, AttentionArgs& a, uint32_t mp, const char* op, ui
 
 extern "C" {
 
-uint32_t lh_attention_padded_dim(uint32_t dim) { return dim <= 32 ? 32u : dim <= 64 ? 64u : (dim + 127) / 128 * 128; }
+uint32_t lh_attention_padded_dim(uint32_t dim) { return dim <= 32 ? 32u : dim <= 64 ? 64u : dim > 128 && dim <= 192 ? 192u : (dim + 127) / 128 * 128; }
 uint32_t lh_attention_padded_vdim(uint32_t vdim) { return vdim <= 32 ? 32u : vdim <= 64 ? 64u : vdim <= 128 ? 128u : (vdim + 255) / 256 * 256; }
 
 int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* keys, const lh_buffer* values, lh_buffer* output, int dtype,
                            const lh_buffer* position, uint32_t max_position, uint32_t rows, uint32_t heads, uint32_t kv_heads, uint32_t maps, uint32_t dim,
-                           uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps) {
+                           uint32_t vdim, uint32_t capacity, float scale, float lambda, float out_scale, float eps,
+                           const lh_buffer* sink, const lh_buffer* gate) {
     const char* op = "attention_rows";
     LH_REQUIRE(batch, "%s: batch is null", op);
     LH_REQUIRE(dtype == LH_F32 || dtype == LH_BF16, "%s: dtype %d", op, dtype);
@@ -577,18 +392,23 @@ int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_buffer*
     a.q = q->ptr; a.keys = keys->ptr; a.values = values->ptr; a.out = output->ptr; a.position = (const uint32_t*)position->ptr;
     a.rows = rows; a.heads = heads; a.kv_heads = kv_heads; a.maps = maps; a.dim = dim; a.vdim = vdim; a.capacity = capacity;
     a.scale = scale; a.lambda = lambda; a.out_scale = out_scale; a.eps = eps;
+    LH_REQUIRE(maps == 1 || (!sink && !gate), "%s: a sink or a gate with two maps", op);
+    if (sink) { LH_NEED(sink, (size_t)heads * 4, op, "sink"); a.sink = (const float*)sink->ptr; }
+    if (gate) { LH_NEED(gate, (size_t)rows * heads * 4, op, "gate"); a.gate = (const float*)gate->ptr; }
     const bool aligned = (((uintptr_t)a.q | (uintptr_t)a.keys | (uintptr_t)a.values | (uintptr_t)a.out) & 15) == 0;
     uint32_t launches = 0;
     int r;
-    if (dtype == LH_BF16 && aligned && a.dq <= 128 && a.dv <= 256) {
+    if (dtype == LH_BF16 && aligned && a.dq <= (maps == 2 ? 128u : 256u) && a.dv <= 256) {
         if (a.dq == 32) r = launch_dv<32>(batch->ctx, a, max_position, op, launches);
         else if (a.dq == 64) r = launch_dv<64>(batch->ctx, a, max_position, op, launches);
-        else r = launch_dv<128>(batch->ctx, a, max_position, op, launches);
+        else if (a.dq == 128) r = launch_dv<128>(batch->ctx, a, max_position, op, launches);
+        else if (a.dq == 192) r = launch_dv<192>(batch->ctx, a, max_position, op, launches);
+        else r = launch_dv<256>(batch->ctx, a, max_position, op, launches);
     } else {
         LH_REQUIRE((uint64_t)rows * heads < 0x7FFFFFFFull, "%s: %u rows", op, rows);
         const size_t lds = (size_t)maps * dim * 4;
-        if (dtype == LH_F32) hipLaunchKernelGGL((attention_plain_kernel<float>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
-        else hipLaunchKernelGGL((attention_plain_kernel<uint16_t>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
+        if (dtype == LH_F32) hipLaunchKernelGGL((attention_plain_kernel<float, float>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
+        else hipLaunchKernelGGL((attention_plain_kernel<uint16_t, uint16_t>), dim3(rows * heads), dim3(256), lds, batch->ctx->stream, a);
         launches = 1;
         r = lh_check_launch(op);
     }

@@ -332,6 +332,32 @@ class RecurrentState:
         self.state.fill_zero()
 
 
+class LatentCache:
+    """The rows of one latent-attention layer for one sequence, in the layout of ``lh_latent_prepare_into``: per position the
+    latent and the rotated key part that all heads share.  Layers that read another layer's rows hold the same object."""
+
+    def __init__(self, ctx, kernels: Kernels, rank: int, rot: int, capacity: int, dtype: int):
+        self.capacity = (capacity + 31) // 32 * 32
+        self.rows = Buffer.empty(ctx, self.capacity * kernels.latent_row(rank, rot) * (4 if dtype == F32 else 2))
+
+    def reset(self) -> None:
+        """Cleared for the same reason as ``BlockKvCache``."""
+        self.rows.fill_zero()
+
+
+class SelectiveState:
+    """The f32 memory of one selective state-space layer for one sequence: the recurrent state, and the last inputs of the
+    convolution in a ring over positions."""
+
+    def __init__(self, ctx, kernels: Kernels, heads: int, state: int, vdim: int, channels: int, taps: int):
+        self.state = Buffer.empty(ctx, heads * vdim * kernels.linear_attention_padded_dim(state) * 4)
+        self.ring = Buffer.empty(ctx, taps * channels * 4)
+
+    def reset(self) -> None:
+        self.state.fill_zero()
+        self.ring.fill_zero()
+
+
 class SequenceSlot:
     """Everything one live sequence holds: a cache or state per layer run, and its position on the host and on the device."""
 
@@ -343,7 +369,7 @@ class SequenceSlot:
         self.graph, self.graph_version, self.graph_ready = None, -1, False
 
     def reset(self) -> None:
-        for m in self.memories:
+        for m in {id(m): m for m in self.memories}.values():      # layers may share one
             m.reset()
         self.position_buf.fill_zero()
         self.position = 0

@@ -55,8 +55,10 @@ class StackedLinear:
     def bytes(self) -> int:
         return self.weight.length()
 
-    def rows_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, m: int, outputs, dtype: int, position=None) -> None:
-        kernels.linear_rows_into(batch, x, x_dtype, self.weight, self.bias, m, self.k, self.segments, outputs, dtype, False, position)
+    def rows_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, m: int, outputs, dtype: int, position=None,
+                  segments: Optional[Segments] = None) -> None:
+        kernels.linear_rows_into(batch, x, x_dtype, self.weight, self.bias, m, self.k, segments or self.segments, outputs, dtype,
+                                 False, position)
 
     def rows_add_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, m: int, residual: Buffer) -> None:
         kernels.linear_rows_into(batch, x, x_dtype, self.weight, self.bias, m, self.k, self.segments, [residual], F32, True)
@@ -64,7 +66,17 @@ class StackedLinear:
     def vector_add_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, residual: Buffer) -> None:
         kernels.linear_vector_into(batch, x, x_dtype, self.weight, self.bias, self.k, self.segments, [residual], F32, True)
 
+    def vector_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, outputs, dtype: int, position=None,
+                    segments: Optional[Segments] = None) -> None:
+        kernels.linear_vector_into(batch, x, x_dtype, self.weight, self.bias, self.k, segments or self.segments, outputs, dtype,
+                                   False, position)
+
+    def residual_vector_into(self, batch, kernels: Kernels, x: Buffer, branch: Buffer, store, norm: Buffer, eps: float, outputs,
+                             dtype: int, position=None, segments: Optional[Segments] = None) -> None:
+        kernels.linear_residual_vector_into(batch, x, branch, store, norm, eps, self.weight, self.bias, self.k,
+                                            segments or self.segments, outputs, dtype, False, position)
+
     def normed_vector_into(self, batch, kernels: Kernels, x: Buffer, norm: Buffer, eps: float, outputs, dtype: int,
-                           position=None, add=None, store=None) -> None:
-        kernels.linear_norm_vector_into(batch, x, add, store, norm, eps, self.weight, self.bias, self.k, self.segments,
-                                        outputs, dtype, False, position)
+                           position=None, add=None, store=None, segments: Optional[Segments] = None) -> None:
+        kernels.linear_norm_vector_into(batch, x, add, store, norm, eps, self.weight, self.bias, self.k,
+                                        segments or self.segments, outputs, dtype, False, position)

@@ -7,7 +7,8 @@ import os
 from typing import Callable, Dict
 
 from . import BF16, Context, InvalidArgument, Io, Kernels
-from .mixers import AttentionSpec, DenseSpec, LayerSpec, LinearAttentionSpec, MoeSpec
+from .mixers import (ACT_NONE, ACT_SILU, AttentionSpec, DenseSpec, GatedSpec, LatentAttentionSpec, LayerSpec, LinearAttentionSpec, MoeSpec,
+                     OutputNormLayer, SelectiveSpec)
 from .safetensors import SafetensorsFile
 from .stack_pipeline import Loop, StackConfig, StackPipeline
 
@@ -67,3 +68,28 @@ def komirax(config: dict) -> StackConfig:
     loop = config.get("loop")
     return StackConfig(config["vocab"], config["width"], config["norm"]["eps"], layers,
                        Loop(loop["start"], loop["stop"], loop["times"]) if loop else None)
+
+
+@register("Vifivik")
+def vifivik(config: dict) -> StackConfig:
+    """Latent-attention, retention and Mamba-2 layers in any order, gated feed-forwards, norms behind the branches, capped logits."""
+    def mixer(kind, m):
+        if kind == "latent_attention":
+            if m["rot"]["dims"] != m["rot_dim"]:
+                raise InvalidArgument(f"{m['rot']['dims']} rotated dimensions of a rotated part of {m['rot_dim']}")
+            return LatentAttentionSpec(m["heads"], m["dim"], m["rot_dim"], m["vdim"], m["kv_rank"], m["rot"]["base"], m["scale"], m.get("kv_from"))
+        if kind == "retention":
+            return LinearAttentionSpec(m["heads"], m["dim"], m["vdim"], list(m["decay"]), ACT_NONE, m["dim"] ** -0.5, ACT_SILU, head_norm=True)
+        if kind == "mamba2":
+            return SelectiveSpec(m["heads"], m["vdim"], m["state"], m["groups"], m["conv"], m["norm_groups"])
+        raise InvalidArgument(f"unknown layer type {kind!r}")
+
+    def feed_forward(f):
+        if f is None:
+            return None
+        if f["kind"] == "dense":
+            return GatedSpec(f["ff"])
+        raise InvalidArgument(f"unknown feed-forward {f['kind']!r}")
+
+    layers = [LayerSpec(mixer(l["type"], l["mixer"]), feed_forward(l.get("mlp"))) for l in config["layers"]]
+    return StackConfig(config["vocab"], config["width"], config["norm"]["eps"], layers, layer=OutputNormLayer, softcap=config["logit_softcap"])

@@ -1,16 +1,16 @@
-"""Pipeline of a stack of pre-norm layers with bf16 weights (mixers.py): embedding, layer runs in order -- a range of layers
-may run several times in a row -- final norm and head, over the caches and states of sequence slots."""
+"""Pipeline of a stack of layers with bf16 weights (mixers.py): embedding, layer runs in order -- a range of layers may run
+several times in a row -- final norm and head, over the caches and states of sequence slots."""
 from __future__ import annotations
 
 from dataclasses import dataclass
-from typing import List, Optional, Sequence, Tuple
+from typing import List, Optional, Sequence, Tuple, Type
 
 import numpy as np
 
 from . import BF16, F32, Buffer, CommandBatch, InvalidArgument, Kernels
 from .kv_cache import SequenceSlot, SlotPool
 from .linear_weight import Segment, StackedLinear
-from .mixers import LayerSpec, Norm, PreNormLayer, Run, Workspace
+from .mixers import LatentAttentionSpec, LayerSpec, Norm, OutputNormLayer, PreNormLayer, Run, Workspace
 
 DEFAULT_MAX_ROWS = 2048     # rows of one pass; longer portions go through in pieces
 
@@ -30,6 +30,8 @@ class StackConfig:
     eps: float
     layers: List[LayerSpec]
     loop: Optional[Loop] = None
+    layer: Type[PreNormLayer] = PreNormLayer     # where the norms are
+    softcap: Optional[float] = None              # logits become softcap * tanh(logits / softcap)
 
     def runs(self) -> List[Tuple[int, bool]]:
         """[(layer, whether the embedding output is added before it)] in running order."""
@@ -42,6 +44,24 @@ class StackConfig:
         return ([(i, False) for i in range(a)] + [(i, p > 0 and i == a) for p in range(t) for i in range(a, b)]
                 + [(i, False) for i in range(b, n)])
 
+    def check(self) -> None:
+        """Refuses what no pipeline can run."""
+        if self.loop is not None and issubclass(self.layer, OutputNormLayer):
+            raise InvalidArgument("layers with norms behind the branches do not repeat")
+        if self.softcap is not None and not self.softcap > 0:
+            raise InvalidArgument(f"logits capped at {self.softcap}")
+        for i, l in enumerate(self.layers):
+            m = l.mixer
+            if not isinstance(m, LatentAttentionSpec) or m.kv_from is None:
+                continue
+            j = self.layers[m.kv_from].mixer if 0 <= m.kv_from < i else None
+            if not isinstance(j, LatentAttentionSpec) or j.kv_from is not None:
+                raise InvalidArgument(f"layer {i} reads the cache of layer {m.kv_from}, which is no earlier layer with one of its own")
+            if (j.kv_rank, j.rot_dim, j.rot_base) != (m.kv_rank, m.rot_dim, m.rot_base):
+                raise InvalidArgument(f"layer {i} reads the cache of layer {m.kv_from}, whose rows are others")
+            if self.loop is not None:
+                raise InvalidArgument("layers that share a cache do not repeat")
+
 
 class StackPipeline:
     """Serves one sequence per slot; the calls are those of generation.SequenceModel."""
@@ -50,11 +70,12 @@ class StackPipeline:
                  max_sequences: int = 1, max_rows: int = DEFAULT_MAX_ROWS, graphs: bool = True):
         if dtype not in (BF16, F32):
             raise InvalidArgument("activations are bf16 or f32")
+        config.check()
         self.ctx, self.kernels, self.config, self.dtype, self.graphs = ctx, kernels, config, dtype, graphs
         self.vocab_size, self.max_rows = config.vocab, max_rows
         self.max_tokens = max(max_tokens, 1)
         w = config.width
-        self.layers = [PreNormLayer(ctx, kernels, s, w, config.eps, tensors, f"l{i}.") for i, s in enumerate(config.layers)]
+        self.layers = [config.layer(ctx, kernels, s, w, config.eps, tensors, f"l{i}.") for i, s in enumerate(config.layers)]
         self.runs = config.runs()
         self.embed = Buffer.from_slice(ctx, tensors.bf16("embed", (config.vocab, w)))
         self.final_norm = Norm(ctx, tensors.f32("final.norm", (w,)), config.eps)
@@ -67,8 +88,12 @@ class StackPipeline:
         self.observe = None          # called with (run index, residual stream buffer, rows) after every layer run
 
     def _new_slot(self) -> SequenceSlot:
-        return SequenceSlot(self.ctx, [self.layers[i].mixer.memory(self.ctx, self.kernels, self.max_tokens, self.dtype)
-                                       for i, _ in self.runs])
+        memories = []
+        for i, _ in self.runs:
+            mixer = self.layers[i].mixer
+            source = getattr(mixer, "source", None)         # the layer whose memory this one reads
+            memories.append(mixer.memory(self.ctx, self.kernels, self.max_tokens, self.dtype) if source is None else memories[source])
+        return SequenceSlot(self.ctx, memories)
 
     # ---- sequences ------------------------------------------------------------------------------------------------------
     def new_sequence(self) -> SequenceSlot:
@@ -120,7 +145,9 @@ class StackPipeline:
                 r.store = (y if r.x is x else x) if n == 1 else r.x
             self.layers[layer].run(r, memory)
             if self.observe is not None:
+                Norm.flush(r)
                 self.observe(i, r.x, n)
+        Norm.flush(r)
         return r.x
 
     def _forward(self, seq: SequenceSlot, tokens, want) -> Optional[np.ndarray]:
@@ -146,12 +173,18 @@ class StackPipeline:
             h = self.ws.get("wanted", m * width * size)
             K.norm_rows_f32_into(batch, x, None, self.final_norm.weight, None, index, h, self.dtype, width, m, self.config.eps)
             self.head.rows_into(batch, K, h, self.dtype, m, [logits], F32)
+            self._encode_cap(batch, logits, m)
         batch.commit_and_wait()
         seq.position += n
         return logits.as_array(np.float32, len(want) * self.vocab_size).reshape(len(want), -1) if want else None
 
     def _encode_head(self, batch, row: Buffer) -> None:
         self.head.normed_vector_into(batch, self.kernels, row, self.final_norm.weight, self.config.eps, [self.logits_buf], F32)
+        self._encode_cap(batch, self.logits_buf, 1)
+
+    def _encode_cap(self, batch, logits: Buffer, rows: int) -> None:
+        if self.config.softcap is not None:
+            self.kernels.softcap_f32_into(batch, logits, rows * self.vocab_size, self.config.softcap)
 
     def _encode_decode(self, batch, seq: SequenceSlot, max_position: int) -> None:
         self._encode_head(batch, self._encode_stack(batch, seq, 1, max_position))
