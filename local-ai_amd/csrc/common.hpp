@@ -7,6 +7,7 @@
 #include <vector>
 #include "../../include/local_hip.h"
 
+struct lh_graph;
 struct lh_context {
     int device;
     hipStream_t stream;
@@ -25,6 +26,8 @@ struct lh_context {
     // Owning buffers released while a capture is open.  A recorded dispatch may reference them, so they live as long as
     // the graph the capture produces (lh_graph_free releases them); when the capture fails they go when it ends.
     std::vector<void*> deferred_free;
+    // Graphs released while a capture is open; they go when it ends.
+    std::vector<lh_graph*> deferred_graphs;
     // Pinned staging for descriptor tables of grouped launches: a small ring of slots, each guarded by an event that is
     // recorded behind the slot's copy, so a slot is rewritten only after the copy that read it has run.
     static constexpr int kDescSlots = 4;

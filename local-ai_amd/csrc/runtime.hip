@@ -453,6 +453,9 @@ int lh_batch_end_capture(lh_batch* batch, lh_graph** out) {
     ctx->capturing = false;
     hipGraph_t graph = nullptr;
     hipError_t e = hipStreamEndCapture(ctx->stream, &graph);
+    std::vector<lh_graph*> graphs;
+    graphs.swap(ctx->deferred_graphs);
+    for (lh_graph* old : graphs) lh_graph_free(old);
     std::vector<void*> released;
     released.swap(ctx->deferred_free);
     auto drop_released = [&]() {   // no graph will replay: nothing can reference them once the stream is idle
@@ -496,6 +499,7 @@ uint32_t lh_graph_dispatch_count(const lh_graph* graph) { return graph ? graph->
 
 void lh_graph_free(lh_graph* graph) {
     if (!graph) return;
+    if (graph->ctx->capturing) { graph->ctx->deferred_graphs.push_back(graph); return; }   // its memory may not be freed inside a capture
     (void)hipStreamSynchronize(graph->ctx->stream);   // a replay may still be running
     (void)hipGraphExecDestroy(graph->exec);
     (void)hipGraphDestroy(graph->graph);

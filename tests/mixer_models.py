@@ -39,9 +39,86 @@ def config(vocab, width, layers, loop=None, eps=1e-5):
     return {"architecture": "Komirax", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers, "loop": loop}
 
 
+# ---- Vifivik -------------------------------------------------------------------------------------------------------------
+def latent(heads, dim, rot, vdim, rank, scale=None, base=10000.0, kv_from=None, ff=None):
+    m = {"heads": heads, "dim": dim, "rot_dim": rot, "vdim": vdim, "kv_rank": rank, "rot": {"base": base, "dims": rot},
+         "scale": (dim + rot) ** -0.5 if scale is None else scale}
+    if kv_from is not None:
+        m["kv_from"] = kv_from
+    return {"type": "latent_attention", "mixer": m, "mlp": ff and dense(ff)}
+
+
+def retention(heads, dim, vdim, decay=None, ff=None):
+    decay = list(1.0 - 2.0 ** -np.linspace(2, 9, heads)) if decay is None else decay
+    return {"type": "retention", "mixer": {"heads": heads, "dim": dim, "vdim": vdim, "decay": decay}, "mlp": ff and dense(ff)}
+
+
+def mamba2(heads, vdim, state, groups=1, conv=4, norm_groups=1, ff=None):
+    return {"type": "mamba2", "mlp": ff and dense(ff), "mixer": {"heads": heads, "vdim": vdim, "state": state, "groups": groups,
+                                                                 "conv": conv, "norm_groups": norm_groups}}
+
+
+def vifivik(vocab, width, layers, eps=1e-5, cap=20.0):
+    return {"architecture": "Vifivik", "vocab": vocab, "width": width, "norm": {"eps": eps}, "layers": layers, "logit_softcap": cap}
+
+
+def vifivik_weights(cfg, seed):
+    """name -> bf16 bits.  Queries and latents are large enough for the softmax to have favourites; sinks, step biases and decay
+    rates differ from head to head."""
+    g = np.random.default_rng(seed)
+    w, v, t = cfg["width"], cfg["vocab"], {}
+
+    def mat(name, rows, cols, scale=1.0):
+        t[name] = g.standard_normal((rows, cols)) * (scale / np.sqrt(cols))
+
+    def norm(name, n, mean=1.0):
+        t[name] = mean + 0.1 * g.standard_normal(n)
+    t["embed"] = g.standard_normal((v, w))
+    for i, l in enumerate(cfg["layers"]):
+        p, m = f"l{i}.mix.", l["mixer"]
+        norm(f"l{i}.norm1", w, 0.5)
+        if l["type"] == "latent_attention":
+            H, d, e, r = m["heads"], m["dim"], m["rot_dim"], m["kv_rank"]
+            mat(p + "q", H * (d + e), w, 1.5)
+            if "kv_from" not in m:
+                mat(p + "dkv", r + e, w)
+                norm(p + "dkv.norm", r)
+            mat(p + "uk", H * d, r)
+            mat(p + "uv", H * m["vdim"], r)
+            t[p + "sink"] = 1.5 * g.standard_normal(H)
+            mat(p + "g", H, w)
+            mat(p + "o", w, H * m["vdim"])
+        elif l["type"] == "retention":
+            nk, nv = m["heads"] * m["dim"], m["heads"] * m["vdim"]
+            for n, c in (("q", nk), ("k", nk), ("v", nv), ("g", nv)):
+                mat(p + n, c, w)
+            mat(p + "o", w, nv)
+        else:
+            inner, ch, H = m["heads"] * m["vdim"], m["heads"] * m["vdim"] + 2 * m["groups"] * m["state"], m["heads"]
+            mat(p + "in", inner + ch + H, w)
+            mat(p + "conv", ch, m["conv"], 1.5)
+            t[p + "conv.b"] = 0.2 * g.standard_normal(ch)
+            t[p + "dt_bias"] = np.linspace(-5.0, -0.5, H) if H > 1 else np.array([-3.0])
+            t[p + "A_log"] = np.linspace(2.0, -1.0, H) if H > 1 else np.array([0.5])
+            t[p + "D"] = g.standard_normal(H)
+            norm(p + "norm", inner)
+            mat(p + "o", w, inner)
+        if l["mlp"]:
+            norm(f"l{i}.norm2", w, 0.5)
+            ff = l["mlp"]["ff"]
+            mat(f"l{i}.mlp.gate", ff, w)
+            mat(f"l{i}.mlp.up", ff, w)
+            mat(f"l{i}.mlp.down", w, ff)
+    norm("final.norm", w)
+    mat("head", v, w, 4.0)
+    return {n: bf16_bits(x) for n, x in t.items()}
+
+
 def weights(cfg, seed):
     """name -> bf16 bits.  Output projections are scaled down and the embeddings carry evenly spaced components along the
     routers' (orthonormal) directions, so that no routing decision is a close call and bf16 runs pick the same experts."""
+    if cfg["architecture"] == "Vifivik":
+        return vifivik_weights(cfg, seed)
     g = np.random.default_rng(seed)
     w, v = cfg["width"], cfg["vocab"]
     t = {}

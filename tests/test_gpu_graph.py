@@ -128,3 +128,25 @@ def test_buffer_released_during_capture_lives_as_long_as_the_graph(pkg, gpu):
         got = out.as_array(np.float16, n).astype(np.float32)
         assert (got == 1.5 + step + 4.0).all(), f"replay {step}: {got[:4]}"
     graph.free()
+
+
+def test_graph_released_during_capture_does_not_disturb_it(pkg, gpu):
+    """An older graph may be collected at any time, also while another is being recorded."""
+    ctx, K = gpu
+    n = 4096
+    a, out = pkg.Buffer.from_slice(ctx, np.full(n, 1.5, np.float16)), pkg.Buffer.empty(ctx, n * 2)
+    batch = pkg.CommandBatch(ctx)
+    batch.begin_capture()
+    K.residual_add_into(batch, a, a, out, n)
+    old = batch.end_capture()
+    batch.begin_capture()
+    K.residual_add_into(batch, a, a, out, n)
+    old.free()
+    K.residual_add_into(batch, out, a, out, n)
+    graph = batch.end_capture()
+    for step in range(3):
+        a.copy_from_bytes(np.full(n, 1.0 + step, np.float16))
+        graph.launch()
+        ctx.synchronize()
+        assert (out.as_array(np.float16, n) == 3.0 + 3 * step).all()
+    graph.free()

@@ -30,6 +30,18 @@ CONFIGS = {
     "attention_only": lambda: M.config(200, 128, [M.attention(8, 2, 64, 128, mlp=M.dense(96)), M.attention(2, 1, 128, 64, mlp=None)]),
     "lightning_only": lambda: M.config(77, 72, [M.lightning(4, 72, 136, mlp=M.moe(3, 3, 48)), M.lightning(5, 33, 40, mlp=M.dense(200))],
                                        {"start": 1, "stop": 2, "times": 1}),
+    # norms behind the branches
+    "latent_and_states": lambda: M.vifivik(90, 80, [M.latent(5, 24, 8, 40, 48, ff=72), M.retention(3, 40, 24, ff=56), M.latent(5, 24, 8, 40, 48, kv_from=0, ff=40),
+                                                    M.mamba2(6, 24, 20, 2, 4, 2, ff=64), M.latent(6, 16, 12, 24, 96)]),
+    "latent_shared": lambda: M.vifivik(64, 96, [M.mamba2(2, 48, 32, 1, 3, 1), M.latent(8, 32, 32, 64, 160, base=500.0, ff=48),
+                                                M.latent(3, 56, 32, 24, 160, base=500.0, kv_from=1, scale=0.3), M.latent(4, 16, 32, 16, 160, base=500.0, kv_from=1, ff=32)],
+                                       eps=1e-3, cap=5.0),
+    # (enough values per branch that none of them happens to vanish, where the norm behind it would amplify rounding)
+    "latent_ragged": lambda: M.vifivik(51, 30, [M.latent(3, 5, 6, 7, 11, ff=13), M.retention(3, 9, 11), M.mamba2(3, 7, 5, 3, 2, 1, ff=9), M.latent(5, 1, 2, 9, 13)]),
+    "latent_wide": lambda: M.vifivik(72, 128, [M.latent(3, 128, 64, 128, 512, ff=96), M.latent(16, 72, 20, 136, 264), M.latent(1, 200, 40, 48, 64)]),
+    "latent_beyond_the_tiles": lambda: M.vifivik(40, 64, [M.latent(2, 40, 72, 24, 96), M.latent(2, 264, 16, 300, 640, ff=24)]),
+    "states_only": lambda: M.vifivik(77, 72, [M.mamba2(6, 20, 130, 3, 5, 2, ff=40), M.mamba2(2, 64, 300, 1, 1, 2), M.retention(2, 128, 64, [1.0, 0.25], ff=64),
+                                              M.mamba2(8, 128, 64, 8, 4, 8), M.retention(4, 33, 72)]),
     "wide_heads": lambda: M.config(40, 64, [M.attention(2, 1, 160, 320), M.lightning(2, 288, 24)]),
 }
 
@@ -82,7 +94,7 @@ def test_prompt_portions_and_decoding_agree_with_the_plain_statement(ai, gpu, na
         check(feed(m, tokens, cuts), want, dtype, f"{name} {what}")
 
 
-@pytest.mark.parametrize("name", ["both", "loop_all"])
+@pytest.mark.parametrize("name", ["both", "loop_all", "latent_and_states", "latent_shared"])
 def test_residual_stream_after_every_layer_run(ai, gpu, name):
     cfg, w, m = build(ai, gpu, name)
     tokens = [int(t) for t in np.random.default_rng(6).integers(0, cfg["vocab"], 23)]
@@ -157,10 +169,88 @@ def test_far_token_decides_through_the_caches(ai, gpu, dtype):
         check(got, want[900:], dtype, f"far token {cuts[:3]}")
 
 
+@pytest.mark.parametrize("sink", [None, 25.0])
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
-def test_slots_used_again_and_interleaved_sequences(ai, gpu, dtype):
+def test_far_token_decides_through_the_latent_cache(ai, gpu, dtype, sink):
+    """As above through latents, in a layer of its own and in one that reads its cache.  With a large sink, which takes nearly all
+    of every softmax, the favourite's share stays in the right proportion to it."""
+    ctx, K = gpu
+    V, W, R = 40, 160, 64
+    layers = [M.latent(1, 32, 2, 32, R, scale=1.0), M.latent(1, 32, 2, 32, R, scale=1.0, kv_from=0)]
+    cfg = M.vifivik(V, W, layers, cap=30.0)
+    t = {n: np.zeros_like(x) for n, x in M.weights(cfg, 3).items()}
+    g = np.random.default_rng(8)
+    keys = np.linalg.qr(g.standard_normal((32, 32)))[0]
+    e = np.zeros((V, W))
+    e[:32, :32] = keys * 6                            # the latent's first half; the second half is the value
+    e[:32, 32:64] = np.eye(32) * 6
+    e[32:, 64:96] = keys[:8] * 6                      # token 32 + i asks for the key of token i
+    t["embed"] = M.bf16_bits(e)
+    for n in ("l0.norm1", "l1.norm1"):
+        t[n] = M.bf16_bits(np.full(W, 0.5))
+    t["final.norm"] = M.bf16_bits(np.ones(W))
+    for i in range(2):
+        p = f"l{i}.mix."
+        q = np.zeros((34, W))
+        q[:32, 64:96] = np.eye(32)
+        t[p + "q"] = M.bf16_bits(q)
+        uk, uv = np.zeros((32, R)), np.zeros((32, R))
+        uk[:, :32], uv[:, 32:] = np.eye(32), np.eye(32)
+        t[p + "uk"], t[p + "uv"] = M.bf16_bits(uk), M.bf16_bits(uv)
+        t[p + "sink"] = M.bf16_bits(np.array([-20.0 if sink is None else sink]))
+        o = np.zeros((W, 32))
+        o[96 + 32 * i:128 + 32 * i] = np.eye(32)
+        t[p + "o"] = M.bf16_bits(o)
+    dkv = np.zeros((R + 2, W))
+    dkv[:R, :R] = np.eye(R)
+    t["l0.mix.dkv"], t["l0.mix.dkv.norm"] = M.bf16_bits(dkv), M.bf16_bits(np.ones(R))
+    head = np.zeros((V, W))
+    head[:32, 96:128], head[:32, 128:160] = np.eye(32) * 3, np.eye(32) * 3
+    t["head"] = M.bf16_bits(head)
+    m = ai.stack_pipeline.StackPipeline(ctx, K, ai.registry.read_config(cfg), M.Tensors(t), 1024, ai.F32 if dtype == "float32" else ai.BF16)
+    w = M.plain_weights(t)
+    places = [0, 1, 31, 32, 33, 63, 64, 500]
+    tokens = [9] * 900
+    for i, p in enumerate(places):
+        tokens[p] = i
+    tokens += [32 + i for i in range(8)]
+    want = O.forward(cfg, w, tokens)
+    assert [int(r[:32].argmax()) for r in want[900:]] == list(range(8)) and np.abs(want[900:]).max() > 1
+    for cuts in ([908], [900] + [1] * 8, [898, 2] + [3, 5], cuts_of(908, [64, 37, 2, 66])):
+        s, at, got = m.new_sequence(), 0, []
+        for c in cuts:
+            wanted = [i for i in range(c) if at + i >= 900]
+            got.append(m.step(s, tokens[at:at + c], wanted))
+            at += c
+        m.end_sequence(s)
+        got = np.concatenate([x for x in got if len(x)])
+        assert [int(r[:32].argmax()) for r in got] == list(range(8)), cuts[:3]
+        check(got, want[900:], dtype, f"far token {cuts[:3]}")
+
+
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_the_first_tokens_reach_the_last_through_the_states(ai, gpu, dtype):
+    """State layers alone, with decays near one: exchanging the very first token moves the last logits, by the plain statement's
+    amount, whether the tokens between were a prompt, portions or decoded."""
+    ctx, K = gpu
+    cfg = M.vifivik(30, 64, [M.retention(2, 32, 32, [1.0, 0.9999]), M.mamba2(2, 32, 32)])
+    t = M.weights(cfg, 4)
+    t["l1.mix.dt_bias"], t["l1.mix.A_log"] = M.bf16_bits(np.array([-4.0, -2.0])), M.bf16_bits(np.array([-6.0, -7.0]))
+    m = ai.stack_pipeline.StackPipeline(ctx, K, ai.registry.read_config(cfg), M.Tensors(t), 400, ai.F32 if dtype == "float32" else ai.BF16)
+    w, tokens = M.plain_weights(t), [int(x) for x in np.random.default_rng(3).integers(0, 30, 300)]
+    other = [(tokens[0] + 1) % 30] + tokens[1:]
+    a, b = O.forward(cfg, w, tokens), O.forward(cfg, w, other)
+    assert np.abs(a[-1] - b[-1]).max() > 0.01 * a.std()
+    for cuts in ([300], [1] * 300, cuts_of(300, [2, 65, 17])):
+        check(feed(m, tokens, cuts), a, dtype, f"{cuts[:3]}")
+        check(feed(m, other, cuts), b, dtype, f"{cuts[:3]}")
+
+
+@pytest.mark.parametrize("name", ["both", "latent_and_states"])
+@pytest.mark.parametrize("dtype", ["float32", "bfloat16"])
+def test_slots_used_again_and_interleaved_sequences(ai, gpu, name, dtype):
     """A long sequence, then shorter ones in the same slot; three live sequences that take turns of unequal size."""
-    cfg, w, m = build(ai, gpu, "both", dtype, max_tokens=300, max_sequences=3)
+    cfg, w, m = build(ai, gpu, name, dtype, max_tokens=300, max_sequences=3)
     g = np.random.default_rng(9)
     seqs = [[int(t) for t in g.integers(0, cfg["vocab"], n)] for n in (290, 3, 77, 1, 150)]
     want = [O.forward(cfg, w, t) for t in seqs]
@@ -180,10 +270,12 @@ def test_slots_used_again_and_interleaved_sequences(ai, gpu, dtype):
     assert m.slots.available() == 3
 
 
-def test_recorded_decoding_equals_unrecorded_bit_for_bit(ai, gpu):
-    """The recorded step is replayed between other sequences' prompts, which also make the scratch buffers move."""
-    cfg, _, m = build(ai, gpu, "both", "bfloat16", max_tokens=400, max_sequences=2)
-    _, _, plain = build(ai, gpu, "both", "bfloat16", max_tokens=400, max_sequences=2, graphs=False)
+@pytest.mark.parametrize("name", ["both", "latent_and_states", "latent_wide"])
+def test_recorded_decoding_equals_unrecorded_bit_for_bit(ai, gpu, name):
+    """The recorded step is replayed between other sequences' prompts, which also make the scratch buffers move.  (So short a cache
+    is not split, so that both forms add up in the same order.)"""
+    cfg, _, m = build(ai, gpu, name, "bfloat16", max_tokens=120, max_sequences=2)
+    _, _, plain = build(ai, gpu, name, "bfloat16", max_tokens=120, max_sequences=2, graphs=False)
     g = np.random.default_rng(10)
     tokens = [int(t) for t in g.integers(0, cfg["vocab"], 120)]
 
@@ -204,8 +296,9 @@ def test_recorded_decoding_equals_unrecorded_bit_for_bit(ai, gpu):
     assert rec_a and not rec_b and np.array_equal(a, b)
 
 
-def test_long_decoding(ai, gpu):
-    cfg, w, m = build(ai, gpu, "loop_all", max_tokens=700)
+@pytest.mark.parametrize("name", ["loop_all", "latent_and_states"])
+def test_long_decoding(ai, gpu, name):
+    cfg, w, m = build(ai, gpu, name, max_tokens=700)
     tokens = [int(t) for t in np.random.default_rng(11).integers(0, cfg["vocab"], 640)]
     want = O.forward(cfg, w, tokens)
     check(feed(m, tokens, [1] * 640), want, "float32", "640 decoded tokens")
@@ -236,9 +329,10 @@ def greedy_of(cfg, w, prompt, n):
     return out
 
 
+@pytest.mark.parametrize("name", ["both", "latent_and_states", "latent_shared"])
 @pytest.mark.parametrize("portion", [5, 512])
-def test_greedy_generation_through_the_scheduler(ai, gpu, portion):
-    cfg, w, m = build(ai, gpu, "both", max_tokens=120, max_sequences=2)
+def test_greedy_generation_through_the_scheduler(ai, gpu, name, portion):
+    cfg, w, m = build(ai, gpu, name, max_tokens=120, max_sequences=2)
     g, gen = np.random.default_rng(13), ai.generation
     prompts = [[int(t) for t in g.integers(0, cfg["vocab"], n)] for n in (4, 33, 1, 70)]
     sch = gen.Scheduler(m, portion)
@@ -252,9 +346,10 @@ def test_greedy_generation_through_the_scheduler(ai, gpu, portion):
     assert r.tokens == reqs[1].tokens[:12]
 
 
-def test_command_line_and_trace_from_a_model_folder(ai, gpu, tmp_path, capsys, monkeypatch):
+@pytest.mark.parametrize("name", ["both", "latent_and_states"])
+def test_command_line_and_trace_from_a_model_folder(ai, gpu, tmp_path, capsys, monkeypatch, name):
     from local_ai_amd import cli, trace
-    cfg = CONFIGS["both"]()
+    cfg = CONFIGS[name]()
     t = M.weights(cfg, 21)
     (tmp_path / "config.json").write_text(json.dumps(cfg))
     ai.safetensors.write(str(tmp_path / "model.safetensors"), t)

@@ -90,6 +90,124 @@ def test_registry_reads_the_configuration(ai):
         ai.stack_pipeline.StackConfig(8, 8, 1e-6, c.layers, ai.stack_pipeline.Loop(2, 5, 2)).runs()
 
 
+def _vifivik():
+    return M.vifivik(23, 16, [M.latent(2, 4, 6, 5, 8, base=100.0, ff=12), M.retention(2, 4, 5, [0.5, 0.75]), M.mamba2(4, 3, 5, 2, 3, 2, ff=7),
+                              M.latent(3, 2, 6, 7, 8, base=100.0, kv_from=0)], cap=9.0)
+
+
+def test_registry_reads_a_stack_with_norms_behind_the_branches(ai):
+    X, c = ai.mixers, ai.registry.read_config(_vifivik())
+    c.check()
+    assert c.layer is X.OutputNormLayer and c.softcap == 9.0 and c.loop is None and (c.vocab, c.width, c.eps) == (23, 16, 1e-5)
+    assert c.layers[0] == X.LayerSpec(X.LatentAttentionSpec(2, 4, 6, 5, 8, 100.0, 10 ** -0.5), X.GatedSpec(12))
+    assert c.layers[1] == X.LayerSpec(X.LinearAttentionSpec(2, 4, 5, [0.5, 0.75], ai.ACT_NONE, 0.5, ai.ACT_SILU, True))
+    assert c.layers[2] == X.LayerSpec(X.SelectiveSpec(4, 3, 5, 2, 3, 2), X.GatedSpec(7)) and c.layers[3].mixer.kv_from == 0
+
+    def broken(change):
+        d = _vifivik()
+        change(d)
+        with pytest.raises(ai.InvalidArgument):
+            ai.registry.read_config(d).check()
+    broken(lambda d: d["layers"][3]["mixer"].update(kv_from=1))        # no latent layer
+    broken(lambda d: d["layers"][3]["mixer"].update(kv_from=3))        # not an earlier one
+    broken(lambda d: d["layers"][3]["mixer"].update(kv_rank=9))
+    broken(lambda d: d["layers"][3]["mixer"]["rot"].update(base=7.0))
+    broken(lambda d: d["layers"][0]["mixer"]["rot"].update(dims=4))
+    broken(lambda d: d["layers"][0].update(type="attention"))
+    broken(lambda d: d["layers"][0]["mlp"].update(kind="moe"))
+    broken(lambda d: d["layers"][2]["mixer"].pop("state"))
+    broken(lambda d: d.update(logit_softcap=0.0))
+
+
+# ---- the plain statement of Vifivik's mechanisms ------------------------------------------------------------------------
+def test_rotation_keeps_lengths_and_depends_on_the_distance():
+    g = np.random.default_rng(1)
+    q, k = g.standard_normal(8), g.standard_normal(8)
+
+    def at(x, p):
+        return O.rotate_pairs(x[None], [p], 50.0)[0]
+    assert np.allclose(at(q, 0), q) and np.isclose(at(q, 17) @ at(q, 17), q @ q)
+    assert np.isclose(at(q, 9) @ at(k, 4), at(q, 105) @ at(k, 100)) and not np.isclose(at(q, 9) @ at(k, 4), at(q, 9) @ at(k, 5))
+    assert np.allclose(at(np.array([1.0, 0, 0, 0]), 2), [np.cos(2), np.sin(2), 0, 0])       # the pair is (0, 1), the angle counts up
+
+
+def test_sink_takes_its_share_once():
+    g = np.random.default_rng(2)
+    q, k, v = g.standard_normal((5, 3)), g.standard_normal((5, 3)), g.standard_normal((5, 4))
+    plain, sunk = O.causal_softmax_attention(q, k, v, 0.7, 0), O.sink_softmax_attention(q, k, v, 0.7, 1.3, 0)
+    for i in range(5):
+        z = np.exp(0.7 * (k[:i + 1] @ q[i])).sum()
+        assert np.allclose(sunk[i], plain[i] * z / (z + np.exp(1.3)))
+    assert np.allclose(O.sink_softmax_attention(q, k, v, 0.7, -100.0, 0), plain)
+
+
+def test_latent_mixer_is_the_same_in_the_latent_space_and_in_portions():
+    """Queries through the key projection and outputs through the value projection give what keys and values of every head give."""
+    g = np.random.default_rng(3)
+    H, d, e, n, r, W, T = 2, 3, 4, 5, 6, 7, 9
+    w = {k: g.standard_normal(s) for k, s in (("q", (H * (d + e), W)), ("dkv", (r + e, W)), ("dkv.norm", (r,)), ("uk", (H * d, r)), ("uv", (H * n, r)),
+                                              ("sink", (H,)), ("g", (H, W)), ("o", (W, H * n)))}
+    h = g.standard_normal((T, W))
+    c, kr = O.latent_rows(h, w, r, 30.0, 1e-5, 0)
+    y = O.latent_mixer(h, w, H, d, e, n, 30.0, 0.4, c, kr, 0)
+    q = (h @ w["q"].T).reshape(T, H, d + e)
+    o = []
+    for i in range(H):
+        ql = np.concatenate([q[:, i, :d] @ w["uk"].reshape(H, d, r)[i], O.rotate_pairs(q[:, i, d:], range(T), 30.0)], axis=1)
+        ol = O.sink_softmax_attention(ql, np.concatenate([c, kr], 1), c, 0.4, w["sink"][i], 0)
+        o.append(O.sigmoid(h @ w["g"][i])[:, None] * (ol @ w["uv"].reshape(H, n, r)[i].T))
+    assert np.allclose(np.concatenate(o, 1) @ w["o"].T, y)
+    c2, kr2 = O.latent_rows(h[4:], w, r, 30.0, 1e-5, 4)
+    assert np.allclose(c2, c[4:]) and np.allclose(kr2, kr[4:])
+    assert np.allclose(O.latent_mixer(h[4:], w, H, d, e, n, 30.0, 0.4, c, kr, 4), y[4:])
+
+
+def test_selective_recurrence_is_the_decayed_sum():
+    g = np.random.default_rng(4)
+    T, H, G, N, e = 7, 4, 2, 3, 2
+    x, B, C, dt = g.standard_normal((T, H, e)), g.standard_normal((T, G, N)), g.standard_normal((T, G, N)), g.random((T, H))
+    a_log, D = g.standard_normal(H), g.standard_normal(H)
+    y, S = O.selective_recurrence(x, B, C, dt, a_log, D)
+    for t in range(T):
+        for h in range(H):
+            want = D[h] * x[t, h]
+            for s in range(t + 1):
+                want = want + np.exp(-np.exp(a_log[h]) * dt[s + 1:t + 1, h].sum()) * dt[s, h] * (B[s, h // 2] @ C[t, h // 2]) * x[s, h]
+            assert np.allclose(y[t, h], want)
+    y1, S1 = O.selective_recurrence(x[:3], B[:3], C[:3], dt[:3], a_log, D)
+    y2, S2 = O.selective_recurrence(x[3:], B[3:], C[3:], dt[3:], a_log, D, S1)
+    assert np.allclose(np.concatenate([y1, y2]), y) and np.allclose(S2, S)
+
+
+@pytest.mark.parametrize("taps", [1, 2, 4])
+def test_causal_convolution_and_grouped_norm(taps):
+    g = np.random.default_rng(5)
+    x, w, b = g.standard_normal((6, 3)), g.standard_normal((3, taps)), g.standard_normal(3)
+    y, past = O.causal_conv(x, np.zeros((taps - 1, 3)), w, b)
+    for c in range(3):
+        assert np.allclose(y[:, c], b[c] + np.convolve(x[:, c], w[c, ::-1])[:6])
+    y1, p1 = O.causal_conv(x[:1], np.zeros((taps - 1, 3)), w, b)
+    y2, p2 = O.causal_conv(x[1:], p1, w, b)
+    assert np.allclose(np.concatenate([y1, y2]), y) and np.allclose(p2, past)
+    v, z = g.standard_normal((2, 6)), g.standard_normal((2, 6))
+    u = v * z / (1 + np.exp(-z))
+    got = O.gated_group_norm(v, z, np.arange(6.0), 2, 0.0)
+    assert np.allclose(got[:, :3], u[:, :3] / np.sqrt((u[:, :3] ** 2).mean(1, keepdims=True)) * np.arange(3.0))
+    assert np.allclose(got[:, 3:], u[:, 3:] / np.sqrt((u[:, 3:] ** 2).mean(1, keepdims=True)) * np.arange(3.0, 6.0))
+
+
+def test_capped_logits_and_portions_of_a_small_stack():
+    cfg = _vifivik()
+    w = M.plain_weights(M.weights(cfg, 6))
+    tokens = [3, 1, 4, 1, 5, 9, 2, 6]
+    whole = O.forward(cfg, w, tokens)
+    assert np.abs(whole).max() < 9.0
+    mem = {}
+    parts = [O.forward(cfg, w, p, mem) for p in (tokens[:3], tokens[3:4], tokens[4:])]
+    assert np.allclose(np.concatenate(parts), whole)
+    assert np.allclose(O.softcap(np.array([1e-3, 50.0]), 9.0), [1e-3, 9.0], atol=1e-3)
+
+
 def test_difference_lambda_matches_the_plain_statement(ai):
     g = np.random.default_rng(3)
     w = {n: g.standard_normal(10) * 0.3 for n in ("lq1", "lk1", "lq2", "lk2")}
