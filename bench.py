@@ -1051,6 +1051,184 @@ def bench_stack_models(pkg, ctx, K, steps, warmup, graphs=True):
     return res
 
 
+def bench_latent_kernels(pkg, ctx, K, steps, warmup):
+    """The kernels of stacks with latent attention, state-space layers and norms behind the branches, each beside the like kernel
+    of the bf16-weight stack with attention caches at the same size: fraction of the HBM peak, or of the dense bf16 matrix peak."""
+    lw, res, batch = pkg.linear_weight, {}, pkg.CommandBatch(ctx)
+    F32, BF16 = pkg.F32, pkg.BF16
+    empty = pkg.Buffer.empty
+
+    def timed(name, fns, byte=None, flop=None):
+        """`fns`: the same call on distinct data, in turn."""
+        it = [0]
+
+        def step():
+            fns[it[0] % len(fns)]()
+            it[0] += 1
+        _, ev = time_steps(pkg, ctx, step, max(steps, len(fns), 20), warmup)
+        r = {"us": ev * 1e3}
+        if byte:
+            r.update(gbs=byte / (ev * 1e-3) * 1e-9, frac_of_hbm_peak=byte / (ev * 1e-3) * 1e-9 / HBM_PEAK_GBS)
+        if flop:
+            r.update(tflops=flop / (ev * 1e-3) * 1e-12, frac_of_mfma_peak=flop / (ev * 1e-3) * 1e-12 / MFMA_F16_PEAK_TFLOPS)
+        res[name] = r
+        log(f"[bench] latent {name}: " + ", ".join(f"{k} {v:.4g}" for k, v in r.items()))
+
+    def floats(n, seed=0):
+        return pkg.Buffer.from_slice(ctx, np.resize(np.random.default_rng(seed).standard_normal(1 << 16).astype(np.float32), n))
+    # one row: products that add the normed branch before, products of gated pairs
+    for n, k in ((2048, 2048), (8192, 2048), (2048, 8192)):
+        byte = n * k * 2
+        reps = max(1, min(64, (1 << 29) // byte))
+        big = random_bits(ctx, pkg, byte * reps)
+        ws = [big.view(i * byte, byte) for i in range(reps)]
+        seg, x, y, s, nw, o = lw.Segments([lw.Segment(n)]), floats(2 * k), floats(k, 1), empty(ctx, k * 4), floats(k, 2), empty(ctx, n * 4)
+        timed(f"row {n}x{k}, norm behind the branch", [lambda w=w: K.linear_residual_vector_into(batch, x, y, s, nw, 1e-6, w, None, k, seg, [o], F32) for w in ws], byte)
+        timed(f"row {n}x{k}, gated pairs", [lambda w=w: K.linear_pairs_vector_into(batch, x, w, None, k, seg, [o], F32) for w in ws], byte)
+        timed(f"row {n}x{k}, norm in front (like)", [lambda w=w: K.linear_norm_vector_into(batch, x, None, None, nw, 1e-6, w, None, k, seg, [o], F32) for w in ws], byte)
+        if n == k:
+            timed(f"row {n}x{k}, gated norm in 16 parts", [lambda w=w: K.linear_gated_vector_into(batch, x, y, F32, None, 1e-6, w, None, k, seg, [o], F32, group=k // 16,
+                                                                                             gate_act=pkg.ACT_SILU) for w in ws], byte)
+        big.free()
+    # latent attention: 16 heads of 128 + 64, values of 128, latents of 512; the like: 16 heads over 4, two maps of 64, values of 128
+    H, D, R, V, C, T = 16, 128, 64, 128, 512, 32768
+    row, cap = K.latent_row(C, R), T + 2304
+    caches = [random_bits(ctx, pkg, cap * row * 2, i) for i in range(8)]
+    like = [(random_bits(ctx, pkg, cap * 4 * 128 * 2, i), random_bits(ctx, pkg, cap * 4 * V * 2, i + 9)) for i in range(8)]
+    q, ql, gate, sink, o = random_bits(ctx, pkg, 2048 * H * 192 * 2, 3), floats(64 * H * row, 4), floats(2048 * H, 5), floats(H, 6), empty(ctx, 2048 * H * C * 4)
+    uk, uv, up = random_bits(ctx, pkg, H * C * D * 2, 1), random_bits(ctx, pkg, H * V * C * 2, 2), random_bits(ctx, pkg, H * (D + V) * C * 2, 3)
+    down, lnorm, freq, qr = floats(2048 * (C + R), 7), floats(C, 8), floats(R // 2, 9), floats(2048 * H * R, 1)
+    for t in (T - 1, 4095):
+        pos = pkg.Buffer.from_slice(ctx, np.array([t], np.uint32))
+        timed(f"latent attention decode, {t + 1} positions", [lambda c=c: K.latent_attention_rows_into(batch, ql, c, o, BF16, pos, t, 1, H, C, R, cap, 0.07, sink, gate)
+                                                              for c in caches], (t + 1) * (C + R) * 2)
+        timed(f"attention decode, {t + 1} positions (like)", [lambda c=c: K.attention_rows_into(batch, q, c[0], c[1], o, BF16, pos, t, 1, H, 4, 2, 64, V, cap, 0.125, 0.3, 0.7,
+                                                                                              1e-6) for c in like], (t + 1) * 4 * (2 * 64 + V) * 2)
+        timed(f"latent attention, 16 rows at {t}", [lambda c=c: K.latent_attention_rows_into(batch, ql, c, o, BF16, pos, t, 16, H, C, R, cap, 0.07, sink, gate)
+                                                    for c in caches], None, 16 * t * H * 2 * (C + R + C))
+    timed("latent prepare, one row", [lambda: K.latent_prepare_into(batch, qr, down, lnorm, freq, pos, ql, F32, caches[0], BF16, 1, H, C, R, row, C, C, cap, 1e-6)])
+    timed("key projection of the queries, one row", [lambda: K.head_linear_into(batch, q, BF16, uk, ql, F32, 1, H, C, D, row)], H * C * D * 2)
+    timed("value projection of the output, one row", [lambda: K.head_linear_into(batch, o, BF16, uv, ql, BF16, 1, H, V, C, V)], H * C * V * 2)
+    keys, values = empty(ctx, cap * H * 192 * 2), empty(ctx, cap * H * V * 2)
+    for t, rows in ((0, 2048), (T, 256), (2048, 2048)):
+        pos, n = pkg.Buffer.from_slice(ctx, np.array([t], np.uint32)), t + rows
+        pairs = rows * t + rows * (rows + 1) / 2
+        timed(f"latent prepare, {rows} rows", [lambda: K.latent_prepare_into(batch, qr, down, lnorm, freq, pos, q, BF16, caches[0], BF16, rows, H, C, R, 192, D, D, cap, 1e-6)],
+              rows * (H * R * (4 + 2) + (C + R) * 4 + row * 2))
+        timed(f"keys and values of {n} positions", [lambda: K.latent_expand_into(batch, caches[0], BF16, up, keys, values, n, H, D, R, V, C)], None, 2.0 * n * H * (D + V) * C)
+        timed(f"attention prefill, {rows} rows at {t}", [lambda: K.attention_rows_into(batch, q, keys, values, o, BF16, pos, t, rows, H, H, 1, D + R, V, cap, 0.07, sink=sink,
+                                                                                       gate=gate)], None, pairs * H * 2 * (D + R + V))
+        timed(f"attention prefill, {rows} rows at {t} (like)", [lambda: K.attention_rows_into(batch, q, like[0][0], like[0][1], o, BF16, pos, t, rows, H, 4, 2, 64, V, cap, 0.125,
+                                                                                            0.3, 0.7, 1e-6)], None, pairs * H * 2 * 2 * (64 + V))
+    del caches, like, keys, values
+    # state space: 64 heads of 64, states of 128, one group; the like: 32 heads of 128 x 128 (the same states)
+    H, V, N, G, taps, rows = 64, 64, 128, 1, 4, 2048
+    inner = H * V
+    ch = inner + 2 * G * N
+    u, uf, ring, tw, tb, pos = random_bits(ctx, pkg, rows * ch * 2), floats(ch), empty(ctx, taps * ch * 4), floats(taps * ch, 1), floats(ch, 2), empty(ctx, 4)
+    x, b, c, dt = (random_bits(ctx, pkg, rows * n * 2, n) for n in (inner, G * N, G * N, 2 * H))
+    dt, args = floats(rows * H, 3), [floats(H, i) for i in range(3)]
+    o, states = empty(ctx, rows * inner * 4), [empty(ctx, H * V * N * 4) for _ in range(64)]
+    steps_buf, work = empty(ctx, K.selective_steps_bytes(rows, H)), empty(ctx, K.linear_attention_workspace_bytes(rows, H, N, V))
+    timed("state space, one row", [lambda s=s: K.selective_step_into(batch, uf, ring, tw, tb, pos, dt, *args, s, o, H, V, G, N, taps) for s in states], 2 * H * V * N * 4)
+    h2, d2 = 16, 128
+    q2, decay = random_bits(ctx, pkg, rows * 32 * d2 * 2, 1), pkg.Buffer.from_slice(ctx, np.full(32, 0.99, np.float32))
+    pw = pkg.Buffer.from_slice(ctx, np.resize(0.99 ** np.arange(65), 32 * 65).astype(np.float32))
+    timed("linear attention, one row (like)", [lambda s=s: K.linear_attention_recurrent_into(batch, q2, q2, q2, BF16, s, decay, o, 1, 32, d2, d2) for s in states], 2 * 32 * d2 * d2 * 4)
+    for n in (256, 2048):
+        timed(f"convolution, {n} rows", [lambda: K.selective_conv_into(batch, u, BF16, ring, tw, tb, pos, x, b, c, n, H, V, G, N, taps)], n * ch * 2 * 2)
+        w = K.linear_attention_workspace_bytes(n, H, N, V)
+        timed(f"state space, {n} rows", [lambda: K.selective_chunked_into(batch, x, b, c, dt, *args, states[0], steps_buf, work, o, n, H, V, G, N)],
+              n * (inner * 2 * 2 + G * N * 2 * 3 + inner * 4) + 4 * w)
+        w = K.linear_attention_workspace_bytes(n, 32, d2, d2)
+        timed(f"linear attention, {n} rows (like)", [lambda: K.linear_attention_chunked_into(batch, q2, q2, q2, states[0], pw, work, o, n, 32, d2, d2)], n * 32 * d2 * (2 * 5 + 4) + 4 * w)
+    # rows around the products
+    f, g, w, y, out = floats(rows * inner), random_bits(ctx, pkg, rows * inner * 2), floats(inner), floats(rows * 2048, 1), empty(ctx, rows * inner * 2)
+    timed(f"gated norm, {rows} x {inner}", [lambda: K.gated_norm_rows_into(batch, f, g, w, out, BF16, inner, rows, 1e-6, None, pkg.ACT_SILU, True)], rows * inner * 8)
+    timed(f"gated norm in 32 parts, {rows} x {inner}", [lambda: K.gated_norm_rows_into(batch, f, g, None, out, BF16, inner, rows, 1e-6, 128, pkg.ACT_SILU)], rows * inner * 8)
+    timed(f"gated norm, {rows} x {inner} (like)", [lambda: K.gated_norm_rows_into(batch, f, g, w, out, BF16, inner, rows, 1e-6)], rows * inner * 8)
+    timed(f"norm behind the branch, {rows} x 2048", [lambda: K.residual_rows_into(batch, f, y, w, f, out, BF16, 2048, rows, 1e-6)], rows * 2048 * 14)
+    timed(f"norm in front, {rows} x 2048 (like)", [lambda: K.norm_rows_f32_into(batch, f, None, w, None, None, out, BF16, 2048, rows, 1e-6)], rows * 2048 * 6)
+    for m in (256, 2048):
+        x, w, y = random_bits(ctx, pkg, m * 2048 * 2, 1), random_bits(ctx, pkg, 8192 * 2048 * 2, 2), empty(ctx, m * 8192 * 2)
+        for name, act in (("gate and up as pairs", pkg.ACT_SILU_PAIRS), ("one activation (like)", pkg.ACT_SILU)):
+            seg = lw.Segments([lw.Segment(8192, act)])
+            timed(f"rows {m}x2048x8192, {name}", [lambda: K.linear_rows_into(batch, x, BF16, w, None, m, 2048, seg, [y], BF16)], None, 2.0 * m * 2048 * 8192)
+    logits = floats(131072)
+    timed("capped logits, 131072", [lambda: K.softcap_f32_into(batch, logits, 131072, 30.0)], 131072 * 8)
+    return res
+
+
+def bench_latent_models(pkg, ctx, K, steps, warmup, graphs=True):
+    """Tokens per second of whole stacks of latent attention, retention and state-space layers with random weights, beside the
+    stack of differential-attention and lightning layers at equal width, depth, context and feed-forward weights."""
+    A, res = pkg.mixers, {}
+    for width, ff in ((1024, 4096), (2048, 8192)):
+        H, T = width // 128, 4096
+        lat = A.LatentAttentionSpec(H, 128, 64, 128, 512, 10000.0, 192 ** -0.5)
+        shared = A.LatentAttentionSpec(H, 128, 64, 128, 512, 10000.0, 192 ** -0.5, 0)
+        decay = list(np.linspace(0.9, 0.999, H))
+        ret = A.LinearAttentionSpec(H, 128, 128, decay, pkg.ACT_NONE, 128 ** -0.5, pkg.ACT_SILU, True)
+        ssm = A.SelectiveSpec(width // 32, 64, 128, 1, 4, 1)
+        gated = A.GatedSpec(ff * 2 // 3 // 64 * 64)
+        attn = A.AttentionSpec(H, max(H // 4, 1), 64, 128, 0.125, maps=2, diff=0.3, bias=True)
+        lin = A.LinearAttentionSpec(H, 128, 128, decay)
+        configs = {"latent": pkg.stack_pipeline.StackConfig(32000, width, 1e-6, [A.LayerSpec(m, gated) for m in (lat, shared, ret, ssm)], layer=A.OutputNormLayer, softcap=30.0),
+                   "like": pkg.stack_pipeline.StackConfig(32000, width, 1e-6, [A.LayerSpec(m, A.DenseSpec(ff)) for m in (attn, attn, lin, lin)])}
+        for name, cfg in configs.items():
+            m = pkg.stack_pipeline.StackPipeline(ctx, K, cfg, RandomTensors(1), T + 512, graphs=graphs)
+            tokens, out = [int(t) for t in np.random.default_rng(2).integers(0, 32000, T)], {}
+            for rows in (256, 2048):
+                m.max_rows = rows
+
+                def prompt():
+                    s = m.new_sequence()
+                    m.step(s, tokens, [T - 1])
+                    m.end_sequence(s)
+                prompt()
+                t0 = time.perf_counter()
+                for _ in range(3):
+                    prompt()
+                out[f"prompt_tokens_per_s_passes_of_{rows}"] = 3 * T / (time.perf_counter() - t0)
+            s = m.new_sequence()
+            m.step(s, tokens)
+            for _ in range(5):
+                m.greedy(s, 1)
+            n = 200
+            t0 = time.perf_counter()
+            for _ in range(n):
+                m.greedy(s, 1)
+            out["decode_us_per_token_with_host"] = (time.perf_counter() - t0) / n * 1e6
+            if graphs:
+                byte = m.head.bytes()
+                for l in m.layers:
+                    mx = l.mixer
+                    byte += mx.out.bytes() + l.ff.up.bytes() + l.ff.down.bytes() + next(getattr(mx, p).bytes() for p in ("qkv", "qkvg", "proj") if hasattr(mx, p))
+                    if isinstance(mx, A.LatentAttention):
+                        byte += mx.up.length() + T * (512 + 64) * 2
+                    elif isinstance(mx, A.SoftmaxAttention):
+                        byte += T * attn.kv_heads * (2 * 64 + 128) * 2
+                    else:
+                        z = mx.spec
+                        byte += 2 * 4 * z.heads * z.vdim * (z.state if isinstance(z, A.SelectiveSpec) else z.dim)
+                settle(ctx, s.graph.launch, 100)
+                e0, e1 = pkg.Event(ctx), pkg.Event(ctx)
+                s.position_buf.copy_from_bytes(np.array([T], np.uint32))
+                e0.record()
+                for _ in range(100):
+                    s.graph.launch()
+                e1.record()
+                ctx.synchronize()
+                us = e0.elapsed_ms(e1) * 10
+                out.update(decode_us_per_token=us, decode_tokens_per_s=1e6 / us, decode_dispatches=s.graph.dispatch_count(), decode_mbytes=byte * 1e-6,
+                           decode_frac_of_hbm_peak=byte / us * 1e-3 / HBM_PEAK_GBS)
+            m.end_sequence(s)
+            del m, s
+            res[f"{name}_width_{width}"] = out
+            log(f"[bench] {name} model width {width}:", out)
+    return res
+
+
 def main():
     global SETTLE_MS
     ap = argparse.ArgumentParser()
@@ -1068,7 +1246,7 @@ def main():
     ap.add_argument("--no-cpu", action="store_true", help="skip the CPU baseline leg")
     ap.add_argument("--legs", default="matvec,attention,sweep,layer,prefill,glue,decode,lanes,chunk,model,model_lanes",
                     help="comma-separated extra measurements to run besides the headline (for profiling one kernel at a time); "
-                         "model_few_lanes (2 .. 16 sequences at 8k context), stack_kernels and stack_models (models with bf16 "
+                         "model_few_lanes (2 .. 16 sequences at 8k context), stack_kernels, stack_models, latent_kernels and latent_models (models with bf16 "
                          "weights beside the quantized decoder) are not in the default set")
     args = ap.parse_args()
     SETTLE_MS = args.settle_ms
@@ -1179,6 +1357,10 @@ def main():
         extra["stack_kernels"] = bench_stack_kernels(pkg, ctx, K, args.steps, args.warmup)
     if "stack_models" in legs:
         extra["stack_models"] = bench_stack_models(pkg, ctx, K, args.steps, args.warmup, graphs=not args.no_graph)
+    if "latent_kernels" in legs:
+        extra["latent_kernels"] = bench_latent_kernels(pkg, ctx, K, args.steps, args.warmup)
+    if "latent_models" in legs:
+        extra["latent_models"] = bench_latent_models(pkg, ctx, K, args.steps, args.warmup, graphs=not args.no_graph)
 
     achieved = head["alg_bytes_per_launch"] / head["ms_per_launch_events"] * 1e-6
     # The other north-star kernels of this run, in the blocks a reader of the line keeps: their rooflines beside the

@@ -97,6 +97,39 @@ __device__ __forceinline__ void store4(const LhLinear& a, uint32_t slot, uint32_
     }
 }
 
+// A finished tile into a value cache: a thread stores a quarter of a block of 32 positions of one column, which is 16 bytes where
+// the tile has all of them.  `tile` as linear_mfma_kernel leaves it.
+template <int BM, int BN>
+__device__ __forceinline__ void store_blocks(const LhLinear& a, uint32_t s, const float* tile, const RowTile& rt, uint32_t n0, uint32_t pos0) {
+    const uint32_t first = pos0 + rt.begin, last = min(pos0 + rt.end, a.seg.rows[s]), b0 = first >> 5;      // positions [first, last)
+    if (first >= last) return;
+    const uint32_t blocks = ((last - 1) >> 5) - b0 + 1, cols = min((uint32_t)BN, a.N - n0);
+    uint16_t* out = static_cast<uint16_t*>(a.seg.out[s]);
+#pragma unroll 1
+    for (uint32_t e = threadIdx.x; e < blocks * cols * 4; e += 256) {
+        const uint32_t g = e & 3, j = (e >> 2) % cols, b = b0 + (e >> 2) / cols, n = n0 + j;
+        uint32_t c = n - a.seg.n0[s];
+        if (a.seg.head[s] != a.seg.padded[s]) { const uint32_t h = c / a.seg.head[s]; c = h * a.seg.padded[s] + (c - h * a.seg.head[s]); }
+        uint16_t* d = out + ((size_t)b * a.seg.ld[s] + c) * 32 + g * 8;
+        const float bias = a.bias ? a.bias[n] : 0.0f;
+        uint16_t v[8];
+        bool all = true, in[8];
+#pragma unroll
+        for (uint32_t i = 0; i < 8; i++) {                    // entries 8 g + i: positions 4 g + i and 16 + 4 g + i - 4
+            const uint32_t p = b * 32 + (i >> 2) * 16 + g * 4 + (i & 3);
+            in[i] = p >= first && p < last;
+            all = all && in[i];
+            const uint32_t m = in[i] ? p - first : 0u;
+            v[i] = lh_f2bf(lh_activate(tile[(m * (BN / 4) + ((j >> 2) ^ (m & 7))) * 4 + (j & 3)] + bias, a.seg.act[s]));
+        }
+        if (all) *reinterpret_cast<uint4*>(d) = make_uint4(v[0] | (uint32_t)v[1] << 16, v[2] | (uint32_t)v[3] << 16, v[4] | (uint32_t)v[5] << 16, v[6] | (uint32_t)v[7] << 16);
+        else {
+#pragma unroll
+            for (uint32_t i = 0; i < 8; i++) if (in[i]) d[i] = v[i];
+        }
+    }
+}
+
 // ---- matrix cores ------------------------------------------------------------------------------------------------------
 // 256 threads, 2 x 2 waves of BM/2 x BN/2 outputs.  A k step is 64 wide: a tile row is eight 16-byte chunks, chunk c of row r
 // kept at place c ^ (r & 7) of its row so that the fragment reads of sixteen rows fall on different banks (the loads
@@ -198,6 +231,11 @@ __global__ __launch_bounds__(256) void linear_mfma_kernel(const LhLinear a) {
         }
     __syncthreads();
     const uint32_t pos0 = a.seg.position ? *a.seg.position : 0u;
+    const uint32_t s = lh_segment_of(a.seg, n0);
+    if (a.seg.layout[s] == LH_BLOCKS_AT_POSITION && !a.seg.f32[s] && s == lh_segment_of(a.seg, min(n0 + BN, a.N) - 1) && a.ex.tiles == nullptr) {
+        store_blocks<BM, BN>(a, s, reinterpret_cast<const float*>(tile), rt, n0, pos0);
+        return;
+    }
 #pragma unroll 1
     for (uint32_t e = tid; e < BM * BN / 4; e += 256) {
         const uint32_t m = e / (BN / 4), c = e % (BN / 4), n = n0 + c * 4, slot = rt.begin + m;

@@ -116,6 +116,7 @@ __global__ __launch_bounds__(256) void head_linear_plain_kernel(const HeadArgs a
 }
 
 // ---- keys of every head: the shared rotated part ---------------------------------------------------------------------------
+// T: as many values as move together.
 template <typename T>
 __global__ __launch_bounds__(256) void expand_rotated_kernel(const T* __restrict__ cache, T* __restrict__ keys, uint32_t heads, uint32_t row, uint32_t dv,
                                                             uint32_t dim, uint32_t rot, uint32_t dq) {
@@ -137,11 +138,12 @@ __device__ __forceinline__ s16x4 transposed4(const void* lds) {
 
 // grid: row tiles x splits; packed row r = head r % heads of query row r / heads.  The blocks of 32 positions of the visible range
 // are dealt out in contiguous runs to the 4 * splits waves of a row tile.  A wave keeps its block in its own part of LDS (so the
-// waves need no barrier): chunk c of 16 bytes of key row k at place c ^ (k & 7).  The scores read it row by row, the values
-// through the transposing LDS read.  A query value enters as the sum of two bf16 terms.
+// waves need no barrier), in tiles of 8 key rows x 8 chunks of 16 bytes, chunk c of row k at place c ^ k of its row: a load fills
+// one tile, and every address is one of a few per lane plus a constant.  The scores read it row by row, the values through the
+// transposing LDS read.  A query value enters as the sum of two bf16 terms.
 template <int DV>
-__global__ __launch_bounds__(256) void latent_split_kernel(const AttentionArgs a) {
-    constexpr int DQ = DV + kRotPad, KC = DQ / 8;
+__global__ __launch_bounds__(256, DV > 256 ? 1 : 2) void latent_split_kernel(const AttentionArgs a) {
+    constexpr int DQ = DV + kRotPad, KC = DQ / 8, KT = KC / 8;
     extern __shared__ __align__(16) uint4 sm[];             // [4 waves][32 * KC]; at the end the partial results [4 waves][16 rows][DV + 4]
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, lc = lane & 15;
     const uint32_t split = blockIdx.x % a.splits, tile = blockIdx.x / a.splits, packed = a.rows * a.heads, start = *a.position;
@@ -151,12 +153,13 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const AttentionArgs a
     const uint32_t per = (nb + 4 * a.splits - 1) / (4 * a.splits), w = split * 4 + wave;
     const uint32_t b0 = min(w * per, nb), b1 = min(b0 + per, nb);
     uint4* mine = sm + wave * (32 * KC);
-    const uint16_t* cache = static_cast<const uint16_t*>(a.keys);
+    const uint16_t* cache = static_cast<const uint16_t*>(a.keys) + ((lane & 7) ^ (lane >> 3)) * 8;
     auto load_block = [&](uint32_t b) {
 #pragma unroll
-        for (int i = 0; i < KC / 2; i++) {
-            const uint32_t c = i * 64 + lane, key = c / KC, ch = (c % KC) ^ (key & 7), p = min(b * 32 + key, last_key);   // keys past the last are masked
-            __builtin_amdgcn_global_load_lds((gvoid*)(cache + (size_t)p * DQ + ch * 8), (lvoid*)(mine + i * 64), 16, 0, 0);
+        for (int k = 0; k < 4; k++) {
+            const uint16_t* row = cache + (size_t)min(b * 32 + k * 8 + (lane >> 3), last_key) * DQ;              // keys past the last are masked
+#pragma unroll
+            for (int i = 0; i < KT; i++) __builtin_amdgcn_global_load_lds((gvoid*)(row + i * 64), (lvoid*)(mine + (k * KT + i) * 64), 16, 0, 0);
         }
     };
     if (b0 < b1) load_block(b0);
@@ -183,21 +186,28 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const AttentionArgs a
     for (int d = 0; d < DV / 16; d++) o[d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
     RowState st{-INFINITY, 0.0f};
     const float scale2 = a.scale * kLog2e;
+    // score operand: key lc (+ 16), chunk 4 c + g; value operand: key 4 g + lc / 4 (+ 16), columns 16 d + 4 (lane & 3) ..
+    const uint4* kp = mine + (lc >> 3) * (KT * 64) + (lc & 7) * 8;
+    const uint32_t vk = g * 4 + (lc >> 2);
+    const char* vp = reinterpret_cast<const char*>(mine + (vk >> 3) * (KT * 64) + (vk & 7) * 8) + (lane & 1) * 8;
 
     for (uint32_t b = b0; b < b1; b++) {
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
-        lh_f32x4 s[2];
+        lh_f32x4 s[2], low[2];                                // four sums that do not wait for each other
 #pragma unroll
-        for (int t = 0; t < 2; t++) {
-            s[t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
-            const uint32_t key = t * 16 + lc;
+        for (int t = 0; t < 2; t++) s[t] = low[t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-            for (int c = 0; c < DQ / 32; c++) {
-                const lh_bf16x8 k = __builtin_bit_cast(lh_bf16x8, mine[key * KC + ((c * 4 + g) ^ (key & 7))]);
-                s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, ql[c], s[t], 0, 0, 0);
+        for (int c = 0; c < DQ / 32; c++)
+#pragma unroll
+            for (int t = 0; t < 2; t++) {
+                const lh_bf16x8 k = __builtin_bit_cast(lh_bf16x8, kp[t * 2 * KT * 64 + (c >> 1) * 64 + (((c & 1) * 4 + g) ^ (lc & 7))]);
+                low[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, ql[c], low[t], 0, 0, 0);
                 s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qh[c], s[t], 0, 0, 0);
             }
-        }
+#pragma unroll
+        for (int t = 0; t < 2; t++)
+#pragma unroll
+            for (int r = 0; r < 4; r++) s[t][r] += low[t][r];
         lh_bf16x8 p[1][3];
         const float alpha = softmax_step<1>(s, st, scale2, b * 32, limit, b * 32 + 31 > first_limit, lane, p);
         if (__ballot(alpha != 1.0f)) {
@@ -206,14 +216,19 @@ __global__ __launch_bounds__(256) void latent_split_kernel(const AttentionArgs a
 #pragma unroll
                 for (int r = 0; r < 4; r++) o[d][r] *= alpha;
         }
-        const uint32_t key = g * 4 + (lc >> 2);               // and key + 16: the same place pattern, as 16 is a multiple of 8
 #pragma unroll
-        for (int d = 0; d < DV / 16; d++) {
-            const char* v0 = reinterpret_cast<const char*>(mine + key * KC + ((2 * d + ((lane & 3) >> 1)) ^ (key & 7))) + (lane & 1) * 8;
-            struct { s16x4 x, y; } v = {transposed4(v0), transposed4(v0 + 16 * KC * 16)};
-            const lh_bf16x8 vf = __builtin_bit_cast(lh_bf16x8, v);
+        for (int d0 = 0; d0 < DV / 16; d0 += 4) {
+            lh_bf16x8 vf[4];
 #pragma unroll
-            for (int z = 2; z >= 0; z--) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf, p[0][z], o[d], 0, 0, 0);
+            for (int d = 0; d < 4; d++) {
+                const char* v0 = vp + (((2 * d + ((lane & 3) >> 1)) ^ (vk & 7)) + (d0 >> 2) * 64) * 16;
+                struct { s16x4 x, y; } v = {transposed4(v0), transposed4(v0 + 2 * KT * 64 * 16)};
+                vf[d] = __builtin_bit_cast(lh_bf16x8, v);
+            }
+#pragma unroll
+            for (int z = 2; z >= 0; z--)
+#pragma unroll
+                for (int d = 0; d < 4; d++) o[d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], p[0][z], o[d0 + d], 0, 0, 0);
         }
         asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");    // the block has been read: the next may overwrite it
         if (b + 1 < b1) load_block(b + 1);
@@ -271,9 +286,8 @@ int launch_split(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const
     hipLaunchKernelGGL((latent_split_kernel<DV>), dim3((uint32_t)(tiles * a.splits)), dim3(256), lds, ctx->stream, a);
     int r = lh_check_launch(op);
     if (r != LH_OK) return r;
-    hipLaunchKernelGGL((attention_merge_kernel<1>), dim3(a.rows * a.heads), dim3(kMergeThreads), 0, ctx->stream, a);
     launches = 2;
-    return lh_check_launch(op);
+    return launch_merge<1>(ctx, a, op);
 }
 
 }  // namespace
@@ -372,12 +386,13 @@ int lh_latent_expand_into(lh_batch* batch, const lh_buffer* cache, int dtype, co
     a.M = positions; a.N = heads * (dim + vdim); a.K = rank; a.lda = row;
     int r = lh_launch_linear(batch->ctx, a, op);
     if (r != LH_OK) return r;
-    if (dtype == LH_F32)
-        hipLaunchKernelGGL((expand_rotated_kernel<float>), dim3(positions), dim3(256), 0, batch->ctx->stream, (const float*)cache->ptr, (float*)keys->ptr, heads, row,
-                           padded_rank(rank), dim, rot, dq);
-    else
-        hipLaunchKernelGGL((expand_rotated_kernel<uint16_t>), dim3(positions), dim3(256), 0, batch->ctx->stream, (const uint16_t*)cache->ptr, (uint16_t*)keys->ptr,
-                           heads, row, padded_rank(rank), dim, rot, dq);
+    const uint32_t dl = padded_rank(rank);
+    const bool aligned = (((uintptr_t)cache->ptr | (uintptr_t)keys->ptr) & 15) == 0;
+#define LH_EXPAND(T, N) hipLaunchKernelGGL((expand_rotated_kernel<T>), dim3(positions), dim3(256), 0, batch->ctx->stream, (const T*)cache->ptr, (T*)keys->ptr, heads, row / N, dl / N, dim / N, rot / N, dq / N)
+    if (dtype == LH_F32) LH_EXPAND(float, 1);
+    else if (aligned && dim % 8 == 0 && rot % 8 == 0) LH_EXPAND(uint4, 8);
+    else LH_EXPAND(uint16_t, 1);
+#undef LH_EXPAND
     r = lh_check_launch(op);
     if (r == LH_OK) batch->dispatch_count += 2;
     return r;

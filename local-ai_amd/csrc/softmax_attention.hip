@@ -315,9 +315,8 @@ int launch_mfma(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const 
     const size_t rec = (size_t)tiles16 * a.kv_heads * MAPS * 16 * (DV + 4) * 4;
     const uint32_t room = (uint32_t)std::min<size_t>(ctx->workspace_bytes / rec, kMaxSplits);
     auto merge = [&]() {
-        hipLaunchKernelGGL((attention_merge_kernel<MAPS>), dim3(a.rows * a.heads), dim3(kMergeThreads), 0, ctx->stream, a);
         launches++;
-        return lh_check_launch(op);
+        return launch_merge<MAPS>(ctx, a, op);
     };
     a.partial = (float*)ctx->workspace;
     launches = 1;

@@ -20,6 +20,7 @@ struct AttentionArgs {
     uint32_t values_in_keys;   // plain form: a position's values are the first columns of its key row
     float* partial;            // records [16-row tile][kv head][split][map][16] of dv unnormalised sums, maximum, sum of weights
     uint32_t splits;
+    uint32_t parts;            // workgroups that share a row's columns in the merge (one map)
 };
 
 constexpr float kLog2e = 1.4426950408889634f;
@@ -73,7 +74,8 @@ template <int MAPS>
 __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const AttentionArgs a) {
     __shared__ float factor[MAPS][512], total[MAPS], scratch[kMergeThreads / 64];
     __shared__ float4 sums[MAPS][kMergeThreads];
-    const uint32_t t = blockIdx.x / a.heads, h = blockIdx.x % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
+    const uint32_t part = blockIdx.x % a.parts, th = blockIdx.x / a.parts, t = th / a.heads, h = th % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
+    const uint32_t cols = a.dv / a.parts, col0 = part * cols;
     const uint32_t kRow = a.dv + 4, rr = row & 15;
     const size_t stride = (size_t)MAPS * 16 * kRow;
     const float* rec = a.partial + (size_t)(((row >> 4) * a.kv_heads + g) * a.splits) * stride + rr * kRow;
@@ -103,7 +105,7 @@ __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const At
         if (lane == 0) total[wave] = 1.0f / l;
     }
     __syncthreads();
-    const uint32_t quads = a.dv / 4, groups = kMergeThreads / quads, grp = threadIdx.x / quads, q = threadIdx.x % quads;   // quads <= 128
+    const uint32_t quads = cols / 4, groups = kMergeThreads / quads, grp = threadIdx.x / quads, q = threadIdx.x % quads;   // quads <= 128
     float4 acc[MAPS];
 #pragma unroll
     for (int mp = 0; mp < MAPS; mp++) acc[mp] = make_float4(0.f, 0.f, 0.f, 0.f);
@@ -111,7 +113,7 @@ __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const At
     for (uint32_t s = grp; s < a.splits; s += groups)
 #pragma unroll
         for (int mp = 0; mp < MAPS; mp++) {
-            const float4 x = *reinterpret_cast<const float4*>(rec + s * stride + mp * 16 * kRow + q * 4);
+            const float4 x = *reinterpret_cast<const float4*>(rec + s * stride + mp * 16 * kRow + col0 + q * 4);
             const float f = factor[mp][s];
             acc[mp].x += f * x.x; acc[mp].y += f * x.y; acc[mp].z += f * x.z; acc[mp].w += f * x.w;
         }
@@ -119,19 +121,28 @@ __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const At
     for (int mp = 0; mp < MAPS; mp++) sums[mp][threadIdx.x] = acc[mp];
     __syncthreads();
     float v = 0.0f;
-    const uint32_t d = threadIdx.x;                           // dv <= 512
-    if (d < a.vdim) {
+    const uint32_t d = col0 + threadIdx.x;                    // dv <= 512
+    const bool on = threadIdx.x < cols && d < a.vdim;
+    if (on) {
         float s[MAPS] = {};
         for (uint32_t i = 0; i < groups; i++)
 #pragma unroll
-            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sums[mp][i * quads])[d];
+            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sums[mp][i * quads])[threadIdx.x];
         v = s[0] * total[0];
         if constexpr (MAPS == 2) v -= a.lambda * (s[MAPS - 1] * total[MAPS - 1]);
     }
     float f = 1.0f;
     if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(v * v, scratch) / (float)a.vdim + a.eps) * a.out_scale;
     if (MAPS == 1 && a.gate) f = lh_sigmoid(a.gate[(size_t)t * a.heads + h]);
-    if (d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
+    if (on) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
+}
+
+template <int MAPS>
+int launch_merge(lh_context* ctx, AttentionArgs& a, const char* op) {
+    a.parts = 1;                                              // two maps: the norm needs all columns
+    if (MAPS == 1) while (a.dv / a.parts > 64 && (uint64_t)a.rows * a.heads * a.parts * 2 <= (uint64_t)ctx->cu_count) a.parts *= 2;
+    hipLaunchKernelGGL((attention_merge_kernel<MAPS>), dim3(a.rows * a.heads * a.parts), dim3(kMergeThreads), 0, ctx->stream, a);
+    return lh_check_launch(op);
 }
 
 // One workgroup per (query row, head), 256 keys at a time; f32 arithmetic throughout.
