@@ -1084,7 +1084,9 @@ def bench_latent_kernels(pkg, ctx, K, steps, warmup):
         ws = [big.view(i * byte, byte) for i in range(reps)]
         seg, x, y, s, nw, o = lw.Segments([lw.Segment(n)]), floats(2 * k), floats(k, 1), empty(ctx, k * 4), floats(k, 2), empty(ctx, n * 4)
         timed(f"row {n}x{k}, norm behind the branch", [lambda w=w: K.linear_residual_vector_into(batch, x, y, s, nw, 1e-6, w, None, k, seg, [o], F32) for w in ws], byte)
-        timed(f"row {n}x{k}, gated pairs", [lambda w=w: K.linear_pairs_vector_into(batch, x, w, None, k, seg, [o], F32) for w in ws], byte)
+        pairs = lw.Segments([lw.Segment(n, pkg.ACT_SILU_PAIRS)])
+        timed(f"row {n}x{k}, norm behind the branch, gate and up as pairs", [lambda w=w: K.linear_residual_vector_into(batch, x, y, s, nw, 1e-6, w, None, k, pairs, [o], F32)
+                                                                             for w in ws], byte)
         timed(f"row {n}x{k}, norm in front (like)", [lambda w=w: K.linear_norm_vector_into(batch, x, None, None, nw, 1e-6, w, None, k, seg, [o], F32) for w in ws], byte)
         if n == k:
             timed(f"row {n}x{k}, gated norm in 16 parts", [lambda w=w: K.linear_gated_vector_into(batch, x, y, F32, None, 1e-6, w, None, k, seg, [o], F32, group=k // 16,
@@ -1106,16 +1108,18 @@ def bench_latent_kernels(pkg, ctx, K, steps, warmup):
                                                                                               1e-6) for c in like], (t + 1) * 4 * (2 * 64 + V) * 2)
         timed(f"latent attention, 16 rows at {t}", [lambda c=c: K.latent_attention_rows_into(batch, ql, c, o, BF16, pos, t, 16, H, C, R, cap, 0.07, sink, gate)
                                                     for c in caches], None, 16 * t * H * 2 * (C + R + C))
-    timed("latent prepare, one row", [lambda: K.latent_prepare_into(batch, qr, down, lnorm, freq, pos, ql, F32, caches[0], BF16, 1, H, C, R, row, C, C, cap, 1e-6)])
-    timed("key projection of the queries, one row", [lambda: K.head_linear_into(batch, q, BF16, uk, ql, F32, 1, H, C, D, row)], H * C * D * 2)
-    timed("value projection of the output, one row", [lambda: K.head_linear_into(batch, o, BF16, uv, ql, BF16, 1, H, V, C, V)], H * C * V * 2)
-    keys, values = empty(ctx, cap * H * 192 * 2), empty(ctx, cap * H * V * 2)
+    timed("value projection of the output, one row", [lambda: K.head_linear_into(batch, o, BF16, uv, q, BF16, 1, H, V, C, V)], H * C * V * 2)
+    timed("latent queries and cache row, one row", [lambda: K.latent_queries_into(batch, q, uk, qr, down, lnorm, freq, pos, ql, caches[0], BF16, 1, H, D, C, R, cap, 1e-6)],
+          H * C * D * 2)
+    keys, values = empty(ctx, cap * H * 256 * 2), empty(ctx, cap * H * V * 2)
     for t, rows in ((0, 2048), (T, 256), (2048, 2048)):
         pos, n = pkg.Buffer.from_slice(ctx, np.array([t], np.uint32)), t + rows
         pairs = rows * t + rows * (rows + 1) / 2
         timed(f"latent prepare, {rows} rows", [lambda: K.latent_prepare_into(batch, qr, down, lnorm, freq, pos, q, BF16, caches[0], BF16, rows, H, C, R, 192, D, D, cap, 1e-6)],
               rows * (H * R * (4 + 2) + (C + R) * 4 + row * 2))
         timed(f"keys and values of {n} positions", [lambda: K.latent_expand_into(batch, caches[0], BF16, up, keys, values, n, H, D, R, V, C)], None, 2.0 * n * H * (D + V) * C)
+        seg = lw.Segments([lw.Segment(H * (D + V))])
+        timed(f"rows {n}x{C}x{H * (D + V)} (like)", [lambda: K.linear_rows_into(batch, caches[0], BF16, up, None, n, C, seg, [keys], BF16)], None, 2.0 * n * H * (D + V) * C)
         timed(f"attention prefill, {rows} rows at {t}", [lambda: K.attention_rows_into(batch, q, keys, values, o, BF16, pos, t, rows, H, H, 1, D + R, V, cap, 0.07, sink=sink,
                                                                                        gate=gate)], None, pairs * H * 2 * (D + R + V))
         timed(f"attention prefill, {rows} rows at {t} (like)", [lambda: K.attention_rows_into(batch, q, like[0][0], like[0][1], o, BF16, pos, t, rows, H, 4, 2, 64, V, cap, 0.125,

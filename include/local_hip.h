@@ -629,7 +629,7 @@ LH_API uint32_t lh_flash_split_count(uint32_t eff_seq_len);
 #define LH_ACT_GELU_TANH 2
 #define LH_ACT_RELU_SQUARED 3
 #define LH_ACT_SIGMOID 4
-#define LH_ACT_SILU_PAIRS 5   /* products of many rows: columns come as (gate, up) pairs and leave as silu(gate) * up */
+#define LH_ACT_SILU_PAIRS 5   /* columns come as (gate, up) pairs and leave as silu(gate) * up; the product's only segment for one row */
 #define LH_ROWS 0
 #define LH_ROWS_AT_POSITION 1
 #define LH_BLOCKS_AT_POSITION 2
@@ -667,7 +667,6 @@ LH_API int lh_linear_rows_into(lh_batch* batch, const lh_buffer* input, int inpu
  *   norm    x = rms_norm(input + add) * norm_weight, input f32, `add` may be null; input + add goes to `store` when given
  *           (which must not be `input`: every workgroup reads it)
  *   residual  x = input + rms_norm(branch) * norm_weight, all f32; x goes to `store` when given (not `input` or `branch`)
- *   pairs   x = silu(input[2i]) * input[2i + 1], input f32 [2 k]
  *   gated   x = the output of lh_gated_norm_rows_into, input f32, gate of gate_dtype; lh_gated_vector_fits(k, group) says
  *           whether the parts suit this form */
 LH_API int lh_linear_vector_into(lh_batch* batch, const lh_buffer* input, int input_dtype, const lh_buffer* weight,
@@ -687,11 +686,6 @@ LH_API int lh_linear_residual_vector_into(lh_batch* batch, const lh_buffer* inpu
                                           const uint32_t* ns, const uint32_t* acts, const uint32_t* heads,
                                           const uint32_t* padded, const uint32_t* layouts, lh_buffer* const* outputs,
                                           int output_dtype, int accumulate, const lh_buffer* position);
-LH_API int lh_linear_pairs_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* weight,
-                                       const lh_buffer* bias, uint32_t k, uint32_t count, const uint32_t* ns,
-                                       const uint32_t* acts, const uint32_t* heads, const uint32_t* padded,
-                                       const uint32_t* layouts, lh_buffer* const* outputs, int output_dtype,
-                                       int accumulate, const lh_buffer* position);
 LH_API uint32_t lh_gated_vector_fits(uint32_t k, uint32_t group);
 LH_API int lh_linear_gated_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* gate, int gate_dtype,
                                        uint32_t gate_act, int gate_first, const lh_buffer* norm_weight,
@@ -732,7 +726,8 @@ LH_API int lh_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_
  *            (keys), then heads * vdim (values)][rank]; keys get the rotated part behind their dim columns
  *   rows     attention of queries that the key projection has been applied to, in the latent space: q f32 [rows, heads,
  *            lh_latent_row], output [rows, heads, rank] of `dtype`, of which the value projection is then taken.  sink and
- *            gate as above. */
+ *            gate as above.
+ *   queries  prepare and the key projection of q [rows, heads, dim] (weight [heads, rank, dim]) into the queries of rows */
 LH_API uint32_t lh_latent_padded_rank(uint32_t rank);
 LH_API uint32_t lh_latent_row(uint32_t rank, uint32_t rot);
 LH_API int lh_latent_prepare_into(lh_batch* batch, const lh_buffer* q_rot, const lh_buffer* down, const lh_buffer* norm_weight,
@@ -748,6 +743,10 @@ LH_API int lh_latent_attention_rows_into(lh_batch* batch, const lh_buffer* q, co
                                          int dtype, const lh_buffer* position, uint32_t max_position, uint32_t rows,
                                          uint32_t heads, uint32_t rank, uint32_t rot, uint32_t capacity, float scale,
                                          const lh_buffer* sink, const lh_buffer* gate);
+LH_API int lh_latent_queries_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* key_weight, const lh_buffer* q_rot,
+                                  const lh_buffer* down, const lh_buffer* norm_weight, const lh_buffer* frequencies,
+                                  const lh_buffer* position, lh_buffer* output, lh_buffer* cache, int dtype, uint32_t rows,
+                                  uint32_t heads, uint32_t dim, uint32_t rank, uint32_t rot, uint32_t capacity, float eps);
 
 /* Linear attention with a fixed decay per head: per token the head's state M shrinks by its decay, takes in the outer
  * product of key and value, and is read with the query (M <- a M + k (x) v, y = q M), from the state the call before left.  q, k [rows, heads, dim_padded], v [rows, heads, vdim] of `dtype`; state f32 [heads, vdim, dim_padded]

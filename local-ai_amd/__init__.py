@@ -814,12 +814,6 @@ class Kernels:
                                                       weight._h, _opt(bias), _u32(k), *segments.args, _handles(outputs),
                                                       C.c_int(output_dtype), C.c_int(bool(accumulate)), _opt(position)))
 
-    def linear_pairs_vector_into(self, batch, input, weight, bias, k, segments, outputs, output_dtype, accumulate=False,
-                                 position=None):
-        _check(self._l.lh_linear_pairs_vector_into(batch._h, input._h, weight._h, _opt(bias), _u32(k), *segments.args,
-                                                   _handles(outputs), C.c_int(output_dtype), C.c_int(bool(accumulate)),
-                                                   _opt(position)))
-
     def gated_vector_fits(self, k, group):
         return bool(self._l.lh_gated_vector_fits(_u32(k), _u32(group)))
 
@@ -888,6 +882,12 @@ class Kernels:
         _check(self._l.lh_latent_attention_rows_into(batch._h, q._h, cache._h, output._h, C.c_int(dtype), position._h,
                                                      _u32(max_position), _u32(rows), _u32(heads), _u32(rank), _u32(rot),
                                                      _u32(capacity), C.c_float(scale), _opt(sink), _opt(gate)))
+
+    def latent_queries_into(self, batch, q, key_weight, q_rot, down, norm_weight, frequencies, position, output, cache, dtype, rows,
+                            heads, dim, rank, rot, capacity, eps):
+        _check(self._l.lh_latent_queries_into(batch._h, q._h, key_weight._h, q_rot._h, _opt(down), _opt(norm_weight),
+                                              frequencies._h, position._h, output._h, cache._h, C.c_int(dtype), _u32(rows),
+                                              _u32(heads), _u32(dim), _u32(rank), _u32(rot), _u32(capacity), C.c_float(eps)))
 
     def selective_steps_bytes(self, rows, heads):
         return int(self._l.lh_selective_steps_bytes(_u32(rows), _u32(heads)))

@@ -311,7 +311,6 @@ template <int STAGE>
 __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, uint32_t K) {
     auto gate = [&](uint32_t k) { return lh_gate(st.gate_f32 ? static_cast<const float*>(st.gate)[k] : lh_bf2f(static_cast<const uint16_t*>(st.gate)[k]), st.gate_act); };
     auto value = [&](uint32_t k) {
-        if constexpr (STAGE == kPairs) { const float2 p = reinterpret_cast<const float2*>(st.x)[k]; return p.x * lh_sigmoid(p.x) * p.y; }
         if constexpr (STAGE == kPlain) return st.x_f32 ? static_cast<const float*>(st.x)[k] : lh_bf2f(static_cast<const uint16_t*>(st.x)[k]);
         float v = static_cast<const float*>(st.x)[k];
         if (STAGE == kNorm && st.add) v += st.add[k];
@@ -333,7 +332,7 @@ __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, u
             xs[x_place(k)] = v;
             if (st.store && blockIdx.x == 0 && k < K) st.store[k] = v;
         }
-    } else if constexpr (STAGE == kPlain || STAGE == kPairs) {
+    } else if constexpr (STAGE == kPlain) {
         for (uint32_t k = threadIdx.x; k < padded; k += blockDim.x) xs[x_place(k)] = k < K ? value(k) : 0.0f;
     } else {
         constexpr int R = 8;                                  // elements a thread keeps between the passes; the rest are read again
@@ -368,22 +367,38 @@ __device__ void stage_vector(const VectorStage& st, float* xs, float* scratch, u
     __syncthreads();
 }
 
+// Which rows a wave (or workgroup) takes: every `count`-th from `first` on; of (gate, up) pairs both.
+struct RowWalk {
+    const uint32_t first, count, pairs;
+    __device__ __forceinline__ uint32_t row(uint32_t i) const { return pairs ? 2 * (first + (i >> 1) * count) + (i & 1) : first + i * count; }
+};
+
+// Stores the finished sums of rows i0 .. i0 + n - 1 of a walk, one per lane.
+__device__ __forceinline__ void store_sums(const LhSegments& seg, const float* bias, const RowWalk& walk, uint32_t i0, uint32_t n, uint32_t lane, float v) {
+    const uint32_t row = walk.row(i0 + lane);
+    if (bias && lane < n) v += bias[row];
+    if (walk.pairs) {                                         // n is even, and a pair's factors are in neighbouring lanes
+        const float up = lh_dpp_f<LH_DPP_QUAD_XOR1>(v);
+        if (lane < n && !(lane & 1)) lh_segment_put(seg, 0, row >> 1, v * lh_sigmoid(v) * up);
+    } else if (lane < n) lh_segment_store(seg, 0, row, v, seg.position ? *seg.position : 0u);
+}
+
 // The finished sums of a wave's rows, one per lane, stored 64 at a time: bias, activation and destination then cost one pass
 // for all of them, and no load of that pass has to wait for weights that were requested in between.
 struct RowSums {
     const LhSegments& seg;
     const float* bias;
-    const uint32_t lane, step;
-    uint32_t row0, n = 0;
+    const RowWalk& walk;
+    const uint32_t lane;
+    uint32_t i0 = 0, n = 0;
     float mine = 0.0f;
     __device__ __forceinline__ void add(float total) {
         mine = n == lane ? total : mine;
         if (++n == 64) flush();
     }
     __device__ __forceinline__ void flush() {
-        const uint32_t row = row0 + lane * step;
-        if (lane < n) lh_segment_store(seg, 0, row, mine + (bias ? bias[row] : 0.0f), seg.position ? *seg.position : 0u);
-        row0 += n * step;
+        store_sums(seg, bias, walk, i0, n, lane, mine);
+        i0 += n;
         n = 0;
     }
 };
@@ -398,11 +413,12 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
     __shared__ float scratch[4];
     const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     stage_vector<STAGE>(st, xs, scratch, K);
-    RowSums sums{seg, bias, lane, gridDim.x * 4, blockIdx.x * 4 + wave};
+    const RowWalk walk{blockIdx.x * 4 + wave, gridDim.x * 4, seg.pairs};
+    RowSums sums{seg, bias, walk, lane};
     if constexpr (VEC) {
         constexpr uint32_t kPass = 512u * NL;
-        const uint32_t ppr = (K + kPass - 1) / kPass, row_step = gridDim.x * 4, last = (K >> 3) - 1;
-        uint32_t row = blockIdx.x * 4 + wave, pass = 0;
+        const uint32_t ppr = (K + kPass - 1) / kPass, last = (K >> 3) - 1;
+        uint32_t at = 0, row = walk.row(0), pass = 0;
         auto issue = [&](uint4 (&v)[NL], uint32_t r, uint32_t ps) {
             const uint16_t* wr = W + (size_t)r * K;
 #pragma unroll
@@ -427,7 +443,7 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
         };
         auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {   // false: that was the wave's last pass
             uint32_t nrow = row, npass = pass + 1;
-            if (npass == ppr) { npass = 0; nrow = row + row_step; }
+            if (npass == ppr) { npass = 0; nrow = walk.row(++at); }
             const bool more = nrow < N;
             if (more) issue(nxt, nrow, npass);
             consume(cur, row, pass);
@@ -440,7 +456,7 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
             while (step(p, q) && step(q, p)) {}
         }
     } else {
-        for (uint32_t row = blockIdx.x * 4 + wave; row < N; row += gridDim.x * 4) {
+        for (uint32_t i = 0, row; (row = walk.row(i)) < N; i++) {
             float acc = 0.0f;
             for (uint32_t k = lane; k < K; k += 64) acc = __builtin_fmaf(lh_bf2f(W[(size_t)row * K + k]), xs[x_place(k)], acc);
             sums.add(lh_group_sum(acc, 64));
@@ -453,35 +469,36 @@ __global__ __launch_bounds__(256) void matvec_bf16_kernel(const VectorStage st, 
 template <int STAGE, int NL>
 __global__ __launch_bounds__(256) void matvec_bf16_reg_kernel(const VectorStage st, const uint16_t* __restrict__ W, const float* __restrict__ bias, const LhSegments seg,
                                                              uint32_t N, uint32_t K) {
-    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, row_step = gridDim.x * 4, last = (K >> 3) - 1;
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, last = (K >> 3) - 1;
+    const RowWalk walk{blockIdx.x * 4 + wave, gridDim.x * 4, seg.pairs};
     auto issue = [&](uint4 (&v)[NL], uint32_t r) {
         const uint16_t* wr = W + (size_t)r * K;
 #pragma unroll
         for (int c = 0; c < NL; c++) v[c] = lh_ld16_stream(wr + 8 * min(64u * c + lane, last));
     };
-    uint32_t row = blockIdx.x * 4 + wave;
-    if (row >= N) return;
+    uint32_t at = 0;
+    if (walk.row(0) >= N) return;
     uint4 p[NL], q[NL];
-    issue(p, row);
-    RowSums sums{seg, bias, lane, row_step, row};
+    issue(p, walk.row(0));
+    RowSums sums{seg, bias, walk, lane};
     float xr[NL][8];
     lh_vector_registers<STAGE, NL>(st, K, lane, blockIdx.x == 0 && wave == 0 && st.store != nullptr, xr);
     auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {   // false: that was the wave's last row
-        const bool more = row + row_step < N;
-        if (more) issue(nxt, row + row_step);
+        const uint32_t next = walk.row(++at);
+        const bool more = next < N;
+        if (more) issue(nxt, next);
         float acc = 0.0f;
 #pragma unroll
         for (int c = 0; c < NL; c++) acc = lh_dot8(cur[c], xr[c], acc);
         sums.add(lh_group_sum(acc, 64));
-        row += row_step;
         return more;
     };
     while (step(p, q) && step(q, p)) {}
     sums.flush();
 }
 
-// Rows longer than a wave's registers: the four waves of a workgroup take a quarter of the columns each, and the quarters of up to 64 rows meet in LDS.  Plain vectors and pairs only: a norm would need all quarters.
-template <int STAGE, int NL>
+// Rows longer than a wave's registers: the four waves of a workgroup take a quarter of the columns each, and the quarters of up to 64 rows meet in LDS.  Plain vectors only: a norm would need all quarters.
+template <int NL>
 __global__ __launch_bounds__(256) void matvec_bf16_quarter_kernel(const VectorStage st, const uint16_t* __restrict__ W, const float* __restrict__ bias, const LhSegments seg,
                                                                  uint32_t N, uint32_t K, uint32_t quarter) {
     __shared__ float sums[4][64];
@@ -492,33 +509,33 @@ __global__ __launch_bounds__(256) void matvec_bf16_quarter_kernel(const VectorSt
 #pragma unroll
         for (int c = 0; c < NL; c++) v[c] = lh_ld16_stream(wr + 8 * min(64u * c + lane, last));
     };
-    uint32_t row = blockIdx.x, base = blockIdx.x, n = 0;
+    const RowWalk walk{blockIdx.x, gridDim.x, seg.pairs};
+    uint32_t at = 0, i0 = 0, n = 0;
+    if (walk.row(0) >= N) return;
     uint4 p[NL], q[NL];
-    issue(p, row);
+    issue(p, walk.row(0));
     VectorStage part = st;
-    part.x = STAGE == kPairs ? (const void*)(static_cast<const float*>(st.x) + 2 * kb) : st.x_f32 ? (const void*)(static_cast<const float*>(st.x) + kb) : (const void*)(static_cast<const uint16_t*>(st.x) + kb);
+    part.x = st.x_f32 ? (const void*)(static_cast<const float*>(st.x) + kb) : (const void*)(static_cast<const uint16_t*>(st.x) + kb);
     float xr[NL][8], mine = 0.0f;
-    lh_vector_registers<STAGE, NL>(part, len, lane, false, xr);
+    lh_vector_registers<kPlain, NL>(part, len, lane, false, xr);
     auto flush = [&]() {
         sums[wave][lane] = mine;
         __syncthreads();
-        const uint32_t r = base + lane * gridDim.x;
-        if (wave == 0 && lane < n)
-            lh_segment_store(seg, 0, r, ((sums[0][lane] + sums[1][lane]) + (sums[2][lane] + sums[3][lane])) + (bias ? bias[r] : 0.0f), seg.position ? *seg.position : 0u);
+        if (wave == 0) store_sums(seg, bias, walk, i0, n, lane, (sums[0][lane] + sums[1][lane]) + (sums[2][lane] + sums[3][lane]));
         __syncthreads();
-        base += n * gridDim.x;
+        i0 += n;
         n = 0;
     };
     auto step = [&](const uint4 (&cur)[NL], uint4 (&nxt)[NL]) {
-        const bool more = row + gridDim.x < N;
-        if (more) issue(nxt, row + gridDim.x);
+        const uint32_t next = walk.row(++at);
+        const bool more = next < N;
+        if (more) issue(nxt, next);
         float acc = 0.0f;
 #pragma unroll
         for (int c = 0; c < NL; c++) acc = lh_dot8(cur[c], xr[c], acc);
         acc = lh_group_sum(acc, 64);
         mine = n == lane ? acc : mine;
         if (++n == 64) flush();
-        row += gridDim.x;
         return more;
     };
     while (step(p, q) && step(q, p)) {}
@@ -531,9 +548,10 @@ template <int STAGE>
 int launch_vector(lh_context* ctx, const VectorStage& st, const uint16_t* W, const float* bias, const LhSegments& seg, uint32_t N, uint32_t K, const char* op) {
     LH_REQUIRE(K > 0 && K <= kMaxVectorK, "%s: k %u outside 1..=%u", op, K, kMaxVectorK);
     const size_t lds = (size_t)(K + 511) / 512 * 512 * 4;
+    const uint32_t takes = seg.pairs ? N / 2 : N;             // rows, or pairs of rows
     const bool vec = K % 8 == 0 && ((uintptr_t)W & 15) == 0;
     if (vec && K <= 4096 && lh_stage_aligned(st)) {
-        const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * (K <= 2048 ? 4 : 2));
+        const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)takes + 3) / 4, (uint64_t)ctx->cu_count * (K <= 2048 ? 4 : 2));
 #define LH_MVR(NLOADS) hipLaunchKernelGGL((matvec_bf16_reg_kernel<STAGE, NLOADS>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K)
         if (K <= 512) LH_MVR(1);
         else if (K <= 1024) LH_MVR(2);
@@ -542,14 +560,14 @@ int launch_vector(lh_context* ctx, const VectorStage& st, const uint16_t* W, con
 #undef LH_MVR
         return lh_check_launch(op);
     }
-    if constexpr (STAGE == kPlain || STAGE == kPairs) if (vec && K <= 16384 && lh_stage_aligned(st)) {
-        const uint32_t quarter = ((K + 3) / 4 + 7) / 8 * 8, grid = (uint32_t)std::min<uint64_t>(N, (uint64_t)ctx->cu_count * 4);
-        if (quarter <= 1024) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 2>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
-        else if (quarter <= 2048) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 4>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
-        else hipLaunchKernelGGL((matvec_bf16_quarter_kernel<STAGE, 8>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+    if constexpr (STAGE == kPlain) if (vec && K <= 16384 && lh_stage_aligned(st)) {
+        const uint32_t quarter = ((K + 3) / 4 + 7) / 8 * 8, grid = (uint32_t)std::min<uint64_t>(takes, (uint64_t)ctx->cu_count * 4);
+        if (quarter <= 1024) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<2>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else if (quarter <= 2048) hipLaunchKernelGGL((matvec_bf16_quarter_kernel<4>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
+        else hipLaunchKernelGGL((matvec_bf16_quarter_kernel<8>), dim3(grid), dim3(256), 0, ctx->stream, st, W, bias, seg, N, K, quarter);
         return lh_check_launch(op);
     }
-    const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)N + 3) / 4, (uint64_t)ctx->cu_count * 4);
+    const uint32_t grid = (uint32_t)std::min<uint64_t>(((uint64_t)takes + 3) / 4, (uint64_t)ctx->cu_count * 4);
 #define LH_MV(NLOADS, V)                                                                                                               \
     do {                                                                                                                               \
         if (lds > 64 * 1024 - 64) {                                                                                                    \
@@ -583,14 +601,13 @@ int vector_entry(lh_batch* batch, const char* op, int stage, const VectorStage& 
                  lh_buffer* const* outputs, int output_dtype, int accumulate, const lh_buffer* position) {
     LhSegments seg;
     LH_TRY(lh_make_segments(seg, op, 1, 0, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position));
-    LH_REQUIRE(!seg.pairs, "%s: pairs are stored as they are for one row", op);
+    LH_REQUIRE(!seg.pairs || seg.count == 1, "%s: pairs beside other segments", op);
     const uint32_t n = seg.n0[seg.count];
     LH_TRY(check_common(batch, weight, bias, k, n, op));
     const uint16_t* W = (const uint16_t*)weight->ptr;
     const float* b = bias ? (const float*)bias->ptr : nullptr;
     int r;
-    if (stage == kPairs) r = launch_vector<kPairs>(batch->ctx, st, W, b, seg, n, k, op);
-    else if (stage == kResidual) r = launch_vector<kResidual>(batch->ctx, st, W, b, seg, n, k, op);
+    if (stage == kResidual) r = launch_vector<kResidual>(batch->ctx, st, W, b, seg, n, k, op);
     else if (stage == kPlain) r = launch_vector<kPlain>(batch->ctx, st, W, b, seg, n, k, op);
     else if (stage == kNorm) r = launch_vector<kNorm>(batch->ctx, st, W, b, seg, n, k, op);
     else r = launch_vector<kGated>(batch->ctx, st, W, b, seg, n, k, op);
@@ -704,17 +721,6 @@ int lh_linear_residual_vector_into(lh_batch* batch, const lh_buffer* input, cons
     st.x = input->ptr; st.x_f32 = 1; st.add = (const float*)branch->ptr; st.store = store ? (float*)store->ptr : nullptr;
     st.norm_weight = (const float*)norm_weight->ptr; st.eps = eps;
     return vector_entry(batch, op, kResidual, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
-}
-
-int lh_linear_pairs_vector_into(lh_batch* batch, const lh_buffer* input, const lh_buffer* weight, const lh_buffer* bias, uint32_t k, uint32_t count,
-                                const uint32_t* ns, const uint32_t* acts, const uint32_t* heads, const uint32_t* padded, const uint32_t* layouts,
-                                lh_buffer* const* outputs, int output_dtype, int accumulate, const lh_buffer* position) {
-    const char* op = "linear_pairs_vector";
-    LH_REQUIRE(batch, "%s: batch is null", op);
-    LH_NEED(input, (size_t)k * 8, op, "input");
-    VectorStage st{};
-    st.x = input->ptr; st.x_f32 = 1;
-    return vector_entry(batch, op, kPairs, st, weight, bias, k, count, ns, acts, heads, padded, layouts, outputs, output_dtype, accumulate, position);
 }
 
 uint32_t lh_gated_vector_fits(uint32_t k, uint32_t group) {

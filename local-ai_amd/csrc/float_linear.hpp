@@ -28,9 +28,9 @@ uint32_t lh_expert_tile_rows(uint32_t slots, uint32_t experts);
 // ---- one row: the activation vector in registers -------------------------------------------------------------------------
 // Up to 4096 columns a wave keeps the vector itself: lane l holds the NL chunks of eight elements 8 (64 c + l), which is what
 // it multiplies in every row.  The norm before the product is then a sum over the wave, with no barrier and no LDS.
-enum { kPlain = 0, kNorm = 1, kGated = 2, kResidual = 3, kPairs = 4 };
+enum { kPlain = 0, kNorm = 1, kGated = 2, kResidual = 3 };
 struct VectorStage {
-    const void* x;             // plain: x_f32 ? f32 : bf16; the others: f32 (pairs: 2 K values, gate and up in turn)
+    const void* x;             // plain: x_f32 ? f32 : bf16; the others: f32
     uint32_t x_f32;
     const float* add;          // norm: may be null; residual: what is normed and added
     float* store;              // norm, residual: receives the sum (workgroup 0), may be null
@@ -63,16 +63,7 @@ __device__ __forceinline__ void lh_vector_registers(const VectorStage& st, uint3
         for (int j = 0; j < 8; j++) xr[c][j] = 0.0f;
         if constexpr (kNormed) s[c] = 0.0f;
         if (k >= K) continue;
-        if constexpr (STAGE == kPairs) {
-            float a[8], b[8];
-            lh_ld8(static_cast<const float*>(st.x) + 2 * k, a);
-            lh_ld8(static_cast<const float*>(st.x) + 2 * k + 8, b);
-#pragma unroll
-            for (int j = 0; j < 4; j++) {
-                xr[c][j] = a[2 * j] * lh_sigmoid(a[2 * j]) * a[2 * j + 1];
-                xr[c][4 + j] = b[2 * j] * lh_sigmoid(b[2 * j]) * b[2 * j + 1];
-            }
-        } else if (STAGE == kPlain && !st.x_f32) lh_ld8(static_cast<const uint16_t*>(st.x) + k, xr[c]);
+        if (STAGE == kPlain && !st.x_f32) lh_ld8(static_cast<const uint16_t*>(st.x) + k, xr[c]);
         else lh_ld8(static_cast<const float*>(st.x) + k, xr[c]);
         if constexpr (STAGE == kNorm) if (st.add) {
             float b[8];

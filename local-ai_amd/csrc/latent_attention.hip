@@ -31,12 +31,11 @@ __device__ __forceinline__ float rotated(const float* v, uint32_t i, float posit
     return i & 1 ? w * c + u * s : u * c - w * s;
 }
 
-// grid (rows, 1 + query workgroups): workgroup y = 0 writes the cache row, the others 1024 columns of the queries each.
+// Row t; piece 0 writes the cache row, the others 1024 columns of the queries each.
 template <typename TQ, typename T>
-__global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepareArgs a) {
-    __shared__ float scratch[4];
-    const uint32_t t = blockIdx.x, pos = *a.position + t;
-    if (blockIdx.y == 0) {
+__device__ __forceinline__ void prepare_piece(const PrepareArgs& a, uint32_t t, uint32_t piece, float* scratch) {
+    const uint32_t pos = *a.position + t;
+    if (piece == 0) {
         if (!a.down || pos >= a.capacity) return;
         const float* d = a.down + (size_t)t * (a.rank + a.rot);
         T* row = static_cast<T*>(a.cache) + (size_t)pos * a.row;
@@ -54,13 +53,19 @@ __global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepareArgs a
     const uint32_t width = a.q_ld - a.clear_column, total = a.heads * width;
 #pragma unroll
     for (uint32_t j = 0; j < 4; j++) {
-        const uint32_t e = (blockIdx.y - 1) * 1024 + j * 256 + threadIdx.x;
+        const uint32_t e = (piece - 1) * 1024 + j * 256 + threadIdx.x;
         if (e >= total) return;
         const uint32_t h = e / width, c = a.clear_column + e % width;
         const float v = c >= a.rot_column && c < a.rot_column + a.rot
                             ? rotated(a.q_rot + ((size_t)t * a.heads + h) * a.rot, c - a.rot_column, (float)pos, a.frequencies) : 0.0f;
         lh_st(static_cast<TQ*>(a.q), ((size_t)t * a.heads + h) * a.q_ld + c, v);
     }
+}
+
+template <typename TQ, typename T>
+__global__ __launch_bounds__(256) void latent_prepare_kernel(const PrepareArgs a) {
+    __shared__ float scratch[4];
+    prepare_piece<TQ, T>(a, blockIdx.x, blockIdx.y, scratch);
 }
 
 // ---- one small product per head --------------------------------------------------------------------------------------------
@@ -82,11 +87,10 @@ __device__ __forceinline__ lh_bf16x8 operand8(const uint16_t* row, uint32_t k, u
     return __builtin_bit_cast(lh_bf16x8, v);
 }
 
-// grid (column tiles, heads, row tiles): 16 columns x 16 rows of one head, the four waves take quarters of K.
+// 16 columns x 16 rows of one head, the four waves take quarters of K.
 template <typename TO>
-__global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a) {
-    __shared__ lh_f32x4 part[4][64];
-    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6, h = blockIdx.y, n0 = blockIdx.x * 16, m0 = blockIdx.z * 16;
+__device__ __forceinline__ void head_tile(const HeadArgs& a, uint32_t h, uint32_t n0, uint32_t m0, lh_f32x4 (&part)[4][64]) {
+    const uint32_t lane = threadIdx.x & 63, wave = threadIdx.x >> 6;
     const uint32_t steps = (a.K + 31) / 32, per = (steps + 3) / 4, s0 = min(wave * per, steps), s1 = min(s0 + per, steps);
     const uint16_t* w = a.W + ((size_t)h * a.N + min(n0 + (lane & 15), a.N - 1)) * a.K;
     const uint16_t* x = static_cast<const uint16_t*>(a.x) + ((size_t)min(m0 + (lane & 15), a.rows - 1) * a.heads + h) * a.K;
@@ -101,6 +105,21 @@ __global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a)
     const uint32_t l = threadIdx.x >> 2, r = threadIdx.x & 3, m = m0 + (l & 15), n = n0 + (l >> 4) * 4 + r;   // thread: one output
     if (m >= a.rows || n >= a.N) return;
     lh_st(static_cast<TO*>(a.out), ((size_t)m * a.heads + h) * a.ld + n, (part[0][l][r] + part[1][l][r]) + (part[2][l][r] + part[3][l][r]));
+}
+
+// grid (column tiles, heads, row tiles)
+template <typename TO>
+__global__ __launch_bounds__(256) void head_linear_mfma_kernel(const HeadArgs a) {
+    __shared__ lh_f32x4 part[4][64];
+    head_tile<TO>(a, blockIdx.y, blockIdx.x * 16, blockIdx.z * 16, part);
+}
+
+// Both steps in front of the attention of few rows: the tiles of the key projection, then the pieces of the preparation.
+__global__ __launch_bounds__(256) void latent_queries_kernel(const HeadArgs a, const PrepareArgs p, uint32_t tiles, uint32_t pieces) {
+    __shared__ lh_f32x4 part[4][64];
+    const uint32_t nt = (a.N + 15) / 16, i = blockIdx.x;
+    if (i < tiles) head_tile<float>(a, i / nt % a.heads, i % nt * 16, i / (nt * a.heads) * 16, part);
+    else prepare_piece<float, uint16_t>(p, (i - tiles) / pieces, (i - tiles) % pieces, reinterpret_cast<float*>(&part[0][0]));
 }
 
 // f32: a wave per output.
@@ -137,38 +156,35 @@ __device__ __forceinline__ s16x4 transposed4(const void* lds) {
 }
 
 // grid: row tiles x splits; packed row r = head r % heads of query row r / heads.  The blocks of 32 positions of the visible range
-// are dealt out in contiguous runs to the 4 * splits waves of a row tile.  A wave keeps its block in its own part of LDS (so the
-// waves need no barrier), in tiles of 8 key rows x 8 chunks of 16 bytes, chunk c of row k at place c ^ k of its row: a load fills
-// one tile, and every address is one of a few per lane plus a constant.  The scores read it row by row, the values through the
-// transposing LDS read.  A query value enters as the sum of two bf16 terms.
+// are dealt out in contiguous runs to the splits of a row tile.  The four waves share a block in LDS, in tiles of 8 key rows x 8
+// chunks of 16 bytes, chunk c of row k at place c ^ k of its row (a load fills one tile, and every address is one of a few per
+// lane plus a constant), while the next block is on its way into a second buffer.  A wave takes every fourth 32 columns of the
+// scores' sums, which meet in LDS, and a quarter of the value columns, which it reads through the transposing LDS read.  A query
+// value enters as the sum of two bf16 terms.
 template <int DV>
-__global__ __launch_bounds__(256, DV > 256 ? 1 : 2) void latent_split_kernel(const AttentionArgs a) {
-    constexpr int DQ = DV + kRotPad, KC = DQ / 8, KT = KC / 8;
-    extern __shared__ __align__(16) uint4 sm[];             // [4 waves][32 * KC]; at the end the partial results [4 waves][16 rows][DV + 4]
+__global__ __launch_bounds__(256) void latent_split_kernel(const AttentionArgs a) {
+    constexpr int DQ = DV + kRotPad, KT = DQ / 64, NC = (DQ / 32 + 3) / 4, ND = DV / 64, kBlock = 4 * KT * 64;
+    extern __shared__ __align__(16) uint4 sm[];             // two blocks, then the partial scores [4 waves][2 tiles][64 lanes]
+    lh_f32x4* sums = reinterpret_cast<lh_f32x4*>(sm + 2 * kBlock);
     const uint32_t tid = threadIdx.x, lane = tid & 63, wave = tid >> 6, g = lane >> 4, lc = lane & 15;
     const uint32_t split = blockIdx.x % a.splits, tile = blockIdx.x / a.splits, packed = a.rows * a.heads, start = *a.position;
     const uint32_t row0 = tile * 16, row_last = min(row0 + 16, packed) - 1, row = row0 + lc;
     const uint32_t last_key = min(start + row_last / a.heads, a.capacity - 1), nb = last_key / 32 + 1;
     const uint32_t limit = min(start + row / a.heads, last_key), first_limit = start + row0 / a.heads;
-    const uint32_t per = (nb + 4 * a.splits - 1) / (4 * a.splits), w = split * 4 + wave;
-    const uint32_t b0 = min(w * per, nb), b1 = min(b0 + per, nb);
-    uint4* mine = sm + wave * (32 * KC);
+    const uint32_t per = (nb + a.splits - 1) / a.splits, b0 = min(split * per, nb), b1 = min(b0 + per, nb);
     const uint16_t* cache = static_cast<const uint16_t*>(a.keys) + ((lane & 7) ^ (lane >> 3)) * 8;
-    auto load_block = [&](uint32_t b) {
+    auto load_block = [&](uint32_t b) {                       // a wave brings in eight key rows
+        const uint16_t* key = cache + (size_t)min(b * 32 + wave * 8 + (lane >> 3), last_key) * DQ;               // keys past the last are masked
+        uint4* to = sm + (b & 1) * kBlock + wave * KT * 64;
 #pragma unroll
-        for (int k = 0; k < 4; k++) {
-            const uint16_t* row = cache + (size_t)min(b * 32 + k * 8 + (lane >> 3), last_key) * DQ;              // keys past the last are masked
-#pragma unroll
-            for (int i = 0; i < KT; i++) __builtin_amdgcn_global_load_lds((gvoid*)(row + i * 64), (lvoid*)(mine + (k * KT + i) * 64), 16, 0, 0);
-        }
+        for (int i = 0; i < KT; i++) __builtin_amdgcn_global_load_lds((gvoid*)(key + i * 64), (lvoid*)(to + i * 64), 16, 0, 0);
     };
-    if (b0 < b1) load_block(b0);
-
-    lh_bf16x8 qh[DQ / 32], ql[DQ / 32];
+    lh_bf16x8 qh[NC], ql[NC];
 #pragma unroll
-    for (int c = 0; c < DQ / 32; c++) {
+    for (int i = 0; i < NC; i++) {
+        const uint32_t c = i * 4 + wave;
         float f[8];
-        if (row < packed) lh_ld8(static_cast<const float*>(a.q) + (size_t)row * DQ + c * 32 + g * 8, f);
+        if (row < packed && c < DQ / 32) lh_ld8(static_cast<const float*>(a.q) + (size_t)row * DQ + c * 32 + g * 8, f);
         else
 #pragma unroll
             for (int j = 0; j < 8; j++) f[j] = 0.0f;
@@ -178,105 +194,83 @@ __global__ __launch_bounds__(256, DV > 256 ? 1 : 2) void latent_split_kernel(con
             h[j] = lh_pack_bf(f[2 * j], f[2 * j + 1]);
             l[j] = lh_pack_bf(f[2 * j] - __builtin_bit_cast(float, h[j] << 16), f[2 * j + 1] - __builtin_bit_cast(float, h[j] & 0xFFFF0000u));
         }
-        qh[c] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
-        ql[c] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
+        qh[i] = __builtin_bit_cast(lh_bf16x8, (u32x4){h[0], h[1], h[2], h[3]});
+        ql[i] = __builtin_bit_cast(lh_bf16x8, (u32x4){l[0], l[1], l[2], l[3]});
     }
-    lh_f32x4 o[DV / 16];
+    if (b0 < b1) load_block(b0);
+    lh_f32x4 o[ND];
 #pragma unroll
-    for (int d = 0; d < DV / 16; d++) o[d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
+    for (int d = 0; d < ND; d++) o[d] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
     RowState st{-INFINITY, 0.0f};
     const float scale2 = a.scale * kLog2e;
     // score operand: key lc (+ 16), chunk 4 c + g; value operand: key 4 g + lc / 4 (+ 16), columns 16 d + 4 (lane & 3) ..
-    const uint4* kp = mine + (lc >> 3) * (KT * 64) + (lc & 7) * 8;
+    const uint4* kp = sm + (lc >> 3) * (KT * 64) + (lc & 7) * 8;
     const uint32_t vk = g * 4 + (lc >> 2);
-    const char* vp = reinterpret_cast<const char*>(mine + (vk >> 3) * (KT * 64) + (vk & 7) * 8) + (lane & 1) * 8;
+    const char* vp = reinterpret_cast<const char*>(sm + (vk >> 3) * (KT * 64) + (vk & 7) * 8) + (lane & 1) * 8;
 
     for (uint32_t b = b0; b < b1; b++) {
         asm volatile("s_waitcnt vmcnt(0)" ::: "memory");
+        lh_lds_barrier();                                     // the block has arrived, and the one before has been read by all
+        if (b + 1 < b1) load_block(b + 1);
+        const uint32_t buf = (b & 1) * kBlock;
         lh_f32x4 s[2], low[2];                                // four sums that do not wait for each other
 #pragma unroll
         for (int t = 0; t < 2; t++) s[t] = low[t] = (lh_f32x4){0.f, 0.f, 0.f, 0.f};
 #pragma unroll
-        for (int c = 0; c < DQ / 32; c++)
+        for (int i = 0; i < NC; i++) {
+            const uint32_t c = i * 4 + wave;
+            if (i * 4 + 3 >= DQ / 32 && c >= DQ / 32) break;
 #pragma unroll
             for (int t = 0; t < 2; t++) {
-                const lh_bf16x8 k = __builtin_bit_cast(lh_bf16x8, kp[t * 2 * KT * 64 + (c >> 1) * 64 + (((c & 1) * 4 + g) ^ (lc & 7))]);
-                low[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, ql[c], low[t], 0, 0, 0);
-                s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qh[c], s[t], 0, 0, 0);
+                const lh_bf16x8 k = __builtin_bit_cast(lh_bf16x8, kp[buf + t * 2 * KT * 64 + (c >> 1) * 64 + (((c & 1) * 4 + g) ^ (lc & 7))]);
+                low[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, ql[i], low[t], 0, 0, 0);
+                s[t] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(k, qh[i], s[t], 0, 0, 0);
             }
+        }
 #pragma unroll
-        for (int t = 0; t < 2; t++)
+        for (int t = 0; t < 2; t++) sums[(wave * 2 + t) * 64 + lane] = s[t] + low[t];
+        lh_lds_barrier();
 #pragma unroll
-            for (int r = 0; r < 4; r++) s[t][r] += low[t][r];
+        for (int t = 0; t < 2; t++) s[t] = (sums[t * 64 + lane] + sums[(2 + t) * 64 + lane]) + (sums[(4 + t) * 64 + lane] + sums[(6 + t) * 64 + lane]);
         lh_bf16x8 p[1][3];
         const float alpha = softmax_step<1>(s, st, scale2, b * 32, limit, b * 32 + 31 > first_limit, lane, p);
         if (__ballot(alpha != 1.0f)) {
 #pragma unroll
-            for (int d = 0; d < DV / 16; d++)
+            for (int d = 0; d < ND; d++)
 #pragma unroll
                 for (int r = 0; r < 4; r++) o[d][r] *= alpha;
         }
+        lh_bf16x8 vf[ND];
 #pragma unroll
-        for (int d0 = 0; d0 < DV / 16; d0 += 4) {
-            lh_bf16x8 vf[4];
-#pragma unroll
-            for (int d = 0; d < 4; d++) {
-                const char* v0 = vp + (((2 * d + ((lane & 3) >> 1)) ^ (vk & 7)) + (d0 >> 2) * 64) * 16;
-                struct { s16x4 x, y; } v = {transposed4(v0), transposed4(v0 + 2 * KT * 64 * 16)};
-                vf[d] = __builtin_bit_cast(lh_bf16x8, v);
-            }
-#pragma unroll
-            for (int z = 2; z >= 0; z--)
-#pragma unroll
-                for (int d = 0; d < 4; d++) o[d0 + d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], p[0][z], o[d0 + d], 0, 0, 0);
+        for (int d = 0; d < ND; d++) {
+            const uint32_t ch = 2 * (wave * ND + d) + ((lane & 3) >> 1);
+            const char* v0 = vp + (buf + ((ch & 7) ^ (vk & 7)) + (ch >> 3) * 64) * 16;
+            struct { s16x4 x, y; } v = {transposed4(v0), transposed4(v0 + 2 * KT * 64 * 16)};
+            vf[d] = __builtin_bit_cast(lh_bf16x8, v);
         }
-        asm volatile("s_waitcnt lgkmcnt(0)" ::: "memory");    // the block has been read: the next may overwrite it
-        if (b + 1 < b1) load_block(b + 1);
+#pragma unroll
+        for (int z = 2; z >= 0; z--)
+#pragma unroll
+            for (int d = 0; d < ND; d++) o[d] = __builtin_amdgcn_mfma_f32_16x16x32_bf16(vf[d], p[0][z], o[d], 0, 0, 0);
     }
-    __syncthreads();
+    const float l = lh_column_sum(st.l);
+    if (row > row_last) return;
     constexpr uint32_t kRow = DV + 4;
-    float* merge = reinterpret_cast<float*>(sm);
-    {
-        const float l = lh_column_sum(st.l);
-        float* d0 = merge + (wave * 16 + lc) * kRow;
-        if (lane < 16) { d0[DV] = st.m; d0[DV + 1] = l; }
+    float* rec = a.partial + (size_t)(tile * a.splits + split) * 16 * kRow + lc * kRow;
 #pragma unroll
-        for (int d = 0; d < DV / 16; d++) *reinterpret_cast<float4*>(d0 + d * 16 + g * 4) = make_float4(o[d][0], o[d][1], o[d][2], o[d][3]);
-    }
-    __syncthreads();
-    float* rec = a.partial + (size_t)(tile * a.splits + split) * 16 * kRow;
-    const uint32_t used = row_last - row0 + 1;
-    for (uint32_t i = tid; i < used * (DV / 4); i += 256) {
-        const uint32_t rr = i / (DV / 4), d = i % (DV / 4) * 4;
-        float m = -INFINITY, l = 0.0f;
-        float4 acc = make_float4(0.f, 0.f, 0.f, 0.f);
-#pragma unroll
-        for (int wv = 0; wv < 4; wv++) m = fmaxf(m, merge[(wv * 16 + rr) * kRow + DV]);
-        const float base = m == -INFINITY ? 0.0f : m;
-#pragma unroll
-        for (int wv = 0; wv < 4; wv++) {
-            const float* s = merge + (wv * 16 + rr) * kRow;
-            const float f = __builtin_amdgcn_exp2f(s[DV] - base);
-            const float4 x = *reinterpret_cast<const float4*>(s + d);
-            l += f * s[DV + 1];
-            acc.x += f * x.x; acc.y += f * x.y; acc.z += f * x.z; acc.w += f * x.w;
-        }
-        float* r = rec + rr * kRow;
-        *reinterpret_cast<float4*>(r + d) = acc;
-        if (d == 0) { r[DV] = m; r[DV + 1] = l; }
-    }
+    for (int d = 0; d < ND; d++) *reinterpret_cast<float4*>(rec + (wave * ND + d) * 16 + g * 4) = make_float4(o[d][0], o[d][1], o[d][2], o[d][3]);
+    if (tid < 16) { rec[DV] = st.m; rec[DV + 1] = l; }
 }
 
 template <int DV>
 int launch_split(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const char* op, uint32_t& launches) {
-    constexpr size_t lds = std::max<size_t>((size_t)4 * 32 * (DV + kRotPad) * 2, (size_t)4 * 16 * (DV + 4) * 4);
-    constexpr uint32_t per_cu = lds > 80 * 1024 ? 1 : lds > 40 * 1024 ? 2 : 3;
-    const uint64_t tiles = ((uint64_t)a.rows * a.heads + 15) / 16, want = (uint64_t)ctx->cu_count * per_cu;
+    constexpr size_t lds = 2 * 32 * (DV + kRotPad) * 2 + 4 * 2 * 64 * 16;
+    const uint64_t tiles = ((uint64_t)a.rows * a.heads + 15) / 16, want = (uint64_t)ctx->cu_count * (tiles > 2 ? 2 : 1);
     const uint32_t max_blocks = (uint32_t)std::min<uint64_t>((uint64_t)max_position + a.rows, a.capacity) / 32 + 1;
     const size_t rec = (size_t)tiles * 16 * (DV + 4) * 4;
     const uint32_t room = (uint32_t)std::min<size_t>(ctx->workspace_bytes / rec, kMaxSplits);
     LH_REQUIRE(room >= 1, "%s: %u rows of %u heads exceed the workspace", op, a.rows, a.heads);
-    a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({max_blocks / 4, (want + tiles - 1) / tiles, room}));   // a block per wave at least
+    a.splits = (uint32_t)std::max<uint64_t>(1, std::min<uint64_t>({max_blocks / 2, (want + tiles - 1) / tiles, room}));
     LH_REQUIRE(tiles * a.splits < 0x7FFFFFFFull && (uint64_t)a.rows * a.heads < 0x7FFFFFFFull, "%s: %u rows", op, a.rows);
     a.partial = (float*)ctx->workspace;
     if (lds > 64 * 1024) {
@@ -288,6 +282,78 @@ int launch_split(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const
     if (r != LH_OK) return r;
     launches = 2;
     return launch_merge<1>(ctx, a, op);
+}
+
+// Checks and arguments of an attention over cache rows; the output is the caller's.
+int latent_args(AttentionArgs& a, const char* op, const lh_buffer* q, const lh_buffer* cache, int dtype, const lh_buffer* position, uint32_t max_position,
+                uint32_t rows, uint32_t heads, uint32_t rank, uint32_t rot, uint32_t capacity, float scale, const lh_buffer* sink, const lh_buffer* gate) {
+    LH_REQUIRE(dtype == LH_F32 || dtype == LH_BF16, "%s: dtype %d", op, dtype);
+    LH_REQUIRE(heads > 0 && rank > 0 && rank <= 1024 && rot > 0 && rot <= 2048, "%s: heads %u, rank %u, rot %u", op, heads, rank, rot);
+    LH_REQUIRE(capacity > 0 && capacity % 32 == 0 && (uint64_t)max_position + rows <= capacity, "%s: positions up to %llu in caches of %u", op,
+               (unsigned long long)max_position + rows, capacity);
+    a = AttentionArgs{};
+    a.dv = padded_rank(rank);
+    a.dq = lh_latent_row(rank, rot);
+    LH_NEED(q, (size_t)rows * heads * a.dq * 4, op, "q");
+    LH_NEED(cache, (size_t)capacity * a.dq * (dtype == LH_F32 ? 4 : 2), op, "cache");
+    LH_NEED(position, 4, op, "position");
+    if (sink) { LH_NEED(sink, (size_t)heads * 4, op, "sink"); a.sink = (const float*)sink->ptr; }
+    if (gate) { LH_NEED(gate, (size_t)rows * heads * 4, op, "gate"); a.gate = (const float*)gate->ptr; }
+    a.q = q->ptr; a.keys = cache->ptr; a.values = cache->ptr; a.position = (const uint32_t*)position->ptr;
+    a.rows = rows; a.heads = heads; a.kv_heads = 1; a.maps = 1; a.dim = a.dq; a.vdim = rank; a.capacity = capacity; a.scale = scale; a.out_scale = 1.0f;
+    a.values_in_keys = 1;
+    return LH_OK;
+}
+bool tiled(const AttentionArgs& a, int dtype, uint32_t rot) {
+    return dtype == LH_BF16 && (((uintptr_t)a.q | (uintptr_t)a.keys) & 15) == 0 && rot <= kRotPad && a.dv <= 512;
+}
+int launch_tiled(lh_context* ctx, AttentionArgs& a, uint32_t max_position, const char* op, uint32_t& launches) {
+    if (a.dv == 64) return launch_split<64>(ctx, a, max_position, op, launches);
+    if (a.dv == 128) return launch_split<128>(ctx, a, max_position, op, launches);
+    if (a.dv == 256) return launch_split<256>(ctx, a, max_position, op, launches);
+    return launch_split<512>(ctx, a, max_position, op, launches);
+}
+
+int prepare_args(PrepareArgs& a, uint32_t& pieces, const char* op, const lh_buffer* q_rot, const lh_buffer* down, const lh_buffer* norm_weight,
+                 const lh_buffer* frequencies, const lh_buffer* position, lh_buffer* q, int q_dtype, lh_buffer* cache, int dtype, uint32_t rows, uint32_t heads,
+                 uint32_t rank, uint32_t rot, uint32_t q_ld, uint32_t rot_column, uint32_t clear_column, uint32_t capacity, float eps) {
+    LH_REQUIRE((dtype == LH_F32 || dtype == LH_BF16) && (q_dtype == LH_F32 || q_dtype == LH_BF16), "%s: dtypes %d, %d", op, q_dtype, dtype);
+    LH_REQUIRE(q_dtype == LH_F32 || dtype == LH_BF16, "%s: bf16 queries of an f32 cache", op);
+    LH_REQUIRE(heads > 0 && rank > 0 && rot > 0 && rot % 2 == 0, "%s: heads %u, rank %u, rot %u", op, heads, rank, rot);
+    LH_REQUIRE(clear_column <= rot_column && (uint64_t)rot_column + rot <= q_ld && (uint64_t)heads * q_ld < 0x7FFFFFFFull, "%s: columns %u and %u of %u", op,
+               clear_column, rot_column, q_ld);
+    const uint32_t row = lh_latent_row(rank, rot);
+    LH_NEED(q_rot, (size_t)rows * heads * rot * 4, op, "q_rot");
+    LH_NEED(frequencies, (size_t)(rot / 2) * 4, op, "frequencies");
+    LH_NEED(position, 4, op, "position");
+    LH_NEED(q, (size_t)rows * heads * q_ld * (q_dtype == LH_F32 ? 4 : 2), op, "q");
+    LH_NEED(cache, (size_t)capacity * row * (dtype == LH_F32 ? 4 : 2), op, "cache");
+    if (down) {
+        LH_NEED(down, (size_t)rows * (rank + rot) * 4, op, "down");
+        LH_NEED(norm_weight, (size_t)rank * 4, op, "norm_weight");
+    }
+    a = PrepareArgs{};
+    a.q_rot = (const float*)q_rot->ptr; a.down = down ? (const float*)down->ptr : nullptr; a.norm_weight = down ? (const float*)norm_weight->ptr : nullptr;
+    a.frequencies = (const float*)frequencies->ptr; a.position = (const uint32_t*)position->ptr; a.q = q->ptr; a.cache = cache->ptr;
+    a.heads = heads; a.rank = rank; a.dv = padded_rank(rank); a.rot = rot; a.row = row; a.q_ld = q_ld; a.rot_column = rot_column; a.clear_column = clear_column;
+    a.capacity = capacity; a.eps = eps;
+    const uint64_t parts = ((uint64_t)heads * (q_ld - clear_column) + 1023) / 1024;
+    LH_REQUIRE(parts < 65535, "%s: %u heads of %u columns", op, heads, q_ld);
+    pieces = (uint32_t)parts + 1;
+    return LH_OK;
+}
+int head_args(HeadArgs& a, const char* op, const lh_buffer* input, int dtype, const lh_buffer* weight, lh_buffer* output, int output_dtype, uint32_t rows,
+              uint32_t heads, uint32_t n, uint32_t k, uint32_t output_ld) {
+    LH_REQUIRE((dtype == LH_F32 && output_dtype == LH_F32) || (dtype == LH_BF16 && (output_dtype == LH_F32 || output_dtype == LH_BF16)), "%s: dtypes %d, %d", op, dtype,
+               output_dtype);
+    LH_REQUIRE(heads > 0 && heads < 65536 && n > 0 && k > 0 && output_ld >= n, "%s: %u heads of %u x %u into %u columns", op, heads, n, k, output_ld);
+    LH_REQUIRE(rows < 65536, "%s: %u rows", op, rows);
+    LH_NEED(input, (size_t)rows * heads * k * (dtype == LH_F32 ? 4 : 2), op, "input");
+    LH_NEED(weight, (size_t)heads * n * k * 2, op, "weight");
+    LH_NEED(output, (size_t)rows * heads * output_ld * (output_dtype == LH_F32 ? 4 : 2), op, "output");
+    a = HeadArgs{input->ptr, (const uint16_t*)weight->ptr, output->ptr, rows, heads, n, k, output_ld,
+                 k % 8 == 0 && (((uintptr_t)input->ptr | (uintptr_t)weight->ptr) & 15) == 0};
+    return LH_OK;
 }
 
 }  // namespace
@@ -302,34 +368,17 @@ int lh_latent_prepare_into(lh_batch* batch, const lh_buffer* q_rot, const lh_buf
                            uint32_t rot, uint32_t q_ld, uint32_t rot_column, uint32_t clear_column, uint32_t capacity, float eps) {
     const char* op = "latent_prepare";
     LH_REQUIRE(batch, "%s: batch is null", op);
-    LH_REQUIRE((dtype == LH_F32 || dtype == LH_BF16) && (q_dtype == LH_F32 || q_dtype == LH_BF16), "%s: dtypes %d, %d", op, q_dtype, dtype);
-    LH_REQUIRE(q_dtype == LH_F32 || dtype == LH_BF16, "%s: bf16 queries of an f32 cache", op);
-    LH_REQUIRE(heads > 0 && rank > 0 && rot > 0 && rot % 2 == 0, "%s: heads %u, rank %u, rot %u", op, heads, rank, rot);
-    LH_REQUIRE(clear_column <= rot_column && (uint64_t)rot_column + rot <= q_ld && (uint64_t)heads * q_ld < 0x7FFFFFFFull, "%s: columns %u and %u of %u", op,
-               clear_column, rot_column, q_ld);
     if (rows == 0) return LH_OK;
-    const uint32_t row = lh_latent_row(rank, rot);
-    LH_NEED(q_rot, (size_t)rows * heads * rot * 4, op, "q_rot");
-    LH_NEED(frequencies, (size_t)(rot / 2) * 4, op, "frequencies");
-    LH_NEED(position, 4, op, "position");
-    LH_NEED(q, (size_t)rows * heads * q_ld * (q_dtype == LH_F32 ? 4 : 2), op, "q");
-    LH_NEED(cache, (size_t)capacity * row * (dtype == LH_F32 ? 4 : 2), op, "cache");
-    if (down) {
-        LH_NEED(down, (size_t)rows * (rank + rot) * 4, op, "down");
-        LH_NEED(norm_weight, (size_t)rank * 4, op, "norm_weight");
-    }
-    PrepareArgs a{};
-    a.q_rot = (const float*)q_rot->ptr; a.down = down ? (const float*)down->ptr : nullptr; a.norm_weight = down ? (const float*)norm_weight->ptr : nullptr;
-    a.frequencies = (const float*)frequencies->ptr; a.position = (const uint32_t*)position->ptr; a.q = q->ptr; a.cache = cache->ptr;
-    a.heads = heads; a.rank = rank; a.dv = padded_rank(rank); a.rot = rot; a.row = row; a.q_ld = q_ld; a.rot_column = rot_column; a.clear_column = clear_column;
-    a.capacity = capacity; a.eps = eps;
-    const uint64_t parts = ((uint64_t)heads * (q_ld - clear_column) + 1023) / 1024;
-    LH_REQUIRE(parts < 65535, "%s: %u heads of %u columns", op, heads, q_ld);
-    const dim3 grid(rows, (uint32_t)parts + 1);
+    PrepareArgs a;
+    uint32_t pieces = 0;
+    int r = prepare_args(a, pieces, op, q_rot, down, norm_weight, frequencies, position, q, q_dtype, cache, dtype, rows, heads, rank, rot, q_ld, rot_column, clear_column,
+                         capacity, eps);
+    if (r != LH_OK) return r;
+    const dim3 grid(rows, pieces);
     if (dtype == LH_F32) hipLaunchKernelGGL((latent_prepare_kernel<float, float>), grid, dim3(256), 0, batch->ctx->stream, a);
     else if (q_dtype == LH_F32) hipLaunchKernelGGL((latent_prepare_kernel<float, uint16_t>), grid, dim3(256), 0, batch->ctx->stream, a);
     else hipLaunchKernelGGL((latent_prepare_kernel<uint16_t, uint16_t>), grid, dim3(256), 0, batch->ctx->stream, a);
-    const int r = lh_check_launch(op);
+    r = lh_check_launch(op);
     if (r == LH_OK) batch->dispatch_count++;
     return r;
 }
@@ -338,23 +387,17 @@ int lh_head_linear_into(lh_batch* batch, const lh_buffer* input, int dtype, cons
                         uint32_t heads, uint32_t n, uint32_t k, uint32_t output_ld) {
     const char* op = "head_linear";
     LH_REQUIRE(batch, "%s: batch is null", op);
-    LH_REQUIRE((dtype == LH_F32 && output_dtype == LH_F32) || (dtype == LH_BF16 && (output_dtype == LH_F32 || output_dtype == LH_BF16)), "%s: dtypes %d, %d", op, dtype,
-               output_dtype);
-    LH_REQUIRE(heads > 0 && heads < 65536 && n > 0 && k > 0 && output_ld >= n, "%s: %u heads of %u x %u into %u columns", op, heads, n, k, output_ld);
     if (rows == 0) return LH_OK;
-    LH_REQUIRE(rows < 65536, "%s: %u rows", op, rows);
-    LH_NEED(input, (size_t)rows * heads * k * (dtype == LH_F32 ? 4 : 2), op, "input");
-    LH_NEED(weight, (size_t)heads * n * k * 2, op, "weight");
-    LH_NEED(output, (size_t)rows * heads * output_ld * (output_dtype == LH_F32 ? 4 : 2), op, "output");
-    HeadArgs a{input->ptr, (const uint16_t*)weight->ptr, output->ptr, rows, heads, n, k, output_ld,
-               k % 8 == 0 && (((uintptr_t)input->ptr | (uintptr_t)weight->ptr) & 15) == 0};
+    HeadArgs a;
+    int r = head_args(a, op, input, dtype, weight, output, output_dtype, rows, heads, n, k, output_ld);
+    if (r != LH_OK) return r;
     if (dtype == LH_F32) hipLaunchKernelGGL(head_linear_plain_kernel, dim3((n + 3) / 4, heads, rows), dim3(256), 0, batch->ctx->stream, a);
     else {
         const dim3 grid((n + 15) / 16, heads, (rows + 15) / 16);
         if (output_dtype == LH_F32) hipLaunchKernelGGL((head_linear_mfma_kernel<float>), grid, dim3(256), 0, batch->ctx->stream, a);
         else hipLaunchKernelGGL((head_linear_mfma_kernel<uint16_t>), grid, dim3(256), 0, batch->ctx->stream, a);
     }
-    const int r = lh_check_launch(op);
+    r = lh_check_launch(op);
     if (r == LH_OK) batch->dispatch_count++;
     return r;
 }
@@ -403,39 +446,48 @@ int lh_latent_attention_rows_into(lh_batch* batch, const lh_buffer* q, const lh_
                                   const lh_buffer* sink, const lh_buffer* gate) {
     const char* op = "latent_attention_rows";
     LH_REQUIRE(batch, "%s: batch is null", op);
-    LH_REQUIRE(dtype == LH_F32 || dtype == LH_BF16, "%s: dtype %d", op, dtype);
-    LH_REQUIRE(heads > 0 && rank > 0 && rank <= 1024 && rot > 0 && rot <= 2048, "%s: heads %u, rank %u, rot %u", op, heads, rank, rot);
     if (rows == 0) return LH_OK;
-    LH_REQUIRE(capacity > 0 && capacity % 32 == 0 && (uint64_t)max_position + rows <= capacity, "%s: positions up to %llu in caches of %u", op,
-               (unsigned long long)max_position + rows, capacity);
-    const size_t es = dtype == LH_F32 ? 4 : 2;
-    AttentionArgs a{};
-    a.dv = padded_rank(rank);
-    a.dq = lh_latent_row(rank, rot);
-    LH_NEED(q, (size_t)rows * heads * a.dq * 4, op, "q");
-    LH_NEED(cache, (size_t)capacity * a.dq * es, op, "cache");
-    LH_NEED(output, (size_t)rows * heads * rank * es, op, "output");
-    LH_NEED(position, 4, op, "position");
-    if (sink) { LH_NEED(sink, (size_t)heads * 4, op, "sink"); a.sink = (const float*)sink->ptr; }
-    if (gate) { LH_NEED(gate, (size_t)rows * heads * 4, op, "gate"); a.gate = (const float*)gate->ptr; }
-    a.q = q->ptr; a.keys = cache->ptr; a.values = cache->ptr; a.out = output->ptr; a.position = (const uint32_t*)position->ptr;
-    a.rows = rows; a.heads = heads; a.kv_heads = 1; a.maps = 1; a.dim = a.dq; a.vdim = rank; a.capacity = capacity; a.scale = scale; a.out_scale = 1.0f;
-    a.values_in_keys = 1;
+    AttentionArgs a;
+    int r = latent_args(a, op, q, cache, dtype, position, max_position, rows, heads, rank, rot, capacity, scale, sink, gate);
+    if (r != LH_OK) return r;
+    LH_NEED(output, (size_t)rows * heads * rank * (dtype == LH_F32 ? 4 : 2), op, "output");
+    a.out = output->ptr;
     uint32_t launches = 1;
-    int r;
-    const bool aligned = (((uintptr_t)a.q | (uintptr_t)a.keys) & 15) == 0;
-    if (dtype == LH_BF16 && aligned && rot <= kRotPad && a.dv <= 512) {
-        if (a.dv == 64) r = launch_split<64>(batch->ctx, a, max_position, op, launches);
-        else if (a.dv == 128) r = launch_split<128>(batch->ctx, a, max_position, op, launches);
-        else if (a.dv == 256) r = launch_split<256>(batch->ctx, a, max_position, op, launches);
-        else r = launch_split<512>(batch->ctx, a, max_position, op, launches);
-    } else {
+    if (tiled(a, dtype, rot)) r = launch_tiled(batch->ctx, a, max_position, op, launches);
+    else {
         LH_REQUIRE((uint64_t)rows * heads < 0x7FFFFFFFull, "%s: %u rows", op, rows);
         if (dtype == LH_F32) hipLaunchKernelGGL((attention_plain_kernel<float, float>), dim3(rows * heads), dim3(256), (size_t)a.dim * 4, batch->ctx->stream, a);
         else hipLaunchKernelGGL((attention_plain_kernel<float, uint16_t>), dim3(rows * heads), dim3(256), (size_t)a.dim * 4, batch->ctx->stream, a);
         r = lh_check_launch(op);
     }
     batch->dispatch_count += launches;
+    return r;
+}
+
+int lh_latent_queries_into(lh_batch* batch, const lh_buffer* q, const lh_buffer* key_weight, const lh_buffer* q_rot, const lh_buffer* down,
+                           const lh_buffer* norm_weight, const lh_buffer* frequencies, const lh_buffer* position, lh_buffer* output, lh_buffer* cache, int dtype,
+                           uint32_t rows, uint32_t heads, uint32_t dim, uint32_t rank, uint32_t rot, uint32_t capacity, float eps) {
+    const char* op = "latent_queries";
+    LH_REQUIRE(batch, "%s: batch is null", op);
+    if (rows == 0) return LH_OK;
+    PrepareArgs p;
+    uint32_t pieces = 0;
+    const uint32_t row = lh_latent_row(rank, rot);
+    int r = prepare_args(p, pieces, op, q_rot, down, norm_weight, frequencies, position, output, LH_F32, cache, dtype, rows, heads, rank, rot, row, padded_rank(rank), rank,
+                         capacity, eps);
+    if (r != LH_OK) return r;
+    HeadArgs a;
+    r = head_args(a, op, q, dtype, key_weight, output, LH_F32, rows, heads, rank, dim, row);
+    if (r != LH_OK) return r;
+    const uint64_t tiles = (uint64_t)((rank + 15) / 16) * heads * ((rows + 15) / 16);
+    if (dtype == LH_F32 || tiles + (uint64_t)rows * pieces >= 0x7FFFFFFFull) {
+        r = lh_head_linear_into(batch, q, dtype, key_weight, output, LH_F32, rows, heads, rank, dim, row);
+        return r != LH_OK ? r : lh_latent_prepare_into(batch, q_rot, down, norm_weight, frequencies, position, output, LH_F32, cache, dtype, rows, heads, rank, rot, row,
+                                                       padded_rank(rank), rank, capacity, eps);
+    }
+    hipLaunchKernelGGL(latent_queries_kernel, dim3((uint32_t)tiles + rows * pieces), dim3(256), 0, batch->ctx->stream, a, p, (uint32_t)tiles, pieces);
+    r = lh_check_launch(op);
+    if (r == LH_OK) batch->dispatch_count++;
     return r;
 }
 

@@ -11,8 +11,9 @@ struct ConvArgs {
     const uint32_t* position;
     void *x, *b, *c;            // [rows, inner], [rows, groups, dq] twice
     uint32_t rows, channels, inner, groups, state, dq, taps;
+    uint32_t tile;              // rows of a workgroup, taps - 1 at least
 };
-constexpr uint32_t kConvRows = 32, kMaxTaps = 32;
+constexpr uint32_t kMaxTaps = 32;
 
 // Where channel ch of row t goes.
 template <typename T>
@@ -22,14 +23,13 @@ __device__ __forceinline__ T* conv_place(const ConvArgs& a, uint32_t ch, size_t 
     return static_cast<T*>(r < n ? a.b : a.c) + (t * a.groups + i / a.state) * a.dq + i % a.state;
 }
 
-// Thread = channel, workgroup = kConvRows rows.  Only the first rows' workgroup reads the ring, and it writes the ring
+// Thread = channel, workgroup = a.tile rows.  Only the first rows' workgroup reads the ring, and it writes the ring
 // afterwards (the inputs it keeps are those of the last rows, which nobody changes).  TAPS 0: any number.
 template <typename T, int TAPS>
 __global__ __launch_bounds__(256) void conv_rows_kernel(const ConvArgs a) {
-    const uint32_t ch = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * kConvRows, t1 = min(t0 + kConvRows, a.rows);
-    const uint32_t n = a.groups * a.state, padding = a.dq - a.state;
+    const uint32_t ch = blockIdx.x * 256 + threadIdx.x, t0 = blockIdx.y * a.tile, t1 = min(t0 + a.tile, a.rows);
     if (ch >= a.channels) {                                   // the threads behind the channels clear the padding of B and C
-        const uint32_t i = ch - a.channels;
+        const uint32_t i = ch - a.channels, padding = a.dq - a.state;
         if (i < 2 * a.groups * padding) {
             T* d = static_cast<T*>(i < a.groups * padding ? a.b : a.c);
             const uint32_t j = i % (a.groups * padding);
@@ -37,7 +37,6 @@ __global__ __launch_bounds__(256) void conv_rows_kernel(const ConvArgs a) {
         }
         return;
     }
-    (void)n;
     const uint32_t taps = TAPS ? TAPS : a.taps, pos0 = *a.position;
     const T* in = static_cast<const T*>(a.input) + ch;
     auto value = [&](int64_t t) {                             // the input of row t, rows before this portion from the ring
@@ -172,7 +171,8 @@ int lh_selective_conv_into(lh_batch* batch, const lh_buffer* input, int dtype, l
     LH_NEED(b, (size_t)rows * groups * a.dq * es, op, "b");
     LH_NEED(c, (size_t)rows * groups * a.dq * es, op, "c");
     a.x = x->ptr; a.b = b->ptr; a.c = c->ptr;
-    const uint32_t threads = a.channels + 2 * groups * (a.dq - state), tiles = (rows + kConvRows - 1) / kConvRows;
+    a.tile = taps > 17 ? 32 : 16;
+    const uint32_t threads = a.channels + 2 * groups * (a.dq - state), tiles = (rows + a.tile - 1) / a.tile;
     LH_REQUIRE(tiles < 65536, "%s: %u rows", op, rows);
     const dim3 grid((threads + 255) / 256, tiles);
 #define LH_CONV(T, N) hipLaunchKernelGGL((conv_rows_kernel<T, N>), grid, dim3(256), 0, batch->ctx->stream, a)

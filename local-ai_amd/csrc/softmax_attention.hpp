@@ -67,15 +67,15 @@ __device__ __forceinline__ float softmax_step(lh_f32x4 (&s)[2 * NB], RowState& s
     return alpha;
 }
 
-// One workgroup per (query row, head): merges the splits of every map, combines the maps, norms and stores.  Groups of dv / 4
-// threads take the splits in turn, four values a thread, several loads on their way; the groups are added through LDS.
+// Merges the splits of every map of one (query row, head) in columns col0 .. col0 + cols - 1 (cols a multiple of 4, at most 512):
+// thread i returns column col0 + i, the maps combined (no norm, no gate).  Groups of cols / 4 threads take the splits in turn,
+// four values a thread, several loads on their way; the groups are added through LDS.
 constexpr uint32_t kMergeThreads = 512;
 template <int MAPS>
-__global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const AttentionArgs a) {
-    __shared__ float factor[MAPS][512], total[MAPS], scratch[kMergeThreads / 64];
-    __shared__ float4 sums[MAPS][kMergeThreads];
-    const uint32_t part = blockIdx.x % a.parts, th = blockIdx.x / a.parts, t = th / a.heads, h = th % a.heads, R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
-    const uint32_t cols = a.dv / a.parts, col0 = part * cols;
+struct MergeSpace { float factor[MAPS][512], total[MAPS]; float4 sums[MAPS][kMergeThreads]; };
+template <int MAPS>
+__device__ __forceinline__ float merge_columns(const AttentionArgs& a, uint32_t t, uint32_t h, uint32_t col0, uint32_t cols, MergeSpace<MAPS>& sp) {
+    const uint32_t R = a.heads / a.kv_heads, g = h / R, row = t * R + h % R;
     const uint32_t kRow = a.dv + 4, rr = row & 15;
     const size_t stride = (size_t)MAPS * 16 * kRow;
     const float* rec = a.partial + (size_t)(((row >> 4) * a.kv_heads + g) * a.splits) * stride + rr * kRow;
@@ -98,11 +98,11 @@ __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const At
         for (uint32_t i = 0; i < 8; i++) {
             if (i * 64 >= a.splits) break;
             const float f = __builtin_amdgcn_exp2f(mine[i] - m);
-            if (i * 64 + lane < a.splits) factor[wave][i * 64 + lane] = f;
+            if (i * 64 + lane < a.splits) sp.factor[wave][i * 64 + lane] = f;
             l += f * ml[i];
         }
         l = lh_group_sum(l, 64) + __builtin_amdgcn_exp2f(sink - m);
-        if (lane == 0) total[wave] = 1.0f / l;
+        if (lane == 0) sp.total[wave] = 1.0f / l;
     }
     __syncthreads();
     const uint32_t quads = cols / 4, groups = kMergeThreads / quads, grp = threadIdx.x / quads, q = threadIdx.x % quads;   // quads <= 128
@@ -114,27 +114,36 @@ __global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const At
 #pragma unroll
         for (int mp = 0; mp < MAPS; mp++) {
             const float4 x = *reinterpret_cast<const float4*>(rec + s * stride + mp * 16 * kRow + col0 + q * 4);
-            const float f = factor[mp][s];
+            const float f = sp.factor[mp][s];
             acc[mp].x += f * x.x; acc[mp].y += f * x.y; acc[mp].z += f * x.z; acc[mp].w += f * x.w;
         }
 #pragma unroll
-    for (int mp = 0; mp < MAPS; mp++) sums[mp][threadIdx.x] = acc[mp];
+    for (int mp = 0; mp < MAPS; mp++) sp.sums[mp][threadIdx.x] = acc[mp];
     __syncthreads();
     float v = 0.0f;
-    const uint32_t d = col0 + threadIdx.x;                    // dv <= 512
-    const bool on = threadIdx.x < cols && d < a.vdim;
-    if (on) {
+    if (threadIdx.x < cols && col0 + threadIdx.x < a.vdim) {
         float s[MAPS] = {};
         for (uint32_t i = 0; i < groups; i++)
 #pragma unroll
-            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sums[mp][i * quads])[threadIdx.x];
-        v = s[0] * total[0];
-        if constexpr (MAPS == 2) v -= a.lambda * (s[MAPS - 1] * total[MAPS - 1]);
+            for (int mp = 0; mp < MAPS; mp++) s[mp] += reinterpret_cast<const float*>(&sp.sums[mp][i * quads])[threadIdx.x];
+        v = s[0] * sp.total[0];
+        if constexpr (MAPS == 2) v -= a.lambda * (s[MAPS - 1] * sp.total[MAPS - 1]);
     }
+    return v;
+}
+
+// One workgroup per (query row, head) and part of the columns: merges, norms or gates, and stores.
+template <int MAPS>
+__global__ __launch_bounds__(kMergeThreads) void attention_merge_kernel(const AttentionArgs a) {
+    __shared__ MergeSpace<MAPS> space;
+    __shared__ float scratch[kMergeThreads / 64];
+    const uint32_t part = blockIdx.x % a.parts, th = blockIdx.x / a.parts, t = th / a.heads, h = th % a.heads;
+    const uint32_t cols = a.dv / a.parts, d = part * cols + threadIdx.x;
+    const float v = merge_columns<MAPS>(a, t, h, part * cols, cols, space);
     float f = 1.0f;
     if constexpr (MAPS == 2) f = rsqrtf(lh_block_sum(v * v, scratch) / (float)a.vdim + a.eps) * a.out_scale;
     if (MAPS == 1 && a.gate) f = lh_sigmoid(a.gate[(size_t)t * a.heads + h]);
-    if (on) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
+    if (threadIdx.x < cols && d < a.vdim) static_cast<uint16_t*>(a.out)[((size_t)t * a.heads + h) * a.vdim + d] = lh_f2bf(v * f);
 }
 
 template <int MAPS>

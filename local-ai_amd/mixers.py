@@ -24,6 +24,7 @@ from .linear_weight import Segment, Segments, StackedLinear
 CHUNK = 64                 # rows per chunk of lh_linear_attention_chunked_into and lh_selective_chunked_into
 CHUNKED_MIN_ROWS = 17      # below this a portion walks the recurrence
 MAX_CHUNKED_DIM = 256
+GATED_IN_PRODUCT = 2048    # longer gated norms are a step of their own: every wave of the product would repeat them
 EXPANDED_MIN_ROWS = 65     # from here on latent attention makes keys and values of every head out of its cache
 
 
@@ -226,7 +227,7 @@ class LatentAttention:
             raise InvalidArgument(f"{s.rot_dim} rotated dimensions do not make pairs")
         self.eps, self.source = eps, s.kv_from
         H, d, e, r = s.heads, s.dim, s.rot_dim, s.kv_rank
-        self.row, self.rot_column = kernels.latent_row(r, e), kernels.latent_padded_rank(r)
+        self.row = kernels.latent_row(r, e)
         self.dq, self.dv = kernels.attention_padded_dim(d + e), kernels.attention_padded_vdim(s.vdim)
         q = tensors.bf16(prefix + "q", (H * (d + e), width)).reshape(H, d + e, width)
         weights = [np.ascontiguousarray(q[:, :d]).reshape(H * d, width), np.ascontiguousarray(q[:, d:]).reshape(H * e, width),
@@ -259,12 +260,9 @@ class LatentAttention:
         q = r.scratch("q", n * H * (self.dq if expanded else s.dim))
         norm.project(r, self.qkvg, [q, q_rot, gate] + ([down] if down else []), r.dtype, self.padded if expanded else None)
         mixed = r.scratch("mixed", n * H * s.vdim)
-
-        def prepare(queries, dtype, ld, rot_column, clear_column):
-            K.latent_prepare_into(b, q_rot, down, self.latent_norm, self.frequencies, r.position, queries, dtype, memory.rows, r.dtype, n,
-                                  H, s.kv_rank, s.rot_dim, ld, rot_column, clear_column, memory.capacity, self.eps)
         if expanded:
-            prepare(q, r.dtype, self.dq, s.dim, s.dim)
+            K.latent_prepare_into(b, q_rot, down, self.latent_norm, self.frequencies, r.position, q, r.dtype, memory.rows, r.dtype, n, H,
+                                  s.kv_rank, s.rot_dim, self.dq, s.dim, s.dim, memory.capacity, self.eps)
             positions = (r.max_position + n + 31) // 32 * 32
             keys, values = r.scratch("latent.keys", positions * H * self.dq), r.scratch("latent.values", positions * H * self.dv)
             K.latent_expand_into(b, memory.rows, r.dtype, self.up, keys, values, positions, H, s.dim, s.rot_dim, s.vdim, s.kv_rank)
@@ -272,8 +270,8 @@ class LatentAttention:
                                   positions, s.scale, sink=self.sink, gate=gate)
         else:
             ql = r.scratch("latent.q", n * H * self.row, f32=True)
-            prepare(ql, F32, self.row, self.rot_column, s.kv_rank)
-            K.head_linear_into(b, q, r.dtype, self.key_up, ql, F32, n, H, s.kv_rank, s.dim, self.row)
+            K.latent_queries_into(b, q, self.key_up, q_rot, down, self.latent_norm, self.frequencies, r.position, ql, memory.rows, r.dtype,
+                                  n, H, s.dim, s.kv_rank, s.rot_dim, memory.capacity, self.eps)
             ol = r.scratch("latent.out", n * H * s.kv_rank)
             K.latent_attention_rows_into(b, ql, memory.rows, ol, r.dtype, r.position, r.max_position, n, H, s.kv_rank, s.rot_dim,
                                          memory.capacity, s.scale, self.sink, gate)
@@ -298,7 +296,7 @@ def finish_gated(r: Run, norm: Norm, out: StackedLinear, o: Buffer, gate: Buffer
                  act: int, gate_first: bool) -> None:
     """Norm in parts of `group` values and gate of o (f32), then the branch's last product."""
     K, b, k = r.kernels, r.batch, out.k
-    if r.rows == 1 and K.gated_vector_fits(k, group):
+    if r.rows == 1 and k <= GATED_IN_PRODUCT and K.gated_vector_fits(k, group):
         dest, add = norm.destination(r)
         K.linear_gated_vector_into(b, o, gate, gate_dtype, weight, eps, out.weight, None, k, out.segments, [dest], F32, add, None, group,
                                    act, gate_first)
@@ -436,20 +434,12 @@ class GatedFeedForward:
         self.spec = spec
         gate, up = tensors.bf16(prefix + "gate", (spec.ff, width)), tensors.bf16(prefix + "up", (spec.ff, width))
         self.up = StackedLinear(ctx, [np.stack([gate, up], 1).reshape(2 * spec.ff, width)], [Segment(2 * spec.ff, ACT_SILU_PAIRS)])
-        self.plain = Segments([Segment(2 * spec.ff)])
         self.down = StackedLinear(ctx, [tensors.bf16(prefix + "down", (width, spec.ff))], [Segment(width)])
 
     def run(self, r: Run, norm: Norm) -> None:
-        ff = self.spec.ff
-        if r.rows == 1:
-            h = r.scratch("pairs", 2 * ff, f32=True)
-            norm.project(r, self.up, [h], F32, self.plain)
-            dest, add = norm.destination(r)
-            r.kernels.linear_pairs_vector_into(r.batch, h, self.down.weight, None, ff, self.down.segments, [dest], F32, add)
-        else:
-            h = r.scratch("hidden", r.rows * ff)
-            norm.project(r, self.up, [h], r.dtype)
-            norm.finish(r, self.down, h, r.dtype)
+        h = r.scratch("hidden", r.rows * self.spec.ff)
+        norm.project(r, self.up, [h], r.dtype)
+        norm.finish(r, self.down, h, r.dtype)
 
 
 @dataclass

@@ -92,4 +92,4 @@ def vifivik(config: dict) -> StackConfig:
         raise InvalidArgument(f"unknown feed-forward {f['kind']!r}")
 
     layers = [LayerSpec(mixer(l["type"], l["mixer"]), feed_forward(l.get("mlp"))) for l in config["layers"]]
-    return StackConfig(config["vocab"], config["width"], config["norm"]["eps"], layers, layer=OutputNormLayer, softcap=config["logit_softcap"])
+    return StackConfig(config["vocab"], config["width"], config["norm"]["eps"], layers, layer=OutputNormLayer, softcap=config.get("logit_softcap"))

@@ -126,6 +126,26 @@ def latent_case(ai, gpu, dtype, heads, rank, rot, start, rows, capacity, spike=N
 
 
 @pytest.mark.parametrize("dtype", ["bf16", "f32"])
+@pytest.mark.parametrize("rows,heads,dim,rank,rot,own", [(1, 1, 3, 5, 2, True), (1, 6, 64, 128, 16, False), (1, 16, 128, 512, 64, True), (40, 3, 40, 96, 20, True)])
+def test_latent_queries_equal_the_two_steps(ai, gpu, dtype, rows, heads, dim, rank, rot, own):
+    ctx, K = gpu
+    dt, g = ai.BF16 if dtype == "bf16" else ai.F32, np.random.default_rng(rank)
+    row, dv, start = K.latent_row(rank, rot), K.latent_padded_rank(rank), 17
+    q, uk = upload(ai, ctx, g.standard_normal((rows, heads, dim)), dt), ai.Buffer.from_slice(ctx, M.bf16_bits(g.standard_normal((heads, rank, dim))))
+    qr, down, nw = f32(ai, ctx, g.standard_normal((rows, heads, rot))), f32(ai, ctx, g.standard_normal((rows, rank + rot))) if own else None, f32(ai, ctx, g.standard_normal(rank))
+    freq, pos, batch = f32(ai, ctx, 30.0 ** -np.arange(rot // 2)), ai.Buffer.from_slice(ctx, np.array([start], np.uint32)), ai.CommandBatch(ctx)
+    caches, outs = [empty(ai, ctx, 64 * row, dt) for _ in range(2)], [empty(ai, ctx, rows * heads * row, ai.F32) for _ in range(2)]
+    K.latent_prepare_into(batch, qr, down, nw, freq, pos, outs[0], ai.F32, caches[0], dt, rows, heads, rank, rot, row, dv, rank, 64, 1e-5)
+    K.head_linear_into(batch, q, dt, uk, outs[0], ai.F32, rows, heads, rank, dim, row)
+    K.latent_queries_into(batch, q, uk, qr, down, nw, freq, pos, outs[1], caches[1], dt, rows, heads, dim, rank, rot, 64, 1e-5)
+    batch.commit_and_wait()
+    for a, b, t in ((*caches, dt), (*outs, ai.F32)):
+        n = 64 * row if a is caches[0] else rows * heads * row
+        assert np.array_equal(download(ai, a, n, t), download(ai, b, n, t))
+    assert own == bool(download(ai, caches[1], 64 * row, dt).any())
+
+
+@pytest.mark.parametrize("dtype", ["bf16", "f32"])
 @pytest.mark.parametrize("heads,rank,rot", [(1, 3, 2), (5, 64, 8), (3, 100, 64), (16, 160, 32), (17, 512, 64), (2, 300, 20), (2, 70, 72), (2, 600, 16)])
 @pytest.mark.parametrize("start,rows", [(0, 1), (31, 1), (32, 2), (95, 34), (0, 64), (600, 1)])
 def test_latent_attention_shapes(ai, gpu, dtype, heads, rank, rot, start, rows):
@@ -193,7 +213,7 @@ def test_softmax_attention_with_sink_and_gate(ai, gpu, dtype, heads, kv_heads, d
 
 
 # ---- selective state space --------------------------------------------------------------------------------------------------
-@pytest.mark.parametrize("heads,vdim,state,groups,taps", [(1, 3, 5, 1, 1), (4, 24, 20, 2, 4), (3, 33, 64, 3, 2), (2, 64, 128, 1, 3), (6, 16, 130, 2, 6), (2, 20, 300, 1, 4)])
+@pytest.mark.parametrize("heads,vdim,state,groups,taps", [(1, 3, 5, 1, 1), (4, 24, 20, 2, 4), (3, 33, 64, 3, 2), (2, 64, 128, 1, 3), (6, 16, 130, 2, 6), (2, 20, 300, 1, 4), (2, 8, 12, 1, 20)])
 @pytest.mark.parametrize("cuts", [[1, 1, 1, 1, 1], [2, 2, 1, 2], [17, 1, 65, 2, 130], [63, 1, 64, 1], [200]])
 def test_selective_state_space(ai, gpu, heads, vdim, state, groups, taps, cuts):
     """The kernels from the projections to the recurrence's output, in portions, and the states left behind: all f32, and bf16
@@ -331,30 +351,43 @@ def test_norm_behind_a_branch(ai, gpu, dtype, dim):
 def test_gate_and_up_in_one_product(ai, gpu, dtype, m, k, n):
     ctx, K = gpu
     dt, g, L = ai.BF16 if dtype == "bf16" else ai.F32, np.random.default_rng(m + n), ai.linear_weight
-    x, a, b, d = stored(g.standard_normal((m, k)), ai, dt), *(M.rounded(g.standard_normal(s) / np.sqrt(s[1])) for s in ((n, k), (n, k), (11, n)))
+    x, a, b = stored(g.standard_normal((m, k)), ai, dt), *(M.rounded(g.standard_normal((n, k)) / np.sqrt(k)) for _ in range(2))
     want = O.silu(x @ a.T) * (x @ b.T)
     both = M.bf16_bits(np.stack([a, b], 1).reshape(2 * n, k))
     lin, h, batch = L.StackedLinear(ctx, [both], [L.Segment(2 * n, ai.ACT_SILU_PAIRS)]), empty(ai, ctx, m * n, dt), ai.CommandBatch(ctx)
     lin.rows_into(batch, K, upload(ai, ctx, x, dt), dt, m, [h], dt)
-    down, raw, y = L.StackedLinear(ctx, [M.bf16_bits(d)], [L.Segment(11)]), empty(ai, ctx, 2 * n, ai.F32), empty(ai, ctx, 11, ai.F32)
-    lin.vector_into(batch, K, upload(ai, ctx, x[0], dt), dt, [raw], ai.F32, segments=L.Segments([L.Segment(2 * n)]))
-    K.linear_pairs_vector_into(batch, raw, down.weight, None, n, down.segments, [y], ai.F32)
     batch.commit_and_wait()
     close(download(ai, h, m * n, dt).reshape(m, n), want, F32_TOL if dt == ai.F32 else BF16_TOL)
-    close(download(ai, y, 11, ai.F32), want[0] @ d.T, F32_TOL, "one row")
-    with pytest.raises(ai.InvalidArgument):
-        lin.vector_into(batch, K, upload(ai, ctx, x[0], dt), dt, [raw], ai.F32)
 
 
-@pytest.mark.parametrize("n", [24, 4096, 6000, 16384, 20008])
-def test_gated_vector_of_every_length(ai, gpu, n):
+@pytest.mark.parametrize("dtype", ["bf16", "f32"])
+@pytest.mark.parametrize("k,n", [(64, 1), (13, 5), (512, 33), (2048, 3000), (4096, 70), (4100, 40), (5000, 1500), (16384, 9), (20008, 17)])
+def test_gate_and_up_of_one_row(ai, gpu, dtype, k, n):
     ctx, K = gpu
-    g, L = np.random.default_rng(n), ai.linear_weight
-    raw, d = g.standard_normal((n, 2)).astype(np.float32), M.rounded(g.standard_normal((9, n)) / np.sqrt(n))
-    down, y, batch = L.StackedLinear(ctx, [M.bf16_bits(d)], [L.Segment(9)]), empty(ai, ctx, 9, ai.F32), ai.CommandBatch(ctx)
-    K.linear_pairs_vector_into(batch, f32(ai, ctx, raw), down.weight, None, n, down.segments, [y], ai.F32)
+    g, L, dt = np.random.default_rng(n), ai.linear_weight, ai.BF16 if dtype == "bf16" else ai.F32
+    x, a, b = stored(g.standard_normal(k), ai, dt), *(M.rounded(g.standard_normal((n, k)) / np.sqrt(k)) for _ in range(2))
+    y, w, s = g.standard_normal(k).astype(np.float32), np.ones(k, np.float32), empty(ai, ctx, k, ai.F32)
+    lin = L.StackedLinear(ctx, [M.bf16_bits(np.stack([a, b], 1).reshape(2 * n, k))], [L.Segment(2 * n, ai.ACT_SILU_PAIRS)])
+    outs, batch = [empty(ai, ctx, n, ai.F32), empty(ai, ctx, n, ai.BF16), empty(ai, ctx, n, ai.F32)], ai.CommandBatch(ctx)
+    xb = upload(ai, ctx, x, dt)
+    lin.vector_into(batch, K, xb, dt, [outs[0]], ai.F32)
+    lin.vector_into(batch, K, xb, dt, [outs[1]], ai.BF16)
+    lin.residual_vector_into(batch, K, f32(ai, ctx, x), f32(ai, ctx, y), s, f32(ai, ctx, w), 1e-5, [outs[2]], ai.F32)
     batch.commit_and_wait()
-    close(download(ai, y, 9, ai.F32), (O.silu(raw[:, 0].astype(np.float64)) * raw[:, 1]) @ d.T, F32_TOL)
+    want = O.silu(a @ x) * (b @ x)
+    close(download(ai, outs[0], n, ai.F32), want, F32_TOL)
+    close(download(ai, outs[1], n, ai.BF16), want, BF16_TOL)
+    x = x + O.unit_rms(y.astype(np.float64), 1e-5)
+    close(download(ai, outs[2], n, ai.F32), O.silu(a @ x) * (b @ x), F32_TOL, "behind a normed branch")
+
+
+def test_pairs_stand_alone_in_a_product_of_one_row(ai, gpu):
+    ctx, K = gpu
+    L, b, batch = ai.linear_weight, ai.Buffer.empty(ctx, 4096), ai.CommandBatch(ctx)
+    with pytest.raises(ai.InvalidArgument):
+        K.linear_vector_into(batch, b, ai.F32, b, None, 8, L.Segments([L.Segment(8, ai.ACT_SILU_PAIRS), L.Segment(8)]), [b, b], ai.F32)
+    with pytest.raises(ai.InvalidArgument):
+        K.linear_vector_into(batch, b, ai.F32, b, None, 8, L.Segments([L.Segment(7, ai.ACT_SILU_PAIRS)]), [b], ai.F32)
 
 
 def test_destinations_of_mixed_types(ai, gpu):
