@@ -63,9 +63,6 @@ class StackedLinear:
     def rows_add_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, m: int, residual: Buffer) -> None:
         kernels.linear_rows_into(batch, x, x_dtype, self.weight, self.bias, m, self.k, self.segments, [residual], F32, True)
 
-    def vector_add_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, residual: Buffer) -> None:
-        kernels.linear_vector_into(batch, x, x_dtype, self.weight, self.bias, self.k, self.segments, [residual], F32, True)
-
     def vector_into(self, batch, kernels: Kernels, x: Buffer, x_dtype: int, outputs, dtype: int, position=None,
                     segments: Optional[Segments] = None) -> None:
         kernels.linear_vector_into(batch, x, x_dtype, self.weight, self.bias, self.k, segments or self.segments, outputs, dtype,

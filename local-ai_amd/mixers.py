@@ -91,7 +91,7 @@ class Norm:
         linear.normed_vector_into(r.batch, r.kernels, x, self.weight, self.eps, outputs, dtype, r.position, add, store)
 
     def project(self, r: Run, linear: StackedLinear, outputs, dtype: int, segments: Optional[Segments] = None) -> None:
-        """The branch's first product.  For one row an f32 run may ask for f32 outputs whatever the run's dtype."""
+        """The branch's first product; `dtype` is that of the outputs, `segments` overrides where they go."""
         if r.rows == 1:
             x, add, store = r.take_input()
             linear.normed_vector_into(r.batch, r.kernels, x, self.weight, self.eps, outputs, dtype, r.position, add, store, segments)
